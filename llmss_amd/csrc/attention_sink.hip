@@ -19,6 +19,12 @@
 // sequence); `vshare` > 1 lets that many neighbouring key heads read one value head (the value cache then holds
 // G / vshare heads) - differential attention caches the two maps of a key head as two key heads over one value head.
 //
+// `window` > 0: position i sees the keys j <= i with i - j < window or j < keep (the first `keep` positions stay
+// visible for good). `sinks` [H]: the unit in the denominator becomes exp(sinks[h]), a learned number per head. What a
+// workgroup's rows see is ONE list of keys - the kept positions before the window of its first row, then the positions from
+// there on - walked in blocks whatever they are. `vcs` [T, vdim / 2, 2] = (cos, sin): every head's result at a row is
+// turned back by the row's angles, pairs (c, c + vdim / 2) - for caches whose values were rotated by their positions.
+//
 // One kernel serves portions of prompts, continued portions and single decoded tokens: a row finds its sequence and
 // position through cu / ctx_lens and reads every key, those of its own step too, from the paged cache.
 // Scores, softmax and sums are fp32; the cache is read in the model's storage type.
@@ -91,7 +97,8 @@ __global__ void sink_attn_kernel(const float* __restrict__ q, const T* __restric
                                  const int* __restrict__ bt, int maxb, const int* __restrict__ cu,
                                  const int* __restrict__ ctx, float* __restrict__ out, int B, int H, int G, int dim,
                                  int vdim, int bs, float scale, float cap, int all, int KB, int Dp, int hchunks,
-                                 int RVchunk, int sink, int chunk, int vshare) {
+                                 int RVchunk, int sink, int chunk, int vshare, const float* __restrict__ sinks,
+                                 int window, int keep) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   T* tile = reinterpret_cast<T*>(smem);
   float* qs = reinterpret_cast<float*>(smem + (((size_t)KB * Dp * sizeof(T) + 15) & ~(size_t)15));
@@ -131,15 +138,19 @@ __global__ void sink_attn_kernel(const float* __restrict__ q, const T* __restric
 #pragma unroll
     for (int i = 0; i < NR2; ++i) acc[hh][i] = 0.f;
   // the sink: score 0, weight exp(0 - m), no value; without it the first block of keys sets the maximum
-  float m = sink ? 0.f : -INFINITY, l = sink ? 1.f : 0.f;
+  float m = sink ? (sinks && live ? sinks[h] : 0.f) : -INFINITY, l = sink ? 1.f : 0.f;
   const float icap = cap > 0.f ? 1.0f / cap : 0.f;
   const int* btr = bt + (int64_t)r.b * maxb;
   const int c0 = wv * cs + lane;  // this lane's first column within the chunk
-  for (int j0 = chunk > 0 ? (r.pos / chunk) * chunk : 0; j0 <= r.pos; j0 += KB) {
-    const int nk = min(KB, r.pos - j0 + 1);
+  const int jlo = max(chunk > 0 ? (r.pos / chunk) * chunk : 0, window > 0 ? r.pos - window + 1 : 0);
+  const int nkp = window > 0 ? min(keep, jlo) : 0;  // kept positions before the window
+  const int total = nkp + r.pos - jlo + 1;
+  for (int u0 = 0; u0 < total; u0 += KB) {
+    const int nk = min(KB, total - u0);
     __syncthreads();
     for (int kk = threadIdx.x; kk < nk; kk += blockDim.x) {
-      const int j = j0 + kk;
+      const int u = u0 + kk;
+      const int j = u < nkp ? u : jlo + (u - nkp);
       srow[kk] = (int64_t)btr[j / bs] * bs + j % bs;
     }
     __syncthreads();
@@ -238,7 +249,8 @@ __global__ void sink_attn_kernel(const float* __restrict__ q, const T* __restric
 template <typename T>
 static void sink_attn_t(const void* q, const void* kc, const void* vc, const void* bt, int maxb, const void* cu,
                         const void* ctx, void* out, int T_, int B, int H, int G, int dim, int vdim, int bs,
-                        float scale, float cap, int all, int sink, int chunk, int vshare, hipStream_t st) {
+                        float scale, float cap, int all, int sink, int chunk, int vshare, const void* sinks, int window,
+                        int keep, hipStream_t st) {
   const int rep = H / G;
   const int NW = rep >= 8 ? 8 : (rep > 2 ? 4 : rep);  // waves = heads per workgroup: 1, 2, 4 or 8
   const int hchunks = (rep + NW - 1) / NW;
@@ -268,7 +280,8 @@ static void sink_attn_t(const void* q, const void* kc, const void* vc, const voi
 #define LAUNCH_SA1(NW_, NR_, WD_)                                                                            \
   sink_attn_kernel<T, NW_, NR_, WD_><<<g, NW_ * 64, bytes(KB), st>>>(                                        \
       (const float*)q, (const T*)kc, (const T*)vc, (const int*)bt, maxb, (const int*)cu, (const int*)ctx,    \
-      (float*)out, B, H, G, dim, vdim, bs, scale, cap, all, KB, Dp, hchunks, RVchunk, sink, chunk, vshare)
+      (float*)out, B, H, G, dim, vdim, bs, scale, cap, all, KB, Dp, hchunks, RVchunk, sink, chunk, vshare, \
+      (const float*)sinks, window, keep)
 #define LAUNCH_SA(NW_, NR_)               \
   do {                                    \
     if (words) LAUNCH_SA1(NW_, NR_, true); \
@@ -294,17 +307,19 @@ static void sink_attn_t(const void* q, const void* kc, const void* vc, const voi
 
 void launch_sink_attn(const void* q, const void* kc, const void* vc, const void* bt, int maxb, const void* cu,
                       const void* ctx, void* out, int T_, int B, int H, int G, int dim, int vdim, int bs, float scale,
-                      float cap, int all, int sink, int chunk, int vshare, int dt, hipStream_t st) {
+                      float cap, int all, int sink, int chunk, int vshare, const void* sinks, int window, int keep,
+                      int dt, hipStream_t st) {
   if (T_ == 0 || B == 0) return;
   if (G < 1 || H % G) throw std::runtime_error("sink attention: heads must be a multiple of the key/value heads");
-  if (vshare < 1 || G % vshare || chunk < 0) throw std::runtime_error("sink attention: bad vshare / chunk");
+  if (vshare < 1 || G % vshare || chunk < 0 || window < 0 || keep < 0)
+    throw std::runtime_error("sink attention: bad vshare / chunk / window");
   DISPATCH_T(dt, T, (sink_attn_t<T>(q, kc, vc, bt, maxb, cu, ctx, out, T_, B, H, G, dim, vdim, bs, scale, cap, all,
-                                    sink, chunk, vshare, st)));
+                                    sink, chunk, vshare, sinks, window, keep, st)));
   HIP_CHECK_LAUNCH();
 }
 
-// The same attention on the matrix cores, for portions of bf16 prompts (key size 32, 64 or 128, value size a
-// multiple of 8). One workgroup serves one key/value group, GE of its query heads and 64 * NS / GE query rows of one
+// The same attention on the matrix cores, over bf16 pages (key size 32, 64 or 128, or with split operands any multiple
+// of 8 up to 128, staged with zeros behind it; value size a multiple of 8). One workgroup serves one key/value group, GE of its query heads and 64 * NS / GE query rows of one
 // sequence: its 64 * NS "slots" enumerate (row, head) pairs, slot s -> row s / GE, head s % GE, so a key tile is
 // staged in LDS once for the whole head group. A wave owns NS groups of 16 neighbouring slots; per group the
 // products are the swapped ones,
@@ -321,12 +336,26 @@ void launch_sink_attn(const void* q, const void* kc, const void* vc, const void*
 // PRECISE: the fp32 queries and the fp32 softmax weights enter the products as the sum of two bf16 numbers (the
 // rounded value and the rounded remainder, two matrix instructions each), so scores and weighted sums are those of
 // 32-bit queries and weights; otherwise both are rounded to bf16 once.
+// nsplit > 1 (steps of single rows): a row's list of keys is cut into nsplit runs of whole tiles, each walked by a
+// workgroup of its own that leaves its sums, maximum and denominator (no sink) in po / pml; attn_finish joins them.
+struct SinkExt {
+  int dim;     // numbers per cached key (<= DK)
+  int window, keep;
+  const float* sinks;
+  int nsplit;
+  float* po;       // [nsplit][rows][H][RVtot], addressed by the step's row numbers (the base is shifted)
+  float* pml;      // [nsplit][rows][H][2]
+  int64_t prows;   // rows * H
+  const float* vcs;  // direct: the turn-back angles or null
+  int direct;      // the result goes straight to out as bf16 rows [T, H * vdim]
+};
+
 template <int DK, int NVT, bool PRECISE, int NS>
 __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
     const float* __restrict__ q, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
     const int* __restrict__ block_tables, int max_blocks, const int* __restrict__ cu_q, const int* __restrict__ ctx_lens,
     float* __restrict__ out, int H, int G, int GE, int vdim, int bs, float scale, float cap, int all, int nvch,
-    int sink, int chunk, int vshare) {
+    int sink, int chunk, int vshare, SinkExt X) {
   constexpr int BKV = 64;
   constexpr int LDK = DK + 16;
   constexpr int VCH = NVT * 16;
@@ -337,6 +366,9 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
   const int rows_per_wg = 64 * NS / GE;
   int bx, by, b;
   causal_block_order(bx, by, b);
+  const int sp = bx % X.nsplit;
+  bx /= X.nsplit;
+  const int dim = X.dim, window = X.window;
   const int vch = by % nvch, hy = by / nvch;
   const int kvh = hy / (rep / GE);
   const int h0 = kvh * rep + (hy % (rep / GE)) * GE;
@@ -352,6 +384,7 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
   const int64_t vrow = (int64_t)GV * vdim;
   const int voff = (all ? 0 : (kvh / vshare) * vdim) + v0;
 
+  constexpr float kLog2e = 1.4426950408889634f;
   // per slot group: the lane's slot, and (the same in every lane) the positions the group's rows span
   int row[NS], hd[NS], qpos[NS], qlo[NS];
   bool valid[NS], grp_rows[NS];
@@ -375,12 +408,12 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
     grp_last[n] = p0 + min(qlen - 1, r0 + (gs + 15) / GE);
     grp_lo[n] = chunk > 0 ? (grp_first[n] / chunk) * chunk : 0;
     grp_hilo[n] = chunk > 0 ? (grp_last[n] / chunk) * chunk : 0;
-    const float* qp = q + ((int64_t)(t0 + (valid[n] ? row[n] : 0)) * H + (valid[n] ? hd[n] : h0)) * DK + 8 * g;
+    const float* qp = q + ((int64_t)(t0 + (valid[n] ? row[n] : 0)) * H + (valid[n] ? hd[n] : h0)) * dim + 8 * g;
 #pragma unroll
     for (int ks = 0; ks < DK / 32; ++ks)
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
-        const float x = qp[32 * ks + j];
+        const float x = 32 * ks + 8 * g < dim ? qp[32 * ks + j] : 0.f;
         const bf16_t hi = f2bf(x);
         qf[n][ks][j] = (short)hi;
         if constexpr (PRECISE) ql[n][ks][j] = (short)f2bf(x - bf2f(hi));
@@ -388,15 +421,20 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
 #pragma unroll
     for (int i = 0; i < NVT; ++i) o[n][i] = f32x4{0.f, 0.f, 0.f, 0.f};
     // the sink: score 0, weight exp(0 - m), no value; without it a masked score's stand-in is the starting maximum
-    m[n] = sink ? 0.f : -1.0e30f;
-    lsum[n] = sink ? 1.f : 0.f;
+    const bool own_sink = sink && X.nsplit == 1;  // split keys: the sink joins when the parts do
+    m[n] = own_sink ? (X.sinks ? X.sinks[valid[n] ? hd[n] : h0] * kLog2e : 0.f) : -1.0e30f;
+    lsum[n] = own_sink ? 1.f : 0.f;
   }
-  constexpr float kLog2e = 1.4426950408889634f;
   const float icap = cap > 0.f ? 1.0f / cap : 0.f;
   const float scale2 = scale * kLog2e;
   const int r_last = min(qlen, r0 + rows_per_wg) - 1;
-  const int kv_end = p0 + r_last + 1;
-  const int kv_begin = chunk > 0 ? ((p0 + r0) / chunk) * chunk : 0;  // the first row's block starts first
+  // the workgroup's keys, numbered u: the kept positions before jlo, then the positions from jlo on
+  const int jlo = max(chunk > 0 ? ((p0 + r0) / chunk) * chunk : 0, window > 0 ? p0 + r0 - window + 1 : 0);
+  const int nkp = window > 0 ? min(X.keep, jlo) : 0;
+  const int total = nkp + p0 + r_last + 1 - jlo;
+  const int tps = ((total + BKV - 1) / BKV + X.nsplit - 1) / X.nsplit;
+  const int u_begin = sp * tps * BKV, u_end = min(total, (sp + 1) * tps * BKV);
+  auto pos_of = [&](int u) { return u < nkp ? u : jlo + (u - nkp); };
   const int* bt = block_tables + (int64_t)b * max_blocks;
   constexpr int CHK = DK / 8, CHV = VCH / 8;
   // Software pipeline: the next tile's 16-byte chunks are fetched into registers while this tile is computed from
@@ -404,20 +442,22 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
   static_assert((BKV * CHK) % 256 == 0 && (BKV * CHV) % 256 == 0, "whole 16-byte chunks per thread");
   constexpr int NCK = BKV * CHK / 256, NCV = BKV * CHV / 256;
   u16x8 kr[NCK], vr[NCV];
-  auto load_tile = [&](int kv0) {
+  auto load_tile = [&](int u0) {
 #pragma unroll
     for (int j = 0; j < NCK; ++j) {
       const int c = threadIdx.x + 256 * j;
       const int r = c / CHK, ch = c % CHK;
-      const int key = min(kv0 + r, kv_end - 1);
+      const int key = pos_of(min(u0 + r, total - 1));
       const int64_t sl = (int64_t)bt[key / bs] * bs + key % bs;
-      kr[j] = *reinterpret_cast<const u16x8*>(kc + (sl * G + kvh) * DK + ch * 8);
+      u16x8 val = {0, 0, 0, 0, 0, 0, 0, 0};
+      if (DK == 32 || ch * 8 < dim) val = *reinterpret_cast<const u16x8*>(kc + (sl * G + kvh) * dim + ch * 8);
+      kr[j] = val;
     }
 #pragma unroll
     for (int j = 0; j < NCV; ++j) {
       const int c = threadIdx.x + 256 * j;
       const int r = c / CHV, ch = c % CHV;
-      const int key = min(kv0 + r, kv_end - 1);
+      const int key = pos_of(min(u0 + r, total - 1));
       const int64_t sl = (int64_t)bt[key / bs] * bs + key % bs;
       u16x8 val = {0, 0, 0, 0, 0, 0, 0, 0};
       if (v0 + ch * 8 < RVtot) val = *reinterpret_cast<const u16x8*>(vc + sl * vrow + voff + ch * 8);
@@ -437,13 +477,15 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
     }
   };
   // one tile of keys from LDS for every slot group of this wave that sees any of it
-  auto compute_tile = [&](int kv0) {
+  auto compute_tile = [&](int u0) {
     bool act[NS];
     bool any = false;
+    const bool kept = u0 < nkp;  // some of the tile are kept positions
+    const int j0 = pos_of(u0), j1 = kept ? j0 : j0 + BKV - 1;
 #pragma unroll
     for (int n = 0; n < NS; ++n) {
-      // not wholly in the group's causal future, not wholly before the block of its first row
-      act[n] = grp_rows[n] && kv0 <= grp_last[n] && kv0 + BKV > grp_lo[n];
+      // not wholly in the group's causal future, not wholly before the block or the window of its first row
+      act[n] = grp_rows[n] && (kept || (j0 <= grp_last[n] && j1 >= grp_lo[n] && !(window > 0 && grp_first[n] - j1 >= window)));
       any = any || act[n];
     }
     if (!any) return;
@@ -462,7 +504,7 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
         }
       }
     }
-    // S^T accumulators: lane (li, g) holds slot li's scores for keys kv0 + 16 kt + 4 g + i.
+    // S^T accumulators: lane (li, g) holds slot li's scores for keys u0 + 16 kt + 4 g + i.
     // The matrix instructions above and below run for every group of the wave (a fragment from LDS serves them all);
     // a group that sees nothing of the tile gets zero weights, which leave its sums as they are.
     s16x8 pf[NS][2], pl[NS][PRECISE ? 2 : 1];
@@ -477,13 +519,15 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
           if constexpr (CAP) {
             const float x = s[n][kt][i] * scale;
             const float e2 = __expf(2.0f * x * icap);  // tanh(x) = 1 - 2 / (exp(2x) + 1)
-            v = cap * (1.0f - 2.0f / (e2 + 1.0f)) * kLog2e;
+            v = cap * (1.0f - 2.0f * __builtin_amdgcn_rcpf(e2 + 1.0f)) * kLog2e;
           } else {
             v = s[n][kt][i] * scale2;
           }
           if constexpr (!WHOLE) {
-            const int key = kv0 + kt * 16 + 4 * g + i;
-            v = (key <= qpos[n] && key >= qlo[n] && key < kv_end) ? v : -1.0e30f;
+            const int u = u0 + kt * 16 + 4 * g + i, key = pos_of(u);
+            const bool vis = key <= qpos[n] && key >= qlo[n] && u < u_end &&
+                             (window == 0 || qpos[n] - key < window || key < X.keep);
+            v = vis ? v : -1.0e30f;
           }
           s[n][kt][i] = v;
           mx = fmaxf(mx, v);
@@ -523,9 +567,12 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
         continue;
       }
       // does every row of the group see the whole tile?
-      const bool whole = kv0 + BKV - 1 <= grp_first[n] && kv0 >= grp_hilo[n];
-      if (cap > 0.f) softmax(n, std::false_type{}, std::true_type{});
-      else if (whole) softmax(n, std::true_type{}, std::false_type{});
+      const bool whole = !kept && u0 + BKV <= u_end && j1 <= grp_first[n] && j0 >= grp_hilo[n] &&
+                         (window == 0 || grp_last[n] - j0 < window);
+      if (cap > 0.f) {
+        if (whole) softmax(n, std::true_type{}, std::true_type{});
+        else softmax(n, std::false_type{}, std::true_type{});
+      } else if (whole) softmax(n, std::true_type{}, std::false_type{});
       else softmax(n, std::false_type{}, std::false_type{});
     }
     const int tq = li >> 2, tp = li & 3;
@@ -546,18 +593,52 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
       }
     }
   };
-  if (kv_end > kv_begin) load_tile(kv_begin);  // (a padded row has no keys at all)
-  for (int kv0 = kv_begin; kv0 < kv_end; kv0 += BKV) {
+  if (u_end > u_begin) load_tile(u_begin);  // (a padded row has no keys at all)
+  for (int u0 = u_begin; u0 < u_end; u0 += BKV) {
     __syncthreads();  // every wave is done reading the previous tile
     store_tile();
     __syncthreads();
-    if (kv0 + BKV < kv_end) load_tile(kv0 + BKV);
-    if (wave_rows) compute_tile(kv0);
+    if (u0 + BKV < u_end) load_tile(u0 + BKV);
+    if (wave_rows) compute_tile(u0);
   }
 #pragma unroll
   for (int n = 0; n < NS; ++n) {
     if (!valid[n]) continue;
-    const float inv = 1.0f / lsum[n];
+    if (X.nsplit > 1) {
+      const int64_t at = (int64_t)sp * X.prows + (int64_t)(t0 + row[n]) * H + hd[n];
+#pragma unroll
+      for (int dt = 0; dt < NVT; ++dt)
+        if (v0 + dt * 16 + 4 * g < RVtot) *reinterpret_cast<f32x4*>(X.po + at * RVtot + v0 + 4 * g + dt * 16) = o[n][dt];
+      if (g == 0 && vch == 0) {
+        X.pml[at * 2] = m[n];
+        X.pml[at * 2 + 1] = lsum[n];
+      }
+      continue;
+    }
+    const float inv = lsum[n] > 0.f ? 1.0f / lsum[n] : 0.f;  // (a padded row has no keys)
+    if (X.direct) {
+      if (X.vcs) {  // (the host takes this path only where the value tile is the whole head: VCH == vdim)
+        const float* cs = X.vcs + (int64_t)(t0 + row[n]) * vdim + 8 * g;
+#pragma unroll
+        for (int dt = 0; dt < NVT / 2; ++dt) {
+          const f32x4 c0 = *reinterpret_cast<const f32x4*>(cs + dt * 32), c1 = *reinterpret_cast<const f32x4*>(cs + dt * 32 + 4);
+          const float co[4] = {c0[0], c0[2], c1[0], c1[2]}, si[4] = {c0[1], c0[3], c1[1], c1[3]};
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const float u = o[n][dt][i], v = o[n][dt + NVT / 2][i];
+            o[n][dt][i] = u * co[i] + v * si[i];
+            o[n][dt + NVT / 2][i] = v * co[i] - u * si[i];
+          }
+        }
+      }
+      bf16_t* ob = reinterpret_cast<bf16_t*>(out) + ((int64_t)(t0 + row[n]) * H + hd[n]) * RVtot + v0 + 4 * g;
+#pragma unroll
+      for (int dt = 0; dt < NVT; ++dt)
+        if (v0 + dt * 16 + 4 * g < RVtot)
+          *reinterpret_cast<u16x4*>(ob + dt * 16) = u16x4{f2bf(o[n][dt][0] * inv), f2bf(o[n][dt][1] * inv),
+                                                          f2bf(o[n][dt][2] * inv), f2bf(o[n][dt][3] * inv)};
+      continue;
+    }
     float* op = out + ((int64_t)(t0 + row[n]) * H + hd[n]) * RVtot + v0 + 4 * g;
 #pragma unroll
     for (int dt = 0; dt < NVT; ++dt)
@@ -566,16 +647,21 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
 }
 
 // Can the matrix-core kernel take this shape? (bf16 storage is the caller's to check.)
-bool sink_attn_mfma_ok(int dim, int vdim) { return (dim == 32 || dim == 64 || dim == 128) && vdim % 8 == 0; }
+bool sink_attn_mfma_ok(int dim, int vdim, int precise) {
+  return (dim == 32 || dim == 64 || dim == 128 || (precise && dim % 8 == 0 && dim > 0 && dim <= 128)) && vdim % 8 == 0;
+}
 
 void launch_sink_attn_mfma(const void* q, const void* kc, const void* vc, const void* bt, int maxb, const void* cu,
                            const void* ctx, void* out, int B, int max_qlen, int H, int G, int dim, int vdim, int bs,
                            float scale, float cap, int all, int sink, int chunk, int vshare, int precise,
-                           hipStream_t st) {
+                           const void* sinks, int window, int keep, int nsplit, void* po, void* pml, int64_t row0,
+                           int64_t rows, const void* vcs, int direct, hipStream_t st) {
   if (B == 0 || max_qlen <= 0) return;
   if (G < 1 || H % G) throw std::runtime_error("sink attention: heads must be a multiple of the key/value heads");
   if (vshare < 1 || G % vshare || chunk < 0) throw std::runtime_error("sink attention: bad vshare / chunk");
-  if (!sink_attn_mfma_ok(dim, vdim)) throw std::runtime_error("sink attention: shape not built for the matrix cores");
+  if (window < 0 || keep < 0 || nsplit < 1 || (nsplit > 1 && (max_qlen != 1 || !po || !pml)))
+    throw std::runtime_error("sink attention: bad window / split");
+  if (!sink_attn_mfma_ok(dim, vdim, precise)) throw std::runtime_error("sink attention: shape not built for the matrix cores");
   const int rep = H / G;
   int GE = 1;
   for (int ge = std::min(rep, 64); ge >= 1; --ge)
@@ -593,11 +679,14 @@ void launch_sink_attn_mfma(const void* q, const void* kc, const void* vc, const 
   const int rows_per_wg = 64 * ns / GE;
   const int64_t gy = (int64_t)G * (rep / GE) * nvch;
   if (gy > 65535 || B > 65535) throw std::runtime_error("sink attention: too many heads or sequences");
-  dim3 grid((max_qlen + rows_per_wg - 1) / rows_per_wg, (unsigned)gy, B);
+  if (direct && vcs && vdim != nvt * 16) throw std::runtime_error("sink attention: the turn-back needs whole heads");
+  dim3 grid((max_qlen + rows_per_wg - 1) / rows_per_wg * nsplit, (unsigned)gy, B);
+  SinkExt X{dim, window, keep, (const float*)sinks, nsplit, po ? (float*)po - row0 * H * RVtot : nullptr,
+            pml ? (float*)pml - row0 * H * 2 : nullptr, rows * H, (const float*)vcs, direct};
 #define LAUNCH_SAM2(DK_, NVT_, PR_, NS_)                                                                            \
   sink_attn_mfma_kernel<DK_, NVT_, PR_, NS_><<<grid, 256, 0, st>>>(                                                 \
       (const float*)q, (const bf16_t*)kc, (const bf16_t*)vc, (const int*)bt, maxb, (const int*)cu, (const int*)ctx, \
-      (float*)out, H, G, GE, vdim, bs, scale, cap, all, nvch, sink, chunk, vshare)
+      (float*)out, H, G, GE, vdim, bs, scale, cap, all, nvch, sink, chunk, vshare, X)
 #define LAUNCH_SAM1(DK_, NVT_, NS_)                                                       \
   do {                                                                                    \
     if (!precise) LAUNCH_SAM2(DK_, NVT_, false, NS_);                                     \
@@ -614,12 +703,74 @@ void launch_sink_attn_mfma(const void* q, const void* kc, const void* vc, const 
       else LAUNCH_SAM1(DK_, 4, 1);            \
     }                                         \
   } while (0)
-  if (dim == 32) LAUNCH_SAM(32);
-  else if (dim == 64) LAUNCH_SAM(64);
+  if (dim <= 32) LAUNCH_SAM(32);
+  else if (dim <= 64) LAUNCH_SAM(64);
   else LAUNCH_SAM(128);
 #undef LAUNCH_SAM
 #undef LAUNCH_SAM1
 #undef LAUNCH_SAM2
+  HIP_CHECK_LAUNCH();
+}
+
+// Joins the parts of a row's keys (nsplit > 1: po [nsplit][rows][H][vdim] sums, pml [..][2] maximum (base 2) and
+// denominator; the sink, exp(sinks[h]) or 1, is added here) or takes the finished fp32 rows O (nsplit 1), turns every head back
+// by vcs [T, vdim / 2, 2] (null: not) and stores rows y [T, H * vdim]. One wave per (row, head); row r of the parts is row
+// row0 + r of the step.
+template <typename T>
+__global__ __launch_bounds__(256) void attn_finish_kernel(const float* __restrict__ po, const float* __restrict__ pml,
+                                                          int nsplit, int64_t prows, int sink,
+                                                          const float* __restrict__ sinks,
+                                                          const float* __restrict__ vcs, T* __restrict__ y,
+                                                          int64_t row0, int H, int vdim) {
+  const int64_t e = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);  // (row, head) of the parts
+  if (e >= prows) return;
+  const int lane = threadIdx.x & 63;
+  const int64_t r = e / H;
+  const int h = (int)(e - r * H);
+  constexpr float kLog2e = 1.4426950408889634f;
+  float M = sink ? (sinks ? sinks[h] * kLog2e : 0.f) : -1.0e30f, inv = 1.0f;
+  float wsp = 1.0f;  // lane sp: the weight of part sp
+  if (nsplit > 1) {
+    const float s0 = M;
+    const float ms = lane < nsplit ? pml[((int64_t)lane * prows + e) * 2] : -1.0e30f;
+    const float ls = lane < nsplit ? pml[((int64_t)lane * prows + e) * 2 + 1] : 0.f;
+    M = fmaxf(M, warp_max(ms));
+    wsp = exp2f(ms - M);
+    const float L = warp_sum(ls * wsp) + (sink ? exp2f(s0 - M) : 0.f);
+    inv = L > 0.f ? 1.0f / L : 0.f;
+  }
+  const int half = (vdim + 1) >> 1;
+  for (int c0 = 0; c0 < half; c0 += 64) {
+    const int c = c0 + lane, c2 = c + half;
+    float u = 0.f, v = 0.f;
+    for (int sp = 0; sp < nsplit; ++sp) {  // (every lane takes part in the exchange)
+      const float w = nsplit > 1 ? __shfl(wsp, sp, 64) : 1.0f;
+      const float* p = po + ((int64_t)sp * prows + e) * vdim;
+      if (c < half) u = fmaf(w, p[c], u);
+      if (c < half && c2 < vdim) v = fmaf(w, p[c2], v);
+    }
+    if (c >= half) continue;
+    u *= inv, v *= inv;
+    if (vcs) {
+      const float co = vcs[(row0 + r) * vdim + 2 * c], si = vcs[(row0 + r) * vdim + 2 * c + 1];
+      const float a = u * co + v * si;
+      v = v * co - u * si;
+      u = a;
+    }
+    T* d = y + ((row0 + r) * H + h) * vdim;
+    El<T>::st(d + c, u);
+    if (c2 < vdim) El<T>::st(d + c2, v);
+  }
+}
+
+void launch_attn_finish(const void* po, const void* pml, int nsplit, int64_t row0, int64_t rows, int sink,
+                        const void* sinks, const void* vcs, void* y, int H, int vdim, int dt, hipStream_t st) {
+  if (rows <= 0) return;
+  if (nsplit < 1 || nsplit > 64) throw std::runtime_error("attn_finish: 1 to 64 parts");
+  if (vcs && vdim % 2) throw std::runtime_error("attn_finish: the turn-back needs an even value size");
+  DISPATCH_T(dt, T, (attn_finish_kernel<T><<<(unsigned)((rows * H + 3) / 4), 256, 0, st>>>(
+      (const float*)po, (const float*)pml, nsplit, rows * H, sink, (const float*)sinks, (const float*)vcs, (T*)y, row0, H,
+      vdim)));
   HIP_CHECK_LAUNCH();
 }
 

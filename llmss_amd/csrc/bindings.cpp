@@ -82,9 +82,9 @@ void launch_resid_add_norm(void* x, const void* a, int64_t lda, const void* b, i
                            hipStream_t st);
 void launch_gemm_any(const void* A, const void* B, void* C, int M, int N, int K, int batch, int64_t sAb, int64_t sAm,
                      int64_t sBb, int64_t sBn, int64_t sBk, int64_t sCb, int64_t sCm, int da, int db, int dc,
-                     hipStream_t st);
+                     const void* bias, hipStream_t st);
 void launch_gemm_tile(const void* A, const void* B, void* C, int M, int N, int K, int batch, int64_t sAb, int64_t sAm,
-                      int64_t sBb, int64_t sBn, int64_t sCb, int64_t sCm, int dc, hipStream_t st);
+                      int64_t sBb, int64_t sBn, int64_t sCb, int64_t sCm, int dc, const void* bias, hipStream_t st);
 void launch_moe_gate_up_tile(const void* h, int64_t ldh, const void* wg, const void* wu, const void* meta,
                              const void* order, void* act, int E, int maxt, int top, int F, int K, float limit,
                              float alpha, int tile_rows, const void* pw, int silu, hipStream_t st);
@@ -98,9 +98,9 @@ void launch_latent_attn(const void* qa, int64_t ldq, const void* cache, const vo
                         const void* ctx_lens, void* out, int64_t ldo, int T_, int B, int H, int R, int bs, int window,
                         float scale, int dt, hipStream_t st);
 void launch_moe_route(const void* z, const void* corr, void* idx, void* wts, int T_, int E, int top, int norm,
-                      hipStream_t st);
+                      int smax, hipStream_t st);
 void launch_moe_router(const void* h, int64_t ldh, const void* wr, const void* corr, void* idx, void* wts, int T_,
-                       int E, int K, int top, int dt, int norm, hipStream_t st);
+                       int E, int K, int top, int dt, int norm, int smax, hipStream_t st);
 void launch_moe_group(const void* idx, int P, int E, int maxt, void* meta, void* order, void* place, int tile_rows,
                       hipStream_t st);
 void launch_moe_gate_up(const void* h, int64_t ldh, const void* wg, const void* wu, const void* meta,
@@ -109,7 +109,7 @@ void launch_moe_gate_up(const void* h, int64_t ldh, const void* wg, const void* 
 void launch_moe_down(const void* act, const void* wd, const void* meta, void* y, int E, int maxt, int N, int F,
                      int dt, hipStream_t st);
 void launch_moe_combine(const void* y, const void* place, const void* wts, const void* shared_, int64_t lds_,
-                        void* out, int T_, int N, int top, int dt, hipStream_t st);
+                        void* out, int T_, int N, int top, int dt, const void* ident, int64_t ldi, hipStream_t st);
 void launch_glu_clamp(const void* gu, int64_t ldg, void* out, int64_t ldo, int T_, int F, float limit, float alpha,
                       int dt, hipStream_t st);
 
@@ -124,19 +124,28 @@ void launch_causal_conv(const void* in, int64_t ldi, const void* w, void* state,
                         int di, int dw, int dout, const void* bias, hipStream_t st);
 void launch_gated_group_norm(const void* o, int64_t ldo, const void* gate, int64_t ldg, const void* w, float eps,
                              int act, float c, void* out, int64_t ldout, int T_, int groups, int n, int dt, int wfull,
-                             int first, hipStream_t st);
+                             int first, const void* den, const void* gates, float qs, hipStream_t st);
 void launch_glu_act(const void* gu, int64_t ldg, void* out, int64_t ldo, int T_, int F, int act, int dt,
                     hipStream_t st);
 void launch_recurrence(int mode, const void* q, const void* k, const void* v, int64_t ldq, int64_t ldk, int64_t ldv,
                        const void* ab, int64_t ldab, int off_a, int off_b, const void* decay, const void* dt_bias,
                        void* state, const void* cu, const void* ctx, const void* sslots, void* out, int64_t ldo, int B,
                        int H, int G, int dim, int vdim, int silu_in, int gates_ready, int dq, int dp, const void* skip,
-                       hipStream_t st);
+                       void* nstate, void* den, hipStream_t st);
+void launch_mlstm_gates(const void* zi, const void* zf, int64_t ld, const void* bi, const void* bf, float cap,
+                        void* mstate, const void* cu, const void* ctx, const void* sslots, void* gates, void* ab, int B,
+                        int H, int dt, hipStream_t st);
+// query / key / value heads on their way into the paged cache
+void launch_head_prep(const void* proj, int64_t ldp, int off_q, int off_k, int off_v, const void* conv, int taps,
+                      void* tail, int single, const void* cu, const void* ctx, const void* sslots, int B, const void* qw,
+                      const void* kw, int vnorm, float eps, const void* cs, int half, const void* vcs, void* q, void* kc,
+                      void* vc, const void* slots, int T_, int H, int G, int dim, int vdim, int dt, hipStream_t st);
 // blocks normed on both sides, token input, windowed sigmoid attention with pooled blocks
 void launch_sandwich_add_norm(void* x, const void* y, int64_t ldy, const void* ey, const void* place, const void* wts,
                               int top, const void* shared_, int64_t lds_, const void* r, int64_t ldr, const void* rb,
                               const void* wpost, const void* add, const void* wnext, void* h, int64_t ldh, float eps,
-                              int T_, int W, int dt, hipStream_t st);
+                              int groups, const void* ident, int64_t ldi, const void* y2, int64_t ldy2, const void* wl,
+                              const void* wr, int T_, int W, int dt, hipStream_t st);
 void launch_token_side_add(void* x, const void* ids, const void* table, int64_t ldt, int vocab, int col0, int d,
                            const void* wg, const void* wp, const void* wn, const void* add, const void* wnext, void* h,
                            int64_t ldh, float eps, int T_, int W, int dt, hipStream_t st);
@@ -164,12 +173,16 @@ void launch_rope_bias_cache(const void* proj, int64_t ldp, int off_q, int off_k,
                             const void* slots, int T_, int H, int G, int dim, int vdim, int dt, hipStream_t st);
 void launch_sink_attn(const void* q, const void* kc, const void* vc, const void* bt, int maxb, const void* cu,
                       const void* ctx, void* out, int T_, int B, int H, int G, int dim, int vdim, int bs, float scale,
-                      float cap, int all, int sink, int chunk, int vshare, int dt, hipStream_t st);
-bool sink_attn_mfma_ok(int dim, int vdim);
+                      float cap, int all, int sink, int chunk, int vshare, const void* sinks, int window, int keep,
+                      int dt, hipStream_t st);
+bool sink_attn_mfma_ok(int dim, int vdim, int precise);
 void launch_sink_attn_mfma(const void* q, const void* kc, const void* vc, const void* bt, int maxb, const void* cu,
                            const void* ctx, void* out, int B, int max_qlen, int H, int G, int dim, int vdim, int bs,
                            float scale, float cap, int all, int sink, int chunk, int vshare, int precise,
-                           hipStream_t st);
+                           const void* sinks, int window, int keep, int nsplit, void* po, void* pml, int64_t row0,
+                           int64_t rows, const void* vcs, int direct, hipStream_t st);
+void launch_attn_finish(const void* po, const void* pml, int nsplit, int64_t row0, int64_t rows, int sink,
+                        const void* sinks, const void* vcs, void* y, int H, int vdim, int dt, hipStream_t st);
 void launch_talk_mix(const void* O, const void* talk, float c, void* y, int64_t ldy, int T_, int H, int G, int vdim,
                      int dt, hipStream_t st);
 
@@ -336,12 +349,12 @@ PYBIND11_MODULE(_C, m) {
   });
   m.def("gemm_any", [](uintptr_t A, uintptr_t B, uintptr_t C, int M, int N, int K, int batch, int64_t sAb, int64_t sAm,
                        int64_t sBb, int64_t sBn, int64_t sBk, int64_t sCb, int64_t sCm, int da, int db, int dc,
-                       uintptr_t st) {
-    launch_gemm_any(CP(A), CP(B), P(C), M, N, K, batch, sAb, sAm, sBb, sBn, sBk, sCb, sCm, da, db, dc, S(st));
+                       uintptr_t bias, uintptr_t st) {
+    launch_gemm_any(CP(A), CP(B), P(C), M, N, K, batch, sAb, sAm, sBb, sBn, sBk, sCb, sCm, da, db, dc, CP(bias), S(st));
   });
   m.def("gemm_tile", [](uintptr_t A, uintptr_t B, uintptr_t C, int M, int N, int K, int batch, int64_t sAb, int64_t sAm,
-                        int64_t sBb, int64_t sBn, int64_t sCb, int64_t sCm, int dc, uintptr_t st) {
-    launch_gemm_tile(CP(A), CP(B), P(C), M, N, K, batch, sAb, sAm, sBb, sBn, sCb, sCm, dc, S(st));
+                        int64_t sBb, int64_t sBn, int64_t sCb, int64_t sCm, int dc, uintptr_t bias, uintptr_t st) {
+    launch_gemm_tile(CP(A), CP(B), P(C), M, N, K, batch, sAb, sAm, sBb, sBn, sCb, sCm, dc, CP(bias), S(st));
   });
   m.def("moe_gate_up_tile", [](uintptr_t h, int64_t ldh, uintptr_t wg, uintptr_t wu, uintptr_t meta, uintptr_t order,
                                uintptr_t act, int E, int maxt, int top, int F, int K, float limit, float alpha,
@@ -369,10 +382,12 @@ PYBIND11_MODULE(_C, m) {
                        scale, dt, S(st));
   });
   m.def("moe_route", [](uintptr_t z, uintptr_t corr, uintptr_t idx, uintptr_t wts, int T, int E, int top, int norm,
-                        uintptr_t st) { launch_moe_route(CP(z), CP(corr), P(idx), P(wts), T, E, top, norm, S(st)); });
+                        int smax, uintptr_t st) {
+    launch_moe_route(CP(z), CP(corr), P(idx), P(wts), T, E, top, norm, smax, S(st));
+  });
   m.def("moe_router", [](uintptr_t h, int64_t ldh, uintptr_t wr, uintptr_t corr, uintptr_t idx, uintptr_t wts, int T,
-                         int E, int K, int top, int dt, int norm, uintptr_t st) {
-    launch_moe_router(CP(h), ldh, CP(wr), CP(corr), P(idx), P(wts), T, E, K, top, dt, norm, S(st));
+                         int E, int K, int top, int dt, int norm, int smax, uintptr_t st) {
+    launch_moe_router(CP(h), ldh, CP(wr), CP(corr), P(idx), P(wts), T, E, K, top, dt, norm, smax, S(st));
   });
   m.def("moe_group", [](uintptr_t idx, int Pn, int E, int maxt, uintptr_t meta, uintptr_t order, uintptr_t place,
                         int tile_rows, uintptr_t st) {
@@ -387,8 +402,8 @@ PYBIND11_MODULE(_C, m) {
   m.def("moe_down", [](uintptr_t act, uintptr_t wd, uintptr_t meta, uintptr_t y, int E, int maxt, int N, int F, int dt,
                        uintptr_t st) { launch_moe_down(CP(act), CP(wd), CP(meta), P(y), E, maxt, N, F, dt, S(st)); });
   m.def("moe_combine", [](uintptr_t y, uintptr_t place, uintptr_t wts, uintptr_t sh, int64_t lds_, uintptr_t out, int T,
-                          int N, int top, int dt, uintptr_t st) {
-    launch_moe_combine(CP(y), CP(place), CP(wts), CP(sh), lds_, P(out), T, N, top, dt, S(st));
+                          int N, int top, int dt, uintptr_t ident, int64_t ldi, uintptr_t st) {
+    launch_moe_combine(CP(y), CP(place), CP(wts), CP(sh), lds_, P(out), T, N, top, dt, CP(ident), ldi, S(st));
   });
   m.def("glu_clamp", [](uintptr_t gu, int64_t ldg, uintptr_t out, int64_t ldo, int T, int F, float limit, float alpha,
                         int dt, uintptr_t st) { launch_glu_clamp(CP(gu), ldg, P(out), ldo, T, F, limit, alpha, dt, S(st)); });
@@ -410,9 +425,9 @@ PYBIND11_MODULE(_C, m) {
   });
   m.def("gated_group_norm", [](uintptr_t o, int64_t ldo, uintptr_t gate, int64_t ldg, uintptr_t w, float eps, int act,
                                float c, uintptr_t out, int64_t ldout, int T, int groups, int n, int dt, int wfull,
-                               int first, uintptr_t st) {
+                               int first, uintptr_t den, uintptr_t gates, float qs, uintptr_t st) {
     launch_gated_group_norm(CP(o), ldo, CP(gate), ldg, CP(w), eps, act, c, P(out), ldout, T, groups, n, dt, wfull,
-                            first, S(st));
+                            first, CP(den), CP(gates), qs, S(st));
   });
   m.def("glu_act", [](uintptr_t gu, int64_t ldg, uintptr_t out, int64_t ldo, int T, int F, int act, int dt,
                       uintptr_t st) { launch_glu_act(CP(gu), ldg, P(out), ldo, T, F, act, dt, S(st)); });
@@ -420,10 +435,25 @@ PYBIND11_MODULE(_C, m) {
                          uintptr_t ab, int64_t ldab, int off_a, int off_b, uintptr_t decay, uintptr_t dtb,
                          uintptr_t state, uintptr_t cu, uintptr_t ctx, uintptr_t ss, uintptr_t out, int64_t ldo, int B,
                          int H, int G, int dim, int vdim, int silu_in, int gates_ready, int dq, int dp, uintptr_t skip,
-                         uintptr_t st) {
+                         uintptr_t nstate, uintptr_t den, uintptr_t st) {
     launch_recurrence(mode, CP(q), CP(k), CP(v), ldq, ldk, ldv, CP(ab), ldab, off_a, off_b, CP(decay), CP(dtb),
                       P(state), CP(cu), CP(ctx), CP(ss), P(out), ldo, B, H, G, dim, vdim, silu_in, gates_ready, dq, dp,
-                      CP(skip), S(st));
+                      CP(skip), P(nstate), P(den), S(st));
+  });
+  m.def("mlstm_gates", [](uintptr_t zi, uintptr_t zf, int64_t ld, uintptr_t bi, uintptr_t bf, float cap, uintptr_t ms,
+                          uintptr_t cu, uintptr_t ctx, uintptr_t ss, uintptr_t gates, uintptr_t ab, int B, int H, int dt,
+                          uintptr_t st) {
+    launch_mlstm_gates(CP(zi), CP(zf), ld, CP(bi), CP(bf), cap, P(ms), CP(cu), CP(ctx), CP(ss), P(gates), P(ab), B, H,
+                       dt, S(st));
+  });
+  m.def("head_prep", [](uintptr_t proj, int64_t ldp, int off_q, int off_k, int off_v, uintptr_t conv, int taps,
+                        uintptr_t tail, int single, uintptr_t cu, uintptr_t ctx, uintptr_t ss, int B, uintptr_t qw,
+                        uintptr_t kw, int vnorm, float eps, uintptr_t cs, int half, uintptr_t vcs, uintptr_t q,
+                        uintptr_t kc, uintptr_t vc, uintptr_t slots, int T, int H, int G, int dim, int vdim, int dt,
+                        uintptr_t st) {
+    launch_head_prep(CP(proj), ldp, off_q, off_k, off_v, CP(conv), taps, P(tail), single, CP(cu), CP(ctx), CP(ss), B,
+                     CP(qw), CP(kw), vnorm, eps, CP(cs), half, CP(vcs), P(q), P(kc), P(vc), CP(slots), T, H, G, dim,
+                     vdim, dt, S(st));
   });
   m.def("silu_f32", [](uintptr_t in, int64_t ldi, uintptr_t out, int64_t ldo, int T, int n, int dt, uintptr_t st) {
     launch_silu_f32(CP(in), ldi, P(out), ldo, T, n, dt, S(st));
@@ -441,17 +471,24 @@ PYBIND11_MODULE(_C, m) {
   });
   m.def("sink_attn", [](uintptr_t q, uintptr_t kc, uintptr_t vc, uintptr_t bt, int maxb, uintptr_t cu, uintptr_t ctx,
                         uintptr_t out, int T, int B, int H, int G, int dim, int vdim, int bs, float scale, float cap,
-                        int all, int sink, int chunk, int vshare, int dt, uintptr_t st) {
+                        int all, int sink, int chunk, int vshare, uintptr_t sinks, int window, int keep, int dt,
+                        uintptr_t st) {
     launch_sink_attn(CP(q), CP(kc), CP(vc), CP(bt), maxb, CP(cu), CP(ctx), P(out), T, B, H, G, dim, vdim, bs, scale,
-                     cap, all, sink, chunk, vshare, dt, S(st));
+                     cap, all, sink, chunk, vshare, CP(sinks), window, keep, dt, S(st));
   });
   m.def("sink_attn_mfma_ok", &sink_attn_mfma_ok);
   m.def("sink_attn_mfma", [](uintptr_t q, uintptr_t kc, uintptr_t vc, uintptr_t bt, int maxb, uintptr_t cu,
                              uintptr_t ctx, uintptr_t out, int B, int max_qlen, int H, int G, int dim, int vdim, int bs,
                              float scale, float cap, int all, int sink, int chunk, int vshare, int precise,
-                             uintptr_t st) {
+                             uintptr_t sinks, int window, int keep, int nsplit, uintptr_t po, uintptr_t pml,
+                             int64_t row0, int64_t rows, uintptr_t vcs, int direct, uintptr_t st) {
     launch_sink_attn_mfma(CP(q), CP(kc), CP(vc), CP(bt), maxb, CP(cu), CP(ctx), P(out), B, max_qlen, H, G, dim, vdim,
-                          bs, scale, cap, all, sink, chunk, vshare, precise, S(st));
+                          bs, scale, cap, all, sink, chunk, vshare, precise, CP(sinks), window, keep, nsplit, P(po),
+                          P(pml), row0, rows, CP(vcs), direct, S(st));
+  });
+  m.def("attn_finish", [](uintptr_t po, uintptr_t pml, int nsplit, int64_t row0, int64_t rows, int sink, uintptr_t sinks,
+                          uintptr_t vcs, uintptr_t y, int H, int vdim, int dt, uintptr_t st) {
+    launch_attn_finish(CP(po), CP(pml), nsplit, row0, rows, sink, CP(sinks), CP(vcs), P(y), H, vdim, dt, S(st));
   });
   m.def("talk_mix", [](uintptr_t O, uintptr_t talk, float c, uintptr_t y, int64_t ldy, int T, int H, int G, int vdim,
                        int dt, uintptr_t st) { launch_talk_mix(CP(O), CP(talk), c, P(y), ldy, T, H, G, vdim, dt, S(st)); });
@@ -484,9 +521,11 @@ PYBIND11_MODULE(_C, m) {
   m.def("sandwich_add_norm", [](uintptr_t x, uintptr_t y, int64_t ldy, uintptr_t ey, uintptr_t place, uintptr_t wts,
                                 int top, uintptr_t sh, int64_t lds_, uintptr_t r, int64_t ldr, uintptr_t rb,
                                 uintptr_t wpost, uintptr_t add, uintptr_t wnext, uintptr_t h, int64_t ldh, float eps,
-                                int T, int W, int dt, uintptr_t st) {
+                                int groups, uintptr_t ident, int64_t ldi, uintptr_t y2, int64_t ldy2, uintptr_t wl,
+                                uintptr_t wr, int T, int W, int dt, uintptr_t st) {
     launch_sandwich_add_norm(P(x), CP(y), ldy, CP(ey), CP(place), CP(wts), top, CP(sh), lds_, CP(r), ldr, CP(rb),
-                             CP(wpost), CP(add), CP(wnext), P(h), ldh, eps, T, W, dt, S(st));
+                             CP(wpost), CP(add), CP(wnext), P(h), ldh, eps, groups, CP(ident), ldi, CP(y2), ldy2,
+                             CP(wl), CP(wr), T, W, dt, S(st));
   });
   m.def("token_side_add", [](uintptr_t x, uintptr_t ids, uintptr_t table, int64_t ldt, int vocab, int col0, int d,
                              uintptr_t wg, uintptr_t wp, uintptr_t wn, uintptr_t add, uintptr_t wnext, uintptr_t h,

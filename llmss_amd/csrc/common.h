@@ -115,13 +115,17 @@ __device__ __forceinline__ float gelu_erf(float x) { return 0.5f * x * (1.f + er
 
 __device__ __forceinline__ float silu(float x) { return x / (1.f + __expf(-x)); }
 
-enum Act : int { ACT_NONE = 0, ACT_GELU_TANH = 1, ACT_GELU = 2, ACT_RELU = 3, ACT_SILU_GLU = 4 };
+enum Act : int { ACT_NONE = 0, ACT_GELU_TANH = 1, ACT_GELU = 2, ACT_RELU = 3, ACT_SILU_GLU = 4, ACT_RELU2 = 5 };
 
 __device__ __forceinline__ float apply_act(float x, int act) {
   switch (act) {
     case ACT_GELU_TANH: return gelu_tanh(x);
     case ACT_GELU: return gelu_erf(x);
     case ACT_RELU: return fmaxf(x, 0.f);
+    case ACT_RELU2: {
+      const float r = fmaxf(x, 0.f);
+      return r * r;
+    }
     default: return x;
   }
 }

@@ -1,6 +1,6 @@
 // Strided, batched matrix product for any shape and either storage type, fp32 accumulation on the vector ALUs:
 //
-//   C[b][m][n] = sum_k A[b][m][k] * B[b][n][k]
+//   C[b][m][n] = sum_k A[b][m][k] * B[b][n][k] (+ bias[n])
 //   A(m, k) = A[b * sAb + m * sAm + k]            (k contiguous)
 //   B(n, k) = B[b * sBb + n * sBn + k * sBk]      (either index may be the contiguous one)
 //   C(m, n) = C[b * sCb + m * sCm + n]
@@ -17,6 +17,7 @@ struct GemmAnyArgs {
   const void* A;
   const void* B;
   void* C;
+  const void* bias;  // [N] in B's storage type, added to every row (null: none)
   int M, N, K;
   int64_t sAb, sAm, sBb, sBn, sBk, sCb, sCm;
 };
@@ -71,7 +72,8 @@ __global__ __launch_bounds__(256) void gemm_any_kernel(GemmAnyArgs p) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
-      if (n < p.N) El<TC>::st(C + (int64_t)m * p.sCm + n, acc[i][j]);
+      if (n < p.N)
+        El<TC>::st(C + (int64_t)m * p.sCm + n, acc[i][j] + (p.bias ? El<TB>::ld((const TB*)p.bias + n) : 0.f));
     }
   }
 }
@@ -86,11 +88,11 @@ static void gemm_any_c(int dc, const GemmAnyArgs& a, dim3 g, hipStream_t st) {
 
 void launch_gemm_any(const void* A, const void* B, void* C, int M, int N, int K, int batch, int64_t sAb, int64_t sAm,
                      int64_t sBb, int64_t sBn, int64_t sBk, int64_t sCb, int64_t sCm, int da, int db, int dc,
-                     hipStream_t st) {
+                     const void* bias, hipStream_t st) {
   if (M <= 0 || N <= 0 || batch <= 0) return;
   if ((da | db | dc) & ~1) throw std::runtime_error("gemm_any: bad dtype code");
   if (batch > 65535 || (M + TV_BM - 1) / TV_BM > 65535) throw std::runtime_error("gemm_any: grid too large");
-  GemmAnyArgs a{A, B, C, M, N, K, sAb, sAm, sBb, sBn, sBk, sCb, sCm};
+  GemmAnyArgs a{A, B, C, bias, M, N, K, sAb, sAm, sBb, sBn, sBk, sCb, sCm};
   dim3 g((N + TV_BN - 1) / TV_BN, (M + TV_BM - 1) / TV_BM, batch);
   if (da == 0 && db == 0) gemm_any_c<bf16_t, bf16_t>(dc, a, g, st);
   else if (da == 1 && db == 0) gemm_any_c<float, bf16_t>(dc, a, g, st);

@@ -2,7 +2,7 @@
 // over strided views, products that keep an fp32 output, and the grouped expert GEMMs of a mixture-of-experts layer
 // (row gather, per-expert weights, the clamped gated activation fused behind the gate / up product).
 //
-//   C[b][m][n] = sum_k A[b][m][k] * B[b][n][k]        A, B bf16 with k contiguous; C bf16 or fp32
+//   C[b][m][n] = sum_k A[b][m][k] * B[b][n][k] (+ bias[n])        A, B bf16 with k contiguous; C bf16 or fp32
 //
 // One 64x64 or 128x128 output tile per 256-thread workgroup, k in steps of 64 through LDS, v_mfma_f32_16x16x32_bf16.
 // Fragment layout: lane (li = lane % 16, g = lane / 16) holds k = 8g .. 8g + 7 of row li
@@ -10,14 +10,15 @@
 // bounds-checked while staging (zero fill), so any M, N, K works; rows that are 16-byte aligned take vector loads.
 //
 // Modes: PLAIN (batched, strided), GATE_UP (grouped: rows of an expert's tile list, A rows gathered through
-// order[] / top, two weight matrices, output glu(gate, up) in bf16) and DOWN (grouped: A = the activation rows,
+// order[] / top, two weight matrices, output glu(gate, up) in bf16), UP (the same with one weight matrix, output
+// gelu(up), the error-function form) and DOWN (grouped: A = the activation rows,
 // fp32 output). The tile list and offsets are those moe_group writes (moe.hip).
 #include "anytype.h"
 
 #define GT_BK 64
 #define GT_LD 72  // bf16 per LDS row: 144 bytes, keeps ds_read_b128 rows 16-byte aligned and spreads the banks
 
-enum { GT_PLAIN = 0, GT_GATE_UP = 1, GT_DOWN = 2 };
+enum { GT_PLAIN = 0, GT_GATE_UP = 1, GT_DOWN = 2, GT_UP = 3 };
 
 struct GemmTileArgs {
   const bf16_t* A;
@@ -33,6 +34,7 @@ struct GemmTileArgs {
   float limit, alpha;
   const float* pw;  // GATE_UP: weight of each (token, slot) pair on the expert's input (null: 1)
   int silu;         // GATE_UP: silu(g) * u instead of the clamped form
+  const bf16_t* bias;  // PLAIN: [N] or null
 };
 
 __device__ __forceinline__ float glu_clamped_t(float g, float u, float limit, float alpha, int silu) {
@@ -101,7 +103,7 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmTileArgs p) {
     arow[i] = nullptr;
     if (sr < rows) {
       if constexpr (MODE == GT_PLAIN) arow[i] = A + (int64_t)(m0 + sr) * p.sAm;
-      else if constexpr (MODE == GT_GATE_UP) arow[i] = A + (int64_t)(p.order[crow0 + sr] / p.top) * p.sAm;
+      else if constexpr (MODE == GT_GATE_UP || MODE == GT_UP) arow[i] = A + (int64_t)(p.order[crow0 + sr] / p.top) * p.sAm;
       else arow[i] = A + (int64_t)(crow0 + sr) * p.sAm;
     }
     avec[i] = arow[i] && ((uintptr_t)arow[i] & 15) == 0;
@@ -182,20 +184,22 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmTileArgs p) {
       if (r >= rows) continue;
       TC* crow = C + (int64_t)((MODE == GT_PLAIN ? m0 : crow0) + r) * p.sCm;
       float sw = 1.0f;
-      if constexpr (MODE == GT_GATE_UP) sw = p.pw ? p.pw[p.order[crow0 + r]] : 1.0f;
+      if constexpr (MODE == GT_GATE_UP || MODE == GT_UP) sw = p.pw ? p.pw[p.order[crow0 + r]] : 1.0f;
 #pragma unroll
       for (int j = 0; j < NB; ++j) {
         const int n = n0 + wn + 16 * j + li;
         if (n >= p.N) continue;
         float v = acc[i][j][q];
         if constexpr (DUAL) v = glu_clamped_t(v * sw, acc2[i][j][q] * sw, p.limit, p.alpha, p.silu);
+        if constexpr (MODE == GT_UP) v = gelu_erf(v * sw);
+        if constexpr (MODE == GT_PLAIN) v += p.bias ? bf2f(p.bias[n]) : 0.f;
         El<TC>::st(crow + n, v);
       }
     }
 }
 
 void launch_gemm_tile(const void* A, const void* B, void* C, int M, int N, int K, int batch, int64_t sAb, int64_t sAm,
-                      int64_t sBb, int64_t sBn, int64_t sCb, int64_t sCm, int dc, hipStream_t st) {
+                      int64_t sBb, int64_t sBn, int64_t sCb, int64_t sCm, int dc, const void* bias, hipStream_t st) {
   if (M <= 0 || N <= 0 || batch <= 0) return;
   const int T = (M >= 512 && N >= 128) ? 128 : 64;  // big tiles where there is enough work to fill the chip
   if (batch > 65535 || (M + T - 1) / T > 65535) throw std::runtime_error("gemm_tile: grid too large");
@@ -203,6 +207,7 @@ void launch_gemm_tile(const void* A, const void* B, void* C, int M, int N, int K
   a.A = (const bf16_t*)A; a.B = (const bf16_t*)B; a.C = C;
   a.M = M; a.N = N; a.K = K;
   a.sAb = sAb; a.sAm = sAm; a.sBb = sBb; a.sBn = sBn; a.sCb = sCb; a.sCm = sCm;
+  a.bias = (const bf16_t*)bias;
   dim3 g((N + T - 1) / T, (M + T - 1) / T, batch);
   if (dc != 0 && dc != 1) throw std::runtime_error("gemm_tile: bad output dtype code");
   if (T == 128) {
@@ -215,7 +220,8 @@ void launch_gemm_tile(const void* A, const void* B, void* C, int M, int N, int K
   HIP_CHECK_LAUNCH();
 }
 
-// act[r, f] = glu(h[order[r] / top] . gate_e[f], h[..] . up_e[f]) over the tile list (bf16); tile_rows = the rows
+// act[r, f] = glu(h[order[r] / top] . gate_e[f], h[..] . up_e[f]) over the tile list (bf16), or gelu(h[..] . up_e[f])
+// where there is no gate (wg null); tile_rows = the rows
 // per tile the list was built with (moe_group): 64 or 128
 void launch_moe_gate_up_tile(const void* h, int64_t ldh, const void* wg, const void* wu, const void* meta,
                              const void* order, void* act, int E, int maxt, int top, int F, int K, float limit,
@@ -230,6 +236,14 @@ void launch_moe_gate_up_tile(const void* h, int64_t ldh, const void* wg, const v
   a.limit = limit; a.alpha = alpha; a.pw = (const float*)pw; a.silu = silu;
   // 128-row tiles are 64 columns wide here: with two accumulator sets (gate and up) a 128x128 tile leaves one
   // workgroup per CU; at 128x64 two to three fit and hide each other's staging
+  if (!wg) {
+    a.B = (const bf16_t*)wu; a.B2 = nullptr;
+    dim3 g((F + tile_rows - 1) / tile_rows, maxt);
+    if (tile_rows == 128) gemm_tile_kernel<GT_UP, bf16_t, 128, 128><<<g, 256, 0, st>>>(a);
+    else gemm_tile_kernel<GT_UP, bf16_t, 64, 64><<<g, 256, 0, st>>>(a);
+    HIP_CHECK_LAUNCH();
+    return;
+  }
   dim3 g((F + 63) / 64, maxt);
   if (tile_rows == 128) gemm_tile_kernel<GT_GATE_UP, bf16_t, 128, 64><<<g, 256, 0, st>>>(a);
   else gemm_tile_kernel<GT_GATE_UP, bf16_t, 64, 64><<<g, 256, 0, st>>>(a);

@@ -1,0 +1,194 @@
+// Query, key and value heads of an attention layer on their way into the paged cache, one launch from the projection row:
+//
+//   u = projection row (q | k | v columns), or a short causal convolution over time of it (no activation):
+//       u[t, c] = sum_k w[k, c] x[t - (taps - 1) + k, c], inputs before the portion from the sequence's tail
+//   q, k: per head  x <- x / sqrt(mean(x^2) + eps) * weight  (optional), then the first 2 * half numbers turned by the
+//         row's angles cs [T, half, 2], number i paired with i + half (optional)
+//   v:    the key columns as they were projected where there is no value projection (off_v == off_k); per head
+//         v <- v / sqrt(mean(v^2) + eps) (optional), then all vdim numbers turned by vcs [T, vdim / 2, 2] (optional)
+//
+// q leaves in fp32 [T, H * dim]; k and v go into the paged caches at slots[t] (< 0: not cached), in the storage type.
+// Norms, angles and the convolution's sum are fp32. One workgroup per row: the row's numbers are formed in LDS, then a wave
+// takes a head at a time. In a step of single rows (tail_here) the workgroup also renews its sequence's tail - nobody
+// else reads it; portions renew theirs in a second launch, after every row has read the old one.
+#include "anytype.h"
+#include "seqrows.h"
+
+struct HeadPrepArgs {
+  const void* proj;
+  int64_t ldp;
+  int off_q, off_k, off_v;
+  const void* conv;  // [taps, nq + nk + nv] (columns q | k | v, contiguous in the projection) or null
+  int taps;
+  float* tail;  // [slots, taps - 1, nq + nk + nv]
+  int tail_here;
+  const int* cu;
+  const int* ctx;
+  const int* sslots;
+  int B;
+  const float* qw;  // [dim] or null
+  const float* kw;
+  int vnorm;
+  float eps;
+  const float* cs;
+  int half;
+  const float* vcs;
+  float* q;
+  void* kc;
+  void* vc;
+  const int64_t* slots;
+  int H, G, dim, vdim;
+};
+
+template <typename T, int V>
+__device__ __forceinline__ void hp_ld(const T* p, float* v) {
+  if constexpr (V == 8) {
+    const u16x8 x = *reinterpret_cast<const u16x8*>(p);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = bf2f(x[i]);
+  } else if constexpr (V == 4) {
+    const f32x4 x = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = x[i];
+  } else {
+    v[0] = El<T>::ld(p);
+  }
+}
+
+// V: numbers per thread and access while the row is formed (8 bf16 or 4 fp32 numbers = 16 bytes, or 1)
+template <typename T, int V>
+__global__ __launch_bounds__(256) void head_prep_kernel(HeadPrepArgs A) {
+  extern __shared__ __attribute__((aligned(16))) float us[];
+  const int t = blockIdx.x, lane = threadIdx.x & 63, wv = threadIdx.x >> 6, nw = blockDim.x >> 6;
+  const int dim = A.dim, vdim = A.vdim, H = A.H, G = A.G;
+  const int nq = H * dim, nk = G * dim, nv = G * vdim;
+  const bool sharev = A.off_v == A.off_k;  // the values are the projected keys
+  const T* row = (const T*)A.proj + (int64_t)t * A.ldp;
+  const int64_t slot = A.slots[t];
+  if (A.conv) {
+    const RowSeq r = row_seq(A.cu, A.ctx, A.B, t);
+    const int C = nq + nk + nv, R = A.taps - 1;
+    const int ss = r.pos >= 0 ? A.sslots[r.b] : -1;
+    float* st = A.tail + (int64_t)max(ss, 0) * R * C;
+    for (int c = threadIdx.x * V; c < C; c += blockDim.x * V) {
+      float acc[V];
+#pragma unroll
+      for (int i = 0; i < V; ++i) acc[i] = 0.f;
+      if (r.pos >= 0) {
+        for (int k = 0; k <= R; ++k) {
+          const int d = R - k;
+          if (r.pos - d < 0) continue;
+          float x[V], w[V];
+          hp_ld<T, V>((const T*)A.conv + (int64_t)k * C + c, w);
+          if (r.j - d >= 0) {
+            hp_ld<T, V>(row - (int64_t)d * A.ldp + A.off_q + c, x);
+          } else {
+#pragma unroll
+            for (int i = 0; i < V; ++i) x[i] = ss >= 0 ? st[(int64_t)(r.j - d + R) * C + c + i] : 0.f;
+          }
+#pragma unroll
+          for (int i = 0; i < V; ++i) acc[i] = fmaf(w[i], x[i], acc[i]);
+        }
+        if (A.tail_here && ss >= 0) {  // one row per sequence: the tail moves up by one and takes this row
+          for (int i = 0; i < R; ++i) {
+            float x[V];
+            if (i + 1 < R) {
+#pragma unroll
+              for (int e = 0; e < V; ++e) x[e] = r.pos > 0 ? st[(int64_t)(i + 1) * C + c + e] : 0.f;
+            } else {
+              hp_ld<T, V>(row + A.off_q + c, x);
+            }
+#pragma unroll
+            for (int e = 0; e < V; ++e) st[(int64_t)i * C + c + e] = x[e];
+          }
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < V; ++i) us[c + i] = acc[i];
+    }
+  } else {
+    for (int c = threadIdx.x * V; c < nq + nk + (sharev ? 0 : nv); c += blockDim.x * V) {
+      const int src = c < nq ? A.off_q + c : (c < nq + nk ? A.off_k + c - nq : A.off_v + c - nq - nk);
+      float x[V];
+      hp_ld<T, V>(row + src, x);
+#pragma unroll
+      for (int i = 0; i < V; ++i) us[c + i] = x[i];
+    }
+  }
+  __syncthreads();
+  const int nvec = H + G + (slot >= 0 ? G : 0);
+  for (int n = wv; n < nvec; n += nw) {
+    const int kind = n < H ? 0 : (n < H + G ? 1 : 2);  // query, key, value
+    if (kind == 1 && slot < 0) continue;
+    const int idx = kind == 0 ? n : (kind == 1 ? n - H : n - H - G);
+    const int N = kind == 2 ? vdim : dim;
+    const float* x = us + (kind == 0 ? idx * dim : (kind == 1 ? nq + idx * dim : (sharev ? nq : nq + nk) + idx * vdim));
+    const float* w = kind == 0 ? A.qw : (kind == 1 ? A.kw : nullptr);
+    float inv = 1.f;
+    if (w || (kind == 2 && A.vnorm)) {
+      float s = 0.f;
+      for (int d = lane; d < N; d += 64) s = fmaf(x[d], x[d], s);
+      inv = 1.0f / sqrtf(warp_sum(s) / (float)N + A.eps);
+    }
+    const float* tab = nullptr;
+    int half = 0;
+    if (kind == 2) {
+      if (A.vcs) half = vdim >> 1, tab = A.vcs + (int64_t)t * half * 2;
+    } else if (A.cs) {
+      half = A.half, tab = A.cs + (int64_t)t * half * 2;
+    }
+    float* qd = A.q + (int64_t)t * nq + idx * dim;
+    T* cd = kind == 2 ? (T*)A.vc + slot * (int64_t)nv + idx * vdim : (T*)A.kc + slot * (int64_t)nk + idx * dim;
+    for (int d = lane; d < N; d += 64) {
+      float v = x[d] * inv * (w ? w[d] : 1.0f);
+      if (d < 2 * half) {
+        const bool lo = d < half;
+        const int i = lo ? d : d - half, od = lo ? d + half : d - half;
+        const float o = x[od] * inv * (w ? w[od] : 1.0f);
+        const float c = tab[2 * i], s = tab[2 * i + 1];
+        v = lo ? v * c - o * s : v * c + o * s;
+      }
+      if (kind == 0) qd[d] = v;
+      else El<T>::st(cd + d, v);
+    }
+  }
+}
+
+void launch_conv_tail(const void* in, int64_t ldi, void* state, const void* cu, const void* ctx, const void* sslots, int B,
+                      int C, int taps, int di, hipStream_t st);
+
+void launch_head_prep(const void* proj, int64_t ldp, int off_q, int off_k, int off_v, const void* conv, int taps,
+                      void* tail, int single, const void* cu, const void* ctx, const void* sslots, int B, const void* qw,
+                      const void* kw, int vnorm, float eps, const void* cs, int half, const void* vcs, void* q, void* kc,
+                      void* vc, const void* slots, int T_, int H, int G, int dim, int vdim, int dt, hipStream_t st) {
+  if (T_ == 0) return;
+  if (G < 1 || H % G) throw std::runtime_error("head_prep: heads must be a multiple of the key heads");
+  if (half < 0 || 2 * half > dim || (vcs && vdim % 2)) throw std::runtime_error("head_prep: rotation wider than a head");
+  const int nq = H * dim, nk = G * dim, nv = G * vdim, C = nq + nk + nv;
+  if (off_v == off_k && (conv || vdim != dim)) throw std::runtime_error("head_prep: shared keys need vdim == dim");
+  if (conv && (off_k != off_q + nq || off_v != off_k + nk || taps < 1 || !sslots || (taps > 1 && !tail)))
+    throw std::runtime_error("head_prep: the convolution takes contiguous q | k | v columns and a tail");
+  const size_t lds = (size_t)C * 4;
+  if (lds > 64 * 1024) throw std::runtime_error("head_prep: rows wider than 16384");
+  HeadPrepArgs A{proj, ldp, off_q, off_k, off_v, conv, taps, (float*)tail, single, (const int*)cu, (const int*)ctx,
+                 (const int*)sslots, B, (const float*)qw, (const float*)kw, vnorm, eps, (const float*)cs, half,
+                 (const float*)vcs, (float*)q, kc, vc, (const int64_t*)slots, H, G, dim, vdim};
+  const int vn = dt == 0 ? 8 : 4;
+  const auto al16 = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+  const bool vec = al16(proj) && al16(conv) && ldp % vn == 0 && off_q % vn == 0 && off_k % vn == 0 && off_v % vn == 0 &&
+                   nq % vn == 0 && nk % vn == 0 && nv % vn == 0;
+  if (dt == 0) {
+    if (vec) head_prep_kernel<bf16_t, 8><<<T_, 256, lds, st>>>(A);
+    else head_prep_kernel<bf16_t, 1><<<T_, 256, lds, st>>>(A);
+  } else if (dt == 1) {
+    if (vec) head_prep_kernel<float, 4><<<T_, 256, lds, st>>>(A);
+    else head_prep_kernel<float, 1><<<T_, 256, lds, st>>>(A);
+  } else {
+    throw std::runtime_error("bad dtype code");
+  }
+  HIP_CHECK_LAUNCH();
+  if (conv && taps > 1 && !single) {
+    const int es = dt == 0 ? 2 : 4;
+    launch_conv_tail((const char*)proj + (int64_t)off_q * es, ldp, tail, cu, ctx, sslots, B, C, taps, dt, st);
+  }
+}

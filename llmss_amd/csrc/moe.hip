@@ -1,8 +1,10 @@
 // Mixture-of-experts feed-forward: routing, grouping of (token, expert) pairs and the grouped expert GEMMs.
 //
 //   z = W_router h (fp32, gemm_any)                                   [T, E]
-//   moe_route:   s = sigmoid(z); the `top` experts with the largest s + correction are chosen (ties: the lower
+//   moe_route:   s = sigmoid(z), or softmax(z) over all experts; the `top` experts with the largest s + correction are chosen (ties: the lower
 //                index); weights = chosen s / (their sum + 1e-20)     -> idx [T, top] int32, wts [T, top] fp32
+//                A router may have more outputs than there are experts: the outputs from E on are identity experts,
+//                whose output is the layer's input row; their pairs are left out of the grouping (place -1).
 //   moe_group:   pairs p = t * top + j are bucketed by expert: off [E + 1], order [P] (pair at each sorted row),
 //                place [P] (sorted row of each pair) and a flat list of row tiles (expert, first row; 64 or 128 rows each) so the
 //                grouped GEMMs launch a grid whose size is known on the host (ceil(P / rows) + E tiles at most)
@@ -35,12 +37,21 @@ __device__ __forceinline__ float glu_value(float g, float u, float limit, float 
 // one wave per token; lanes over experts
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ z, const float* __restrict__ corr,
                                                        int* __restrict__ idx, float* __restrict__ wts, int E, int top,
-                                                       int norm) {
+                                                       int norm, int smax) {
   extern __shared__ float sc[];  // [E] scores, [E] choice values
   float* ch = sc + E;
   const int t = blockIdx.x, lane = threadIdx.x;
+  float mx = 0.f, den = 1.f;
+  if (smax) {
+    mx = -INFINITY, den = 0.f;
+    for (int e = lane; e < E; e += 64) mx = fmaxf(mx, z[(int64_t)t * E + e]);
+    mx = warp_max(mx);
+    for (int e = lane; e < E; e += 64) den += expf(z[(int64_t)t * E + e] - mx);
+    den = warp_sum(den);
+  }
   for (int e = lane; e < E; e += 64) {
-    const float s = 1.f / (1.f + expf(-z[(int64_t)t * E + e]));
+    const float ze = z[(int64_t)t * E + e];
+    const float s = smax ? expf(ze - mx) / den : 1.f / (1.f + expf(-ze));
     sc[e] = s;
     ch[e] = s + (corr ? corr[e] : 0.f);
   }
@@ -81,11 +92,11 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
 }
 
 void launch_moe_route(const void* z, const void* corr, void* idx, void* wts, int T_, int E, int top, int norm,
-                      hipStream_t st) {
+                      int smax, hipStream_t st) {
   if (T_ == 0) return;
   if (top > E || top <= 0) throw std::runtime_error("moe_route: top must be in [1, experts]");
   moe_route_kernel<<<T_, 64, 2 * E * sizeof(float), st>>>((const float*)z, (const float*)corr, (int*)idx, (float*)wts,
-                                                           E, top, norm);
+                                                           E, top, norm, smax);
   HIP_CHECK_LAUNCH();
 }
 
@@ -96,7 +107,7 @@ template <typename T>
 __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ h, int64_t ldh, const T* __restrict__ wr,
                                                          const float* __restrict__ corr, int* __restrict__ idx,
                                                          float* __restrict__ wts, int E, int K, int top, bool vec,
-                                                         int norm) {
+                                                         int norm, int smax) {
   extern __shared__ float sc[];  // [E] scores, [E] choice values
   float* ch = sc + E;
   const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, nw = blockDim.x >> 6;
@@ -114,12 +125,26 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ 
     }
     acc = warp_sum(acc);
     if (lane == 0) {
-      const float s = 1.f / (1.f + expf(-acc));
+      const float s = smax ? acc : 1.f / (1.f + expf(-acc));
       sc[e] = s;
       ch[e] = s + (corr ? corr[e] : 0.f);
     }
   }
   __syncthreads();
+  if (smax) {  // sc holds the logits: every wave forms their maximum and sum, then the scores replace them
+    float mx = -INFINITY, den = 0.f;
+    for (int e = lane; e < E; e += 64) mx = fmaxf(mx, sc[e]);
+    mx = warp_max(mx);
+    for (int e = lane; e < E; e += 64) den += expf(sc[e] - mx);
+    den = warp_sum(den);
+    __syncthreads();
+    for (int e = tid; e < E; e += blockDim.x) {
+      const float s = expf(sc[e] - mx) / den;
+      sc[e] = s;
+      ch[e] = s + (corr ? corr[e] : 0.f);
+    }
+    __syncthreads();
+  }
   float sum = 0.f;
   for (int j = 0; j < top; ++j) {
     float best = -INFINITY;
@@ -157,7 +182,7 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ 
 }
 
 void launch_moe_router(const void* h, int64_t ldh, const void* wr, const void* corr, void* idx, void* wts, int T_,
-                       int E, int K, int top, int dt, int norm, hipStream_t st) {
+                       int E, int K, int top, int dt, int norm, int smax, hipStream_t st) {
   if (T_ == 0) return;
   if (top > E || top <= 0) throw std::runtime_error("moe_router: top must be in [1, experts]");
   const int es = dt == 0 ? 2 : 4;
@@ -165,7 +190,7 @@ void launch_moe_router(const void* h, int64_t ldh, const void* wr, const void* c
   const int threads = E >= 16 ? 1024 : (E >= 8 ? 512 : 256);  // a wave per expert up to 16 waves
   DISPATCH_T(dt, T, (moe_router_kernel<T><<<T_, threads, 2 * E * sizeof(float), st>>>(
                         (const T*)h, ldh, (const T*)wr, (const float*)corr, (int*)idx, (float*)wts, E, K, top, vec,
-                        norm)));
+                        norm, smax)));
   HIP_CHECK_LAUNCH();
 }
 
@@ -182,7 +207,8 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int* __restrict__
   int* tile_r = tile_e + maxt;
   for (int e = threadIdx.x; e < E; e += blockDim.x) cnt[e] = 0;
   __syncthreads();
-  for (int p = threadIdx.x; p < P; p += blockDim.x) atomicAdd(&cnt[idx[p]], 1);
+  for (int p = threadIdx.x; p < P; p += blockDim.x)
+    if (idx[p] < E) atomicAdd(&cnt[idx[p]], 1);
   __syncthreads();
   if (threadIdx.x == 0) {
     int o = 0, nt = 0;
@@ -205,6 +231,10 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int* __restrict__
   // rows within an expert take whatever order the atomics give: every pair's row is computed on its own, so the
   // values do not depend on where the row lands
   for (int p = threadIdx.x; p < P; p += blockDim.x) {
+    if (idx[p] >= E) {  // an identity expert: no row of its own
+      place[p] = -1;
+      continue;
+    }
     const int o = atomicAdd(&cur[idx[p]], 1);
     order[o] = p;
     place[p] = o;
@@ -222,6 +252,7 @@ void launch_moe_group(const void* idx, int P, int E, int maxt, void* meta, void*
 }
 
 // ------------------------------------------------------------------------------------------------ grouped GEMMs
+// (wg null: experts without a gate, act = gelu(up), the error-function form)
 // grid (ceil(F / 64), maxt): tile y of the list covers sorted rows [row0, min(row0 + 64, off[e + 1])) of expert e.
 template <typename T>
 __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ h, int64_t ldh,
@@ -240,7 +271,7 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ 
   const int rows = min(TV_BM, off[e + 1] - row0);
   const int n0 = blockIdx.x * TV_BN;
   const int tid = threadIdx.x;
-  const T* G = wg + (int64_t)e * F * K;
+  const T* G = wg ? wg + (int64_t)e * F * K : nullptr;
   const T* U = wu + (int64_t)e * F * K;
   const int r = tid >> 2, kq = (tid & 3) * 4;
   const T* arow = r < rows ? h + (int64_t)(order[row0 + r] / top) * ldh : nullptr;
@@ -252,7 +283,7 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ 
       const int k = k0 + kq + i;
       const bool kin = k < K;
       As[kq + i][r] = (arow && kin) ? El<T>::ld(arow + k) : 0.f;
-      Gs[kq + i][r] = (n < F && kin) ? El<T>::ld(G + (int64_t)n * K + k) : 0.f;
+      Gs[kq + i][r] = (G && n < F && kin) ? El<T>::ld(G + (int64_t)n * K + k) : 0.f;
       Us[kq + i][r] = (n < F && kin) ? El<T>::ld(U + (int64_t)n * K + k) : 0.f;
     }
     __syncthreads();
@@ -269,7 +300,9 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ 
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int f = n0 + tx * 4 + j;
-      if (f < F) El<T>::st(act + (int64_t)(row0 + m) * F + f, glu_value(ag[i][j] * sw, au[i][j] * sw, limit, alpha, silu));
+      if (f >= F) continue;
+      const float v = wg ? glu_value(ag[i][j] * sw, au[i][j] * sw, limit, alpha, silu) : gelu_erf(au[i][j] * sw);
+      El<T>::st(act + (int64_t)(row0 + m) * F + f, v);
     }
   }
 }
@@ -343,22 +376,27 @@ void launch_moe_down(const void* act, const void* wd, const void* meta, void* y,
 template <typename T>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ y, const int* __restrict__ place,
                                                           const float* __restrict__ wts, const T* __restrict__ shared_,
-                                                          int64_t lds_, float* __restrict__ out, int N, int top) {
+                                                          int64_t lds_, float* __restrict__ out, int N, int top,
+                                                          const T* __restrict__ ident, int64_t ldi) {
   const int t = blockIdx.x;
   for (int c = threadIdx.x; c < N; c += blockDim.x) {
     float a = 0.f;
-    for (int j = 0; j < top; ++j)
-      a = fmaf(wts ? wts[(int64_t)t * top + j] : 1.0f, y[(int64_t)place[(int64_t)t * top + j] * N + c], a);
+    for (int j = 0; j < top; ++j) {
+      const int pl = place[(int64_t)t * top + j];
+      const float e = pl >= 0 ? y[(int64_t)pl * N + c] : (ident ? El<T>::ld(ident + (int64_t)t * ldi + c) : 0.f);
+      a = fmaf(wts ? wts[(int64_t)t * top + j] : 1.0f, e, a);
+    }
     if (shared_) a += El<T>::ld(shared_ + (int64_t)t * lds_ + c);
     out[(int64_t)t * N + c] = a;
   }
 }
 
 void launch_moe_combine(const void* y, const void* place, const void* wts, const void* shared_, int64_t lds_,
-                        void* out, int T_, int N, int top, int dt, hipStream_t st) {
+                        void* out, int T_, int N, int top, int dt, const void* ident, int64_t ldi, hipStream_t st) {
   if (T_ == 0) return;
   DISPATCH_T(dt, T, (moe_combine_kernel<T><<<T_, 256, 0, st>>>((const float*)y, (const int*)place, (const float*)wts,
-                                                                (const T*)shared_, lds_, (float*)out, N, top)));
+                                                                (const T*)shared_, lds_, (float*)out, N, top,
+                                                                (const T*)ident, ldi)));
   HIP_CHECK_LAUNCH();
 }
 

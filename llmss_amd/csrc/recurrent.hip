@@ -8,6 +8,10 @@
 //                    beta = sigmoid(b), g = exp(-exp(A_log[head]) softplus(a + dt_bias[head]))
 //   ssd   (MODE 2):  d = softplus(a + dt_bias[head]); S <- exp(-exp(A_log[head]) d) S + d k v^T
 //                    o = S^T q + D[head] v             (k = B, q = C of the head's group, v = the head's input x)
+//   exponential gates (mlstm, also MODE 2): S <- g S + e k v^T, n <- g n + e k, o = S^T q, den = n . q, where g and e
+//                    come ready from mlstm_gates: with the log gates i and f and a running maximum m (0 before the
+//                    sequence), m' = max(f + m, i), g = exp(f + m - m'), e = exp(i - m'). n is one more state column
+//                    whose value is always 1, walked by a workgroup of its own.
 //
 // Both updates act on the columns of S independently: column c needs only v[c] and the whole k and q. So a thread
 // owns one column, split over 1, 2 or 4 neighbouring lanes (32 to 128 state values in registers each) that reduce
@@ -62,7 +66,9 @@ struct RecArgs {
   int64_t ldo;
   int H, G, dim, vdim, silu_in;
   int gates_ready;  // delta: a / b already hold g / beta (delta_gates_kernel), nothing left to compute while staging
-  const float* skip;  // ssd: D [H]
+  const float* skip;  // ssd: D [H] (null: no skip term)
+  float* nstate;      // mlstm: [slots, H, dim] or null
+  float* den;         // mlstm: [T, H]
 };
 
 // TQ: storage of q / k / v; TP: storage of a / b. R: state values per lane, P lanes per column. Staging: every
@@ -81,21 +87,25 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecArgs A, int P, int c
   if (qlen <= 0) return;
   const int t0 = A.cu[b], n = A.ctx[b], slot = A.sslots[b];
   const int cidx = min((int)threadIdx.x / P, cols - 1);
-  const int col = zb * cols + cidx, part = threadIdx.x % P;
-  const bool live = col < vdim && (int)threadIdx.x < cols * P;
+  const bool ncol = MODE == 2 && A.nstate && zb == (int)gridDim.y - 1;  // the normaliser's column
+  const int col = ncol ? 0 : zb * cols + cidx, part = threadIdx.x % P;
+  const bool live = ncol ? (int)threadIdx.x < P : (col < vdim && (int)threadIdx.x < cols * P);
+  const int svd = ncol ? 1 : vdim;  // columns of the state walked here
+  float* outp = ncol ? A.den + h : A.out + (int64_t)h * vdim + col;
+  const int64_t ldo = ncol ? A.H : A.ldo;
   if (slot < 0 || n <= 0) {
     if (live && part == 0)
-      for (int j = 0; j < qlen; ++j) A.out[(int64_t)(t0 + j) * A.ldo + (int64_t)h * vdim + col] = 0.f;
+      for (int j = 0; j < qlen; ++j) outp[(int64_t)(t0 + j) * ldo] = 0.f;
     return;
   }
   const int p0 = n - qlen;
   const int d0 = part * R;  // this lane's rows of the column: d0 .. d0 + R - 1
   float S[R];
-  float* sp = A.state + (((int64_t)slot * A.H + h) * dim) * vdim;
+  float* sp = (ncol ? A.nstate : A.state) + (((int64_t)slot * A.H + h) * dim) * svd;
   if (p0 > 0) {  // rows past dim and lanes without a column read a valid address and drop the value
-    const int cc = min(col, vdim - 1);
+    const int cc = min(col, svd - 1);
 #pragma unroll
-    for (int i = 0; i < R; ++i) S[i] = sp[(int64_t)min(d0 + i, dim - 1) * vdim + cc];
+    for (int i = 0; i < R; ++i) S[i] = sp[(int64_t)min(d0 + i, dim - 1) * svd + cc];
 #pragma unroll
     for (int i = 0; i < R; ++i) S[i] = (live && d0 + i < dim) ? S[i] : 0.f;
   } else {
@@ -107,12 +117,12 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecArgs A, int P, int c
   const int per = (2 * dimp + cols + 2 + 3) & ~3;
   float a_const = 0.f, dtb = 0.f;
   if (MODE == 0) a_const = A.decay[h];
-  else {
+  else if (A.decay) {
     a_const = expf(A.decay[h]);
     dtb = A.dt_bias[h];
   }
   const float qmul = MODE == 1 ? 1.0f / sqrtf((float)dim) : 1.0f;
-  const float dskip = MODE == 2 ? A.skip[h] : 0.f;
+  const float dskip = MODE == 2 && A.skip ? A.skip[h] : 0.f;
   // this thread's staged numbers: slots 0 .. REC_NE - 2 hold k / q / v entries (storage TQ), the last slot the
   // head's two per-token scalars (storage TP, threads 0 and 1). A slot without an entry points at a valid address
   // all the same, so every load is unconditional and the whole batch is in flight together.
@@ -185,7 +195,7 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecArgs A, int P, int c
     for (int jj = 0; jj < nt; ++jj) {
       const float* ks = sm + jj * per;
       const float* qs = ks + dimp;
-      const float vv = ks[2 * dimp + cidx];
+      const float vv = ncol ? 1.0f : ks[2 * dimp + cidx];
       // k and q come from LDS 32 numbers at a time by 16-byte reads issued together (a wave alone on its SIMD has
       // nobody to hide a read's latency behind), sums run in four partial accumulators
       float o4[4] = {0.f, 0.f, 0.f, 0.f};
@@ -262,13 +272,13 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecArgs A, int P, int c
       float o = (o4[0] + o4[1]) + (o4[2] + o4[3]);
       o = part_sum(o, P);
       if (MODE == 2) o = fmaf(dskip, vv, o);
-      if (live && part == 0) A.out[(int64_t)(t0 + j0 + jj) * A.ldo + (int64_t)h * vdim + col] = o;
+      if (live && part == 0) outp[(int64_t)(t0 + j0 + jj) * ldo] = o;
     }
   }
   if (live) {
 #pragma unroll
     for (int i = 0; i < R; ++i)
-      if (d0 + i < dim) sp[(int64_t)(d0 + i) * vdim + col] = S[i];
+      if (d0 + i < dim) sp[(int64_t)(d0 + i) * svd + col] = S[i];
   }
 }
 
@@ -286,7 +296,7 @@ static void recurrence_t(const RecArgs& A, int B, hipStream_t st) {
   const int per = (2 * dimp + cols + 2 + 3) & ~3;
   const int threads = ((std::max(cols * P, (2 * dimp + cols + REC_NE - 2) / (REC_NE - 1)) + 63) / 64) * 64;
   if (threads > 256) throw std::runtime_error("recurrence: too many numbers per token to stage");
-  dim3 g(A.H, (vdim + cols - 1) / cols, B);
+  dim3 g(A.H, (vdim + cols - 1) / cols + (MODE == 2 && A.nstate ? 1 : 0), B);
   if (B > 65535 || g.y > 65535) throw std::runtime_error("recurrence: too many sequences or columns");
   const size_t lds = ((size_t)REC_CT * per + 4 * 128) * 4;  // + room for the last token's reads past its k / q
   if (R == 32) recurrence_kernel<TQ, TP, 32, MODE><<<g, threads, lds, st>>>(A, P, cols);
@@ -298,12 +308,12 @@ void launch_recurrence(int mode, const void* q, const void* k, const void* v, in
                        const void* ab, int64_t ldab, int off_a, int off_b, const void* decay, const void* dt_bias,
                        void* state, const void* cu, const void* ctx, const void* sslots, void* out, int64_t ldo, int B,
                        int H, int G, int dim, int vdim, int silu_in, int gates_ready, int dq, int dp, const void* skip,
-                       hipStream_t st) {
+                       void* nstate, void* den, hipStream_t st) {
   if (B == 0) return;
   if (G < 1 || H % G) throw std::runtime_error("recurrence: heads must be a multiple of the key heads");
   RecArgs A{q, k, v, ldq, ldk, ldv, ab, ldab, off_a, off_b, (const float*)decay, (const float*)dt_bias, (float*)state,
             (const int*)cu, (const int*)ctx, (const int*)sslots, (float*)out, ldo, H, G, dim, vdim, silu_in, gates_ready,
-            (const float*)skip};
+            (const float*)skip, (float*)nstate, (float*)den};
   if (mode == 0) DISPATCH_T(dq, TQ, (recurrence_t<TQ, float, 0>(A, B, st)));
   else if (mode == 2) DISPATCH_T(dq, TQ, DISPATCH_T(dp, TP, (recurrence_t<TQ, TP, 2>(A, B, st))));
   else DISPATCH_T(dq, TQ, DISPATCH_T(dp, TP, (recurrence_t<TQ, TP, 1>(A, B, st))));
@@ -348,5 +358,67 @@ void launch_delta_gates(const void* a, const void* b, int64_t ld, const void* A_
   if (T_ == 0) return;
   DISPATCH_T(dt, T, (delta_gates_kernel<T><<<(T_ * H + 255) / 256, 256, 0, st>>>(
       (const T*)a, (const T*)b, ld, (const float*)A_log, (const float*)dt_bias, (float*)gates, T_, H)));
+  HIP_CHECK_LAUNCH();
+}
+
+// Gates of the exponential-gate recurrence (mlstm). Per token and head, from the projections' columns zi and zf:
+//   i = cap tanh((zi + bi) / cap), f = logsigmoid(cap tanh((zf + bf) / cap)), m' = max(f + m, i), m = 0 before position 0
+// out: gates [T, H, 4] = (f, i, m', m) and ab [T, 2H] = (g | e) = (exp(f + m - m') | exp(i - m')); the sequence's running
+// maximum [slots, H] is read from and renewed in its slot. (sum of f, m) pairs compose associatively - first (F1, M1), then
+// (F2, M2) give (F1 + F2, max(F2 + M1, M2)) - so a wave scans 64 tokens at a time: one wave per (head, sequence).
+template <typename T>
+__global__ __launch_bounds__(64) void mlstm_gates_kernel(const T* __restrict__ zi, const T* __restrict__ zf, int64_t ld,
+                                                         const float* __restrict__ bi, const float* __restrict__ bf,
+                                                         float cap, float* __restrict__ mstate,
+                                                         const int* __restrict__ cu, const int* __restrict__ ctx,
+                                                         const int* __restrict__ sslots, f32x4* __restrict__ gates,
+                                                         float* __restrict__ ab, int H) {
+  const int h = blockIdx.x, b = blockIdx.y, lane = threadIdx.x;
+  const int t0 = cu[b], qlen = cu[b + 1] - t0, n = ctx[b], slot = sslots[b];
+  if (qlen <= 0) return;
+  const bool real = slot >= 0 && n > 0;
+  float m = real && n > qlen ? mstate[(int64_t)slot * H + h] : 0.f;
+  const float icap = 1.0f / cap;
+  for (int j0 = 0; j0 < qlen; j0 += 64) {
+    const int j = j0 + lane;
+    const bool in = j < qlen;
+    float f = 0.f, i = -INFINITY;  // past the end: the pair that changes nothing
+    if (in) {
+      i = cap * tanhf((El<T>::ld(zi + (int64_t)(t0 + j) * ld + h) + bi[h]) * icap);
+      const float z = cap * tanhf((El<T>::ld(zf + (int64_t)(t0 + j) * ld + h) + bf[h]) * icap);
+      f = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+    }
+    float F = f, M = i;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const float F1 = __shfl_up(F, o, 64), M1 = __shfl_up(M, o, 64);
+      if (lane >= o) {
+        M = fmaxf(F + M1, M);
+        F += F1;
+      }
+    }
+    const float mt = fmaxf(F + m, M);
+    float mp = __shfl_up(mt, 1, 64);
+    if (lane == 0) mp = m;
+    if (in) {
+      const int64_t e = (int64_t)(t0 + j) * H + h;
+      gates[e] = f32x4{f, i, mt, mp};
+      ab[(int64_t)(t0 + j) * 2 * H + h] = expf(f + mp - mt);
+      ab[(int64_t)(t0 + j) * 2 * H + H + h] = expf(i - mt);
+    }
+    m = __shfl(mt, min(63, qlen - 1 - j0), 64);
+  }
+  if (real && lane == 0) mstate[(int64_t)slot * H + h] = m;
+}
+
+void launch_mlstm_gates(const void* zi, const void* zf, int64_t ld, const void* bi, const void* bf, float cap,
+                        void* mstate, const void* cu, const void* ctx, const void* sslots, void* gates, void* ab, int B,
+                        int H, int dt, hipStream_t st) {
+  if (B == 0) return;
+  if (B > 65535) throw std::runtime_error("mlstm_gates: too many sequences");
+  dim3 g(H, B);
+  DISPATCH_T(dt, T, (mlstm_gates_kernel<T><<<g, 64, 0, st>>>(
+      (const T*)zi, (const T*)zf, ld, (const float*)bi, (const float*)bf, cap, (float*)mstate, (const int*)cu,
+      (const int*)ctx, (const int*)sslots, (f32x4*)gates, (float*)ab, H)));
   HIP_CHECK_LAUNCH();
 }

@@ -6,9 +6,14 @@
 //   token_side_add:     e = table[id, col0 : col0 + d]; g = gelu_tanh(Wg x) * e; y = Wp g;
 //                       x += rms_norm(y) * wn, then the same optional `add` and `h`
 //
+// A norm may be taken in `groups` equal consecutive parts of the row, each divided by its own root mean square
+// (groups = 1: the whole row); both norms of a launch take the same number of parts.
+//
 // so a sublayer's closing op also forms the next reader's input, as add_norm does for the uniform families. y is
 // either a dense row in the storage type, or the still uncombined output of a mixture-of-experts layer (moe.hip):
 // y[t] = sum_j (wts ? wts[t, j] : 1) * ey[place[t * top + j]] (+ shared[t]), j ascending, then the shared expert.
+// A pair whose place is negative chose an identity expert: its output is ident[t], the sublayer's own input row. Or y
+// is the result of two mixers side by side, y = 1/2 (rms_norm(y) * wl + rms_norm(y2) * wr), both norms over the whole row.
 // Norm weights, biases and layer scales are fp32. One workgroup per row; the gated row lives in LDS between the
 // pass that sums its squares and the pass that adds it, and the updated x between that pass and the norm.
 #include "anytype.h"
@@ -33,6 +38,13 @@ struct SandwichArgs {
   int64_t ldh;
   float eps;
   int W;
+  int groups;
+  const void* ident;  // [T, W] in the storage type
+  int64_t ldi;
+  const void* y2;
+  int64_t ldy2;
+  const float* wl;
+  const float* wr;
 };
 
 template <typename T, int V>
@@ -58,18 +70,38 @@ __device__ __forceinline__ void stv(T* p, const float* v) {
   }
 }
 
+// 1 / root mean square of every part of the row in buf, left behind the row: buf[W + g]. A wave per part.
+__device__ __forceinline__ void part_inv(float* buf, const SandwichArgs& p) {
+  const int n = p.W / p.groups, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
+  __syncthreads();
+  for (int g = threadIdx.x >> 6; g < p.groups; g += nw) {
+    float s = 0.f;
+    for (int c = lane; c < n; c += 64) s = fmaf(buf[g * n + c], buf[g * n + c], s);
+    s = warp_sum(s);
+    if (lane == 0) buf[p.W + g] = 1.0f / sqrtf(s / (float)n + p.eps);
+  }
+  __syncthreads();
+}
+
 // the tail both kernels share: buf holds the updated x row; writes h = rms_norm(x) * wnext
 template <typename T, int V>
-__device__ __forceinline__ void norm_out(const float* buf, float ss, const SandwichArgs& p, int t, float* red) {
+__device__ __forceinline__ void norm_out(float* buf, float ss, const SandwichArgs& p, int t, float* red) {
   if (!p.wnext) return;
-  ss = block_sum(ss, red);
-  const float inv = 1.0f / sqrtf(ss / (float)p.W + p.eps);
+  float inv = 0.f;
+  const float* invs = nullptr;
+  if (p.groups > 1) {
+    part_inv(buf, p);
+    invs = buf + p.W;
+  } else {
+    ss = block_sum(ss, red);
+    inv = 1.0f / sqrtf(ss / (float)p.W + p.eps);
+  }
   T* hr = (T*)p.h + (int64_t)t * p.ldh;
   for (int c = threadIdx.x * V; c < p.W; c += blockDim.x * V) {
     float w[V], o[V];
     ldv<float, V>(p.wnext + c, w);
 #pragma unroll
-    for (int i = 0; i < V; ++i) o[i] = buf[c + i] * inv * w[i];
+    for (int i = 0; i < V; ++i) o[i] = buf[c + i] * (invs ? invs[(c + i) / (p.W / p.groups)] : inv) * w[i];
     stv<T, V>(hr + c, o);
   }
 }
@@ -77,7 +109,7 @@ __device__ __forceinline__ void norm_out(const float* buf, float ss, const Sandw
 template <typename T, int V>
 __global__ __launch_bounds__(256) void sandwich_add_norm_kernel(SandwichArgs p) {
   extern __shared__ __attribute__((aligned(16))) float buf[];
-  __shared__ float red[16];
+  __shared__ float red[32];
   const int t = blockIdx.x, W = p.W;
   float* xr = p.x + (int64_t)t * W;
   const bool has_y = p.y != nullptr || p.ey != nullptr;
@@ -86,18 +118,46 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_kernel(SandwichArgs p) 
     const T* yr = p.y ? (const T*)p.y + (int64_t)t * p.ldy : nullptr;
     const T* sr = p.shared_ ? (const T*)p.shared_ + (int64_t)t * p.lds_ : nullptr;
     const T* rr = p.r ? (const T*)p.r + (int64_t)t * p.ldr : nullptr;
+    const T* y2r = p.y2 ? (const T*)p.y2 + (int64_t)t * p.ldy2 : nullptr;
+    float il = 0.f, ir = 0.f;
+    if (y2r) {  // two mixers: the root mean square of each row first
+      float sl = 0.f, sr2 = 0.f;
+      for (int c = threadIdx.x * V; c < W; c += blockDim.x * V) {
+        float a[V], b[V];
+        ldv<T, V>(yr + c, a);
+        ldv<T, V>(y2r + c, b);
+#pragma unroll
+        for (int i = 0; i < V; ++i) {
+          sl = fmaf(a[i], a[i], sl);
+          sr2 = fmaf(b[i], b[i], sr2);
+        }
+      }
+      const f32x2 s2 = block_sum2(sl, sr2, red);
+      il = 0.5f / sqrtf(s2[0] / (float)W + p.eps);
+      ir = 0.5f / sqrtf(s2[1] / (float)W + p.eps);
+    }
     float ss = 0.f;
     for (int c = threadIdx.x * V; c < W; c += blockDim.x * V) {
       float v[V];
-      if (yr) {
+      if (y2r) {
+        float a[V], b[V], wa[V], wb[V];
+        ldv<T, V>(yr + c, a);
+        ldv<T, V>(y2r + c, b);
+        ldv<float, V>(p.wl + c, wa);
+        ldv<float, V>(p.wr + c, wb);
+#pragma unroll
+        for (int i = 0; i < V; ++i) v[i] = fmaf(a[i] * il, wa[i], b[i] * ir * wb[i]);
+      } else if (yr) {
         ldv<T, V>(yr + c, v);
       } else {
 #pragma unroll
         for (int i = 0; i < V; ++i) v[i] = 0.f;
         for (int j = 0; j < p.top; ++j) {
           const float wj = p.wts ? p.wts[(int64_t)t * p.top + j] : 1.0f;
+          const int pl = p.place[(int64_t)t * p.top + j];
           float e[V];
-          ldv<float, V>(p.ey + (int64_t)p.place[(int64_t)t * p.top + j] * W + c, e);
+          if (pl >= 0) ldv<float, V>(p.ey + (int64_t)pl * W + c, e);
+          else ldv<T, V>((const T*)p.ident + (int64_t)t * p.ldi + c, e);
 #pragma unroll
           for (int i = 0; i < V; ++i) v[i] = fmaf(wj, e[i], v[i]);
         }
@@ -121,10 +181,15 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_kernel(SandwichArgs p) 
         ss = fmaf(v[i], v[i], ss);
       }
     }
-    ss = block_sum(ss, red);
-    inv = 1.0f / sqrtf(ss / (float)W + p.eps);
+    if (p.groups > 1) {
+      part_inv(buf, p);
+    } else {
+      ss = block_sum(ss, red);
+      inv = 1.0f / sqrtf(ss / (float)W + p.eps);
+    }
   }
   const float* ar = p.add ? p.add + (int64_t)t * W : nullptr;
+  const int part = W / p.groups;
   float ss2 = 0.f;
   for (int c = threadIdx.x * V; c < W; c += blockDim.x * V) {
     float xv[V];
@@ -133,7 +198,7 @@ __global__ __launch_bounds__(256) void sandwich_add_norm_kernel(SandwichArgs p) 
       float w[V];
       ldv<float, V>(p.wpost + c, w);
 #pragma unroll
-      for (int i = 0; i < V; ++i) xv[i] = fmaf(buf[c + i] * inv, w[i], xv[i]);
+      for (int i = 0; i < V; ++i) xv[i] = fmaf(buf[c + i] * (p.groups > 1 ? buf[W + (c + i) / part] : inv), w[i], xv[i]);
     }
     if (ar) {
       float a[V];
@@ -156,16 +221,20 @@ static bool al16(const void* p) { return ((uintptr_t)p & 15) == 0; }
 void launch_sandwich_add_norm(void* x, const void* y, int64_t ldy, const void* ey, const void* place, const void* wts,
                               int top, const void* shared_, int64_t lds_, const void* r, int64_t ldr, const void* rb,
                               const void* wpost, const void* add, const void* wnext, void* h, int64_t ldh, float eps,
-                              int T_, int W, int dt, hipStream_t st) {
+                              int groups, const void* ident, int64_t ldi, const void* y2, int64_t ldy2, const void* wl,
+                              const void* wr, int T_, int W, int dt, hipStream_t st) {
   if (T_ == 0) return;
-  if ((size_t)W * 4 > 64 * 1024) throw std::runtime_error("sandwich_add_norm: rows wider than 16384");
+  if (groups < 1 || W % groups) throw std::runtime_error("sandwich_add_norm: the norm's parts must divide the row");
+  if (((size_t)W + groups) * 4 > 64 * 1024) throw std::runtime_error("sandwich_add_norm: rows wider than 16384");
   SandwichArgs p{(float*)x, y, ldy, (const float*)ey, (const int*)place, (const float*)wts, top, shared_, lds_, r, ldr,
-                 (const float*)rb, (const float*)wpost, (const float*)add, (const float*)wnext, h, ldh, eps, W};
+                 (const float*)rb, (const float*)wpost, (const float*)add, (const float*)wnext, h, ldh, eps, W, groups, ident, ldi, y2, ldy2,
+                 (const float*)wl, (const float*)wr};
   const int es = dt == 0 ? 2 : 4;
   const auto alv = [&](const void* q, int64_t ld) { return !q || (((uintptr_t)q % (4 * es)) == 0 && ld % 4 == 0); };
   const bool vec = W % 4 == 0 && al16(x) && al16(ey) && al16(rb) && al16(wpost) && al16(add) && al16(wnext) &&
-                   alv(y, ldy) && alv(shared_, lds_) && alv(r, ldr) && alv(h, ldh);
-  const size_t lds = (size_t)W * 4;
+                   alv(y, ldy) && alv(shared_, lds_) && alv(r, ldr) && alv(h, ldh) && alv(ident, ldi) && alv(y2, ldy2) &&
+                   al16(wl) && al16(wr);
+  const size_t lds = ((size_t)W + (groups > 1 ? groups : 0)) * 4;
   DISPATCH_T(dt, T, {
     if (vec) sandwich_add_norm_kernel<T, 4><<<T_, 256, lds, st>>>(p);
     else sandwich_add_norm_kernel<T, 1><<<T_, 256, lds, st>>>(p);
@@ -274,7 +343,7 @@ void launch_token_side_add(void* x, const void* ids, const void* table, int64_t 
   const size_t lds = ((size_t)2 * W + d) * 4;
   if (lds > 64 * 1024) throw std::runtime_error("token_side_add: rows too wide");
   SandwichArgs p{};
-  p.x = (float*)x; p.add = (const float*)add; p.wnext = (const float*)wnext; p.h = h; p.ldh = ldh; p.eps = eps; p.W = W;
+  p.x = (float*)x; p.add = (const float*)add; p.wnext = (const float*)wnext; p.h = h; p.ldh = ldh; p.eps = eps; p.W = W; p.groups = 1;
   SideArgs s{(const int64_t*)ids, table, ldt, vocab, col0, d, wg, wp, (const float*)wn};
   const int es = dt == 0 ? 2 : 4;
   const bool vec = W % 4 == 0 && al16(x) && al16(wn) && al16(add) && al16(wnext) && ((uintptr_t)wg % (4 * es)) == 0 &&

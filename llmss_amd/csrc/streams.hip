@@ -330,6 +330,17 @@ static void causal_conv_t(const void* in, int64_t ldi, const void* w, void* stat
   }
 }
 
+// The tail's renewal alone (head_prep.hip forms the convolution's output itself)
+void launch_conv_tail(const void* in, int64_t ldi, void* state, const void* cu, const void* ctx, const void* sslots, int B,
+                      int C, int taps, int di, hipStream_t st) {
+  if (B == 0 || taps <= 1) return;
+  if (taps - 1 > MAX_TAIL) throw std::runtime_error("conv_tail: 1 to 17 taps");
+  dim3 g(B, (C + 255) / 256);
+  DISPATCH_T(di, TI, (conv_tail_kernel<TI><<<g, 256, 0, st>>>((const TI*)in, ldi, (float*)state, (const int*)cu,
+                                                              (const int*)ctx, (const int*)sslots, C, taps)));
+  HIP_CHECK_LAUNCH();
+}
+
 // di / dw / dout: storage types of the input, the weights and the output (0 bf16, 1 fp32)
 void launch_causal_conv(const void* in, int64_t ldi, const void* w, void* state, const void* cu, const void* ctx,
                         const void* sslots, void* out, int64_t ldo, int T_, int B, int C, int taps, int res, int silu,
@@ -345,12 +356,15 @@ void launch_causal_conv(const void* in, int64_t ldi, const void* w, void* state,
 // out[t, g * n + i] = c * o[t, g * n + i] / sqrt(mean_i(o[t, g, :]^2) + eps) * w[i] * act(gate[t, g * n + i])
 // act 0: sigmoid, 1: silu. o fp32; gate, w and out in the storage type. wfull: w holds a weight per column, w[g * n +
 // i]. first: the gate comes before the norm, out = c * u / sqrt(mean(u^2) + eps) * w with u = o * act(gate).
+// den [T, groups] with gates [T, groups, 4] (the exponential-gate recurrence, recurrent.hip): o and den are numerator
+// and normaliser of a group and token, o <- qs * o / (max(|qs * den|, exp(-gates[2])) + 1e-6) comes first.
 template <typename T>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __restrict__ o, int64_t ldo,
                                                                const T* __restrict__ gate, int64_t ldg,
                                                                const T* __restrict__ w, float eps, int act, float c,
                                                                T* __restrict__ out, int64_t ldout, int n, int wfull,
-                                                               int first) {
+                                                               int first, const float* __restrict__ den,
+                                                               const f32x4* __restrict__ gates, float qs) {
   __shared__ float red[32];
   const int t = blockIdx.x, g = blockIdx.y;
   const float* row = o + (int64_t)t * ldo + (int64_t)g * n;
@@ -361,13 +375,18 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
     const float sg = 1.0f / (1.0f + expf(-z));
     return act ? z * sg : sg;
   };
+  float pre = 1.0f;
+  if (den) {
+    const int64_t e = (int64_t)t * gridDim.y + g;
+    pre = qs / (fmaxf(fabsf(qs * den[e]), expf(-gates[e][2])) + 1e-6f);
+  }
   float ss = 0.f;
   for (int i = threadIdx.x; i < n; i += blockDim.x) {
-    const float u = first ? row[i] * gate_of(i) : row[i];
+    const float u = (first ? row[i] * gate_of(i) : row[i]) * pre;
     ss = fmaf(u, u, ss);
   }
   ss = block_sum(ss, red);
-  const float inv = c / sqrtf(ss / (float)n + eps);
+  const float inv = pre * c / sqrtf(ss / (float)n + eps);
   T* dst = out + (int64_t)t * ldout + (int64_t)g * n;
   for (int i = threadIdx.x; i < n; i += blockDim.x)
     El<T>::st(dst + i, row[i] * inv * El<T>::ld(wr + i) * gate_of(i));
@@ -375,14 +394,15 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
 
 void launch_gated_group_norm(const void* o, int64_t ldo, const void* gate, int64_t ldg, const void* w, float eps,
                              int act, float c, void* out, int64_t ldout, int T_, int groups, int n, int dt, int wfull,
-                             int first, hipStream_t st) {
+                             int first, const void* den, const void* gates, float qs, hipStream_t st) {
   if (T_ == 0) return;
   if (groups > 65535) throw std::runtime_error("gated_group_norm: too many groups");
   dim3 g(T_, groups);
   const int threads = n >= 256 ? 256 : ((n + 63) / 64) * 64;
   DISPATCH_T(dt, T, (gated_group_norm_kernel<T><<<g, threads, 0, st>>>((const float*)o, ldo, (const T*)gate, ldg,
                                                                         (const T*)w, eps, act, c, (T*)out, ldout, n,
-                                                                        wfull, first)));
+                                                                        wfull, first, (const float*)den,
+                                                                        (const f32x4*)gates, qs)));
   HIP_CHECK_LAUNCH();
 }
 
@@ -410,9 +430,12 @@ void launch_glu_act(const void* gu, int64_t ldg, void* out, int64_t ldo, int T_,
 
 // out[t, f] = act(x[t, f]), no gate. act 0: tanh-form GELU, 1: SiLU, 2: xIELU with the two coefficients (a, b):
 //   z > 0: a z^2 + z / 2;   z <= 0: b (exp(z) - 1 - z) + z / 2
+// 3: error-function GELU, 4: the square of relu
 __device__ __forceinline__ float act_value(float z, int act, float a, float b) {
   if (act == 0) return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
   if (act == 1) return z / (1.0f + expf(-z));
+  if (act == 3) return gelu_erf(z);
+  if (act == 4) return apply_act(z, ACT_RELU2);
   return z > 0.f ? fmaf(a * z, z, 0.5f * z) : fmaf(b, expm1f(z) - z, 0.5f * z);
 }
 

@@ -35,6 +35,13 @@ Families (``MODEL_REGISTRY`` keys, reference ``custom_modeling/__init__.py:4-7``
                     neighbour-pair rotation) and ``mamba2`` (state-space duality: decayed matrix state per head, short
                     convolution, gate before a grouped norm); feed-forward dense SiLU-gated or mixture of experts whose
                     sigmoid score multiplies the expert's input; scaled logits, untied head.
+* ``tefudra``     - per-layer description: blocks normed before and after each sublayer, the norms taken in equal parts of
+                    the row; mixers ``window_attention`` (normed, half-rotated queries and keys, the projected keys as values,
+                    a sliding window that keeps the first positions, a learned sink per head) and ``pair`` (soft-capped
+                    window attention with projection biases, short convolutions and normed, rotated values beside a matrix
+                    memory with exponential gates, ``mlstm``, each normed over the row and averaged); feed-forward dense
+                    squared-relu or mixture of ungated GELU experts with softmax scores and identity experts; layers may
+                    share another layer's weights; tied head.
 """
 from __future__ import annotations
 
@@ -83,9 +90,12 @@ class MoESpec:
     expert: ExpertSpec
     shared: Optional[ExpertSpec] = None
     kind: str = "moe"
-    act: str = "glu_clamp"  # "glu_clamp": g sigmoid(1.702 g) (u + 1) with clamps; "silu": silu(g) u, no clamps
+    # "glu_clamp": g sigmoid(1.702 g) (u + 1) with clamps; "silu": silu(g) u, no clamps; "gelu": no gate, gelu(u)
+    act: str = "glu_clamp"
     normalize: bool = True  # the chosen scores are divided by their sum
     weight_input: bool = False  # the score multiplies the expert's input (sum_e expert_e(w_e h)), not its output
+    score: str = "sigmoid"  # or "softmax" over all router outputs
+    identity: int = 0  # router outputs after the experts': identity experts, whose output is the layer's input
 
 
 @dataclass
@@ -155,6 +165,62 @@ class PoolAttnSpec:
 
 
 @dataclass
+class WindowAttnSpec:
+    """Softmax attention over a paged key/value cache: ``heads`` query heads on ``kv_heads`` key/value heads, scores times
+    ``scale``, soft-capped when ``softcap`` > 0. Position i sees j <= i with i - j < ``window`` (0: all) or j <
+    ``keep_first``. ``rot``: rotation of the halves of the first ``rot.dims`` numbers of every query and key head;
+    ``qk_norm``: queries and keys RMS-normed per head with a learned weight before it; ``shared_kv``: no value projection,
+    the values are the keys as projected; ``sink``: exp of a learned number per head in the softmax denominator; ``bias``:
+    the projections (output too) have biases; ``conv`` > 0: q, k and v pass a causal convolution of that many taps first;
+    ``v_norm``: values divided per head by their root mean square; ``rot_values``: values turned by their position over
+    all vdim numbers (the keys' base) and every head's result turned back by its own."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int = 0
+    keep_first: int = 0
+    softcap: float = 0.0
+    rot: Optional[RotarySpec] = None
+    qk_norm: bool = False
+    shared_kv: bool = False
+    sink: bool = False
+    bias: bool = False
+    conv: int = 0
+    v_norm: bool = False
+    rot_values: bool = False
+    kind: str = "window_attention"
+
+    @property
+    def qkv_columns(self) -> int:
+        return self.heads * self.dim + self.kv_heads * (self.dim + (0 if self.shared_kv else self.vdim))
+
+
+@dataclass
+class MLSTMSpec:
+    """Matrix memory with exponential gates: a matrix state [dim, vdim], a normaliser [dim] and a running maximum per head;
+    log input and forget gates soft-capped by ``gate_cap``; the heads' results are RMS-normed per head and gated."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+    kind: str = "mlstm"
+
+
+@dataclass
+class PairMixerSpec:
+    """Two mixers reading the same input; the result is half the sum of the two, each RMS-normed over the row first."""
+    left: Any
+    right: Any
+    kind: str = "pair"
+
+    @property
+    def heads(self) -> int:
+        return self.left.heads
+
+
+@dataclass
 class SSDSpec:
     """State-space mixer with a scalar decay per head and token: a matrix state [state, vdim] per head, ``groups``
     input / output vectors (B, C) shared by heads / groups heads each, x | B | C through a causal convolution of
@@ -221,7 +287,8 @@ class ParallelMixerSpec:
 @dataclass
 class DenseMLPSpec:
     """Feed-forward down(act(gate h) * (up h)), or, ``gated`` false, down(act(up h)). ``act``: ``gelu_tanh``,
-    ``silu`` or ``xielu`` (two learned numbers per layer)."""
+    ``silu``, ``xielu`` (two learned numbers per layer) or, ungated, ``gelu`` (error function) and ``relu2`` (the square of
+    relu)."""
     ff: int
     act: str = "gelu_tanh"
     kind: str = "dense"
@@ -284,6 +351,8 @@ class ModelConfig:
     token_side_dim: int = 0  # > 0: after the feed-forward a layer adds a normed projection of its slice of a second token table
     loop: Optional[tuple] = None  # (start, stop, times): layers start .. stop - 1 run ``times`` times in a row
     logit_scale: float = 1.0
+    norm_groups: int = 1  # sandwich blocks: every norm is taken in that many equal consecutive parts of the row
+    weights_of: Optional[List[int]] = None  # per layer: the layer whose weights it uses (itself: its own)
 
     def layer_runs(self) -> List[int]:
         """Layer index of every layer run, in order: a looped stretch repeats with the same weights, each pass with
@@ -313,11 +382,11 @@ class ModelConfig:
 
     def num_params(self) -> int:
         h, f, v = self.hidden_size, self.intermediate_size, self.vocab_size
-        if self.layer_specs and self.model_type in ("babotar", "lamisun", "fizelix"):
-            from .weights import babotar_shapes, fizelix_shapes, lamisun_shapes
+        if self.layer_specs and self.model_type in ("babotar", "lamisun", "fizelix", "tefudra"):
+            from .weights import babotar_shapes, fizelix_shapes, lamisun_shapes, tefudra_shapes
 
-            shapes = {"babotar": babotar_shapes, "lamisun": lamisun_shapes, "fizelix": fizelix_shapes}[
-                self.model_type](self)
+            shapes = {"babotar": babotar_shapes, "lamisun": lamisun_shapes, "fizelix": fizelix_shapes,
+                      "tefudra": tefudra_shapes}[self.model_type](self)
             return sum(math.prod(shp) for shp in shapes.values())
         if self.layer_specs:
             n = v * h + h
@@ -351,6 +420,8 @@ class ModelConfig:
             return _lamisun(cls, d)
         if mt is None and d.get("architecture") == "Fizelix":
             return _fizelix(cls, d)
+        if mt is None and d.get("architecture") == "Tefudra":
+            return _tefudra(cls, d)
         common = dict(
             bos_token_id=d.get("bos_token_id"),
             eos_token_id=_first(d.get("eos_token_id")),
@@ -637,6 +708,91 @@ def _fizelix(cls, d: Dict[str, Any]) -> "ModelConfig":
     )
 
 
+def _tefudra(cls, d: Dict[str, Any]) -> "ModelConfig":
+    """``{"architecture": "Tefudra", "vocab", "width", "norm": {"eps", "groups"}, "layers": [{"type": "attention" |
+    "parallel", "mixer": {...}, "mlp": {"kind": "dense", "ff"} | {"kind": "moe", "router": {"experts", "top", "identity"},
+    "expert": {"ff"}, "shared": {"ff"}} | null, "weights_of"}]}``. An attention mixer gives heads, kv_heads, dim, vdim,
+    scale, mask: {size, keep_first}, rot: {base, dims}; a parallel one ``left`` (heads, kv_heads, dim, vdim, scale,
+    softcap, conv, mask: {size}, rot: {base, dims}) and ``right`` (heads, dim, vdim, gate_cap). Keys a config leaves out
+    switch their mechanism off (no window, no kept positions, no cap, no rotation, one norm part, no identity experts, no
+    shared expert)."""
+    specs: List[LayerSpec] = []
+
+    def attn(i, where, m, **fixed):
+        rot = None
+        if m.get("rot") and int(m["rot"].get("dims") or 0):
+            rot = RotarySpec(int(m["rot"]["dims"]), float(m["rot"]["base"]))
+            if rot.dims % 2 or rot.dims > int(m["dim"]):
+                raise ValueError(f"Tefudra layer {i}{where}: {rot.dims} rotary dimensions on heads of {m['dim']}")
+        mask = m.get("mask") or {}
+        a = WindowAttnSpec(int(m["heads"]), int(m.get("kv_heads") or m["heads"]), int(m["dim"]),
+                           int(m.get("vdim") or m["dim"]), float(m["scale"]) if "scale" in m else int(m["dim"]) ** -0.5,
+                           int(mask.get("size") or 0), int(mask.get("keep_first") or 0), float(m.get("softcap") or 0.0),
+                           rot, **fixed)
+        if a.heads % a.kv_heads:
+            raise ValueError(f"Tefudra layer {i}{where}: {a.heads} heads on {a.kv_heads} key heads")
+        return a
+    for i, L in enumerate(d["layers"]):
+        m, typ = L["mixer"], L.get("type")
+        if typ == "attention":
+            mixer = attn(i, "", m, qk_norm=True, shared_kv=True, sink=True)
+            if mixer.vdim != mixer.dim:
+                raise ValueError(f"Tefudra layer {i}: the values are the keys, {mixer.vdim} is not {mixer.dim}")
+        elif typ == "parallel":
+            a, r = m["left"], m["right"]
+            left = attn(i, " left", a, bias=True, conv=max(1, int(a.get("conv") or 1)), v_norm=True,
+                        rot_values=bool(a.get("rot")))
+            if left.rot_values and (left.vdim % 2 or left.rot is None):
+                raise ValueError(f"Tefudra layer {i} left: rotated values need an even value size and a rotation")
+            mixer = PairMixerSpec(left, MLSTMSpec(int(r["heads"]), int(r["dim"]), int(r["vdim"]), float(r["gate_cap"])))
+        else:
+            raise ValueError(f"Tefudra layer {i}: unsupported mixer type {typ!r}")
+        f, mlp = L.get("mlp"), None
+        if f is not None:
+            kind = f.get("kind", "dense")
+            if kind == "dense":
+                mlp = DenseMLPSpec(int(f["ff"]), "relu2", gated=False)
+            elif kind == "moe":
+                sh, r = f.get("shared"), f["router"]
+                mlp = MoESpec(int(r["experts"]), int(r["top"]), ExpertSpec(int(f["expert"]["ff"])),
+                              None if not sh else ExpertSpec(int(sh["ff"])), act="gelu", score="softmax",
+                              identity=int(r.get("identity") or 0))
+                if not 1 <= mlp.top <= mlp.experts + mlp.identity:
+                    raise ValueError(f"Tefudra layer {i}: top {mlp.top} of {mlp.experts + mlp.identity} router outputs")
+            else:
+                raise ValueError(f"Tefudra layer {i}: unsupported feed-forward kind {kind!r}")
+        specs.append(LayerSpec(mixer, mlp))
+    if not specs:
+        raise ValueError("Tefudra: no layers")
+    owners = []
+    for i in range(len(specs)):
+        j, seen = i, set()
+        while d["layers"][j].get("weights_of") is not None:
+            if j in seen:
+                raise ValueError(f"Tefudra layer {i}: weights_of goes round in a circle")
+            seen.add(j)
+            j = int(d["layers"][j]["weights_of"])
+            if not 0 <= j < len(specs):
+                raise ValueError(f"Tefudra layer {i}: weights_of {j} of {len(specs)} layers")
+        if specs[j] != specs[i]:
+            raise ValueError(f"Tefudra layer {i}: it uses the weights of layer {j} but is described differently")
+        owners.append(j)
+    groups = int((d.get("norm") or {}).get("groups") or 1)
+    if int(d["width"]) % groups:
+        raise ValueError(f"Tefudra: width {d['width']} in {groups} norm parts")
+    ffs = [s.mlp.ff if s.mlp.kind == "dense" else s.mlp.expert.ff for s in specs if s.mlp]
+    return cls(
+        model_type="tefudra", vocab_size=int(d["vocab"]), hidden_size=int(d["width"]), num_layers=len(specs),
+        num_heads=max(s.mixer.heads for s in specs), num_kv_heads=1, head_dim=1, intermediate_size=max(ffs or [0]),
+        max_position_embeddings=1 << 20,  # the design has no positional limit of its own
+        norm="rmsnorm", norm_eps=float(d["norm"]["eps"]), activation="relu2", position="none", rotary_dim=0,
+        parallel_block=False, tie_word_embeddings=True, layer_specs=specs, residual_fp32=True, sandwich=True,
+        norm_groups=groups, weights_of=owners,
+        bos_token_id=d.get("bos_token_id"), eos_token_id=_first(d.get("eos_token_id")),
+        pad_token_id=d.get("pad_token_id"),
+    )
+
+
 def _first(x):
     if isinstance(x, (list, tuple)):
         return x[0] if x else None
@@ -758,6 +914,26 @@ _PRESETS: Dict[str, Dict[str, Any]] = {
                                            shared=dict(ff=12))),
                              dict(type="mamba2",
                                   mixer=dict(heads=3, vdim=16, state=12, groups=1, conv=2, norm_groups=1), mlp=None),
+                         ]),
+    # sandwich-normed per-layer design with norms in parts: window attention with kept positions and a sink, a layer of
+    # attention beside an exponential-gate memory, dense and expert feed-forwards, a layer that shares weights
+    "tiny-tefudra": dict(architecture="Tefudra", vocab=211, width=48, norm=dict(eps=1e-5, groups=3),
+                         layers=[
+                             dict(type="parallel",
+                                  mixer=dict(left=dict(heads=4, kv_heads=2, dim=8, vdim=12, scale=0.3, softcap=15.0,
+                                                       conv=4, mask=dict(size=9), rot=dict(base=1000.0, dims=6)),
+                                             right=dict(heads=3, dim=8, vdim=16, gate_cap=10.0)),
+                                  mlp=dict(kind="dense", ff=64)),
+                             dict(type="attention",
+                                  mixer=dict(heads=4, kv_heads=1, dim=12, vdim=12, scale=0.25,
+                                             mask=dict(size=7, keep_first=2), rot=dict(base=500.0, dims=8)),
+                                  mlp=dict(kind="moe", router=dict(experts=5, top=2, identity=2), expert=dict(ff=20),
+                                           shared=dict(ff=12))),
+                             dict(type="attention", weights_of=1,
+                                  mixer=dict(heads=4, kv_heads=1, dim=12, vdim=12, scale=0.25,
+                                             mask=dict(size=7, keep_first=2), rot=dict(base=500.0, dims=8)),
+                                  mlp=dict(kind="moe", router=dict(experts=5, top=2, identity=2), expert=dict(ff=20),
+                                           shared=dict(ff=12))),
                          ]),
     # TP up to 8 (16 q / kv heads: 2 per rank at TP=8, as Llama-2-7B's 32 give 4)
     "tiny-llama16h": dict(model_type="llama", hidden_size=256, num_hidden_layers=2, num_attention_heads=16,

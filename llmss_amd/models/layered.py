@@ -1,7 +1,7 @@
 """Decoder whose layers are described one by one (``ModelConfig.layer_specs``) over an fp32 residual stream.
 
 The uniform families run through :class:`~llmss_amd.models.decoder.DecoderLM`; a per-layer design (Timisun, Babotar,
-Lamisun, Fizelix) runs through :class:`LayeredLM`, which offers the engine the same surface (``hidden_states`` / ``logits`` over a
+Lamisun, Fizelix, Tefudra) runs through :class:`LayeredLM`, which offers the engine the same surface (``hidden_states`` / ``logits`` over a
 :class:`StepInput`, ``allocate_kv_cache``, ``kv_bytes_per_block``, ``plan``) and so shares its scheduler, paged
 cache pool, decode graphs and sampler. A layer is either a parallel block (``cfg.parallel_block``)
 
@@ -18,9 +18,11 @@ on each sublayer's output,
 
 optionally followed by a depth average: what goes on to the next layer is sum_j dwa[j] X_j over the results X_j of
 this and all earlier layers (X_0 the embedding); or (``cfg.sandwich``) a sequential block normed on both sides of
-each sublayer, its result gated per channel and scaled,
+each sublayer, its result optionally gated per channel and scaled,
 
     h = norm_a(x) ;  x <- x + post * rms_norm(sigmoid(W_g h + b) * sublayer(h))          post = norm_b weight * layer scale
+
+the norms optionally taken in ``cfg.norm_groups`` equal parts of the row; layers may share weights (``cfg.weights_of``),
 
 optionally followed by a token input (x <- x + rms_norm(W_p (gelu(W_s x) * e)) * w, e the layer's slice of a second
 token table); a stretch of such layers may run several times in a row with the same weights (``cfg.loop``), each pass
@@ -55,6 +57,12 @@ attention without a softmax - a visible key weighs sigmoid(score + bias_h) - ove
 one mean key / value per block of ``pool`` positions that has wholly left the window; the means live in a pooled cache
 beside the pages (one row per block, written when the block's last position is). Mixer ``mamba2`` (causal_conv with
 bias, ssd_recurrence, gated_group_norm gate-first): S <- exp(-exp(A) dt) S + dt B x^T, y = S^T C + D x per head.
+
+Mixer ``window_attention`` (ops: linear_f, rope_angles, head_prep_cache, window_attn): softmax attention over a sliding
+window that keeps the sequence's first positions, with a learned sink per head, soft cap, short convolutions on q / k / v,
+query / key / value norms, rotated keys and values - each by the spec. Mixer ``mlstm`` (linear_f, mlstm_mix): matrix memory
+with exponential gates and a running maximum. Mixer ``pair``: two mixers on the same input, one input GEMM for both; their
+results go unjoined (``ops.PairPending``) into the block's closing op, which norms and averages them.
 
 Feed-forward ``moe`` (ops: moe_router -> fp32 router logits and routing, moe_experts, glu_clamp): sigmoid scores, the
 choice made on score + correction, weights = chosen scores normalised; experts and the shared expert use the clamped
@@ -152,8 +160,13 @@ class MoEFeedForward:
     @staticmethod
     def forward(model: "LayeredLM", W, spec, h):
         dt = model.dtype
-        idx, wts = ops.moe_router(h, W.router, W.correction, spec.top, spec.normalize)
+        idx, wts = ops.moe_router(h, W.router, W.correction, spec.top, spec.normalize, spec.score)
         sh = None
+        if spec.act == "gelu":  # experts without a gate
+            if W.shared_gu is not None:
+                sh = ops.linear_f(ops.linear_f(h, W.shared_gu, dt, act="gelu"), W.shared_down, dt)
+            return ops.moe_experts(h, idx, wts, None, W.up, W.down, 0.0, 0.0, shared=sh, combine=False, act="gelu",
+                                   identity=spec.identity > 0)
         if W.shared_gu is not None:
             # (a sandwich block's gate logits ride in this GEMM as extra columns: model.proj)
             gu = model.proj = ops.linear_f(h, W.shared_gu, dt)
@@ -254,6 +267,8 @@ class DenseFeedForward:
     @staticmethod
     def forward(model: "LayeredLM", W, spec, h):
         dt = model.dtype
+        if not spec.gated and spec.act in ("gelu", "relu2"):  # the activation rides in the GEMM's epilogue
+            return ops.linear_f(ops.linear_f(h, W.gu, dt, act=spec.act), W.down, dt)
         if not spec.gated:
             return ops.linear_f(ops.act_fn(ops.linear_f(h, W.gu, dt), spec.act, W.act_params), W.down, dt)
         gu = model.proj = ops.linear_f(h, W.gu, dt)  # (columns past 2 ff: a sandwich block's gate logits)
@@ -343,8 +358,111 @@ class SSDMixer:
         return ops.linear_f(y, W.o, dt)
 
 
+class WindowAttention:
+    """Mixer ``window_attention``: softmax attention over a sliding window with kept first positions."""
+
+    @staticmethod
+    def cache_row(spec) -> Optional[int]:
+        return spec.kv_heads * (spec.dim + spec.vdim)
+
+    @staticmethod
+    def allocate(model: "LayeredLM", spec, num_blocks: int, block_size: int, num_slots: int):
+        dt, dev = model.dtype, model.device
+        st = {}
+        if spec.conv > 1:
+            st["tail"] = torch.zeros(num_slots, spec.conv - 1, spec.qkv_columns, dtype=torch.float32, device=dev)
+        return (torch.zeros(num_blocks, block_size, spec.kv_heads * spec.dim, dtype=dt, device=dev),
+                torch.zeros(num_blocks, block_size, spec.kv_heads * spec.vdim, dtype=dt, device=dev), st)
+
+    @staticmethod
+    def state_bytes(spec) -> int:
+        return 4 * max(spec.conv - 1, 0) * spec.qkv_columns
+
+    @staticmethod
+    def mix(model: "LayeredLM", W, spec, proj, inp: StepInput, cu, cache):
+        """The heads' results [T, heads * vdim], before the output projection, from the projection rows."""
+        c, (kc, vc, st) = W.cols, cache
+        single = inp.kind == "decode"
+        cs = model.angles(inp, W.rot_key, W.freqs) if W.freqs is not None else None
+        vcs = model.angles(inp, W.vrot_key, W.vfreqs) if W.vfreqs is not None else None
+        q = ops.head_prep_cache(proj, c["q"], c["k"], c["v"], W.conv, st.get("tail"), W.q_norm, W.k_norm, spec.v_norm,
+                                model.cfg.norm_eps, cs, vcs, kc, vc, inp.slots, spec.heads, spec.kv_heads, spec.dim,
+                                spec.vdim, cu, inp.ctx_lens, inp.state_slots, single=single or inp.max_seqlen <= 1)
+        return ops.window_attn(q, kc, vc, inp.block_tables, cu, inp.ctx_lens, spec.heads, spec.kv_heads, spec.dim,
+                               spec.vdim, spec.scale, spec.softcap, spec.window, spec.keep_first, W.sink, vcs,
+                               model.dtype, max_qlen=1 if single else max(1, inp.max_seqlen),
+                               num_decode=0 if single else inp.num_decode, max_ctx=inp.max_ctx)
+
+    @staticmethod
+    def forward(model: "LayeredLM", i: int, W, spec, h, inp: StepInput, cu, caches):
+        dt = model.dtype
+        y = WindowAttention.mix(model, W, spec, ops.linear_f(h, W.proj, dt, bias=W.bias), inp, cu, caches[i])
+        return ops.linear_f(y, W.o, dt, bias=W.o_bias)
+
+
+class MLSTMMixer:
+    """Mixer ``mlstm``: matrix memory with exponential gates, per-head norm, output gate."""
+
+    @staticmethod
+    def cache_row(spec) -> Optional[int]:
+        return None
+
+    @staticmethod
+    def allocate(model: "LayeredLM", spec, num_blocks: int, block_size: int, num_slots: int):
+        def z(*shape):
+            return torch.zeros(num_slots, spec.heads, *shape, dtype=torch.float32, device=model.device)
+        return None, None, {"S": z(spec.dim, spec.vdim), "n": z(spec.dim), "m": z()}
+
+    @staticmethod
+    def state_bytes(spec) -> int:
+        return 4 * spec.heads * (spec.dim * spec.vdim + spec.dim + 1)
+
+    @staticmethod
+    def mix(model: "LayeredLM", W, spec, proj, inp: StepInput, cu, cache):
+        c, st = W.cols, cache[2]
+        H, nqk, nv = spec.heads, spec.heads * spec.dim, spec.heads * spec.vdim
+        part = lambda n, w: proj[:, c[n]:c[n] + w]  # noqa: E731
+        return ops.mlstm_mix(part("q", nqk), part("k", nqk), part("v", nv), part("i", H), part("f", H), W.bi, W.bf,
+                             spec.gate_cap, st["S"], st["n"], st["m"], cu, inp.ctx_lens, inp.state_slots, H, spec.dim,
+                             spec.vdim, part("g", nv), W.norm, model.cfg.norm_eps, model.dtype,
+                             max_qlen=1 if inp.kind == "decode" else max(1, inp.max_seqlen))
+
+    @staticmethod
+    def forward(model: "LayeredLM", i: int, W, spec, h, inp: StepInput, cu, caches):
+        dt = model.dtype
+        return ops.linear_f(MLSTMMixer.mix(model, W, spec, ops.linear_f(h, W.proj, dt), inp, cu, caches[i]), W.o, dt)
+
+
+class PairMixer:
+    """Mixer ``pair``: two mixers side by side, each result RMS-normed over the row, averaged. One GEMM holds the input
+    projections of both; the join happens inside the block's closing op."""
+
+    @staticmethod
+    def cache_row(spec) -> Optional[int]:
+        return sum(MIXERS[s.kind].cache_row(s) or 0 for s in (spec.left, spec.right)) or None
+
+    @staticmethod
+    def allocate(model: "LayeredLM", spec, num_blocks: int, block_size: int, num_slots: int):
+        l, r = (MIXERS[s.kind].allocate(model, s, num_blocks, block_size, num_slots) for s in (spec.left, spec.right))
+        return l[0], l[1], {**l[2], **r[2]}
+
+    @staticmethod
+    def state_bytes(spec) -> int:
+        return sum(MIXERS[s.kind].state_bytes(s) for s in (spec.left, spec.right))
+
+    @staticmethod
+    def forward(model: "LayeredLM", i: int, W, spec, h, inp: StepInput, cu, caches):
+        dt = model.dtype
+        proj = ops.linear_f(h, W.proj, dt, bias=W.bias)
+        yl = MIXERS[spec.left.kind].mix(model, W.left, spec.left, proj, inp, cu, caches[i])
+        yr = MIXERS[spec.right.kind].mix(model, W.right, spec.right, proj, inp, cu, caches[i])
+        return ops.PairPending(ops.linear_f(yl, W.left.o, dt, bias=W.left.o_bias), ops.linear_f(yr, W.right.o, dt), W.out_l,
+                               W.out_r)
+
+
 MIXERS = {"latent_attention": LatentAttention, "parallel": ParallelMixer, "lightning": DecayMixer,
-          "attention": DiffAttention, "pool_attention": PoolAttention, "mamba2": SSDMixer}
+          "attention": DiffAttention, "pool_attention": PoolAttention, "mamba2": SSDMixer,
+          "window_attention": WindowAttention, "mlstm": MLSTMMixer, "pair": PairMixer}
 FFNS = {"moe": MoEFeedForward, "dense": DenseFeedForward}
 
 
@@ -404,9 +522,10 @@ class LayeredLM:
             if K % 16 == 0 and N % 8 == 0 and (N, K) not in {(s.N, s.K) for s in out.values()}:
                 out[f"{name}_{N}x{K}"] = GemmShape(N, K)
         for L in self.w.layers:
-            for nm in ("qc", "proj", "o"):
-                if hasattr(L.mix, nm):
-                    put(nm, getattr(L.mix, nm))
+            for mx in (L.mix, getattr(L.mix, "left", None), getattr(L.mix, "right", None)):
+                for nm in ("qc", "proj", "o"):
+                    if getattr(mx, nm, None) is not None:
+                        put(nm, getattr(mx, nm))
             for nm in ("shared_gu", "shared_down", "gu", "down"):
                 if getattr(L, "mlp", None) is not None and getattr(L.mlp, nm, None) is not None and \
                         getattr(L.mlp, nm).dim() == 2:
@@ -432,15 +551,19 @@ class LayeredLM:
     @property
     def needs_state(self) -> bool:
         """Some mixer keeps per-sequence state besides its pages: steps must carry the sequences' state slots."""
-        return any(hasattr(MIXERS[s.mixer.kind], "state_bytes") for s in self.cfg.layer_specs) or \
+        return any(self._mixer_state_bytes(s) > 0 for s in self.cfg.layer_specs) or \
             bool(self.cfg.canon_taps > 1) or self.cfg.bigram is not None
+
+    @staticmethod
+    def _mixer_state_bytes(s) -> int:
+        mx = MIXERS[s.mixer.kind]
+        return mx.state_bytes(s.mixer) if hasattr(mx, "state_bytes") else 0
 
     def _canon_sublayers(self) -> int:
         return 2 if self.cfg.canon_ffn else 1
 
     def state_bytes_per_slot(self) -> int:
-        n = sum(MIXERS[s.mixer.kind].state_bytes(s.mixer) for s in self._run_specs()
-                if hasattr(MIXERS[s.mixer.kind], "state_bytes"))
+        n = sum(self._mixer_state_bytes(s) for s in self._run_specs())
         n += 8 if self.cfg.bigram is not None else 0
         return n + 4 * max(self.cfg.canon_taps - 1, 0) * self.cfg.hidden_size * len(self.cfg.layer_specs) * \
             self._canon_sublayers()
@@ -455,7 +578,7 @@ class LayeredLM:
         for s, r in zip(self._run_specs(), self._cache_rows()):
             mx = MIXERS[s.mixer.kind]
             if hasattr(mx, "allocate"):
-                if num_slots <= 0 and hasattr(mx, "state_bytes"):
+                if num_slots <= 0 and self._mixer_state_bytes(s) > 0:
                     raise ValueError(f"{self.cfg.model_type}: the cache needs state slots (num_slots)")
                 caches.append(mx.allocate(self, s.mixer, num_blocks, block_size, num_slots))
             elif r:
@@ -606,8 +729,8 @@ class LayeredLM:
         runs = cfg.layer_runs()
         x = ops.embed_scaled(inp.input_ids, w.wte, cfg.embedding_scale)
         x0 = x.clone() if cfg.loop else None
-        W_ = cfg.hidden_size
-        h = ops.sandwich_add_norm(x, None, None, None, None, eps, None, w.layers[runs[0]].norm1, dt)
+        W_, ng = cfg.hidden_size, cfg.norm_groups
+        h = ops.sandwich_add_norm(x, None, None, None, None, eps, None, w.layers[runs[0]].norm1, dt, ng)
         for r, i in enumerate(runs):
             L, spec = w.layers[i], cfg.layer_specs[i]
             last = r + 1 == len(runs)
@@ -620,20 +743,20 @@ class LayeredLM:
                 tail = (add, nxt)
             side = L.side_gate is not None
             y = MIXERS[spec.mixer.kind].forward(self, r, L.mix, spec.mixer, h, inp, cu, kv_caches)
-            c0 = L.mix.cols["rg"]
+            gate = None if L.rg1_b is None else self.proj[:, L.mix.cols["rg"]:L.mix.cols["rg"] + W_]
             after = (None, L.norm2) if spec.mlp is not None else ((None, None) if side else tail)
-            h = ops.sandwich_add_norm(x, y, self.proj[:, c0:c0 + W_], L.rg1_b, L.post1, eps, *after, dt)
+            h = ops.sandwich_add_norm(x, y, gate, L.rg1_b, L.post1, eps, *after, dt, ng)
             if spec.mlp is not None:
                 y = FFNS[spec.mlp.kind].forward(self, L.mlp, spec.mlp, h)
                 after = (None, None) if side else tail
-                h = ops.sandwich_add_norm(x, y, self.proj[:, L.rg2_col:L.rg2_col + W_], L.rg2_b, L.post2, eps, *after,
-                                          dt)
+                gate = None if L.rg2_b is None else self.proj[:, L.rg2_col:L.rg2_col + W_]
+                h = ops.sandwich_add_norm(x, y, gate, L.rg2_b, L.post2, eps, *after, dt, ng)
             if side:
                 h = ops.token_side_add(x, inp.input_ids, w.extra["side"], L.side_col, L.side_gate, L.side_proj,
                                        L.side_norm, eps, *tail, dt)
             if self.tap is not None:
                 self.tap(r, x)
-                h = ops.sandwich_add_norm(x, None, None, None, None, eps, add, nxt, dt)
+                h = ops.sandwich_add_norm(x, None, None, None, None, eps, add, nxt, dt, ng)
         self._angles = {}
         self.proj = None
         return h

@@ -22,7 +22,7 @@ from .config import ModelConfig
 from .decoder import StepInput
 from .layered import create_model
 from .weights import (load_babotar_weights, load_fizelix_weights, load_hf_weights, load_lamisun_weights,
-                      load_timisun_weights)
+                      load_tefudra_weights, load_timisun_weights)
 
 
 @dataclass
@@ -55,9 +55,9 @@ class CausalLM:
     def __init__(self, config, weights, max_blocks: int = 4096, block_size: int = 16, max_seqs: int = 16):
         cfg = config if isinstance(config, ModelConfig) else ModelConfig.from_hf_dict(config.to_dict())
         tp = getattr(weights, "tp", None) or TPGroup()
-        if cfg.layer_specs:  # per-layer designs (Timisun, Babotar, Lamisun, Fizelix)
+        if cfg.layer_specs:  # per-layer designs (Timisun, Babotar, Lamisun, Fizelix, Tefudra)
             load = {"babotar": load_babotar_weights, "lamisun": load_lamisun_weights,
-                    "fizelix": load_fizelix_weights}.get(cfg.model_type, load_timisun_weights)
+                    "fizelix": load_fizelix_weights, "tefudra": load_tefudra_weights}.get(cfg.model_type, load_timisun_weights)
             w = load(cfg, weights.reader, device=weights.device, dtype=weights.dtype)
         else:
             w = load_hf_weights(cfg, weights.reader, tp.size, tp.rank, device=weights.device, dtype=weights.dtype)
@@ -291,6 +291,13 @@ class FizelixForCausalLM(_FamilyLM):
     model_type = "fizelix"
 
 
+class TefudraForCausalLM(_FamilyLM):
+    """Per-layer design: blocks normed in parts on both sides of their sublayers, window attention with kept positions and a
+    sink, attention over rotated values beside a matrix memory with exponential gates, experts with identity experts
+    (models/layered.py)."""
+    model_type = "tefudra"
+
+
 MODEL_REGISTRY = {c.model_type: c for c in (GPT2LMHeadModel, GPTJForCausalLM, GPTBigCodeForCausalLM,
                                             LlamaForCausalLM, TimisunForCausalLM, BabotarForCausalLM,
-                                            LamisunForCausalLM, FizelixForCausalLM)}
+                                            LamisunForCausalLM, FizelixForCausalLM, TefudraForCausalLM)}

@@ -562,12 +562,12 @@ class LatentAttnWeights:
 
 @dataclass
 class MoEWeights:
-    """Experts stacked: ``gate`` / ``up`` [E, F, H], ``down`` [E, H, F]; ``router`` [E, H]; ``correction`` fp32 [E]
-    (added to the scores for the choice only); the shared expert as one gate | up matrix ``shared_gu`` [2 Fs, H]
-    and ``shared_down`` [H, Fs]."""
+    """Experts stacked: ``gate`` / ``up`` [E, F, H] (``gate`` None: ungated experts), ``down`` [E, H, F]; ``router`` [E (+
+    identity experts), H]; ``correction`` fp32 [router rows] (added to the scores for the choice only); the shared expert as
+    one gate | up matrix ``shared_gu`` [2 Fs, H] (ungated: [Fs, H]) and ``shared_down`` [H, Fs]."""
     router: torch.Tensor
     correction: Optional[torch.Tensor]
-    gate: torch.Tensor
+    gate: Optional[torch.Tensor]
     up: torch.Tensor
     down: torch.Tensor
     shared_gu: Optional[torch.Tensor] = None
@@ -858,7 +858,7 @@ def _cat_rows(parts, pad_to: int = 8):
         n += t.shape[0]
     mats = [t for _, t in parts]
     if n % pad_to:
-        mats.append(torch.zeros(pad_to - n % pad_to, mats[0].shape[1], dtype=mats[0].dtype))
+        mats.append(torch.zeros(pad_to - n % pad_to, mats[0].shape[1], dtype=mats[0].dtype, device=mats[0].device))
     return torch.cat(mats, 0), cols
 
 
@@ -1210,7 +1210,7 @@ class SandwichBlockWeights:
     type, ``side_norm`` fp32 [W], ``side_col`` the layer's first column in the token table."""
     norm1: torch.Tensor
     post1: torch.Tensor
-    rg1_b: torch.Tensor
+    rg1_b: Optional[torch.Tensor]  # None: the results are not gated
     mix: object
     norm2: Optional[torch.Tensor] = None
     post2: Optional[torch.Tensor] = None
@@ -1223,8 +1223,8 @@ class SandwichBlockWeights:
     side_col: int = 0
 
     def tensors(self):
-        out = [self.norm1, self.post1, self.rg1_b] + self.mix.tensors()
-        for t in (self.norm2, self.post2, self.rg2_b, self.side_gate, self.side_proj, self.side_norm):
+        out = [self.norm1, self.post1] + self.mix.tensors()
+        for t in (self.rg1_b, self.norm2, self.post2, self.rg2_b, self.side_gate, self.side_proj, self.side_norm):
             if t is not None:
                 out.append(t)
         if self.mlp is not None:
@@ -1394,3 +1394,216 @@ def fizelix_state_dict(cfg: ModelConfig, seed: int = 0) -> Dict[str, torch.Tenso
     """The random weights of :func:`random_fizelix_weights` under their checkpoint names (bf16; tests, examples)."""
     get = _fizelix_random(cfg, seed)
     return {n: get(n).to(torch.bfloat16) for n in fizelix_shapes(cfg)}
+
+
+# ------------------------------------------------- sandwich-normed per-layer designs with norms in parts (Tefudra)
+@dataclass
+class WindowAttnWeights:
+    """Window attention: ``proj`` [q | k (| v) rows padded to 8, W] with ``bias`` (one GEMM; both None inside a pair, whose
+    own matrix holds the rows), ``cols`` the first row of each part (shared keys and values: cols["v"] = cols["k"]);
+    ``conv`` [taps, q + k + v columns] or None; ``q_norm`` / ``k_norm`` fp32 [dim] or None; ``sink`` fp32 [heads] or None;
+    ``freqs`` / ``vfreqs`` fp32 the angular steps per position of the key and value pairs (None: no rotation),
+    ``rot_key`` / ``vrot_key`` (dims, base): layers with the same rotation share a step's angles; ``o`` [W, heads * vdim]
+    with ``o_bias``."""
+    proj: Optional[torch.Tensor]
+    bias: Optional[torch.Tensor]
+    cols: Dict[str, int]
+    conv: Optional[torch.Tensor]
+    q_norm: Optional[torch.Tensor]
+    k_norm: Optional[torch.Tensor]
+    sink: Optional[torch.Tensor]
+    freqs: Optional[torch.Tensor]
+    rot_key: Optional[tuple]
+    vfreqs: Optional[torch.Tensor]
+    vrot_key: Optional[tuple]
+    o: torch.Tensor
+    o_bias: Optional[torch.Tensor]
+
+    def tensors(self):
+        return [t for t in (self.proj, self.bias, self.conv, self.q_norm, self.k_norm, self.sink, self.freqs, self.vfreqs,
+                            self.o, self.o_bias) if t is not None]
+
+
+@dataclass
+class MLSTMWeights:
+    """Matrix memory with exponential gates: ``proj`` [q | k | v | g | i | f rows padded to 8, W] (None inside a pair),
+    ``cols`` the first row of each part; ``bi`` / ``bf`` fp32 [heads] the gates' biases; ``norm`` [heads * vdim]; ``o``
+    [W, heads * vdim]."""
+    proj: Optional[torch.Tensor]
+    cols: Dict[str, int]
+    bi: torch.Tensor
+    bf: torch.Tensor
+    norm: torch.Tensor
+    o: torch.Tensor
+
+    def tensors(self):
+        return [t for t in (self.proj, self.bi, self.bf, self.norm, self.o) if t is not None]
+
+
+@dataclass
+class PairWeights:
+    """Two mixers reading the same rows: ``proj`` [every input projection of both, rows padded to 8, W] with ``bias``, ``out_l``
+    / ``out_r`` fp32 [W] the weights of the norms their results pass before they are averaged."""
+    proj: torch.Tensor
+    bias: Optional[torch.Tensor]
+    left: WindowAttnWeights
+    right: MLSTMWeights
+    out_l: torch.Tensor
+    out_r: torch.Tensor
+
+    def tensors(self):
+        return [t for t in (self.proj, self.bias, self.out_l, self.out_r) if t is not None] + self.left.tensors() + \
+            self.right.tensors()
+
+
+def tefudra_shapes(cfg: ModelConfig) -> Dict[str, tuple]:
+    """Checkpoint tensor names of a Tefudra config and their shapes (a layer that shares weights has none)."""
+    W = cfg.hidden_size
+    out = {"embed": (cfg.vocab_size, W), "final.norm": (W,)}
+    for i, spec in enumerate(cfg.layer_specs):
+        if cfg.weights_of[i] != i:
+            continue
+        p, m = f"l{i}.", spec.mixer
+        out[p + "norm1"] = out[p + "norm1b"] = (W,)
+        if m.kind == "window_attention":
+            out.update({p + "mix.q": (m.heads * m.dim, W), p + "mix.k": (m.kv_heads * m.dim, W),
+                        p + "mix.q.norm": (m.dim,), p + "mix.k.norm": (m.dim,), p + "mix.sink": (m.heads,),
+                        p + "mix.o": (W, m.heads * m.vdim)})
+        else:
+            a, r, pl, pr = m.left, m.right, p + "mix.left.", p + "mix.right."
+            for n, c in (("q", a.heads * a.dim), ("k", a.kv_heads * a.dim), ("v", a.kv_heads * a.vdim)):
+                out.update({pl + n: (c, W), pl + n + ".b": (c,), pl + n + ".conv": (c, a.conv)})
+            out.update({pl + "o": (W, a.heads * a.vdim), pl + "o.b": (W,), pl + "out": (W,),
+                        pr + "q": (r.heads * r.dim, W), pr + "k": (r.heads * r.dim, W), pr + "v": (r.heads * r.vdim, W),
+                        pr + "g": (r.heads * r.vdim, W), pr + "o": (W, r.heads * r.vdim),
+                        pr + "norm": (r.heads * r.vdim,), pr + "out": (W,)})
+            for n in "if":
+                out.update({pr + n: (r.heads, W), pr + n + ".b": (r.heads,)})
+        f = spec.mlp
+        if f is None:
+            continue
+        out[p + "norm2"] = out[p + "norm2b"] = (W,)
+        if f.kind == "dense":
+            out.update({p + "mlp.up": (f.ff, W), p + "mlp.down": (W, f.ff)})
+        else:
+            E = f.experts + f.identity
+            out.update({p + "mlp.router": (E, W), p + "mlp.correction": (E,)})
+            for k in range(f.experts):
+                out.update({f"{p}mlp.e{k}.up": (f.expert.ff, W), f"{p}mlp.e{k}.down": (W, f.expert.ff)})
+            if f.shared is not None:
+                out.update({p + "mlp.shared.up": (f.shared.ff, W), p + "mlp.shared.down": (W, f.shared.ff)})
+    return out
+
+
+def _tefudra_finish(cfg: ModelConfig, get, device, dtype) -> ModelWeights:
+    """``get(name)`` returns the checkpoint tensor of that name. Shapes are checked against the config. All input
+    projections of a mixer (both branches of a pair) become one matrix with one bias vector; the convolutions' weights are
+    laid side by side with the taps first; norm weights, sinks and gate biases are kept in fp32. A layer that uses another
+    layer's weights holds that layer's objects."""
+    shapes = tefudra_shapes(cfg)
+
+    def g(name):
+        t = get(name)
+        if tuple(t.shape) != shapes[name]:
+            raise ValueError(f"{name} has shape {tuple(t.shape)}, the config says {shapes[name]}")
+        return t
+
+    def dev(t, dt=dtype):
+        return None if t is None else t.to(device=device, dtype=dt).contiguous()
+
+    def f32(t):
+        return dev(t.float(), torch.float32)
+
+    def steps(dims, base):
+        return f32(torch.tensor([base ** (-2.0 * j / dims) for j in range(dims // 2)], dtype=torch.float64))
+
+    def attn(a, p, proj, bias, cols):
+        rot, turn = a.rot is not None, a.rot is not None and a.rot_values
+        return WindowAttnWeights(
+            proj, bias, cols,
+            dev(torch.cat([g(p + n + ".conv") for n in "qkv"], 0).t()) if a.conv else None,
+            f32(g(p + "q.norm")) if a.qk_norm else None, f32(g(p + "k.norm")) if a.qk_norm else None,
+            f32(g(p + "sink")) if a.sink else None, steps(a.rot.dims, a.rot.base) if rot else None,
+            (a.rot.dims, a.rot.base) if rot else None, steps(a.vdim, a.rot.base) if turn else None,
+            (a.vdim, a.rot.base) if turn else None, dev(g(p + "o")), dev(g(p + "o.b")) if a.bias else None)
+    layers: list = [None] * len(cfg.layer_specs)
+    for i, spec in enumerate(cfg.layer_specs):
+        if cfg.weights_of[i] != i:
+            continue
+        p, m = f"l{i}.", spec.mixer
+        if m.kind == "window_attention":
+            proj, cols = _cat_rows([(n, g(p + "mix." + n)) for n in "qk"])
+            mix = attn(m, p + "mix.", dev(proj), None, {**cols, "v": cols["k"]})
+        else:
+            pl, pr = p + "mix.left.", p + "mix.right."
+            proj, cols = _cat_rows([("l" + n, g(pl + n)) for n in "qkv"] + [("r" + n, g(pr + n)) for n in "qkvgif"])
+            bias = torch.cat([g(pl + n + ".b") for n in "qkv"])
+            bias = torch.cat([bias, torch.zeros(proj.shape[0] - bias.numel(), dtype=bias.dtype, device=bias.device)])
+            right = MLSTMWeights(None, {n: cols["r" + n] for n in "qkvgif"}, f32(g(pr + "i.b")), f32(g(pr + "f.b")),
+                                 dev(g(pr + "norm")), dev(g(pr + "o")))
+            mix = PairWeights(dev(proj), dev(bias), attn(m.left, pl, None, None, {n: cols["l" + n] for n in "qkv"}), right,
+                              f32(g(pl + "out")), f32(g(pr + "out")))
+        blk = SandwichBlockWeights(f32(g(p + "norm1")), f32(g(p + "norm1b")), None, mix)
+        f, q = spec.mlp, p + "mlp."
+        if f is not None:
+            blk.norm2, blk.post2 = f32(g(p + "norm2")), f32(g(p + "norm2b"))
+            if f.kind == "dense":
+                blk.mlp = DenseMLPWeights(dev(g(q + "up")), dev(g(q + "down")))
+            else:
+                E, sh = f.experts, f.shared is not None
+                blk.mlp = MoEWeights(
+                    router=dev(g(q + "router")), correction=f32(g(q + "correction")), gate=None,
+                    up=dev(torch.stack([g(f"{q}e{k}.up") for k in range(E)])),
+                    down=dev(torch.stack([g(f"{q}e{k}.down") for k in range(E)])),
+                    shared_gu=dev(g(q + "shared.up")) if sh else None,
+                    shared_down=dev(g(q + "shared.down")) if sh else None)
+        layers[i] = blk
+    layers = [layers[o] for o in cfg.weights_of]
+    wte, head = _tied_head(cfg, g("embed"), device, dtype)
+    return ModelWeights(wte=wte, wpe=None, layers=layers, lnf_w=f32(g("final.norm")), lnf_b=None, head=head)
+
+
+def load_tefudra_weights(cfg: ModelConfig, reader, device="cpu", dtype=torch.bfloat16) -> ModelWeights:
+    return _tefudra_finish(cfg, lambda n: reader.get(n), device, dtype)
+
+
+def _tefudra_random(cfg: ModelConfig, seed: int, device="cpu"):
+    import zlib
+
+    shapes = tefudra_shapes(cfg)
+
+    def get(name: str) -> torch.Tensor:
+        gen = torch.Generator(device=device)
+        gen.manual_seed((seed * 1000003 + zlib.crc32(name.encode())) & 0x7FFFFFFF)
+        shp = shapes[name]
+        t = torch.randn(*shp, generator=gen, dtype=torch.float32, device=device)
+        last = name.split(".")[-1]
+        if last.startswith("norm") or last == "out":
+            t = 1.0 + 0.1 * t
+        elif name.endswith("right.f.b"):
+            t = 3.0 + 0.5 * t  # a memory of tens of tokens
+        elif last == "b":
+            t = 0.3 * t
+        elif last == "correction":
+            t = 0.02 * t
+        elif last == "sink":
+            t = 0.5 * t
+        elif last == "conv":
+            t = t * shp[1] ** -0.5
+        elif len(shp) == 2 and name != "embed":
+            t = t * shp[1] ** -0.5
+        return t.to(torch.bfloat16).float()
+    return get
+
+
+def random_tefudra_weights(cfg: ModelConfig, device="cpu", dtype=torch.bfloat16, seed: int = 0) -> ModelWeights:
+    """Random-init weights of a Tefudra config (values rounded to bf16, so a bf16 and an fp32 run hold the same model):
+    projections ~ N(0, 1 / fan_in), norm weights around one."""
+    gen = device if torch.device(device).type == "cuda" else "cpu"  # large models: draw on the GPU
+    return _tefudra_finish(cfg, _tefudra_random(cfg, seed, gen), device, dtype)
+
+
+def tefudra_state_dict(cfg: ModelConfig, seed: int = 0) -> Dict[str, torch.Tensor]:
+    """The random weights of :func:`random_tefudra_weights` under their checkpoint names (bf16; tests, examples)."""
+    get = _tefudra_random(cfg, seed)
+    return {n: get(n).to(torch.bfloat16) for n in tefudra_shapes(cfg)}

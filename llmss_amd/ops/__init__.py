@@ -205,3 +205,9 @@ rope_pairs_cache = _route("rope_pairs_cache")
 pool_update = _route("pool_update")
 pool_window_attn = _route("pool_window_attn")
 ssd_recurrence = _route("ssd_recurrence")
+
+# ---------- heads on their way into the cache / softmax over a window with kept positions / exponential-gate recurrence
+PairPending = ref.PairPending
+head_prep_cache = _route("head_prep_cache")
+window_attn = _route("window_attn")
+mlstm_mix = _route("mlstm_mix")

@@ -16,6 +16,7 @@ from typing import Optional
 import torch
 
 from . import reference as _ref
+from .reference import PairPending
 
 _C = None
 _ERR = None
@@ -388,7 +389,7 @@ def reserve_workspace(device, gemm_bytes: int = 64 << 20, decode_rows: int = 0, 
         _DECODE_WS.get(decode_rows, nh, nsplit, D, device)
 
 
-_ACT = {"none": 0, None: 0, "gelu_tanh": 1, "gelu": 2, "relu": 3}
+_ACT = {"none": 0, None: 0, "gelu_tanh": 1, "gelu": 2, "relu": 3, "relu2": 5}
 
 
 class PartialSum:
@@ -822,9 +823,10 @@ class MoEPending:
     pair, ``wts`` [T, top], ``shared`` [T, N] or None. resid_add_norm takes it as its fp32 addend and combines while
     it adds to the stream."""
 
-    __slots__ = ("y", "place", "wts", "shared", "top")
+    __slots__ = ("y", "place", "wts", "shared", "top", "ident")
 
-    def __init__(self, y, place, wts, shared, top=None):
+    def __init__(self, y, place, wts, shared, top=None, ident=None):
+        self.ident = ident  # [T, N]: the output of the identity experts (pairs whose place is -1)
         self.y, self.place, self.wts, self.shared = y, place, wts, shared
         self.top = top if top is not None else wts.shape[1]  # wts None: the outputs are summed unweighted
 
@@ -838,7 +840,7 @@ def resid_add_norm(x, a, b, w, woff, eps, out_dtype, want_y=True):
         _check(a.shape[0] == T, "a rows")
     pend = b if isinstance(b, MoEPending) else None
     if pend is not None:
-        _check(pend.wts is not None, "resid_add_norm combines weighted expert outputs")
+        _check(pend.wts is not None and pend.ident is None, "resid_add_norm combines weighted expert outputs")
         top = pend.wts.shape[1]
         _check(pend.y.shape == (T * top, H) and pend.y.is_contiguous() and pend.place.numel() == T * top
                and pend.wts.shape[0] == T, "pending expert outputs do not fit the stream")
@@ -862,16 +864,17 @@ def resid_add_norm(x, a, b, w, woff, eps, out_dtype, want_y=True):
     return y
 
 
-def gemm_any(A, B, C, M, N, K, batch, sAb, sAm, sBb, sBn, sBk, sCb, sCm):
+def gemm_any(A, B, C, M, N, K, batch, sAb, sAm, sBb, sBn, sBk, sCb, sCm, bias=None):
     """C[b][m][n] = sum_k A[b][m][k] B[b][n][k] over element strides; the caller has checked that every index stays
     inside its tensor. bf16 operands with k contiguous run on the matrix cores (csrc/gemm_tile.hip), everything else
     (fp32 storage, k-major B) on the vector ALUs (csrc/gemm_any.hip)."""
     if A.dtype == torch.bfloat16 and B.dtype == torch.bfloat16 and sBk == 1:
         lib().gemm_tile(A.data_ptr(), B.data_ptr(), C.data_ptr(), int(M), int(N), int(K), int(batch), int(sAb),
-                        int(sAm), int(sBb), int(sBn), int(sCb), int(sCm), _dt(C, "C"), _stream())
+                        int(sAm), int(sBb), int(sBn), int(sCb), int(sCm), _dt(C, "C"), _ptr(bias), _stream())
         return C
     lib().gemm_any(A.data_ptr(), B.data_ptr(), C.data_ptr(), int(M), int(N), int(K), int(batch), int(sAb), int(sAm),
-                   int(sBb), int(sBn), int(sBk), int(sCb), int(sCm), _dt(A, "A"), _dt(B, "B"), _dt(C, "C"), _stream())
+                   int(sBb), int(sBn), int(sBk), int(sCb), int(sCm), _dt(A, "A"), _dt(B, "B"), _dt(C, "C"), _ptr(bias),
+                   _stream())
     return C
 
 
@@ -882,20 +885,24 @@ def _mfma_ok(x, w, out_dtype) -> bool:
             and x.data_ptr() % 16 == 0 and (x.stride(0) * 2) % 16 == 0 and w.data_ptr() % 16 == 0)
 
 
-def linear_f(x, w, out_dtype):
-    """x [M, K] . w [N, K]^T -> [M, N] in ``out_dtype`` with fp32 accumulation: the MFMA GEMM where it applies,
-    else the strided VALU GEMM (fp32 storage, fp32 output, odd shapes)."""
+def linear_f(x, w, out_dtype, bias=None, act="none"):
+    """act(x [M, K] . w [N, K]^T + bias) -> [M, N] in ``out_dtype`` with fp32 accumulation: the MFMA GEMM where it applies
+    (bias and activation in its epilogue), else the tile GEMM or the strided VALU GEMM (fp32 storage, fp32 output, odd
+    shapes) and the activation in a launch of its own."""
     M, K = x.shape
     N = w.shape[0]
     _rows(x, "x")
     _rows(w, "w", K)
     _check(w.is_contiguous(), "w contiguous")
+    if bias is not None:
+        _check(bias.dtype == w.dtype and bias.is_contiguous() and bias.numel() == N and bias.is_cuda, "bias [N] in w's type")
     if M == 0:
         return torch.empty(0, N, dtype=out_dtype, device=x.device)
     if _mfma_ok(x, w, out_dtype):
-        return linear(x, w)
+        return linear(x, w, bias, act)
     y = torch.empty(M, N, dtype=out_dtype, device=x.device)
-    return gemm_any(x, w, y, M, N, K, 1, 0, x.stride(0), 0, K, 1, 0, N)
+    gemm_any(x, w, y, M, N, K, 1, 0, x.stride(0), 0, K, 1, 0, N, bias)
+    return y if act in ("none", None) else act_fn(y, act)
 
 
 def head_absorb(q, uk_t, out_dtype=torch.float32, extra=0):
@@ -1017,7 +1024,7 @@ def glu_clamp(gu, F, limit, alpha):
     return out
 
 
-def moe_route(z, corr, top, normalize=True):
+def moe_route(z, corr, top, normalize=True, score="sigmoid"):
     T, E = z.shape
     _rows(z, "z", dtype=torch.float32)
     _check(z.is_contiguous(), "router logits contiguous")
@@ -1027,20 +1034,21 @@ def moe_route(z, corr, top, normalize=True):
                "correction fp32 [E]")
     idx = torch.empty(T, top, dtype=torch.int32, device=z.device)
     wts = torch.empty(T, top, dtype=torch.float32, device=z.device)
-    lib().moe_route(z.data_ptr(), _ptr(corr), idx.data_ptr(), wts.data_ptr(), T, E, top, int(bool(normalize)), _stream())
+    lib().moe_route(z.data_ptr(), _ptr(corr), idx.data_ptr(), wts.data_ptr(), T, E, top, int(bool(normalize)),
+                    int(score == "softmax"), _stream())
     return idx, wts
 
 
 ROUTER_FUSED_MAX_ROWS = 1024  # steps of at most this many tokens compute logits and routing in one launch
 
 
-def moe_router(h, router, corr, top, normalize=True):
+def moe_router(h, router, corr, top, normalize=True, score="sigmoid"):
     """(idx [T, top] int32, wts [T, top] fp32) from the layer input: fp32 router logits, then moe_route. Few rows (a
     decode step): one fused launch; a prompt: the matrix-core GEMM with fp32 output, then moe_route."""
     T, K = h.shape
     E = router.shape[0]
     if T > ROUTER_FUSED_MAX_ROWS:
-        return moe_route(linear_f(h, router, torch.float32), corr, top, normalize)
+        return moe_route(linear_f(h, router, torch.float32), corr, top, normalize, score)
     _rows(h, "h")
     _check(router.dtype == h.dtype and router.is_contiguous() and router.shape == (E, K) and router.is_cuda,
            "router [E, K] in h's storage type")
@@ -1051,22 +1059,23 @@ def moe_router(h, router, corr, top, normalize=True):
     idx = torch.empty(T, top, dtype=torch.int32, device=h.device)
     wts = torch.empty(T, top, dtype=torch.float32, device=h.device)
     lib().moe_router(h.data_ptr(), h.stride(0), router.data_ptr(), _ptr(corr), idx.data_ptr(), wts.data_ptr(), T, E, K,
-                     top, _dt(h, "h"), int(bool(normalize)), _stream())
+                     top, _dt(h, "h"), int(bool(normalize)), int(score == "softmax"), _stream())
     return idx, wts
 
 
 def moe_experts(h, idx, wts, gate, up, down, limit, alpha, shared=None, combine=True, act="glu_clamp",
-                weight_input=False):
-    """``combine=False``: leave the weighting and summing to the next residual add (returns a :class:`MoEPending`).
+                weight_input=False, identity=False):
+    """``identity``: indices from E on are identity experts. ``combine=False``: leave the weighting and summing to the next residual add (returns a :class:`MoEPending`).
     ``weight_input``: the weights scale the two input products in the gate / up epilogue (the experts have no
     biases), and the outputs are summed plainly (``MoEPending.wts`` is None)."""
     T, K = h.shape
-    E, F, _ = gate.shape
+    E, F, _ = up.shape
     N = down.shape[1]
     top = idx.shape[1]
     dt = _dt(h, "h")
     _rows(h, "h")
-    for t, nm, shp in ((gate, "gate", (E, F, K)), (up, "up", (E, F, K)), (down, "down", (E, N, F))):
+    _check((gate is None) == (act == "gelu"), "experts without a gate: act gelu")
+    for t, nm, shp in ((up if gate is None else gate, "gate", (E, F, K)), (up, "up", (E, F, K)), (down, "down", (E, N, F))):
         _check(t.dtype == h.dtype and t.is_contiguous() and tuple(t.shape) == shp and t.is_cuda, f"{nm} {shp}")
     _check(idx.dtype == torch.int32 and idx.is_contiguous() and idx.shape == (T, top) and idx.is_cuda, "idx")
     _check(wts.dtype == torch.float32 and wts.is_contiguous() and wts.shape == (T, top) and wts.is_cuda, "wts")
@@ -1087,24 +1096,26 @@ def moe_experts(h, idx, wts, gate, up, down, limit, alpha, shared=None, combine=
     place = torch.empty(P, dtype=torch.int32, device=dev)
     act_ = torch.empty(P, F, dtype=h.dtype, device=dev)
     y = torch.empty(P, N, dtype=torch.float32, device=dev)
-    _check(act in ("glu_clamp", "silu"), "expert activation: glu_clamp or silu")
+    _check(act in ("glu_clamp", "silu", "gelu"), "expert activation: glu_clamp, silu or gelu (no gate)")
+    _check(not identity or (K == N and not weight_input), "identity experts give the input row itself")
     pw, silu = (wts.data_ptr() if weight_input else 0), int(act == "silu")
     L = lib()
     st = _stream()
     L.moe_group(idx.data_ptr(), P, E, maxt, meta.data_ptr(), order.data_ptr(), place.data_ptr(), rows, st)
     if h.dtype == torch.bfloat16:  # matrix cores (csrc/gemm_tile.hip)
-        L.moe_gate_up_tile(h.data_ptr(), h.stride(0), gate.data_ptr(), up.data_ptr(), meta.data_ptr(),
+        L.moe_gate_up_tile(h.data_ptr(), h.stride(0), _ptr(gate), up.data_ptr(), meta.data_ptr(),
                            order.data_ptr(), act_.data_ptr(), E, maxt, top, F, K, float(limit), float(alpha), rows, pw,
                            silu, st)
         L.moe_down_tile(act_.data_ptr(), down.data_ptr(), meta.data_ptr(), y.data_ptr(), E, maxt, N, F, rows, st)
     else:
-        L.moe_gate_up(h.data_ptr(), h.stride(0), gate.data_ptr(), up.data_ptr(), meta.data_ptr(), order.data_ptr(),
+        L.moe_gate_up(h.data_ptr(), h.stride(0), _ptr(gate), up.data_ptr(), meta.data_ptr(), order.data_ptr(),
                       act_.data_ptr(), E, maxt, top, F, K, float(limit), float(alpha), dt, pw, silu, st)
         L.moe_down(act_.data_ptr(), down.data_ptr(), meta.data_ptr(), y.data_ptr(), E, maxt, N, F, dt, st)
     if not combine:
-        return MoEPending(y, place, None if weight_input else wts, shared, top)
+        return MoEPending(y, place, None if weight_input else wts, shared, top, h if identity else None)
     L.moe_combine(y.data_ptr(), place.data_ptr(), 0 if weight_input else wts.data_ptr(), _ptr(shared),
-                  shared.stride(0) if shared is not None else 0, out.data_ptr(), T, N, top, dt, st)
+                  shared.stride(0) if shared is not None else 0, out.data_ptr(), T, N, top, dt,
+                  h.data_ptr() if identity else 0, h.stride(0), st)
     return out
 
 
@@ -1203,7 +1214,7 @@ def gated_group_norm(o, gate, w, eps, act, c, out=None, out_dtype=None, groups=0
     _check(gate.dtype == w.dtype == out.dtype and gate.shape[0] == T and out.shape[0] == T, "gate / w / out types, rows")
     lib().gated_group_norm(o.data_ptr(), o.stride(0), gate.data_ptr(), gate.stride(0), w.data_ptr(), float(eps),
                            {"sigmoid": 0, "silu": 1}[act], float(c), out.data_ptr(), out.stride(0), T, N // n, n,
-                           _dt(w, "w"), int(bool(groups)), int(bool(gate_first)), _stream())
+                           _dt(w, "w"), int(bool(groups)), int(bool(gate_first)), 0, 0, 1.0, _stream())
     return out
 
 
@@ -1248,7 +1259,7 @@ def decay_recurrence(q, k, v, decay, state, cu, ctx_lens, state_slots, heads, di
         lib().recurrence(0, q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0), 0, 0, 0, 0,
                          decay.data_ptr(), 0, state.data_ptr(), cu.data_ptr(), ctx_lens.data_ptr(),
                          state_slots.data_ptr(), out.data_ptr(), heads * vdim, B, heads, heads, dim, vdim,
-                         int(bool(silu_in)), 0, _dt(q, "q"), 0, 0, _stream())
+                         int(bool(silu_in)), 0, _dt(q, "q"), 0, 0, 0, 0, _stream())
     return out
 
 
@@ -1273,7 +1284,8 @@ def delta_recurrence(q, k, v, a, b_, A_log, dt_bias, state, cu, ctx_lens, state_
         lib().recurrence(1, q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0),
                          a.data_ptr(), a.stride(0), 0, int(off_b), A_log.data_ptr(), dt_bias.data_ptr(),
                          state.data_ptr(), cu.data_ptr(), ctx_lens.data_ptr(), state_slots.data_ptr(), out.data_ptr(),
-                         heads * vdim, B, heads, kv_heads, dim, vdim, 0, ready, _dt(q, "q"), _dt(a, "a"), 0, _stream())
+                         heads * vdim, B, heads, kv_heads, dim, vdim, 0, ready, _dt(q, "q"), _dt(a, "a"), 0, 0, 0,
+                         _stream())
     return out
 
 
@@ -1330,7 +1342,7 @@ def sink_attn(q, k_cache, v_cache, block_tables, cu, ctx_lens, heads, kv_heads, 
     out = torch.empty(T, heads, R, dtype=torch.float32, device=q.device)
     nd = int(num_decode)
     _check(0 <= nd <= B, "num_decode outside the step")
-    mfma = (k_cache.dtype == torch.bfloat16 and max_qlen > 0 and lib().sink_attn_mfma_ok(dim, vdim)
+    mfma = (k_cache.dtype == torch.bfloat16 and max_qlen > 0 and lib().sink_attn_mfma_ok(dim, vdim, int(bool(precise)))
             and k_cache.data_ptr() % 16 == 0 and v_cache.data_ptr() % 16 == 0 and _SINK_MFMA)
     common = (heads, kv_heads, dim, vdim, k_cache.shape[1], float(scale), float(softcap or 0.0), int(bool(all_groups)),
               int(bool(sink)), int(chunk), int(vshare))
@@ -1343,10 +1355,10 @@ def sink_attn(q, k_cache, v_cache, block_tables, cu, ctx_lens, heads, kv_heads, 
                 lib().sink_attn_mfma(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
                                      block_tables.data_ptr() + 4 * first * maxb, maxb, cu.data_ptr() + 4 * first,
                                      ctx_lens.data_ptr() + 4 * first, out.data_ptr(), n, ql, *common,
-                                     int(bool(precise)), _stream())
+                                     int(bool(precise)), 0, 0, 0, 1, 0, 0, 0, 0, 0, 0, _stream())
     else:
         lib().sink_attn(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), block_tables.data_ptr(),
-                        block_tables.shape[1], cu.data_ptr(), ctx_lens.data_ptr(), out.data_ptr(), T, B, *common,
+                        block_tables.shape[1], cu.data_ptr(), ctx_lens.data_ptr(), out.data_ptr(), T, B, *common, 0, 0, 0,
                         _dt(k_cache, "k cache"), _stream())
     return out
 
@@ -1428,7 +1440,7 @@ def act_fn(x, act, params=()):
     _rows(x, "x")
     out = torch.empty(T, F, dtype=x.dtype, device=x.device)
     a, b = (float(params[0]), float(params[1])) if act == "xielu" else (0.0, 0.0)
-    lib().act_fn(x.data_ptr(), x.stride(0), out.data_ptr(), F, T, F, {"gelu_tanh": 0, "silu": 1, "xielu": 2}[act], a, b,
+    lib().act_fn(x.data_ptr(), x.stride(0), out.data_ptr(), F, T, F, {"gelu_tanh": 0, "silu": 1, "xielu": 2, "gelu": 3, "relu2": 4}[act], a, b,
                  _dt(x, "x"), _stream())
     return out
 
@@ -1465,17 +1477,31 @@ def diff_combine(O, lam, eps, mult, heads, kv_heads, vdim, out_dtype):
 
 
 # ------------------- blocks normed on both sides / token input / windowed sigmoid attention with pooled blocks / SSD
-def sandwich_add_norm(x, y, r, rb, wpost, eps, add, wnext, out_dtype):
-    """``y``: rows in the storage type, or a :class:`MoEPending` (combined while it is read)."""
+def sandwich_add_norm(x, y, r, rb, wpost, eps, add, wnext, out_dtype, groups=1):
+    """``y``: rows in the storage type, a :class:`MoEPending` (combined while it is read) or a ``PairPending`` (the results
+    of two mixers, normed and joined while they are read)."""
     T, W = x.shape
     _rows(x, "x", dtype=torch.float32)
     _check(x.is_contiguous(), "x contiguous")
     _check(out_dtype in _DT, "storage type bf16 / fp32")
     pend = y if isinstance(y, MoEPending) else None
+    pair = y if isinstance(y, PairPending) else None
     sh = None
+    if pair is not None:
+        for t_, nm in ((pair.yl, "left"), (pair.yr, "right")):
+            _rows(t_, nm, W, out_dtype)
+            _check(t_.shape[0] == T, "pair rows")
+        for t_ in (pair.wl, pair.wr):
+            _f32c(t_, "pair weights")
+            _check(t_.numel() == W, "pair weights [W]")
+        y = pair.yl
+    _check(groups >= 1 and W % groups == 0, "the norm's parts must divide the row")
     if pend is not None:
         _check(pend.y.shape == (T * pend.top, W) and pend.y.is_contiguous() and pend.place.numel() == T * pend.top,
                "pending expert outputs do not fit the stream")
+        if pend.ident is not None:
+            _rows(pend.ident, "ident", W, out_dtype)
+            _check(pend.ident.shape[0] == T, "ident rows")
         if pend.wts is not None:
             _check(tuple(pend.wts.shape) == (T, pend.top) and pend.wts.is_contiguous(), "pending weights [T, top]")
         sh = pend.shared
@@ -1505,7 +1531,10 @@ def sandwich_add_norm(x, y, r, rb, wpost, eps, add, wnext, out_dtype):
                             _ptr(pend.wts) if pend else 0, pend.top if pend else 0, _ptr(sh),
                             sh.stride(0) if sh is not None else 0, _ptr(r) if y is not None else 0,
                             r.stride(0) if (r is not None and y is not None) else 0, _ptr(rb), _ptr(wpost), _ptr(add),
-                            _ptr(wnext), _ptr(h), W, float(eps), T, W, _DT[out_dtype], _stream())
+                            _ptr(wnext), _ptr(h), W, float(eps), int(groups),
+                            _ptr(pend.ident) if pend else 0, pend.ident.stride(0) if pend and pend.ident is not None else 0,
+                            _ptr(pair.yr) if pair else 0, pair.yr.stride(0) if pair else 0, _ptr(pair.wl) if pair else 0,
+                            _ptr(pair.wr) if pair else 0, T, W, _DT[out_dtype], _stream())
     return h
 
 
@@ -1660,5 +1689,154 @@ def ssd_recurrence(x, Bm, Cm, dt, A_log, dt_bias, D, state, cu, ctx_lens, state_
         lib().recurrence(2, Cm.data_ptr(), Bm.data_ptr(), x.data_ptr(), Cm.stride(0), Bm.stride(0), x.stride(0),
                          dt.data_ptr(), dt.stride(0), 0, 0, A_log.data_ptr(), dt_bias.data_ptr(), state.data_ptr(),
                          cu.data_ptr(), ctx_lens.data_ptr(), state_slots.data_ptr(), out.data_ptr(), heads * vdim, B,
-                         heads, groups, N, vdim, 0, 0, _dt(x, "x"), _dt(dt, "dt"), D.data_ptr(), _stream())
+                         heads, groups, N, vdim, 0, 0, _dt(x, "x"), _dt(dt, "dt"), D.data_ptr(), 0, 0,
+                         _stream())
     return out
+
+
+# ---------- heads on their way into the cache / softmax over a window with kept positions / exponential-gate recurrence
+def head_prep_cache(proj, off_q, off_k, off_v, conv, tail, qw, kw, v_norm, eps, cs, vcs, k_cache, v_cache, slots, heads,
+                    kv_heads, dim, vdim, cu, ctx_lens, state_slots, single=False):
+    """``single``: every sequence of the step has one row - its workgroup then renews the convolution's tail as well."""
+    T = proj.shape[0]
+    _rows(proj, "proj")
+    nq, nk, nv = heads * dim, kv_heads * dim, kv_heads * vdim
+    _check(min(off_q, off_k, off_v) >= 0 and max(off_q + nq, off_k + nk, off_v + nv) <= proj.shape[1],
+           "q / k / v columns outside the projection")
+    for c, n, nm in ((k_cache, nk, "k cache"), (v_cache, nv, "v cache")):
+        _check(c.dtype == proj.dtype and c.is_contiguous() and c.dim() == 3 and c.shape[2] == n and c.is_cuda,
+               f"{nm} [blocks, block_size, {n}] in the model's storage type")
+    _check(slots.dtype == torch.int64 and slots.is_contiguous() and slots.is_cuda and slots.numel() == T, "slots")
+    for w_, nm in ((qw, "q norm"), (kw, "k norm")):
+        if w_ is not None:
+            _f32c(w_, nm)
+            _check(w_.numel() == dim, f"{nm} [dim]")
+    half = 0
+    if cs is not None:
+        _f32c(cs, "angles")
+        _check(cs.dim() == 3 and cs.shape[0] == T and cs.shape[2] == 2 and 2 * cs.shape[1] <= dim,
+               "angles [T, rotated dims / 2, 2], rotated dims <= dim")
+        half = cs.shape[1]
+    if vcs is not None:
+        _f32c(vcs, "value angles")
+        _check(tuple(vcs.shape) == (T, vdim // 2, 2) and vdim % 2 == 0, "value angles [T, vdim / 2, 2]")
+    B = cu.numel() - 1
+    taps = 0
+    if conv is not None:
+        taps = conv.shape[0]
+        _check(conv.dtype == proj.dtype and conv.is_contiguous() and conv.is_cuda
+               and tuple(conv.shape) == (taps, nq + nk + nv), "conv weight [taps, q | k | v columns]")
+        _i32(cu, "cu")
+        _i32(ctx_lens, "ctx_lens", B)
+        _i32(state_slots, "state_slots", B)
+        if taps > 1:
+            _f32c(tail, "tail")
+            _check(tail.dim() == 3 and tuple(tail.shape[1:]) == (taps - 1, nq + nk + nv), "tail [slots, taps - 1, columns]")
+        _check(not single or T == B, "single: one row per sequence")
+    q = torch.empty(T, nq, dtype=torch.float32, device=proj.device)
+    lib().head_prep(proj.data_ptr(), proj.stride(0), int(off_q), int(off_k), int(off_v), _ptr(conv), taps,
+                    _ptr(tail) if taps > 1 else 0, int(bool(single)), cu.data_ptr(), ctx_lens.data_ptr(),
+                    _ptr(state_slots) if conv is not None else 0, B, _ptr(qw), _ptr(kw), int(bool(v_norm)), float(eps),
+                    _ptr(cs), half, _ptr(vcs), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), slots.data_ptr(), T,
+                    heads, kv_heads, dim, vdim, _dt(proj, "proj"), _stream())
+    return q
+
+
+def window_attn(q, k_cache, v_cache, block_tables, cu, ctx_lens, heads, kv_heads, dim, vdim, scale, softcap, window,
+                keep_first, sinks, vcs, out_dtype, max_qlen=0, num_decode=0, max_ctx=0):
+    """The sink attention kernels (csrc/attention_sink.hip) over a window with kept first positions. ``max_qlen`` (the longest
+    portion, known on the host) > 0: bf16 pages of a shape the matrix-core kernel takes run on it, the ``num_decode``
+    leading single-row sequences in one launch - their keys split over workgroups when ``max_ctx`` (an upper bound of every
+    context length) is given - and the portions in another; everything else runs the vector kernel."""
+    T = q.shape[0]
+    _rows(q, "q", heads * dim, torch.float32)
+    _check(q.is_contiguous(), "q contiguous")
+    B = cu.numel() - 1
+    _i32(cu, "cu")
+    _i32(ctx_lens, "ctx_lens", B)
+    _i32(block_tables, "block_tables")
+    _check(block_tables.dim() == 2 and block_tables.shape[0] >= B, "block tables [B, blocks]")
+    _check(k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dtype == v_cache.dtype and k_cache.is_cuda
+           and k_cache.dim() == 3 and k_cache.shape[2] == kv_heads * dim and v_cache.shape[2] == kv_heads * vdim
+           and k_cache.shape[:2] == v_cache.shape[:2], "k / v cache [blocks, block_size, kv_heads * dim | vdim]")
+    _check(window >= 0 and keep_first >= 0 and out_dtype in _DT, "window, kept positions, out type")
+    if sinks is not None:
+        _f32c(sinks, "sinks")
+        _check(sinks.numel() == heads, "sinks [heads]")
+    if vcs is not None:
+        _f32c(vcs, "value angles")
+        _check(tuple(vcs.shape) == (T, vdim // 2, 2) and vdim % 2 == 0, "value angles [T, vdim / 2, 2]")
+    y = torch.empty(T, heads * vdim, dtype=out_dtype, device=q.device)
+    if T == 0:
+        return y
+    nd = int(num_decode)
+    _check(0 <= nd <= B, "num_decode outside the step")
+    sink, od = int(sinks is not None), _DT[out_dtype]
+    maxb, bs = block_tables.shape[1], k_cache.shape[1]
+    shape = (heads, kv_heads, dim, vdim, bs, float(scale), float(softcap or 0.0), 0, sink, 0, 1)
+    L, st = lib(), _stream()
+    if not (k_cache.dtype == torch.bfloat16 and max_qlen > 0 and L.sink_attn_mfma_ok(dim, vdim, 1) and _SINK_MFMA
+            and k_cache.data_ptr() % 16 == 0 and v_cache.data_ptr() % 16 == 0):
+        O = torch.empty(T, heads, vdim, dtype=torch.float32, device=q.device)
+        L.sink_attn(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), block_tables.data_ptr(), maxb, cu.data_ptr(),
+                    ctx_lens.data_ptr(), O.data_ptr(), T, B, *shape, _ptr(sinks), int(window), int(keep_first),
+                    _dt(k_cache, "k cache"), st)
+        L.attn_finish(O.data_ptr(), 0, 1, 0, T, sink, _ptr(sinks), _ptr(vcs), y.data_ptr(), heads, vdim, od, st)
+        return y
+    for first, n, ql in ((0, nd, 1), (nd, B - nd, int(max_qlen))):
+        if n <= 0:
+            continue
+        row0 = first  # single-row sequences come first: sequence b's row is row b
+        rows = n if ql == 1 else T - row0
+        nsplit = pool_key_split(n, kv_heads, int(window) + int(keep_first) if window else 0, 0, int(max_ctx)) \
+            if ql == 1 and max_ctx > 0 else 1
+        # straight into the result rows where no join and no turn-back over separate value tiles is left to do
+        direct = nsplit == 1 and out_dtype == torch.bfloat16 and (vcs is None or vdim in (64, 128, 256)) and vdim % 4 == 0
+        O = y if direct else torch.empty(nsplit, rows, heads, vdim, dtype=torch.float32, device=q.device)
+        ml = torch.empty(nsplit, rows, heads, 2, dtype=torch.float32, device=q.device) if nsplit > 1 else None
+        # (a finished fp32 block is addressed by the step's rows too: shift its base to row 0)
+        out_ptr = y.data_ptr() if direct else O.data_ptr() - 4 * row0 * heads * vdim
+        L.sink_attn_mfma(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), block_tables.data_ptr() + 4 * first * maxb,
+                         maxb, cu.data_ptr() + 4 * first, ctx_lens.data_ptr() + 4 * first, out_ptr, n, ql, *shape, 1,
+                         _ptr(sinks), int(window), int(keep_first), nsplit, O.data_ptr() if nsplit > 1 else 0, _ptr(ml),
+                         row0, rows, _ptr(vcs), int(direct), st)
+        if not direct:
+            L.attn_finish(O.data_ptr(), _ptr(ml), nsplit, row0, rows, sink, _ptr(sinks), _ptr(vcs), y.data_ptr(), heads,
+                          vdim, od, st)
+    return y
+
+
+def mlstm_mix(q, k, v, zi, zf, bi, bf, cap, S, n, m, cu, ctx_lens, state_slots, heads, dim, vdim, gate, w, eps, out_dtype,
+              max_qlen=0):
+    """Gates by a wave per (head, sequence), the matrix-state recurrence with the normaliser as one more column, the joined
+    per-head norm and gate."""
+    T, B, num = _rec_common(q, k, v, S, cu, ctx_lens, state_slots, heads, heads, dim, vdim)
+    for t, nm, shp in ((n, "n", (heads, dim)), (m, "m", (heads,))):
+        _f32c(t, nm)
+        _check(tuple(t.shape[1:]) == shp and t.shape[0] == S.shape[0], f"{nm} [slots, ...]")
+    for t, nm in ((zi, "zi"), (zf, "zf")):
+        _rows(t, nm, heads)
+        _check(t.shape[0] == T and t.dtype == q.dtype and t.stride(0) == zi.stride(0), "gate columns of one projection")
+    for t, nm in ((bi, "bi"), (bf, "bf")):
+        _f32c(t, nm)
+        _check(t.numel() == heads, f"{nm} [heads]")
+    N = heads * vdim
+    _rows(gate, "gate", N)
+    _check(w.is_contiguous() and w.numel() == N and gate.dtype == w.dtype == out_dtype and gate.shape[0] == T,
+           "gate / norm weight / out in one storage type")
+    y = torch.empty(T, N, dtype=out_dtype, device=q.device)
+    if T == 0:
+        return y
+    gates = torch.empty(T, heads, 4, dtype=torch.float32, device=q.device)
+    ab = torch.empty(T, 2 * heads, dtype=torch.float32, device=q.device)
+    den = torch.empty(T, heads, dtype=torch.float32, device=q.device)
+    L, st, dt = lib(), _stream(), _dt(q, "q")
+    L.mlstm_gates(zi.data_ptr(), zf.data_ptr(), zi.stride(0), bi.data_ptr(), bf.data_ptr(), float(cap), m.data_ptr(),
+                  cu.data_ptr(), ctx_lens.data_ptr(), state_slots.data_ptr(), gates.data_ptr(), ab.data_ptr(), B, heads,
+                  dt, st)
+    L.recurrence(2, q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0), ab.data_ptr(),
+                 2 * heads, 0, heads, 0, 0, S.data_ptr(), cu.data_ptr(), ctx_lens.data_ptr(), state_slots.data_ptr(),
+                 num.data_ptr(), N, B, heads, heads, dim, vdim, 0, 1, dt, 1, 0, n.data_ptr(), den.data_ptr(), st)
+    L.gated_group_norm(num.data_ptr(), N, gate.data_ptr(), gate.stride(0), w.data_ptr(), float(eps), 0, 1.0, y.data_ptr(),
+                       N, T, heads, vdim, _dt(w, "w"), 1, 0, den.data_ptr(), gates.data_ptr(), float(dim) ** -0.5, st)
+    return y

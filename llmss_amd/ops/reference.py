@@ -14,7 +14,7 @@ import numpy as np
 import torch
 import torch.nn.functional as F
 
-ACTS = {"none": 0, "gelu_tanh": 1, "gelu": 2, "relu": 3, "silu_glu": 4}
+ACTS = {"none": 0, "gelu_tanh": 1, "gelu": 2, "relu": 3, "silu_glu": 4, "relu2": 5}
 
 
 def _act(x: torch.Tensor, act: str) -> torch.Tensor:
@@ -26,6 +26,8 @@ def _act(x: torch.Tensor, act: str) -> torch.Tensor:
         return F.gelu(x)
     if act == "relu":
         return F.relu(x)
+    if act == "relu2":
+        return F.relu(x).square()
     raise ValueError(act)
 
 
@@ -471,9 +473,11 @@ def resid_add_norm(x: torch.Tensor, a, b, w, woff: float, eps: float, out_dtype,
     return y.to(out_dtype)
 
 
-def linear_f(x: torch.Tensor, w: torch.Tensor, out_dtype) -> torch.Tensor:
-    """x [M, K] . w [N, K]^T with fp32 accumulation -> [M, N] in ``out_dtype``."""
-    return (x.float() @ w.float().t()).to(out_dtype)
+def linear_f(x: torch.Tensor, w: torch.Tensor, out_dtype, bias: Optional[torch.Tensor] = None,
+             act: str = "none") -> torch.Tensor:
+    """act(x [M, K] . w [N, K]^T + bias [N]) with fp32 accumulation -> [M, N] in ``out_dtype``."""
+    y = x.float() @ w.float().t()
+    return _act(y if bias is None else y + bias.float(), act).to(out_dtype)
 
 
 def head_absorb(q: torch.Tensor, uk_t: torch.Tensor, out_dtype=torch.float32, extra: int = 0) -> torch.Tensor:
@@ -574,11 +578,13 @@ def glu_clamp(gu: torch.Tensor, F_: int, limit: float, alpha: float) -> torch.Te
     return glu_clamped(gu[:, :F_].float(), gu[:, F_:2 * F_].float(), limit, alpha).to(gu.dtype)
 
 
-def moe_route(z: torch.Tensor, corr: Optional[torch.Tensor], top: int, normalize: bool = True):
-    """fp32 router logits [T, E] -> (idx int32 [T, top], weights fp32 [T, top]): scores sigmoid(z), the ``top``
+def moe_route(z: torch.Tensor, corr: Optional[torch.Tensor], top: int, normalize: bool = True,
+              score: str = "sigmoid"):
+    """fp32 router logits [T, E] -> (idx int32 [T, top], weights fp32 [T, top]): scores sigmoid(z) (``score``
+    "softmax": softmax(z) over all outputs), the ``top``
     largest of score + corr chosen (ties: lower index), weights = chosen scores / (their sum + 1e-20), or the chosen
     scores themselves (``normalize`` false)."""
-    s = torch.sigmoid(z.float())
+    s = torch.softmax(z.float(), -1) if score == "softmax" else torch.sigmoid(z.float())
     ch = s if corr is None else s + corr.float()
     # descending by value, ascending by index among equals
     order = torch.argsort(ch, dim=-1, descending=True, stable=True)
@@ -590,19 +596,22 @@ def moe_route(z: torch.Tensor, corr: Optional[torch.Tensor], top: int, normalize
 
 
 def moe_router(h: torch.Tensor, router: torch.Tensor, corr: Optional[torch.Tensor], top: int,
-               normalize: bool = True):
+               normalize: bool = True, score: str = "sigmoid"):
     """Router logits in fp32 from the layer input, then :func:`moe_route`."""
-    return moe_route(linear_f(h, router, torch.float32), corr, top, normalize)
+    return moe_route(linear_f(h, router, torch.float32), corr, top, normalize, score)
 
 
 def moe_experts(h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, gate: torch.Tensor, up: torch.Tensor,
                 down: torch.Tensor, limit: float, alpha: float, shared: Optional[torch.Tensor] = None,
-                combine: bool = True, act: str = "glu_clamp", weight_input: bool = False) -> torch.Tensor:
+                combine: bool = True, act: str = "glu_clamp", weight_input: bool = False,
+                identity: bool = False) -> torch.Tensor:
     """sum_j wts[t, j] * down_e(glu(gate_e h, up_e h)) (+ shared) with e = idx[t, j] -> fp32 [T, N]. Stacked expert
     weights gate / up [E, F, K], down [E, N, F]; the activation is rounded to the storage type between the
     products, as the grouped GEMMs do. ``act`` "silu": silu(g) * u without clamps. ``weight_input``: the weight
     multiplies the expert's input instead, sum_j down_e(act(w gate_e h, w up_e h)) (experts have no biases, so the
-    weight is applied to the two products)."""
+    weight is applied to the two products). ``act`` "gelu": experts without a gate (``gate`` None), down_e(gelu(up_e
+    h)), the error-function form. ``identity``: an index from E on is an
+    identity expert, its output is h[t] itself."""
     T = h.shape[0]
     N = down.shape[1]
     out = torch.zeros(T, N, dtype=torch.float32, device=h.device)
@@ -611,6 +620,13 @@ def moe_experts(h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, gate: tor
         for e in idx[:, j].unique().tolist():
             rows = torch.nonzero(idx[:, j] == e).flatten()
             x = hf[rows]
+            if e >= up.shape[0]:
+                out[rows] += x * wts[rows, j:j + 1]
+                continue
+            if act == "gelu":
+                a = F.gelu(x @ up[e].float().t()).to(h.dtype).float()
+                out[rows] += (a @ down[e].float().t()) * wts[rows, j:j + 1]
+                continue
             g_, u_ = x @ gate[e].float().t(), x @ up[e].float().t()
             if weight_input:
                 g_, u_ = g_ * wts[rows, j:j + 1], u_ * wts[rows, j:j + 1]
@@ -969,20 +985,39 @@ def diff_combine(O, lam: float, eps: float, mult: float, heads: int, kv_heads: i
 
 
 # ------------------- blocks normed on both sides / token input / windowed sigmoid attention with pooled blocks / SSD
-def sandwich_add_norm(x, y, r, rb, wpost, eps: float, add, wnext, out_dtype):
+class PairPending:
+    """The results of two mixers side by side before they are joined: y = 1/2 (rms_norm(yl) * wl + rms_norm(yr) * wr), the
+    norms over the whole row. sandwich_add_norm takes it as its ``y`` and joins while it reads."""
+
+    __slots__ = ("yl", "yr", "wl", "wr")
+
+    def __init__(self, yl, yr, wl, wr):
+        self.yl, self.yr, self.wl, self.wr = yl, yr, wl, wr
+
+
+def _rms_parts(x, eps: float, groups: int):
+    xg = x.view(*x.shape[:-1], groups, x.shape[-1] // groups)
+    return (xg * torch.rsqrt(xg.pow(2).mean(-1, keepdim=True) + eps)).view(x.shape)
+
+
+def sandwich_add_norm(x, y, r, rb, wpost, eps: float, add, wnext, out_dtype, groups: int = 1):
     """x fp32 [T, W], in place: with ``y`` [T, W], x += rms_norm(y * sigmoid(r + rb)) * wpost (``r`` [T, W] gate
     logits and ``rb`` [W] their bias, or None for no gate; ``wpost`` fp32 [W]); with ``add`` (fp32 [T, W]) x += add;
-    with ``wnext`` (fp32 [W]) returns rms_norm(x) * wnext in ``out_dtype``, else None."""
+    with ``wnext`` (fp32 [W]) returns rms_norm(x) * wnext in ``out_dtype``, else None. ``groups``: both norms are taken in
+    that many equal consecutive parts of the row. ``y`` may be a :class:`PairPending`."""
+    if isinstance(y, PairPending):
+        l, rr = y.yl.float(), y.yr.float()
+        y = 0.5 * (_rms_parts(l, eps, 1) * y.wl.float() + _rms_parts(rr, eps, 1) * y.wr.float())
     if y is not None:
         yf = y.float()
         if r is not None:
             yf = yf * torch.sigmoid(r.float() + rb.float())
-        x.add_(yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps) * wpost.float())
+        x.add_(_rms_parts(yf, eps, groups) * wpost.float())
     if add is not None:
         x.add_(add)
     if wnext is None:
         return None
-    return (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * wnext.float()).to(out_dtype)
+    return (_rms_parts(x, eps, groups) * wnext.float()).to(out_dtype)
 
 
 def token_side_add(x, ids, table, col0: int, gate_w, proj_w, norm_w, eps: float, add, wnext, out_dtype):
@@ -1094,3 +1129,111 @@ def ssd_recurrence(x, Bm, Cm, dt, A_log, dt_bias, D, state, cu, ctx_lens, state_
             out[t0 + j] = (torch.einsum("hdv,hd->hv", S, CC[j]) + D.float()[:, None] * xx[j]).reshape(-1)
         state[slots[b]] = S
     return out
+
+
+# ------------- heads on their way into the cache / softmax over a window with kept positions / exponential-gate recurrence
+def _turn_half(x: torch.Tensor, cs: torch.Tensor, back: bool = False) -> torch.Tensor:
+    """x [T, n, dim] with the pairs (i, i + half), half = cs.shape[1], turned by cs [T, half, 2] = (cos, sin), or back."""
+    half = cs.shape[1]
+    c, s = cs[:, None, :, 0], cs[:, None, :, 1] * (-1.0 if back else 1.0)
+    u, v = x[..., :half], x[..., half:2 * half]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * half:]], -1)
+
+
+def head_prep_cache(proj, off_q: int, off_k: int, off_v: int, conv, tail, qw, kw, v_norm: bool, eps: float, cs, vcs,
+                    k_cache, v_cache, slots, heads: int, kv_heads: int, dim: int, vdim: int, cu, ctx_lens, state_slots,
+                    single: bool = False):
+    """From the projection rows (q | k | v columns): with ``conv`` [taps, q + k + v columns] a causal convolution over time
+    of all three, continuing from ``tail`` (fp32 [slots, taps - 1, columns], renewed here); queries and keys divided per
+    head by their root mean square and multiplied by ``qw`` / ``kw`` [dim] (None: left), then their first pairs turned by
+    ``cs`` [T, half, 2] (None: not); values (the projected key columns when off_v == off_k) divided per head by their
+    root mean square (``v_norm``) and turned whole by ``vcs`` [T, vdim / 2, 2] (None: not). Returns q fp32 [T, heads *
+    dim]; k / v go into the paged caches at ``slots`` (< 0: not cached). ``single`` (every sequence has one row) only
+    steers the GPU kernels."""
+    T = proj.shape[0]
+    nq, nk, nv = heads * dim, kv_heads * dim, kv_heads * vdim
+    if conv is not None:
+        u = causal_conv(proj[:, off_q:off_q + nq + nk + nv], conv.t().contiguous(), tail, cu, ctx_lens, state_slots, False,
+                        False, torch.float32)
+        q, k, v = u[:, :nq], u[:, nq:nq + nk], u[:, nq + nk:]
+    else:
+        q, k, v = (proj[:, o:o + n].float() for o, n in ((off_q, nq), (off_k, nk), (off_v, nv)))
+    q, k, v = q.reshape(T, heads, dim), k.reshape(T, kv_heads, dim), v.reshape(T, kv_heads, vdim)
+    if qw is not None:
+        q = _rms_parts(q, eps, 1) * qw.float()
+    if kw is not None:
+        k = _rms_parts(k, eps, 1) * kw.float()
+    if v_norm:
+        v = _rms_parts(v, eps, 1)
+    if cs is not None:
+        q, k = _turn_half(q, cs), _turn_half(k, cs)
+    if vcs is not None:
+        v = _turn_half(v, vcs)
+    keep = slots >= 0
+    k_cache.view(-1, nk)[slots[keep]] = k.reshape(T, nk)[keep].to(k_cache.dtype)
+    v_cache.view(-1, nv)[slots[keep]] = v.reshape(T, nv)[keep].to(v_cache.dtype)
+    return q.reshape(T, nq).contiguous()
+
+
+def window_attn(q, k_cache, v_cache, block_tables, cu, ctx_lens, heads: int, kv_heads: int, dim: int, vdim: int,
+                scale: float, softcap: float, window: int, keep_first: int, sinks, vcs, out_dtype, max_qlen: int = 0,
+                num_decode: int = 0, max_ctx: int = 0):
+    """Softmax attention of every row over its sequence's cached keys: the row at position i sees the positions j <= i with
+    i - j < ``window`` (0: all) or j < ``keep_first``. ``softcap`` > 0: scores softcap * tanh(s / softcap); ``sinks``
+    (fp32 [heads]): exp(sinks[h]) is added to the denominator; ``vcs`` [T, vdim / 2, 2]: every head's result is turned back
+    by the row's angles. Returns [T, heads * vdim] in ``out_dtype``. ``max_qlen``, ``num_decode`` and ``max_ctx`` only
+    steer the GPU kernels."""
+    T = q.shape[0]
+    bs = k_cache.shape[1]
+    rep = heads // kv_heads
+    out = torch.zeros(T, heads, vdim, dtype=torch.float32)
+    for b, t0, n, p0 in _seq_rows(cu, ctx_lens):
+        L = p0 + n
+        blocks = block_tables[b, : -(-L // bs)].long()
+        K = k_cache[blocks].reshape(-1, kv_heads, dim)[:L].float()
+        V = v_cache[blocks].reshape(-1, kv_heads, vdim)[:L].float()
+        s = torch.einsum("nhd,lhd->hnl", q[t0:t0 + n].view(n, heads, dim).float(), K.repeat_interleave(rep, 1)) * scale
+        if softcap:
+            s = softcap * torch.tanh(s / softcap)
+        i, j = (p0 + torch.arange(n))[:, None], torch.arange(L)[None, :]
+        vis = j <= i
+        if window:
+            vis = vis & ((i - j < window) | (j < keep_first))
+        s = s.masked_fill(~vis, float("-inf"))
+        if sinks is not None:
+            s = torch.cat([s, sinks.float()[:, None, None].expand(heads, n, 1)], -1)
+        out[t0:t0 + n] = torch.einsum("hnl,lhv->nhv", torch.softmax(s, -1)[..., :L], V.repeat_interleave(rep, 1))
+    if vcs is not None:
+        out = _turn_half(out, vcs, back=True)
+    return out.reshape(T, heads * vdim).to(out_dtype)
+
+
+def mlstm_mix(q, k, v, zi, zf, bi, bf, cap: float, S, n, m, cu, ctx_lens, state_slots, heads: int, dim: int, vdim: int,
+              gate, w, eps: float, out_dtype, max_qlen: int = 0):
+    """Matrix memory with exponential gates, per head: log gates i = cap tanh((zi + bi) / cap) and f = logsigmoid(cap
+    tanh((zf + bf) / cap)); m' = max(f + m, i); S <- exp(f + m - m') S + exp(i - m') k v^T, n likewise with k alone; o =
+    S^T q / (max(|n . q|, exp(-m')) + 1e-6) with q times dim^-1/2. S fp32 [slots, heads, dim, vdim], n [slots, heads, dim],
+    m [slots, heads], carried in the sequence's slot (zero when the portion starts at position 0). Then every head is
+    divided by its root mean square; times w [heads * vdim], times sigmoid(gate) -> [T, heads * vdim] in ``out_dtype``."""
+    T = q.shape[0]
+    out = torch.zeros(T, heads * vdim, dtype=torch.float32)
+    slots = state_slots.tolist()
+    for b, t0, L, p0 in _seq_rows(cu, ctx_lens):
+        sl = slots[b]
+        Sb = S[sl].clone() if p0 > 0 else torch.zeros(heads, dim, vdim)
+        nb = n[sl].clone() if p0 > 0 else torch.zeros(heads, dim)
+        mb = m[sl].clone() if p0 > 0 else torch.zeros(heads)
+        qq = q[t0:t0 + L].float().view(L, heads, dim) * dim ** -0.5
+        kk, vv = k[t0:t0 + L].float().view(L, heads, dim), v[t0:t0 + L].float().view(L, heads, vdim)
+        gi = cap * torch.tanh((zi[t0:t0 + L].float() + bi) / cap)
+        gf = F.logsigmoid(cap * torch.tanh((zf[t0:t0 + L].float() + bf) / cap))
+        for j in range(L):
+            mt = torch.maximum(gf[j] + mb, gi[j])
+            a, e = torch.exp(gf[j] + mb - mt), torch.exp(gi[j] - mt)
+            Sb = a[:, None, None] * Sb + (e[:, None] * kk[j])[:, :, None] * vv[j][:, None, :]
+            nb = a[:, None] * nb + e[:, None] * kk[j]
+            mb = mt
+            den = torch.maximum((nb * qq[j]).sum(-1).abs(), torch.exp(-mb)) + 1e-6
+            out[t0 + j] = (torch.einsum("hdv,hd->hv", Sb, qq[j]) / den[:, None]).reshape(-1)
+        S[sl], n[sl], m[sl] = Sb, nb, mb
+    return gated_group_norm(out, gate, w, eps, "sigmoid", 1.0, out_dtype=out_dtype, groups=heads)
