@@ -484,8 +484,10 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
     const int j0 = pos_of(u0), j1 = kept ? j0 : j0 + BKV - 1;
 #pragma unroll
     for (int n = 0; n < NS; ++n) {
-      // not wholly in the group's causal future, not wholly before the block or the window of its first row
-      act[n] = grp_rows[n] && (kept || (j0 <= grp_last[n] && j1 >= grp_lo[n] && !(window > 0 && grp_first[n] - j1 >= window)));
+      // not wholly in the group's causal future, not wholly before the block or the window of its first row (a kept
+      // position is never before the window)
+      act[n] = grp_rows[n] && (kept || (j0 <= grp_last[n] && j1 >= grp_lo[n] &&
+                                        !(window > 0 && j0 >= X.keep && grp_first[n] - j1 >= window)));
       any = any || act[n];
     }
     if (!any) return;

@@ -3,6 +3,7 @@
 It takes the config as the dictionary a ``config.json`` holds and the weights as a dictionary of checkpoint names, and
 shares no code with the framework's model path. Slow on purpose: every function is the equation it stands for.
 """
+import functools
 import math
 
 import torch
@@ -44,17 +45,17 @@ def rotate_half(x, positions, dims, base, sign=1.0):
 def causal_conv(u, w):
     """u [T, C], w [C, taps]: y_t = sum_j w[:, j] u_(t - taps + 1 + j), zeros before the start."""
     T, taps = u.shape[0], w.shape[1]
-    y = torch.zeros_like(u)
-    for t in range(T):
-        for j in range(taps):
-            s = t - taps + 1 + j
-            if s >= 0:
-                y[t] += w[:, j] * u[s]
-    return y
+    full = torch.cat([torch.zeros(taps - 1, u.shape[1], dtype=F64), u])
+    return sum(w[:, j] * full[j:j + T] for j in range(taps))
 
 
 def visible(i, j, size, keep_first):
     return j <= i and ((not size) or i - j < size or j < keep_first)
+
+
+@functools.lru_cache(maxsize=64)
+def visibility(T, size, keep_first):
+    return torch.tensor([[visible(i, j, size, keep_first) for j in range(T)] for i in range(T)])
 
 
 def softmax_attention(q, k, v, scale, size, keep_first=0, softcap=0.0, sink=None):
@@ -63,18 +64,16 @@ def softmax_attention(q, k, v, scale, size, keep_first=0, softcap=0.0, sink=None
     T, H, _ = q.shape
     G = k.shape[1]
     out = torch.zeros(T, H, v.shape[2], dtype=F64)
+    seen = visibility(T, size, keep_first)
     for h in range(H):
         g = h // (H // G)
-        for i in range(T):
-            js = [j for j in range(i + 1) if visible(i, j, size, keep_first)]
-            s = (k[js, g] @ q[i, h]) * scale
-            if softcap:
-                s = softcap * torch.tanh(s / softcap)
-            if sink is None:
-                p = torch.softmax(s, 0)
-            else:
-                p = torch.softmax(torch.cat([s, sink[h:h + 1]]), 0)[:-1]
-            out[i, h] = p @ v[js, g]
+        s = (q[:, h] @ k[:, g].T) * scale
+        if softcap:
+            s = softcap * torch.tanh(s / softcap)
+        s = torch.where(seen, s, torch.tensor(-math.inf, dtype=F64))
+        if sink is not None:  # one more entry in the denominator, without a value
+            s = torch.cat([s, sink[h].expand(T, 1)], 1)
+        out[:, h] = torch.softmax(s, 1)[:, :T] @ v[:, g]
     return out
 
 
