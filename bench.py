@@ -90,7 +90,22 @@ def main():
                     help="instead of the headline workload: prefill / decode throughput of the Fizelix design beside "
                          "the Llama family at equal size (bench/fizelix_compare.py), sizes by name, one GPU")
     ap.add_argument("--fizelix-kinds", default="fizelix,dense", help="which of the two models --fizelix runs")
+    ap.add_argument("--tefudra", nargs="?", const="w1024,w2048,w4096", default="",
+                    help="instead of the headline workload: prefill / decode throughput of the Tefudra design beside "
+                         "the Llama family at equal size (bench/tefudra_compare.py), sizes by name, one GPU")
+    ap.add_argument("--tefudra-kinds", default="tefudra,dense", help="which of the two models --tefudra runs")
     args = ap.parse_args()
+
+    if args.tefudra:
+        sys.path.insert(0, os.path.join(ROOT, "bench"))
+        import tefudra_compare
+
+        res = tefudra_compare.run(args.tefudra.split(","), args.batch_per_gpu, args.prompt_len, args.gen_len,
+                                  args.timisun_rounds,
+                                  lambda m: print(f"[bench] {m}", file=sys.stderr, flush=True),
+                                  kinds=tuple(args.tefudra_kinds.split(",")))
+        print(json.dumps(res), flush=True)
+        return
 
     if args.fizelix:
         sys.path.insert(0, os.path.join(ROOT, "bench"))
