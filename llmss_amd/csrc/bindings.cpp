@@ -135,6 +135,15 @@ void launch_recurrence(int mode, const void* q, const void* k, const void* v, in
 void launch_mlstm_gates(const void* zi, const void* zf, int64_t ld, const void* bi, const void* bf, float cap,
                         void* mstate, const void* cu, const void* ctx, const void* sslots, void* gates, void* ab, int B,
                         int H, int dt, hipStream_t st);
+bool mlstm_step_ok(int dim, int vdim);
+void launch_mlstm_step(const void* q, const void* k, const void* v, int64_t ldq, int64_t ldk, int64_t ldv, const void* zi,
+                       const void* zf, int64_t ldz, const void* bi, const void* bf, float cap, void* S, void* n, void* m,
+                       const void* cu, const void* ctx, const void* sslots, const void* gate, int64_t ldg, const void* w,
+                       float eps, float qs, void* y, int64_t ldy, int B, int H, int dim, int vdim, int dt, hipStream_t st);
+bool mlstm_chunk_ok(int dim, int vdim);
+void launch_mlstm_chunk(const void* q, const void* k, const void* v, int64_t ldq, int64_t ldk, int64_t ldv,
+                        const void* gates, void* S, void* n, const void* cu, const void* ctx, const void* sslots,
+                        void* num, void* den, int B, int H, int dim, int vdim, hipStream_t st);
 // query / key / value heads on their way into the paged cache
 void launch_head_prep(const void* proj, int64_t ldp, int off_q, int off_k, int off_v, const void* conv, int taps,
                       void* tail, int single, const void* cu, const void* ctx, const void* sslots, int B, const void* qw,
@@ -445,6 +454,22 @@ PYBIND11_MODULE(_C, m) {
                           uintptr_t st) {
     launch_mlstm_gates(CP(zi), CP(zf), ld, CP(bi), CP(bf), cap, P(ms), CP(cu), CP(ctx), CP(ss), P(gates), P(ab), B, H,
                        dt, S(st));
+  });
+  m.def("mlstm_step_ok", &mlstm_step_ok);
+  m.def("mlstm_chunk_ok", &mlstm_chunk_ok);
+  m.def("mlstm_step", [](uintptr_t q, uintptr_t k, uintptr_t v, int64_t ldq, int64_t ldk, int64_t ldv, uintptr_t zi,
+                         uintptr_t zf, int64_t ldz, uintptr_t bi, uintptr_t bf, float cap, uintptr_t Sp, uintptr_t n,
+                         uintptr_t ms, uintptr_t cu, uintptr_t ctx, uintptr_t ss, uintptr_t gate, int64_t ldg, uintptr_t w,
+                         float eps, float qs, uintptr_t y, int64_t ldy, int B, int H, int dim, int vdim, int dt,
+                         uintptr_t st) {
+    launch_mlstm_step(CP(q), CP(k), CP(v), ldq, ldk, ldv, CP(zi), CP(zf), ldz, CP(bi), CP(bf), cap, P(Sp), P(n), P(ms),
+                      CP(cu), CP(ctx), CP(ss), CP(gate), ldg, CP(w), eps, qs, P(y), ldy, B, H, dim, vdim, dt, S(st));
+  });
+  m.def("mlstm_chunk", [](uintptr_t q, uintptr_t k, uintptr_t v, int64_t ldq, int64_t ldk, int64_t ldv, uintptr_t gates,
+                          uintptr_t Sp, uintptr_t n, uintptr_t cu, uintptr_t ctx, uintptr_t ss, uintptr_t num,
+                          uintptr_t den, int B, int H, int dim, int vdim, uintptr_t st) {
+    launch_mlstm_chunk(CP(q), CP(k), CP(v), ldq, ldk, ldv, CP(gates), P(Sp), P(n), CP(cu), CP(ctx), CP(ss), P(num), P(den),
+                       B, H, dim, vdim, S(st));
   });
   m.def("head_prep", [](uintptr_t proj, int64_t ldp, int off_q, int off_k, int off_v, uintptr_t conv, int taps,
                         uintptr_t tail, int single, uintptr_t cu, uintptr_t ctx, uintptr_t ss, int B, uintptr_t qw,

@@ -425,7 +425,8 @@ class MLSTMMixer:
         return ops.mlstm_mix(part("q", nqk), part("k", nqk), part("v", nv), part("i", H), part("f", H), W.bi, W.bf,
                              spec.gate_cap, st["S"], st["n"], st["m"], cu, inp.ctx_lens, inp.state_slots, H, spec.dim,
                              spec.vdim, part("g", nv), W.norm, model.cfg.norm_eps, model.dtype,
-                             max_qlen=1 if inp.kind == "decode" else max(1, inp.max_seqlen))
+                             max_qlen=1 if inp.kind == "decode" else max(1, inp.max_seqlen),
+                             num_decode=0 if inp.kind == "decode" else inp.num_decode)
 
     @staticmethod
     def forward(model: "LayeredLM", i: int, W, spec, h, inp: StepInput, cu, caches):

@@ -1806,10 +1806,14 @@ def window_attn(q, k_cache, v_cache, block_tables, cu, ctx_lens, heads, kv_heads
     return y
 
 
+_MLSTM_MFMA = os.environ.get("LLMSS_MLSTM_MFMA", "1") != "0"  # 0: portions token by token (A/B runs)
+
+
 def mlstm_mix(q, k, v, zi, zf, bi, bf, cap, S, n, m, cu, ctx_lens, state_slots, heads, dim, vdim, gate, w, eps, out_dtype,
-              max_qlen=0):
-    """Gates by a wave per (head, sequence), the matrix-state recurrence with the normaliser as one more column, the joined
-    per-head norm and gate."""
+              max_qlen=0, num_decode=0):
+    """The ``num_decode`` leading single-row sequences (all of them when ``max_qlen`` is 1) take one fused launch; portions
+    the gates' scan, then bf16 rows the chunked form on the matrix cores and everything else the token-by-token recurrence
+    with the normaliser as one more column, then the per-head norm and gate."""
     T, B, num = _rec_common(q, k, v, S, cu, ctx_lens, state_slots, heads, heads, dim, vdim)
     for t, nm, shp in ((n, "n", (heads, dim)), (m, "m", (heads,))):
         _f32c(t, nm)
@@ -1827,16 +1831,34 @@ def mlstm_mix(q, k, v, zi, zf, bi, bf, cap, S, n, m, cu, ctx_lens, state_slots, 
     y = torch.empty(T, N, dtype=out_dtype, device=q.device)
     if T == 0:
         return y
+    L, st, dt, es = lib(), _stream(), _dt(q, "q"), y.element_size()
+    nd = B if max_qlen == 1 else int(num_decode)
+    _check(0 <= nd <= B and (nd < B or T == B), "num_decode outside the step")
+    if not (L.mlstm_step_ok(dim, vdim) and S.data_ptr() % 16 == 0):
+        nd = 0
+    zs = (zi.data_ptr(), zf.data_ptr(), zi.stride(0), bi.data_ptr(), bf.data_ptr(), float(cap))
+    if nd:
+        L.mlstm_step(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0), *zs, S.data_ptr(),
+                     n.data_ptr(), m.data_ptr(), cu.data_ptr(), ctx_lens.data_ptr(), state_slots.data_ptr(),
+                     gate.data_ptr(), gate.stride(0), w.data_ptr(), float(eps), float(dim) ** -0.5, y.data_ptr(), N, nd,
+                     heads, dim, vdim, dt, st)
+    if nd == B:
+        return y
+    # the portions: rows nd .. T - 1 (single-row sequences come first)
+    seqs = (cu.data_ptr() + 4 * nd, ctx_lens.data_ptr() + 4 * nd, state_slots.data_ptr() + 4 * nd)
     gates = torch.empty(T, heads, 4, dtype=torch.float32, device=q.device)
     ab = torch.empty(T, 2 * heads, dtype=torch.float32, device=q.device)
     den = torch.empty(T, heads, dtype=torch.float32, device=q.device)
-    L, st, dt = lib(), _stream(), _dt(q, "q")
-    L.mlstm_gates(zi.data_ptr(), zf.data_ptr(), zi.stride(0), bi.data_ptr(), bf.data_ptr(), float(cap), m.data_ptr(),
-                  cu.data_ptr(), ctx_lens.data_ptr(), state_slots.data_ptr(), gates.data_ptr(), ab.data_ptr(), B, heads,
-                  dt, st)
-    L.recurrence(2, q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0), ab.data_ptr(),
-                 2 * heads, 0, heads, 0, 0, S.data_ptr(), cu.data_ptr(), ctx_lens.data_ptr(), state_slots.data_ptr(),
-                 num.data_ptr(), N, B, heads, heads, dim, vdim, 0, 1, dt, 1, 0, n.data_ptr(), den.data_ptr(), st)
-    L.gated_group_norm(num.data_ptr(), N, gate.data_ptr(), gate.stride(0), w.data_ptr(), float(eps), 0, 1.0, y.data_ptr(),
-                       N, T, heads, vdim, _dt(w, "w"), 1, 0, den.data_ptr(), gates.data_ptr(), float(dim) ** -0.5, st)
+    L.mlstm_gates(*zs, m.data_ptr(), *seqs, gates.data_ptr(), ab.data_ptr(), B - nd, heads, dt, st)
+    qkv = (q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0))
+    if (q.dtype == torch.bfloat16 and _MLSTM_MFMA and L.mlstm_chunk_ok(dim, vdim)
+            and not any(p % 16 for p in qkv[:3]) and not any(x % 8 for x in qkv[3:])):
+        L.mlstm_chunk(*qkv, gates.data_ptr(), S.data_ptr(), n.data_ptr(), *seqs, num.data_ptr(), den.data_ptr(), B - nd,
+                      heads, dim, vdim, st)
+    else:
+        L.recurrence(2, *qkv, ab.data_ptr(), 2 * heads, 0, heads, 0, 0, S.data_ptr(), *seqs, num.data_ptr(), N, B - nd,
+                     heads, heads, dim, vdim, 0, 1, dt, 1, 0, n.data_ptr(), den.data_ptr(), st)
+    L.gated_group_norm(num.data_ptr() + 4 * nd * N, N, gate.data_ptr() + es * nd * gate.stride(0), gate.stride(0),
+                       w.data_ptr(), float(eps), 0, 1.0, y.data_ptr() + es * nd * N, N, T - nd, heads, vdim, _dt(w, "w"), 1,
+                       0, den.data_ptr() + 4 * nd * heads, gates.data_ptr() + 16 * nd * heads, float(dim) ** -0.5, st)
     return y

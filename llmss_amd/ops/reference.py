@@ -1209,12 +1209,13 @@ def window_attn(q, k_cache, v_cache, block_tables, cu, ctx_lens, heads: int, kv_
 
 
 def mlstm_mix(q, k, v, zi, zf, bi, bf, cap: float, S, n, m, cu, ctx_lens, state_slots, heads: int, dim: int, vdim: int,
-              gate, w, eps: float, out_dtype, max_qlen: int = 0):
+              gate, w, eps: float, out_dtype, max_qlen: int = 0, num_decode: int = 0):
     """Matrix memory with exponential gates, per head: log gates i = cap tanh((zi + bi) / cap) and f = logsigmoid(cap
     tanh((zf + bf) / cap)); m' = max(f + m, i); S <- exp(f + m - m') S + exp(i - m') k v^T, n likewise with k alone; o =
     S^T q / (max(|n . q|, exp(-m')) + 1e-6) with q times dim^-1/2. S fp32 [slots, heads, dim, vdim], n [slots, heads, dim],
     m [slots, heads], carried in the sequence's slot (zero when the portion starts at position 0). Then every head is
-    divided by its root mean square; times w [heads * vdim], times sigmoid(gate) -> [T, heads * vdim] in ``out_dtype``."""
+    divided by its root mean square; times w [heads * vdim], times sigmoid(gate) -> [T, heads * vdim] in ``out_dtype``.
+    ``max_qlen`` and ``num_decode`` only steer the GPU kernels."""
     T = q.shape[0]
     out = torch.zeros(T, heads * vdim, dtype=torch.float32)
     slots = state_slots.tolist()

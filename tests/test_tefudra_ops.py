@@ -335,7 +335,8 @@ class Memory:
             wide[:, 8:8 + self.n] = rows
             q, k, v, g, zi, zf = self.parts(wide[:, 8:8 + self.n])
             y = ops.mlstm_mix(q, k, v, zi, zf, to(self.bi, dev), to(self.bf, dev), self.cap, S, n, m, cu, ctx, ss, H, dim,
-                              vdim, g, to(self.w, dev, dt), self.eps, dt, max_qlen=max(c for _, _, c in step))
+                              vdim, g, to(self.w, dev, dt), self.eps, dt, max_qlen=max(c for _, _, c in step),
+                              num_decode=sum(1 for e in step if e[2] == 1 and e[1] > 0))
             at = 0
             for s, _, c in step:
                 got[s].append(y[at:at + c])
