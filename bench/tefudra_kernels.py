@@ -99,17 +99,17 @@ def main():
         pa = rn(T, nq + nk)
         single = phase == "decode"
         f_att = lambda: ops.head_prep_cache(pa, 0, nq, nq, None, None, qw, kw, False, 1e-6, cs_h, None, kc, vc, slots, H, G, D,
-                                            D, cu, cl, ss, single=single)
+                                            D, cu, cl, ss, single=single, q_dtype=bf)
         t = timed(f_att)
-        add("head_prep (q / k norm, rotation, cache)", phase, t, bytes_=T * ((nq + nk) * 2 + nq * 4 + 2 * nk * 2))
+        add("head_prep (q / k norm, rotation, cache)", phase, t, bytes_=T * ((nq + nk) * 2 + nq * 2 + 2 * nk * 2))
         qf = f_att()
         proj = rn(T, s["pcols"])
         conv, tail = rn(4, nq + 2 * nk, std=0.5), torch.zeros(B, 3, nq + 2 * nk, device=dev)
         f_par = lambda: ops.head_prep_cache(proj, 0, nq, nq + nk, conv, tail, None, None, True, 1e-6, cs, cs, kc, vc, slots, H,
-                                            G, D, D, cu, cl, ss, single=single)
+                                            G, D, D, cu, cl, ss, single=single, q_dtype=bf)
         t = timed(f_par)
         add("head_prep (4-tap convolution, value norm, rotations, cache)", phase, t,
-            bytes_=T * ((nq + 2 * nk) * 2 + nq * 4 + 2 * nk * 2))
+            bytes_=T * ((nq + 2 * nk) * 2 + nq * 2 + 2 * nk * 2))
         for nm, wnd, kp, cap, sk, vcs in (("window_attn (kept positions, sinks)", win, keep, 0.0, sinks, None),
                                           ("window_attn (soft cap, turned back)", lwin, 0, 30.0, None, cs)):
             vis = lambda p: min(p + 1, wnd) + min(kp, max(0, p + 1 - wnd))
@@ -118,7 +118,7 @@ def main():
                                          max_ctx=ctx if single else 0)
             t = timed(fa, iters=3, warm=1)
             add(nm, phase, t, flops=pairs * H * 4 * D,
-                bytes_=(T * nq * 4 + B * 2 * nk * min(ctx, wnd + kp) * 2 + T * nq * 2) if single else 0)
+                bytes_=(T * nq * 2 + B * 2 * nk * min(ctx, wnd + kp) * 2 + T * nq * 2) if single else 0)
         kc2, vc2 = rn(B * nblk, G, bs, D), rn(B * nblk, G, bs, D)
         qkv = rn(T, (H + 2 * G) * D)
         if phase == "prompt":

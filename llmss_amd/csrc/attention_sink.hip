@@ -333,9 +333,10 @@ void launch_sink_attn(const void* q, const void* kc, const void* vc, const void*
 // and one barrier per tile, measured the same as one tile and two barriers, and is not kept.)
 // The value tile holds VCH = 16 * NVT columns of the key's value row - all groups side by side when the heads'
 // weights are mixed afterwards - and blockIdx.y also enumerates the column chunks.
-// PRECISE: the fp32 queries and the fp32 softmax weights enter the products as the sum of two bf16 numbers (the
+// PRECISE 1: the fp32 queries and the fp32 softmax weights enter the products as the sum of two bf16 numbers (the
 // rounded value and the rounded remainder, two matrix instructions each), so scores and weighted sums are those of
-// 32-bit queries and weights; otherwise both are rounded to bf16 once.
+// 32-bit queries and weights. PRECISE 2: the queries are bf16 rows (as the keys they meet are), the weights enter as two
+// numbers. PRECISE 0: fp32 queries and weights are both rounded to bf16 once.
 // nsplit > 1 (steps of single rows): a row's list of keys is cut into nsplit runs of whole tiles, each walked by a
 // workgroup of its own that leaves its sums, maximum and denominator (no sink) in po / pml; attn_finish joins them.
 struct SinkExt {
@@ -350,9 +351,9 @@ struct SinkExt {
   int direct;      // the result goes straight to out as bf16 rows [T, H * vdim]
 };
 
-template <int DK, int NVT, bool PRECISE, int NS>
+template <int DK, int NVT, int PRECISE, int NS>
 __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
-    const float* __restrict__ q, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
+    const void* __restrict__ qv, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
     const int* __restrict__ block_tables, int max_blocks, const int* __restrict__ cu_q, const int* __restrict__ ctx_lens,
     float* __restrict__ out, int H, int G, int GE, int vdim, int bs, float scale, float cap, int all, int nvch,
     int sink, int chunk, int vshare, SinkExt X) {
@@ -389,7 +390,7 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
   int row[NS], hd[NS], qpos[NS], qlo[NS];
   bool valid[NS], grp_rows[NS];
   int grp_first[NS], grp_last[NS], grp_lo[NS], grp_hilo[NS];
-  s16x8 qf[NS][DK / 32], ql[NS][PRECISE ? DK / 32 : 1];
+  s16x8 qf[NS][DK / 32], ql[NS][PRECISE == 1 ? DK / 32 : 1];
   f32x4 o[NS][NVT];
   float m[NS], lsum[NS];
   bool wave_rows = false;
@@ -408,16 +409,23 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
     grp_last[n] = p0 + min(qlen - 1, r0 + (gs + 15) / GE);
     grp_lo[n] = chunk > 0 ? (grp_first[n] / chunk) * chunk : 0;
     grp_hilo[n] = chunk > 0 ? (grp_last[n] / chunk) * chunk : 0;
-    const float* qp = q + ((int64_t)(t0 + (valid[n] ? row[n] : 0)) * H + (valid[n] ? hd[n] : h0)) * dim + 8 * g;
+    const int64_t qat = ((int64_t)(t0 + (valid[n] ? row[n] : 0)) * H + (valid[n] ? hd[n] : h0)) * dim + 8 * g;
 #pragma unroll
-    for (int ks = 0; ks < DK / 32; ++ks)
+    for (int ks = 0; ks < DK / 32; ++ks) {
+      const bool in = 32 * ks + 8 * g < dim;
+      if constexpr (PRECISE == 2) {
+        const s16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
+        qf[n][ks] = in ? *reinterpret_cast<const s16x8*>((const bf16_t*)qv + qat + 32 * ks) : z;
+      } else {
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const float x = 32 * ks + 8 * g < dim ? qp[32 * ks + j] : 0.f;
-        const bf16_t hi = f2bf(x);
-        qf[n][ks][j] = (short)hi;
-        if constexpr (PRECISE) ql[n][ks][j] = (short)f2bf(x - bf2f(hi));
+        for (int j = 0; j < 8; ++j) {
+          const float x = in ? ((const float*)qv)[qat + 32 * ks + j] : 0.f;
+          const bf16_t hi = f2bf(x);
+          qf[n][ks][j] = (short)hi;
+          if constexpr (PRECISE == 1) ql[n][ks][j] = (short)f2bf(x - bf2f(hi));
+        }
       }
+    }
 #pragma unroll
     for (int i = 0; i < NVT; ++i) o[n][i] = f32x4{0.f, 0.f, 0.f, 0.f};
     // the sink: score 0, weight exp(0 - m), no value; without it a masked score's stand-in is the starting maximum
@@ -502,7 +510,7 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
 #pragma unroll
         for (int n = 0; n < NS; ++n) {
           s[n][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[n][ks], s[n][kt], 0, 0, 0);
-          if constexpr (PRECISE) s[n][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, ql[n][ks], s[n][kt], 0, 0, 0);
+          if constexpr (PRECISE == 1) s[n][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, ql[n][ks], s[n][kt], 0, 0, 0);
         }
       }
     }
@@ -676,7 +684,7 @@ void launch_sink_attn_mfma(const void* q, const void* kc, const void* vc, const 
   const int nvch = (RVtot + nvt * 16 - 1) / (nvt * 16);
   // two slot groups per wave where a portion has more rows than one group each would hold (the widest value tile,
   // and 128-wide keys with split queries beside the middle one, keep one: two groups would not fit the registers)
-  const bool two_fit = nvt <= 4 || (nvt == 8 && !(dim == 128 && precise));
+  const bool two_fit = nvt <= 4 || (nvt == 8 && !(dim > 64 && precise == 1));
   const int ns = (two_fit && max_qlen > 64 / GE) ? 2 : 1;
   const int rows_per_wg = 64 * ns / GE;
   const int64_t gy = (int64_t)G * (rep / GE) * nvch;
@@ -687,12 +695,13 @@ void launch_sink_attn_mfma(const void* q, const void* kc, const void* vc, const 
             pml ? (float*)pml - row0 * H * 2 : nullptr, rows * H, (const float*)vcs, direct};
 #define LAUNCH_SAM2(DK_, NVT_, PR_, NS_)                                                                            \
   sink_attn_mfma_kernel<DK_, NVT_, PR_, NS_><<<grid, 256, 0, st>>>(                                                 \
-      (const float*)q, (const bf16_t*)kc, (const bf16_t*)vc, (const int*)bt, maxb, (const int*)cu, (const int*)ctx, \
+      q, (const bf16_t*)kc, (const bf16_t*)vc, (const int*)bt, maxb, (const int*)cu, (const int*)ctx,               \
       (float*)out, H, G, GE, vdim, bs, scale, cap, all, nvch, sink, chunk, vshare, X)
 #define LAUNCH_SAM1(DK_, NVT_, NS_)                                                       \
   do {                                                                                    \
-    if (!precise) LAUNCH_SAM2(DK_, NVT_, false, NS_);                                     \
-    else LAUNCH_SAM2(DK_, NVT_, true, (DK_ == 128 && NVT_ == 8 && NS_ == 2) ? 1 : NS_);   \
+    if (precise == 0) LAUNCH_SAM2(DK_, NVT_, 0, NS_);                                     \
+    else if (precise == 2) LAUNCH_SAM2(DK_, NVT_, 2, NS_);                                \
+    else LAUNCH_SAM2(DK_, NVT_, 1, (DK_ == 128 && NVT_ == 8 && NS_ == 2) ? 1 : NS_);      \
   } while (0)
 #define LAUNCH_SAM(DK_)                       \
   do {                                        \

@@ -147,8 +147,9 @@ void launch_mlstm_chunk(const void* q, const void* k, const void* v, int64_t ldq
 // query / key / value heads on their way into the paged cache
 void launch_head_prep(const void* proj, int64_t ldp, int off_q, int off_k, int off_v, const void* conv, int taps,
                       void* tail, int single, const void* cu, const void* ctx, const void* sslots, int B, const void* qw,
-                      const void* kw, int vnorm, float eps, const void* cs, int half, const void* vcs, void* q, void* kc,
-                      void* vc, const void* slots, int T_, int H, int G, int dim, int vdim, int dt, hipStream_t st);
+                      const void* kw, int vnorm, float eps, const void* cs, int half, const void* vcs, void* q, int q_bf,
+                      void* kc, void* vc, const void* slots, int T_, int H, int G, int dim, int vdim, int dt,
+                      hipStream_t st);
 // blocks normed on both sides, token input, windowed sigmoid attention with pooled blocks
 void launch_sandwich_add_norm(void* x, const void* y, int64_t ldy, const void* ey, const void* place, const void* wts,
                               int top, const void* shared_, int64_t lds_, const void* r, int64_t ldr, const void* rb,
@@ -474,11 +475,11 @@ PYBIND11_MODULE(_C, m) {
   m.def("head_prep", [](uintptr_t proj, int64_t ldp, int off_q, int off_k, int off_v, uintptr_t conv, int taps,
                         uintptr_t tail, int single, uintptr_t cu, uintptr_t ctx, uintptr_t ss, int B, uintptr_t qw,
                         uintptr_t kw, int vnorm, float eps, uintptr_t cs, int half, uintptr_t vcs, uintptr_t q,
-                        uintptr_t kc, uintptr_t vc, uintptr_t slots, int T, int H, int G, int dim, int vdim, int dt,
+                        int q_bf, uintptr_t kc, uintptr_t vc, uintptr_t slots, int T, int H, int G, int dim, int vdim, int dt,
                         uintptr_t st) {
     launch_head_prep(CP(proj), ldp, off_q, off_k, off_v, CP(conv), taps, P(tail), single, CP(cu), CP(ctx), CP(ss), B,
-                     CP(qw), CP(kw), vnorm, eps, CP(cs), half, CP(vcs), P(q), P(kc), P(vc), CP(slots), T, H, G, dim,
-                     vdim, dt, S(st));
+                     CP(qw), CP(kw), vnorm, eps, CP(cs), half, CP(vcs), P(q), q_bf, P(kc), P(vc), CP(slots), T, H, G,
+                     dim, vdim, dt, S(st));
   });
   m.def("silu_f32", [](uintptr_t in, int64_t ldi, uintptr_t out, int64_t ldo, int T, int n, int dt, uintptr_t st) {
     launch_silu_f32(CP(in), ldi, P(out), ldo, T, n, dt, S(st));

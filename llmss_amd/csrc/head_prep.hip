@@ -7,7 +7,7 @@
 //   v:    the key columns as they were projected where there is no value projection (off_v == off_k); per head
 //         v <- v / sqrt(mean(v^2) + eps) (optional), then all vdim numbers turned by vcs [T, vdim / 2, 2] (optional)
 //
-// q leaves in fp32 [T, H * dim]; k and v go into the paged caches at slots[t] (< 0: not cached), in the storage type.
+// q leaves in fp32 [T, H * dim] or, for the matrix-core attention kernel, in bf16; k and v go into the paged caches at slots[t] (< 0: not cached), in the storage type.
 // Norms, angles and the convolution's sum are fp32. One workgroup per row: the row's numbers are formed in LDS, then a wave
 // takes a head at a time. In a step of single rows (tail_here) the workgroup also renews its sequence's tail - nobody
 // else reads it; portions renew theirs in a second launch, after every row has read the old one.
@@ -33,7 +33,8 @@ struct HeadPrepArgs {
   const float* cs;
   int half;
   const float* vcs;
-  float* q;
+  void* q;
+  int q_bf;
   void* kc;
   void* vc;
   const int64_t* slots;
@@ -55,9 +56,63 @@ __device__ __forceinline__ void hp_ld(const T* p, float* v) {
   }
 }
 
+// Heads whose vectors are whole 16-byte pieces: N / 8 neighbouring lanes (a power of two) share a vector, each lane takes
+// eight numbers and, where they are turned, the eight they are paired with; the sum of squares is added up over the lanes.
+template <typename T>
+__device__ __forceinline__ void head_vec(const HeadPrepArgs& A, const float* x0, int heads, int N, const float* w, bool norm,
+                                         int half, const float* tab, int kind, int64_t dst) {
+  const int L = N >> 3, sub = threadIdx.x & (L - 1), per = blockDim.x / L, d = 8 * sub;
+  const bool turn = d < 2 * half, lo = d < half;
+  const int od = lo ? d + half : d - half;
+  for (int n = threadIdx.x / L; n < heads; n += per) {
+    const float* x = x0 + n * N;
+    float a[8], o[8];
+    *reinterpret_cast<f32x4*>(a) = *reinterpret_cast<const f32x4*>(x + d);
+    *reinterpret_cast<f32x4*>(a + 4) = *reinterpret_cast<const f32x4*>(x + d + 4);
+    float inv = 1.f;
+    if (norm) {
+      float s = 0.f;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) s = fmaf(a[i], a[i], s);
+      for (int m = L >> 1; m > 0; m >>= 1) s += __shfl_xor(s, m, 64);
+      inv = 1.0f / sqrtf(s / (float)N + A.eps);
+    }
+    if (w) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) a[i] *= inv * w[d + i];
+    } else {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) a[i] *= inv;
+    }
+    if (turn) {
+      *reinterpret_cast<f32x4*>(o) = *reinterpret_cast<const f32x4*>(x + od);
+      *reinterpret_cast<f32x4*>(o + 4) = *reinterpret_cast<const f32x4*>(x + od + 4);
+      const float* tb = tab + 2 * (lo ? d : od);
+#pragma unroll
+      for (int i = 0; i < 8; i += 2) {
+        const f32x4 cs = *reinterpret_cast<const f32x4*>(tb + 2 * i);
+        const float o0 = o[i] * inv * (w ? w[od + i] : 1.0f), o1 = o[i + 1] * inv * (w ? w[od + i + 1] : 1.0f);
+        a[i] = lo ? a[i] * cs[0] - o0 * cs[1] : a[i] * cs[0] + o0 * cs[1];
+        a[i + 1] = lo ? a[i + 1] * cs[2] - o1 * cs[3] : a[i + 1] * cs[2] + o1 * cs[3];
+      }
+    }
+    const int64_t at = dst + (int64_t)n * N + d;
+    if (sizeof(T) == 2 && (kind != 0 || A.q_bf)) {
+      u16x8 y;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) y[i] = f2bf(a[i]);
+      *reinterpret_cast<u16x8*>((bf16_t*)(kind == 0 ? A.q : kind == 1 ? A.kc : A.vc) + at) = y;
+    } else {
+      float* p = (float*)(kind == 0 ? A.q : kind == 1 ? A.kc : A.vc) + at;
+      *reinterpret_cast<f32x4*>(p) = *reinterpret_cast<f32x4*>(a);
+      *reinterpret_cast<f32x4*>(p + 4) = *reinterpret_cast<f32x4*>(a + 4);
+    }
+  }
+}
+
 // V: numbers per thread and access while the row is formed (8 bf16 or 4 fp32 numbers = 16 bytes, or 1)
 template <typename T, int V>
-__global__ __launch_bounds__(256) void head_prep_kernel(HeadPrepArgs A) {
+__global__ __launch_bounds__(512) void head_prep_kernel(HeadPrepArgs A, int vec) {
   extern __shared__ __attribute__((aligned(16))) float us[];
   const int t = blockIdx.x, lane = threadIdx.x & 63, wv = threadIdx.x >> 6, nw = blockDim.x >> 6;
   const int dim = A.dim, vdim = A.vdim, H = A.H, G = A.G;
@@ -116,6 +171,16 @@ __global__ __launch_bounds__(256) void head_prep_kernel(HeadPrepArgs A) {
     }
   }
   __syncthreads();
+  if (vec) {
+    const float* kt = A.cs ? A.cs + (int64_t)t * A.half * 2 : nullptr;
+    head_vec<T>(A, us, H, dim, A.qw, A.qw != nullptr, kt ? A.half : 0, kt, 0, (int64_t)t * nq);
+    if (slot < 0) return;
+    head_vec<T>(A, us + nq, G, dim, A.kw, A.kw != nullptr, kt ? A.half : 0, kt, 1, slot * (int64_t)nk);
+    const float* vt = A.vcs ? A.vcs + (int64_t)t * vdim : nullptr;
+    head_vec<T>(A, us + (sharev ? nq : nq + nk), G, vdim, nullptr, A.vnorm != 0, vt ? vdim >> 1 : 0, vt, 2,
+                slot * (int64_t)nv);
+    return;
+  }
   const int nvec = H + G + (slot >= 0 ? G : 0);
   for (int n = wv; n < nvec; n += nw) {
     const int kind = n < H ? 0 : (n < H + G ? 1 : 2);  // query, key, value
@@ -137,7 +202,7 @@ __global__ __launch_bounds__(256) void head_prep_kernel(HeadPrepArgs A) {
     } else if (A.cs) {
       half = A.half, tab = A.cs + (int64_t)t * half * 2;
     }
-    float* qd = A.q + (int64_t)t * nq + idx * dim;
+    const int64_t qd = (int64_t)t * nq + idx * dim;
     T* cd = kind == 2 ? (T*)A.vc + slot * (int64_t)nv + idx * vdim : (T*)A.kc + slot * (int64_t)nk + idx * dim;
     for (int d = lane; d < N; d += 64) {
       float v = x[d] * inv * (w ? w[d] : 1.0f);
@@ -148,7 +213,8 @@ __global__ __launch_bounds__(256) void head_prep_kernel(HeadPrepArgs A) {
         const float c = tab[2 * i], s = tab[2 * i + 1];
         v = lo ? v * c - o * s : v * c + o * s;
       }
-      if (kind == 0) qd[d] = v;
+      if (kind == 0 && A.q_bf) ((bf16_t*)A.q)[qd + d] = f2bf(v);
+      else if (kind == 0) ((float*)A.q)[qd + d] = v;
       else El<T>::st(cd + d, v);
     }
   }
@@ -159,8 +225,9 @@ void launch_conv_tail(const void* in, int64_t ldi, void* state, const void* cu, 
 
 void launch_head_prep(const void* proj, int64_t ldp, int off_q, int off_k, int off_v, const void* conv, int taps,
                       void* tail, int single, const void* cu, const void* ctx, const void* sslots, int B, const void* qw,
-                      const void* kw, int vnorm, float eps, const void* cs, int half, const void* vcs, void* q, void* kc,
-                      void* vc, const void* slots, int T_, int H, int G, int dim, int vdim, int dt, hipStream_t st) {
+                      const void* kw, int vnorm, float eps, const void* cs, int half, const void* vcs, void* q, int q_bf,
+                      void* kc, void* vc, const void* slots, int T_, int H, int G, int dim, int vdim, int dt,
+                      hipStream_t st) {
   if (T_ == 0) return;
   if (G < 1 || H % G) throw std::runtime_error("head_prep: heads must be a multiple of the key heads");
   if (half < 0 || 2 * half > dim || (vcs && vdim % 2)) throw std::runtime_error("head_prep: rotation wider than a head");
@@ -172,17 +239,23 @@ void launch_head_prep(const void* proj, int64_t ldp, int off_q, int off_k, int o
   if (lds > 64 * 1024) throw std::runtime_error("head_prep: rows wider than 16384");
   HeadPrepArgs A{proj, ldp, off_q, off_k, off_v, conv, taps, (float*)tail, single, (const int*)cu, (const int*)ctx,
                  (const int*)sslots, B, (const float*)qw, (const float*)kw, vnorm, eps, (const float*)cs, half,
-                 (const float*)vcs, (float*)q, kc, vc, (const int64_t*)slots, H, G, dim, vdim};
+                 (const float*)vcs, q, q_bf, kc, vc, (const int64_t*)slots, H, G, dim, vdim};
   const int vn = dt == 0 ? 8 : 4;
   const auto al16 = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
   const bool vec = al16(proj) && al16(conv) && ldp % vn == 0 && off_q % vn == 0 && off_k % vn == 0 && off_v % vn == 0 &&
                    nq % vn == 0 && nk % vn == 0 && nv % vn == 0;
+  // whole 16-byte pieces per head: sizes 8 to 512 that are powers of two, turned parts of whole pieces
+  const auto pow2 = [](int n) { return n >= 8 && n <= 512 && (n & (n - 1)) == 0; };
+  const int hv = pow2(dim) && pow2(vdim) && half % 8 == 0 && (!vcs || vdim % 16 == 0) && al16(q) && al16(kc) && al16(vc) &&
+                 al16(cs) && al16(vcs) && (dt == 0 || !q_bf);
+  const int th = T_ <= 512 ? 512 : 256;  // few rows: more waves to a row
+  if (q_bf && dt != 0) throw std::runtime_error("head_prep: bf16 queries come from bf16 rows");
   if (dt == 0) {
-    if (vec) head_prep_kernel<bf16_t, 8><<<T_, 256, lds, st>>>(A);
-    else head_prep_kernel<bf16_t, 1><<<T_, 256, lds, st>>>(A);
+    if (vec) head_prep_kernel<bf16_t, 8><<<T_, th, lds, st>>>(A, hv);
+    else head_prep_kernel<bf16_t, 1><<<T_, th, lds, st>>>(A, hv);
   } else if (dt == 1) {
-    if (vec) head_prep_kernel<float, 4><<<T_, 256, lds, st>>>(A);
-    else head_prep_kernel<float, 1><<<T_, 256, lds, st>>>(A);
+    if (vec) head_prep_kernel<float, 4><<<T_, th, lds, st>>>(A, hv);
+    else head_prep_kernel<float, 1><<<T_, th, lds, st>>>(A, hv);
   } else {
     throw std::runtime_error("bad dtype code");
   }

@@ -365,22 +365,23 @@ void launch_delta_gates(const void* a, const void* b, int64_t ld, const void* A_
 //   i = cap tanh((zi + bi) / cap), f = logsigmoid(cap tanh((zf + bf) / cap)), m' = max(f + m, i), m = 0 before position 0
 // out: gates [T, H, 4] = (f, i, m', m) and ab [T, 2H] = (g | e) = (exp(f + m - m') | exp(i - m')); the sequence's running
 // maximum [slots, H] is read from and renewed in its slot. (sum of f, m) pairs compose associatively - first (F1, M1), then
-// (F2, M2) give (F1 + F2, max(F2 + M1, M2)) - so a wave scans 64 tokens at a time: one wave per (head, sequence).
+// (F2, M2) give (F1 + F2, max(F2 + M1, M2)) - so a workgroup per (head, sequence) scans 256 tokens at a time, 64 by each wave.
 template <typename T>
-__global__ __launch_bounds__(64) void mlstm_gates_kernel(const T* __restrict__ zi, const T* __restrict__ zf, int64_t ld,
+__global__ __launch_bounds__(256) void mlstm_gates_kernel(const T* __restrict__ zi, const T* __restrict__ zf, int64_t ld,
                                                          const float* __restrict__ bi, const float* __restrict__ bf,
                                                          float cap, float* __restrict__ mstate,
                                                          const int* __restrict__ cu, const int* __restrict__ ctx,
                                                          const int* __restrict__ sslots, f32x4* __restrict__ gates,
                                                          float* __restrict__ ab, int H) {
-  const int h = blockIdx.x, b = blockIdx.y, lane = threadIdx.x;
+  __shared__ float wF[4], wM[4], last;
+  const int h = blockIdx.x, b = blockIdx.y, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
   const int t0 = cu[b], qlen = cu[b + 1] - t0, n = ctx[b], slot = sslots[b];
   if (qlen <= 0) return;
   const bool real = slot >= 0 && n > 0;
   float m = real && n > qlen ? mstate[(int64_t)slot * H + h] : 0.f;
   const float icap = 1.0f / cap;
-  for (int j0 = 0; j0 < qlen; j0 += 64) {
-    const int j = j0 + lane;
+  for (int j0 = 0; j0 < qlen; j0 += 256) {
+    const int j = j0 + threadIdx.x;
     const bool in = j < qlen;
     float f = 0.f, i = -INFINITY;  // past the end: the pair that changes nothing
     if (in) {
@@ -397,18 +398,24 @@ __global__ __launch_bounds__(64) void mlstm_gates_kernel(const T* __restrict__ z
         F += F1;
       }
     }
-    const float mt = fmaxf(F + m, M);
+    if (lane == 63) wF[wv] = F, wM[wv] = M;
+    __syncthreads();
+    float mw = m;  // the running maximum before this wave's tokens
+    for (int u = 0; u < wv; ++u) mw = fmaxf(wF[u] + mw, wM[u]);
+    const float mt = fmaxf(F + mw, M);
     float mp = __shfl_up(mt, 1, 64);
-    if (lane == 0) mp = m;
+    if (lane == 0) mp = mw;
     if (in) {
       const int64_t e = (int64_t)(t0 + j) * H + h;
       gates[e] = f32x4{f, i, mt, mp};
       ab[(int64_t)(t0 + j) * 2 * H + h] = expf(f + mp - mt);
       ab[(int64_t)(t0 + j) * 2 * H + H + h] = expf(i - mt);
     }
-    m = __shfl(mt, min(63, qlen - 1 - j0), 64);
+    if ((int)threadIdx.x == min(255, qlen - 1 - j0)) last = mt;
+    __syncthreads();
+    m = last;
   }
-  if (real && lane == 0) mstate[(int64_t)slot * H + h] = m;
+  if (real && threadIdx.x == 0) mstate[(int64_t)slot * H + h] = m;
 }
 
 void launch_mlstm_gates(const void* zi, const void* zf, int64_t ld, const void* bi, const void* bf, float cap,
@@ -417,7 +424,7 @@ void launch_mlstm_gates(const void* zi, const void* zf, int64_t ld, const void* 
   if (B == 0) return;
   if (B > 65535) throw std::runtime_error("mlstm_gates: too many sequences");
   dim3 g(H, B);
-  DISPATCH_T(dt, T, (mlstm_gates_kernel<T><<<g, 64, 0, st>>>(
+  DISPATCH_T(dt, T, (mlstm_gates_kernel<T><<<g, 256, 0, st>>>(
       (const T*)zi, (const T*)zf, ld, (const float*)bi, (const float*)bf, cap, (float*)mstate, (const int*)cu,
       (const int*)ctx, (const int*)sslots, (f32x4*)gates, (float*)ab, H)));
   HIP_CHECK_LAUNCH();

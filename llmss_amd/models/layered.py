@@ -387,7 +387,8 @@ class WindowAttention:
         vcs = model.angles(inp, W.vrot_key, W.vfreqs) if W.vfreqs is not None else None
         q = ops.head_prep_cache(proj, c["q"], c["k"], c["v"], W.conv, st.get("tail"), W.q_norm, W.k_norm, spec.v_norm,
                                 model.cfg.norm_eps, cs, vcs, kc, vc, inp.slots, spec.heads, spec.kv_heads, spec.dim,
-                                spec.vdim, cu, inp.ctx_lens, inp.state_slots, single=single or inp.max_seqlen <= 1)
+                                spec.vdim, cu, inp.ctx_lens, inp.state_slots, single=single or inp.max_seqlen <= 1,
+                                q_dtype=ops.window_q_dtype(kc, spec.dim, spec.vdim))
         return ops.window_attn(q, kc, vc, inp.block_tables, cu, inp.ctx_lens, spec.heads, spec.kv_heads, spec.dim,
                                spec.vdim, spec.scale, spec.softcap, spec.window, spec.keep_first, W.sink, vcs,
                                model.dtype, max_qlen=1 if single else max(1, inp.max_seqlen),

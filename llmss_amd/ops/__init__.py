@@ -210,4 +210,5 @@ ssd_recurrence = _route("ssd_recurrence")
 PairPending = ref.PairPending
 head_prep_cache = _route("head_prep_cache")
 window_attn = _route("window_attn")
+window_q_dtype = _route("window_q_dtype")
 mlstm_mix = _route("mlstm_mix")

@@ -1696,7 +1696,7 @@ def ssd_recurrence(x, Bm, Cm, dt, A_log, dt_bias, D, state, cu, ctx_lens, state_
 
 # ---------- heads on their way into the cache / softmax over a window with kept positions / exponential-gate recurrence
 def head_prep_cache(proj, off_q, off_k, off_v, conv, tail, qw, kw, v_norm, eps, cs, vcs, k_cache, v_cache, slots, heads,
-                    kv_heads, dim, vdim, cu, ctx_lens, state_slots, single=False):
+                    kv_heads, dim, vdim, cu, ctx_lens, state_slots, single=False, q_dtype=torch.float32):
     """``single``: every sequence of the step has one row - its workgroup then renews the convolution's tail as well."""
     T = proj.shape[0]
     _rows(proj, "proj")
@@ -1733,13 +1733,21 @@ def head_prep_cache(proj, off_q, off_k, off_v, conv, tail, qw, kw, v_norm, eps, 
             _f32c(tail, "tail")
             _check(tail.dim() == 3 and tuple(tail.shape[1:]) == (taps - 1, nq + nk + nv), "tail [slots, taps - 1, columns]")
         _check(not single or T == B, "single: one row per sequence")
-    q = torch.empty(T, nq, dtype=torch.float32, device=proj.device)
+    _check(q_dtype == torch.float32 or q_dtype == proj.dtype, "queries in fp32 or the storage type")
+    q = torch.empty(T, nq, dtype=q_dtype, device=proj.device)
     lib().head_prep(proj.data_ptr(), proj.stride(0), int(off_q), int(off_k), int(off_v), _ptr(conv), taps,
                     _ptr(tail) if taps > 1 else 0, int(bool(single)), cu.data_ptr(), ctx_lens.data_ptr(),
                     _ptr(state_slots) if conv is not None else 0, B, _ptr(qw), _ptr(kw), int(bool(v_norm)), float(eps),
-                    _ptr(cs), half, _ptr(vcs), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), slots.data_ptr(), T,
-                    heads, kv_heads, dim, vdim, _dt(proj, "proj"), _stream())
+                    _ptr(cs), half, _ptr(vcs), q.data_ptr(), int(q_dtype == torch.bfloat16), k_cache.data_ptr(),
+                    v_cache.data_ptr(), slots.data_ptr(), T, heads, kv_heads, dim, vdim, _dt(proj, "proj"), _stream())
     return q
+
+
+def window_q_dtype(k_cache, dim, vdim) -> torch.dtype:
+    """Storage type window_attn wants its queries in: bf16 where the matrix-core kernel runs, else fp32."""
+    ok = k_cache.dtype == torch.bfloat16 and _SINK_MFMA and lib().sink_attn_mfma_ok(dim, vdim, 1) and \
+        k_cache.data_ptr() % 16 == 0
+    return torch.bfloat16 if ok else torch.float32
 
 
 def window_attn(q, k_cache, v_cache, block_tables, cu, ctx_lens, heads, kv_heads, dim, vdim, scale, softcap, window,
@@ -1749,8 +1757,8 @@ def window_attn(q, k_cache, v_cache, block_tables, cu, ctx_lens, heads, kv_heads
     leading single-row sequences in one launch - their keys split over workgroups when ``max_ctx`` (an upper bound of every
     context length) is given - and the portions in another; everything else runs the vector kernel."""
     T = q.shape[0]
-    _rows(q, "q", heads * dim, torch.float32)
-    _check(q.is_contiguous(), "q contiguous")
+    _rows(q, "q", heads * dim)
+    _check(q.is_contiguous() and q.dtype in _DT, "q contiguous, fp32 or bf16")
     B = cu.numel() - 1
     _i32(cu, "cu")
     _i32(ctx_lens, "ctx_lens", B)
@@ -1777,6 +1785,7 @@ def window_attn(q, k_cache, v_cache, block_tables, cu, ctx_lens, heads, kv_heads
     L, st = lib(), _stream()
     if not (k_cache.dtype == torch.bfloat16 and max_qlen > 0 and L.sink_attn_mfma_ok(dim, vdim, 1) and _SINK_MFMA
             and k_cache.data_ptr() % 16 == 0 and v_cache.data_ptr() % 16 == 0):
+        _check(q.dtype == torch.float32, "bf16 queries: matrix-core shapes and max_qlen only")
         O = torch.empty(T, heads, vdim, dtype=torch.float32, device=q.device)
         L.sink_attn(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), block_tables.data_ptr(), maxb, cu.data_ptr(),
                     ctx_lens.data_ptr(), O.data_ptr(), T, B, *shape, _ptr(sinks), int(window), int(keep_first),
@@ -1797,7 +1806,8 @@ def window_attn(q, k_cache, v_cache, block_tables, cu, ctx_lens, heads, kv_heads
         # (a finished fp32 block is addressed by the step's rows too: shift its base to row 0)
         out_ptr = y.data_ptr() if direct else O.data_ptr() - 4 * row0 * heads * vdim
         L.sink_attn_mfma(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), block_tables.data_ptr() + 4 * first * maxb,
-                         maxb, cu.data_ptr() + 4 * first, ctx_lens.data_ptr() + 4 * first, out_ptr, n, ql, *shape, 1,
+                         maxb, cu.data_ptr() + 4 * first, ctx_lens.data_ptr() + 4 * first, out_ptr, n, ql, *shape,
+                         2 if q.dtype == torch.bfloat16 else 1,
                          _ptr(sinks), int(window), int(keep_first), nsplit, O.data_ptr() if nsplit > 1 else 0, _ptr(ml),
                          row0, rows, _ptr(vcs), int(direct), st)
         if not direct:

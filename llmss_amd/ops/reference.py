@@ -1142,13 +1142,13 @@ def _turn_half(x: torch.Tensor, cs: torch.Tensor, back: bool = False) -> torch.T
 
 def head_prep_cache(proj, off_q: int, off_k: int, off_v: int, conv, tail, qw, kw, v_norm: bool, eps: float, cs, vcs,
                     k_cache, v_cache, slots, heads: int, kv_heads: int, dim: int, vdim: int, cu, ctx_lens, state_slots,
-                    single: bool = False):
+                    single: bool = False, q_dtype=torch.float32):
     """From the projection rows (q | k | v columns): with ``conv`` [taps, q + k + v columns] a causal convolution over time
     of all three, continuing from ``tail`` (fp32 [slots, taps - 1, columns], renewed here); queries and keys divided per
     head by their root mean square and multiplied by ``qw`` / ``kw`` [dim] (None: left), then their first pairs turned by
     ``cs`` [T, half, 2] (None: not); values (the projected key columns when off_v == off_k) divided per head by their
-    root mean square (``v_norm``) and turned whole by ``vcs`` [T, vdim / 2, 2] (None: not). Returns q fp32 [T, heads *
-    dim]; k / v go into the paged caches at ``slots`` (< 0: not cached). ``single`` (every sequence has one row) only
+    root mean square (``v_norm``) and turned whole by ``vcs`` [T, vdim / 2, 2] (None: not). Returns q [T, heads *
+    dim] in ``q_dtype``; k / v go into the paged caches at ``slots`` (< 0: not cached). ``single`` (every sequence has one row) only
     steers the GPU kernels."""
     T = proj.shape[0]
     nq, nk, nv = heads * dim, kv_heads * dim, kv_heads * vdim
@@ -1172,7 +1172,11 @@ def head_prep_cache(proj, off_q: int, off_k: int, off_v: int, conv, tail, qw, kw
     keep = slots >= 0
     k_cache.view(-1, nk)[slots[keep]] = k.reshape(T, nk)[keep].to(k_cache.dtype)
     v_cache.view(-1, nv)[slots[keep]] = v.reshape(T, nv)[keep].to(v_cache.dtype)
-    return q.reshape(T, nq).contiguous()
+    return q.reshape(T, nq).contiguous().to(q_dtype)
+
+
+def window_q_dtype(k_cache, dim: int, vdim: int) -> torch.dtype:
+    return torch.float32
 
 
 def window_attn(q, k_cache, v_cache, block_tables, cu, ctx_lens, heads: int, kv_heads: int, dim: int, vdim: int,

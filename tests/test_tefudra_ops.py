@@ -131,7 +131,7 @@ class Attn:
     """A layer's attention over scattered pages, fed in portions through head_prep_cache and window_attn."""
 
     def __init__(self, device, dtype, H, G, dim, vdim, scale, window, keep=0, cap=0.0, sink=False, qk_norm=False,
-                 shared_kv=False, conv=0, v_norm=False, rot=0, base=100.0, rotv=False, bs=16, seed=0):
+                 shared_kv=False, conv=0, v_norm=False, rot=0, base=100.0, rotv=False, bs=16, seed=0, q_storage=True):
         self.__dict__.update(locals())
         n = H * dim + G * dim + (0 if shared_kv else G * vdim)
         self.cols = n
@@ -189,7 +189,8 @@ class Attn:
             q = ops.head_prep_cache(proj, 8, ok, ok if self.shared_kv else ok + G * dim,
                                     to(self.w.t(), dev, dt) if self.conv else None, tail if self.conv > 1 else None,
                                     to(self.qw, dev), to(self.kw, dev), self.v_norm, self.eps, cs, vcs, kc, vc, sl, H, G,
-                                    dim, vdim, cu, ctx, ss, single=ql == 1)
+                                    dim, vdim, cu, ctx, ss, single=ql == 1,
+                                    q_dtype=ops.window_q_dtype(kc, dim, vdim) if self.q_storage else torch.float32)
             y = ops.window_attn(q, kc, vc, pg.bt([s for s, _, _ in step]), cu, ctx, H, G, dim, vdim, self.scale, self.cap,
                                 self.window, self.keep, to(self.sinks, dev), vcs, dt, max_qlen=ql,
                                 num_decode=nd if nd < len(step) else 0,
@@ -232,6 +233,8 @@ def test_attention_over_portions_and_single_rows(device, dtype, name):
     for cuts in ([T], [2, 2, 3, 16, 15, 17, 2, 1, 1, 16], [1] * 6 + [40] + [1] * 29):
         close(a.run([x], [cuts], slots=[2])[0], want, dtype, f"cuts {cuts}")
     close(a.run([x], [[60] + [1] * 15], split=False)[0], want, dtype, "single rows without the key split")
+    a.q_storage = False  # fp32 queries, split into two numbers on the matrix cores
+    close(a.run([x], [[60] + [1] * 15])[0], want, dtype, "fp32 queries")
 
 
 @pytest.mark.parametrize("device,dtype", RUNS)
