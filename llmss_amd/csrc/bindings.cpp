@@ -88,6 +88,8 @@ void launch_gemm_tile(const void* A, const void* B, void* C, int M, int N, int K
 void launch_moe_gate_up_tile(const void* h, int64_t ldh, const void* wg, const void* wu, const void* meta,
                              const void* order, void* act, int E, int maxt, int top, int F, int K, float limit,
                              float alpha, int tile_rows, const void* pw, int silu, hipStream_t st);
+void launch_moe_pp(int mode, const void* A, int64_t lda, const void* W, const void* meta, const void* order, void* C, int E,
+                   int maxt, int top, int N, int K, int act, hipStream_t st);
 void launch_moe_down_tile(const void* act, const void* wd, const void* meta, void* y, int E, int maxt, int N, int F,
                           int tile_rows, hipStream_t st);
 void launch_latent_norm_cache(const void* src, int64_t ld, int off, const void* w, float eps, void* cache,
@@ -371,6 +373,10 @@ PYBIND11_MODULE(_C, m) {
                                int tile_rows, uintptr_t pw, int silu, uintptr_t st) {
     launch_moe_gate_up_tile(CP(h), ldh, CP(wg), CP(wu), CP(meta), CP(order), P(act), E, maxt, top, F, K, limit, alpha,
                             tile_rows, CP(pw), silu, S(st));
+  });
+  m.def("moe_pp", [](int mode, uintptr_t A, int64_t lda, uintptr_t W, uintptr_t meta, uintptr_t order, uintptr_t C, int E,
+                     int maxt, int top, int N, int K, int act, uintptr_t st) {
+    launch_moe_pp(mode, CP(A), lda, CP(W), CP(meta), CP(order), P(C), E, maxt, top, N, K, act, S(st));
   });
   m.def("moe_down_tile", [](uintptr_t act, uintptr_t wd, uintptr_t meta, uintptr_t y, int E, int maxt, int N, int F,
                             int tile_rows, uintptr_t st) {

@@ -901,6 +901,9 @@ __global__ __launch_bounds__(512, 1) void gemm_big_kernel(const void* __restrict
 // LDS-DMA + fragment-read traffic through the LDS costs ~25 % each on top of the MFMA/barrier skeleton.
 // K % 8 == 0: a partial last K-tile reads zeros (zpage) for the chunks past K; rows beyond M / N are clamped on load
 // and masked on store.
+// GRP: the grouped expert products of a mixture-of-experts layer (moe.hip's tile list, tiles of 256 rows): 1 - rows of A
+// gathered through order[] / top, activation in the epilogue, bf16 rows in expert order; 2 - A rows already in expert
+// order, fp32 output. Every die takes a contiguous run of the list's tiles with all their column tiles.
 // -------------------------------------------------------------------------------------------
 __device__ __forceinline__ void pp_barrier() {
   __builtin_amdgcn_sched_barrier(0);
@@ -908,12 +911,20 @@ __device__ __forceinline__ void pp_barrier() {
   __builtin_amdgcn_sched_barrier(0);
 }
 
-template <bool KTAIL>
+struct PpGroup {
+  const int* meta = nullptr;
+  const int* order = nullptr;
+  int E = 0, maxt = 0, top = 1;
+  int64_t sB = 0;         // elements between the experts' weights
+  float* Yf = nullptr;    // GRP 2
+};
+
+template <bool KTAIL, int GRP = 0>
 __global__ __launch_bounds__(512, 1) void gemm_pp_kernel(const bf16_t* __restrict__ A, int64_t lda,
                                                          const bf16_t* __restrict__ B, int64_t ldb,
                                                          const bf16_t* __restrict__ bias, bf16_t* __restrict__ Y,
                                                          int64_t ldy, int M, int N, int K, int act, int glu,
-                                                         int group_m, const char* __restrict__ zpage) {
+                                                         int group_m, const char* __restrict__ zpage, PpGroup gr) {
   constexpr int SLOT = 16384, BUF = 4 * SLOT;
   __shared__ __attribute__((aligned(16))) char smem[2 * BUF];
   const int lane = threadIdx.x & 63;
@@ -922,10 +933,22 @@ __global__ __launch_bounds__(512, 1) void gemm_pp_kernel(const bf16_t* __restric
   const int wr = w >> 2, wc = w & 3;
   const int ntn = (N + 255) / 256, ntm = (M + 255) / 256;
   const int GM = group_m;  // XCD-contiguous tile ranges, GM M-tiles per group (as gemm_big)
-  const int tile = xcd_remap(blockIdx.x, ntn * ntm);
-  const int grp = tile / (GM * ntn), gidx = tile - grp * (GM * ntn);
-  const int gm = min(GM, ntm - grp * GM);
-  const int m0 = (grp * GM + gidx % gm) * 256, n0 = (gidx / gm) * 256;
+  int m0, n0;
+  if constexpr (GRP != 0) {
+    const int nt = gr.meta[0];
+    if ((int)blockIdx.x >= nt * ntn) return;
+    const int id = xcd_remap(blockIdx.x, nt * ntn), ty = id / ntn;
+    const int e = gr.meta[1 + (gr.E + 1) + ty];
+    n0 = (id - ty * ntn) * 256;
+    m0 = gr.meta[1 + (gr.E + 1) + gr.maxt + ty];
+    M = gr.meta[1 + e + 1];
+    B += (int64_t)e * gr.sB;
+  } else {
+    const int tile = xcd_remap(blockIdx.x, ntn * ntm);
+    const int grp = tile / (GM * ntn), gidx = tile - grp * (GM * ntn);
+    const int gm = min(GM, ntm - grp * GM);
+    m0 = (grp * GM + gidx % gm) * 256, n0 = (gidx / gm) * 256;
+  }
   const int nk = (K + 63) / 64;
 
   // staging: slot h, instruction i (0, 1) = 8 local rows x 128 B, local row lr = (8 i + w) * 8 + lane / 8;
@@ -940,8 +963,9 @@ __global__ __launch_bounds__(512, 1) void gemm_pp_kernel(const bf16_t* __restric
     const int gc = (lane & 7) ^ (lr & 7);
     lofs[i] = inst * 1024;
     kcol[i] = gc * 8;
-    const int ar0 = min(m0 + (lr >> 6) * 128 + (lr & 63), M - 1);
-    const int ar1 = min(m0 + (lr >> 6) * 128 + 64 + (lr & 63), M - 1);
+    int ar0 = min(m0 + (lr >> 6) * 128 + (lr & 63), M - 1);
+    int ar1 = min(m0 + (lr >> 6) * 128 + 64 + (lr & 63), M - 1);
+    if constexpr (GRP == 1) ar0 = gr.order[ar0] / gr.top, ar1 = gr.order[ar1] / gr.top;
     const int bc0 = min(n0 + (lr >> 5) * 64 + (lr & 31), N - 1);
     const int bc1 = min(n0 + (lr >> 5) * 64 + 32 + (lr & 31), N - 1);
     soff[0][i] = (int64_t)ar0 * lda * 2 + gc * 16;
@@ -1040,8 +1064,23 @@ __global__ __launch_bounds__(512, 1) void gemm_pp_kernel(const bf16_t* __restric
   if (w < 4) pp_barrier();  // balances the stagger barrier
   __builtin_amdgcn_s_setprio(0);
   wait_vmcnt<0>();
-  tile_store_lds<256, 256, 8, 4, 512, 2 * BUF>(acc, smem, wr * 128, wc * 64, m0, n0, M, N, nullptr, Y, ldy, bias,
-                                               act, glu);
+  if constexpr (GRP == 2) {
+#pragma unroll
+    for (int a = 0; a < 8; ++a)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int row = m0 + wr * 128 + a * 16 + 4 * g + i;
+        if (row >= M) continue;
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+          const int col = n0 + wc * 64 + b * 16 + li;
+          if (col < N) gr.Yf[(int64_t)row * ldy + col] = acc[a][b][i];
+        }
+      }
+  } else {
+    tile_store_lds<256, 256, 8, 4, 512, 2 * BUF>(acc, smem, wr * 128, wc * 64, m0, n0, M, N, nullptr, Y, ldy, bias,
+                                                 act, glu);
+  }
 }
 
 // -------------------------------------------------------------------------------------------
@@ -1872,10 +1911,10 @@ int launch_tiled(const bf16_t* X, int64_t ldx, const void* W, int64_t ldw, const
   if (tsel == 4) {
     if (K & 63)
       gemm_pp_kernel<true><<<tiles_of(M, N, 256, 256), 512, 0, st>>>(X, ldx, (const bf16_t*)W, ldw, B, Y, ldy, M, N, K,
-                                                                     act, g, g_big_group_m, zero_page());
+                                                                     act, g, g_big_group_m, zero_page(), PpGroup{});
     else
       gemm_pp_kernel<false><<<tiles_of(M, N, 256, 256), 512, 0, st>>>(X, ldx, (const bf16_t*)W, ldw, B, Y, ldy, M, N, K,
-                                                                      act, g, g_big_group_m, nullptr);
+                                                                      act, g, g_big_group_m, nullptr, PpGroup{});
     HIP_CHECK_LAUNCH();
     return 0;
   }
@@ -2077,3 +2116,31 @@ void gemm_plan(int M, int N, int K, bool w_fp8, int* nt, int* splitk) {
   }
 }
 
+// Grouped expert products on the ping-pong kernel, over a tile list of 256 rows per tile (moe_group): C = act(A[order / top]
+// W_e^T) in bf16 (mode 1) or C = A W_e^T in fp32 (mode 2). A [rows, K] with row stride lda, W [E, N, K].
+void launch_moe_pp(int mode, const void* A, int64_t lda, const void* W, const void* meta, const void* order, void* C, int E,
+                   int maxt, int top, int N, int K, int act, hipStream_t st) {
+  if (maxt <= 0) return;
+  if (K % 8 || lda % 8 || (((uintptr_t)A | (uintptr_t)W) & 15)) throw std::runtime_error("moe_pp: rows must be 16-byte aligned");
+  const int64_t nwg = (int64_t)maxt * ((N + 255) / 256);
+  if (nwg > 0x7fffffff) throw std::runtime_error("moe_pp: grid too large");
+  PpGroup gr;
+  gr.meta = (const int*)meta, gr.order = (const int*)order, gr.E = E, gr.maxt = maxt, gr.top = top;
+  gr.sB = (int64_t)N * K;
+  gr.Yf = (float*)C;
+  const char* z = K & 63 ? zero_page() : nullptr;
+#define LAUNCH_PPG(KT_, G_)                                                                                         \
+  gemm_pp_kernel<KT_, G_><<<(unsigned)nwg, 512, 0, st>>>((const bf16_t*)A, lda, (const bf16_t*)W, K, nullptr, (bf16_t*)C, \
+                                                         N, 0, N, K, act, 0, 1, z, gr)
+  if (mode == 1) {
+    if (K & 63) LAUNCH_PPG(true, 1);
+    else LAUNCH_PPG(false, 1);
+  } else if (mode == 2) {
+    if (K & 63) LAUNCH_PPG(true, 2);
+    else LAUNCH_PPG(false, 2);
+  } else {
+    throw std::runtime_error("moe_pp: mode");
+  }
+#undef LAUNCH_PPG
+  HIP_CHECK_LAUNCH();
+}

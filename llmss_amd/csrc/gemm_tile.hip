@@ -59,12 +59,12 @@ __device__ __forceinline__ u16x8 gt_load(const bf16_t* row, int k, int K, bool v
   return v;
 }
 
-// BM x BN output tile per 256-thread workgroup (64x64 or 128x128), waves in a 2x2 grid: each wave owns a
+// BM x BN output tile per 256-thread workgroup (64x64, 128x128, or 128x256 where LDS reads would otherwise bound it), waves in a 2x2 grid: each wave owns a
 // (BM/2) x (BN/2) block = MB x NB accumulators of 16x16. Per 32 of k a wave reads MB A fragments and NB B
 // fragments from LDS for MB * NB MFMAs (two such halves per staged k step of 64). The next k step's global loads are issued into registers before the current
 // step's MFMAs and written to LDS after them, so memory latency overlaps the matrix work.
 template <int MODE, typename TC, int BM, int BN>
-__global__ __launch_bounds__(256) void gemm_tile_kernel(GemmTileArgs p) {
+__global__ __launch_bounds__(256, BM * BN > 128 * 128 ? 2 : 1) void gemm_tile_kernel(GemmTileArgs p) {
   constexpr int MB = BM / 32, NB = BN / 32;   // 16x16 blocks per wave, rows x columns
   constexpr int CA = BM / 32, CB = BN / 32;   // 16-byte chunks per thread per staged tile
   constexpr bool DUAL = MODE == GT_GATE_UP;
@@ -73,7 +73,7 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmTileArgs p) {
   __shared__ __attribute__((aligned(16))) bf16_t B2s[DUAL ? BN * GT_LD : 8];
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, li = lane & 15, g = lane >> 4;
   const int wm = (w >> 1) * (BM / 2), wn = (w & 1) * (BN / 2);
-  const int n0 = blockIdx.x * BN;
+  int n0 = blockIdx.x * BN;
   int m0 = 0, rows = 0, crow0 = 0;
   const bf16_t* A = p.A;
   const bf16_t* B = p.B;
@@ -85,8 +85,13 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmTileArgs p) {
     B += (int64_t)blockIdx.z * p.sBb;
   } else {
     if ((int)blockIdx.y >= p.meta[0]) return;
-    const int e = p.meta[1 + (p.E + 1) + blockIdx.y];
-    crow0 = p.meta[1 + (p.E + 1) + p.maxt + blockIdx.y];
+    // every die takes a contiguous run of the list's tiles, all their column tiles with them: an expert's weights then
+    // pass through few L2s, and a row tile's rows stay in one
+    const int id = xcd_remap(blockIdx.y * gridDim.x + blockIdx.x, p.meta[0] * gridDim.x);
+    const int ty = id / gridDim.x;
+    n0 = (id % gridDim.x) * BN;
+    const int e = p.meta[1 + (p.E + 1) + ty];
+    crow0 = p.meta[1 + (p.E + 1) + p.maxt + ty];
     rows = min(BM, p.meta[1 + e + 1] - crow0);
     B += (int64_t)e * p.sBb;
     if constexpr (DUAL) B2 += (int64_t)e * p.sBb;
@@ -238,8 +243,10 @@ void launch_moe_gate_up_tile(const void* h, int64_t ldh, const void* wg, const v
   // workgroup per CU; at 128x64 two to three fit and hide each other's staging
   if (!wg) {
     a.B = (const bf16_t*)wu; a.B2 = nullptr;
-    dim3 g((F + tile_rows - 1) / tile_rows, maxt);
-    if (tile_rows == 128) gemm_tile_kernel<GT_UP, bf16_t, 128, 128><<<g, 256, 0, st>>>(a);
+    const int bn = tile_rows == 128 && F >= 512 ? 256 : tile_rows;
+    dim3 g((F + bn - 1) / bn, maxt);
+    if (bn == 256) gemm_tile_kernel<GT_UP, bf16_t, 128, 256><<<g, 256, 0, st>>>(a);
+    else if (tile_rows == 128) gemm_tile_kernel<GT_UP, bf16_t, 128, 128><<<g, 256, 0, st>>>(a);
     else gemm_tile_kernel<GT_UP, bf16_t, 64, 64><<<g, 256, 0, st>>>(a);
     HIP_CHECK_LAUNCH();
     return;
@@ -260,8 +267,10 @@ void launch_moe_down_tile(const void* act, const void* wd, const void* meta, voi
   a.A = (const bf16_t*)act; a.B = (const bf16_t*)wd; a.C = y;
   a.N = N; a.K = F; a.sAm = F; a.sBb = (int64_t)N * F; a.sBn = F; a.sCm = N;
   a.meta = (const int*)meta; a.E = E; a.maxt = maxt; a.top = 1;
-  dim3 g((N + tile_rows - 1) / tile_rows, maxt);
-  if (tile_rows == 128) gemm_tile_kernel<GT_DOWN, float, 128, 128><<<g, 256, 0, st>>>(a);
+  const int bn = tile_rows == 128 && N >= 512 ? 256 : tile_rows;
+  dim3 g((N + bn - 1) / bn, maxt);
+  if (bn == 256) gemm_tile_kernel<GT_DOWN, float, 128, 256><<<g, 256, 0, st>>>(a);
+  else if (tile_rows == 128) gemm_tile_kernel<GT_DOWN, float, 128, 128><<<g, 256, 0, st>>>(a);
   else gemm_tile_kernel<GT_DOWN, float, 64, 64><<<g, 256, 0, st>>>(a);
   HIP_CHECK_LAUNCH();
 }

@@ -1063,6 +1063,9 @@ def moe_router(h, router, corr, top, normalize=True, score="sigmoid"):
     return idx, wts
 
 
+_MOE_PP = os.environ.get("LLMSS_MOE_PP", "1") != "0"  # 0: grouped products on the tile kernel at every size (A/B runs)
+
+
 def moe_experts(h, idx, wts, gate, up, down, limit, alpha, shared=None, combine=True, act="glu_clamp",
                 weight_input=False, identity=False):
     """``identity``: indices from E on are identity experts. ``combine=False``: leave the weighting and summing to the next residual add (returns a :class:`MoEPending`).
@@ -1088,6 +1091,11 @@ def moe_experts(h, idx, wts, gate, up, down, limit, alpha, shared=None, combine=
     P = T * top
     # rows per tile of the grouped GEMMs: 128 where the experts get enough rows to fill big tiles (bf16 only)
     rows = 128 if h.dtype == torch.bfloat16 and P >= 128 * E else 64
+    # ungated experts with still more rows each: the dense GEMMs' 256x256 ping-pong kernel
+    pp = (gate is None and h.dtype == torch.bfloat16 and P >= 384 * E and min(F, N) >= 256 and F % 8 == 0 and K % 8 == 0
+          and h.stride(0) % 8 == 0 and not weight_input and h.data_ptr() % 16 == 0 and _MOE_PP)
+    if pp:
+        rows = 256
     maxt = -(-P // rows) + min(E, P)
     _check(maxt <= 65535, "too many (token, expert) pairs in one step")
     dev = h.device
@@ -1102,7 +1110,12 @@ def moe_experts(h, idx, wts, gate, up, down, limit, alpha, shared=None, combine=
     L = lib()
     st = _stream()
     L.moe_group(idx.data_ptr(), P, E, maxt, meta.data_ptr(), order.data_ptr(), place.data_ptr(), rows, st)
-    if h.dtype == torch.bfloat16:  # matrix cores (csrc/gemm_tile.hip)
+    if pp:
+        L.moe_pp(1, h.data_ptr(), h.stride(0), up.data_ptr(), meta.data_ptr(), order.data_ptr(), act_.data_ptr(), E, maxt,
+                 top, F, K, _ACT["gelu"], st)
+        L.moe_pp(2, act_.data_ptr(), F, down.data_ptr(), meta.data_ptr(), order.data_ptr(), y.data_ptr(), E, maxt, 1, N, F,
+                 0, st)
+    elif h.dtype == torch.bfloat16:  # matrix cores (csrc/gemm_tile.hip)
         L.moe_gate_up_tile(h.data_ptr(), h.stride(0), _ptr(gate), up.data_ptr(), meta.data_ptr(),
                            order.data_ptr(), act_.data_ptr(), E, maxt, top, F, K, float(limit), float(alpha), rows, pw,
                            silu, st)

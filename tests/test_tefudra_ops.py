@@ -91,7 +91,7 @@ def test_softmax_router_chooses_over_experts_and_identity_experts(device, dtype,
 
 
 @pytest.mark.parametrize("device,dtype", RUNS)
-@pytest.mark.parametrize("E,ident,top,W,F,T", [(4, 2, 2, 48, 24, 11), (3, 3, 3, 50, 17, 9), (2, 1, 1, 64, 160, 700),
+@pytest.mark.parametrize("E,ident,top,W,F,T", [(4, 2, 2, 48, 24, 11), (3, 3, 3, 50, 17, 9), (2, 1, 1, 64, 160, 700), (2, 1, 2, 264, 328, 1500),
                                                 (5, 0, 2, 40, 8, 6)])
 @pytest.mark.parametrize("shared", [False, True])
 def test_ungated_experts_and_identity_experts(device, dtype, E, ident, top, W, F, T, shared):
