@@ -433,7 +433,7 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
     m[n] = own_sink ? (X.sinks ? X.sinks[valid[n] ? hd[n] : h0] * kLog2e : 0.f) : -1.0e30f;
     lsum[n] = own_sink ? 1.f : 0.f;
   }
-  const float icap = cap > 0.f ? 1.0f / cap : 0.f;
+  const float capx = cap > 0.f ? 2.0f * kLog2e * scale / cap : 0.f, capy = -2.0f * cap * kLog2e;
   const float scale2 = scale * kLog2e;
   const int r_last = min(qlen, r0 + rows_per_wg) - 1;
   // the workgroup's keys, numbered u: the kept positions before jlo, then the positions from jlo on
@@ -527,9 +527,8 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(
         for (int i = 0; i < 4; ++i) {
           float v;
           if constexpr (CAP) {
-            const float x = s[n][kt][i] * scale;
-            const float e2 = __expf(2.0f * x * icap);  // tanh(x) = 1 - 2 / (exp(2x) + 1)
-            v = cap * (1.0f - 2.0f * __builtin_amdgcn_rcpf(e2 + 1.0f)) * kLog2e;
+            const float e2 = __builtin_amdgcn_exp2f(s[n][kt][i] * capx);  // tanh(x) = 1 - 2 / (exp(2x) + 1)
+            v = fmaf(capy, __builtin_amdgcn_rcpf(e2 + 1.0f), -0.5f * capy);
           } else {
             v = s[n][kt][i] * scale2;
           }

@@ -110,6 +110,26 @@ __device__ __forceinline__ void head_vec(const HeadPrepArgs& A, const float* x0,
   }
 }
 
+// V numbers of a tail row (fp32; whole 16-byte pieces where V is one)
+template <int V>
+__device__ __forceinline__ void hp_ldf(const float* p, float* v) {
+  if constexpr (V >= 4) {
+#pragma unroll
+    for (int i = 0; i < V; i += 4) *reinterpret_cast<f32x4*>(v + i) = *reinterpret_cast<const f32x4*>(p + i);
+  } else {
+    v[0] = p[0];
+  }
+}
+template <int V>
+__device__ __forceinline__ void hp_stf(float* p, const float* v) {
+  if constexpr (V >= 4) {
+#pragma unroll
+    for (int i = 0; i < V; i += 4) *reinterpret_cast<f32x4*>(p + i) = *reinterpret_cast<const f32x4*>(v + i);
+  } else {
+    p[0] = v[0];
+  }
+}
+
 // V: numbers per thread and access while the row is formed (8 bf16 or 4 fp32 numbers = 16 bytes, or 1)
 template <typename T, int V>
 __global__ __launch_bounds__(512) void head_prep_kernel(HeadPrepArgs A, int vec) {
@@ -138,8 +158,7 @@ __global__ __launch_bounds__(512) void head_prep_kernel(HeadPrepArgs A, int vec)
           if (r.j - d >= 0) {
             hp_ld<T, V>(row - (int64_t)d * A.ldp + A.off_q + c, x);
           } else {
-#pragma unroll
-            for (int i = 0; i < V; ++i) x[i] = ss >= 0 ? st[(int64_t)(r.j - d + R) * C + c + i] : 0.f;
+            hp_ldf<V>(st + (int64_t)(r.j - d + R) * C + c, x);  // (a row without a slot reads slot 0 and is not used)
           }
 #pragma unroll
           for (int i = 0; i < V; ++i) acc[i] = fmaf(w[i], x[i], acc[i]);
@@ -148,13 +167,16 @@ __global__ __launch_bounds__(512) void head_prep_kernel(HeadPrepArgs A, int vec)
           for (int i = 0; i < R; ++i) {
             float x[V];
             if (i + 1 < R) {
+              if (r.pos > 0) {
+                hp_ldf<V>(st + (int64_t)(i + 1) * C + c, x);
+              } else {
 #pragma unroll
-              for (int e = 0; e < V; ++e) x[e] = r.pos > 0 ? st[(int64_t)(i + 1) * C + c + e] : 0.f;
+                for (int e = 0; e < V; ++e) x[e] = 0.f;
+              }
             } else {
               hp_ld<T, V>(row + A.off_q + c, x);
             }
-#pragma unroll
-            for (int e = 0; e < V; ++e) st[(int64_t)i * C + c + e] = x[e];
+            hp_stf<V>(st + (int64_t)i * C + c, x);
           }
         }
       }
@@ -242,7 +264,7 @@ void launch_head_prep(const void* proj, int64_t ldp, int off_q, int off_k, int o
                  (const float*)vcs, q, q_bf, kc, vc, (const int64_t*)slots, H, G, dim, vdim};
   const int vn = dt == 0 ? 8 : 4;
   const auto al16 = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
-  const bool vec = al16(proj) && al16(conv) && ldp % vn == 0 && off_q % vn == 0 && off_k % vn == 0 && off_v % vn == 0 &&
+  const bool vec = al16(proj) && al16(conv) && al16(tail) && ldp % vn == 0 && off_q % vn == 0 && off_k % vn == 0 && off_v % vn == 0 &&
                    nq % vn == 0 && nk % vn == 0 && nv % vn == 0;
   // whole 16-byte pieces per head: sizes 8 to 512 that are powers of two, turned parts of whole pieces
   const auto pow2 = [](int n) { return n >= 8 && n <= 512 && (n & (n - 1)) == 0; };

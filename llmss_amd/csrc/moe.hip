@@ -207,8 +207,18 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int* __restrict__
   int* tile_r = tile_e + maxt;
   for (int e = threadIdx.x; e < E; e += blockDim.x) cnt[e] = 0;
   __syncthreads();
-  for (int p = threadIdx.x; p < P; p += blockDim.x)
-    if (idx[p] < E) atomicAdd(&cnt[idx[p]], 1);
+  constexpr int U = 8;  // pairs per thread whose loads and atomics are in flight together
+  for (int p0 = threadIdx.x; p0 < P; p0 += blockDim.x * U) {
+    int e[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int p = p0 + u * blockDim.x;
+      e[u] = p < P ? idx[p] : E;
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (e[u] < E) atomicAdd(&cnt[e[u]], 1);
+  }
   __syncthreads();
   if (threadIdx.x == 0) {
     int o = 0, nt = 0;
@@ -230,14 +240,22 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int* __restrict__
   __syncthreads();
   // rows within an expert take whatever order the atomics give: every pair's row is computed on its own, so the
   // values do not depend on where the row lands
-  for (int p = threadIdx.x; p < P; p += blockDim.x) {
-    if (idx[p] >= E) {  // an identity expert: no row of its own
-      place[p] = -1;
-      continue;
+  for (int p0 = threadIdx.x; p0 < P; p0 += blockDim.x * U) {
+    int e[U], o[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int p = p0 + u * blockDim.x;
+      e[u] = p < P ? idx[p] : E;
     }
-    const int o = atomicAdd(&cur[idx[p]], 1);
-    order[o] = p;
-    place[p] = o;
+#pragma unroll
+    for (int u = 0; u < U; ++u) o[u] = e[u] < E ? atomicAdd(&cur[e[u]], 1) : -1;  // (-1: an identity expert, no row of its own)
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int p = p0 + u * blockDim.x;
+      if (p >= P) continue;
+      if (o[u] >= 0) order[o[u]] = p;
+      place[p] = o[u];
+    }
   }
 }
 

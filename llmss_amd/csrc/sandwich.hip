@@ -107,7 +107,7 @@ __device__ __forceinline__ void norm_out(float* buf, float ss, const SandwichArg
 }
 
 template <typename T, int V>
-__global__ __launch_bounds__(256) void sandwich_add_norm_kernel(SandwichArgs p) {
+__global__ __launch_bounds__(512) void sandwich_add_norm_kernel(SandwichArgs p) {
   extern __shared__ __attribute__((aligned(16))) float buf[];
   __shared__ float red[32];
   const int t = blockIdx.x, W = p.W;
@@ -235,9 +235,10 @@ void launch_sandwich_add_norm(void* x, const void* y, int64_t ldy, const void* e
                    alv(y, ldy) && alv(shared_, lds_) && alv(r, ldr) && alv(h, ldh) && alv(ident, ldi) && alv(y2, ldy2) &&
                    al16(wl) && al16(wr);
   const size_t lds = ((size_t)W + (groups > 1 ? groups : 0)) * 4;
+  const int th = T_ <= 512 && W > 1024 ? 512 : 256;  // few rows: more waves to a row
   DISPATCH_T(dt, T, {
-    if (vec) sandwich_add_norm_kernel<T, 4><<<T_, 256, lds, st>>>(p);
-    else sandwich_add_norm_kernel<T, 1><<<T_, 256, lds, st>>>(p);
+    if (vec) sandwich_add_norm_kernel<T, 4><<<T_, th, lds, st>>>(p);
+    else sandwich_add_norm_kernel<T, 1><<<T_, th, lds, st>>>(p);
   });
   HIP_CHECK_LAUNCH();
 }
