@@ -392,14 +392,14 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
     El<T>::st(dst + i, row[i] * inv * El<T>::ld(wr + i) * gate_of(i));
 }
 
-// The same with a wave per group and 16-byte accesses of the fp32 rows, for groups of up to 1024 columns (whole fours): the
+// The same, the gate after the norm, with a wave per group and 16-byte accesses, for groups of up to 1024 columns (whole fours): the
 // group's numbers stay in registers between the sum of squares and the result.
 template <typename T>
 __global__ __launch_bounds__(256) void gated_group_norm_vec_kernel(const float* __restrict__ o, int64_t ldo,
                                                                    const T* __restrict__ gate, int64_t ldg,
                                                                    const T* __restrict__ w, float eps, int act, float c,
                                                                    T* __restrict__ out, int64_t ldout, int n, int wfull,
-                                                                   int first, const float* __restrict__ den,
+                                                                   const float* __restrict__ den,
                                                                    const f32x4* __restrict__ gates, float qs, int groups) {
   const int t = blockIdx.x, g = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (g >= groups) return;
@@ -424,8 +424,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_vec_kernel(const float* 
       const float sg = 1.0f / (1.0f + expf(-ga[j][i]));
       ga[j][i] = act ? ga[j][i] * sg : sg;
       u[j][i] *= pre;
-      const float x = first ? u[j][i] * ga[j][i] : u[j][i];
-      ss = fmaf(x, x, ss);
+      ss = fmaf(u[j][i], u[j][i], ss);
     }
   }
   const float inv = c / sqrtf(warp_sum(ss) / (float)n + eps);
@@ -449,11 +448,11 @@ void launch_gated_group_norm(const void* o, int64_t ldo, const void* gate, int64
   if (groups > 65535) throw std::runtime_error("gated_group_norm: too many groups");
   const int es = dt == 0 ? 2 : 4;
   const auto al = [](const void* p, int64_t b) { return ((uintptr_t)p % b) == 0; };
-  if (n % 4 == 0 && n <= 1024 && n >= 64 && ldo % 4 == 0 && ldg % 4 == 0 && ldout % 4 == 0 && al(o, 16) && al(gate, 4 * es) &&
+  if (!first && n % 4 == 0 && n <= 1024 && n >= 64 && ldo % 4 == 0 && ldg % 4 == 0 && ldout % 4 == 0 && al(o, 16) && al(gate, 4 * es) &&
       al(w, 4 * es) && al(out, 4 * es)) {
     dim3 gv(T_, (groups + 3) / 4);
     DISPATCH_T(dt, T, (gated_group_norm_vec_kernel<T><<<gv, 256, 0, st>>>(
-        (const float*)o, ldo, (const T*)gate, ldg, (const T*)w, eps, act, c, (T*)out, ldout, n, wfull, first,
+        (const float*)o, ldo, (const T*)gate, ldg, (const T*)w, eps, act, c, (T*)out, ldout, n, wfull,
         (const float*)den, (const f32x4*)gates, qs, groups)));
     HIP_CHECK_LAUNCH();
     return;
