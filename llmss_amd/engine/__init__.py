@@ -10,8 +10,8 @@ from ..models.config import ModelConfig, get_preset
 from ..models.decoder import DecoderLM
 from ..models.layered import LayeredLM, create_model
 from ..models.weights import (load_babotar_weights, load_fizelix_weights, load_hf_weights, load_lamisun_weights,
-                              load_shard, load_tefudra_weights, load_timisun_weights, random_babotar_weights,
-                              random_fizelix_weights, random_lamisun_weights, random_tefudra_weights,
+                              load_nolavik_weights, load_shard, load_tefudra_weights, load_timisun_weights, random_babotar_weights,
+                              random_fizelix_weights, random_lamisun_weights, random_nolavik_weights, random_tefudra_weights,
                               random_timisun_weights, random_weights, save_shard, shard_cache_path)
 from ..parallel.dist import TPGroup
 from ..utils.checkpoint import CheckpointReader, weight_files
@@ -53,7 +53,8 @@ def build_model(model: str, tp: Optional[TPGroup] = None, dtype: str = "bf16", d
         rand, load = {"babotar": (random_babotar_weights, load_babotar_weights),
                       "lamisun": (random_lamisun_weights, load_lamisun_weights),
                       "fizelix": (random_fizelix_weights, load_fizelix_weights),
-                      "tefudra": (random_tefudra_weights, load_tefudra_weights)}.get(
+                      "tefudra": (random_tefudra_weights, load_tefudra_weights),
+                      "nolavik": (random_nolavik_weights, load_nolavik_weights)}.get(
             cfg.model_type, (random_timisun_weights, load_timisun_weights))
         if random_init:
             w = rand(cfg, device=device, dtype=tdtype, seed=seed)

@@ -42,6 +42,12 @@ Families (``MODEL_REGISTRY`` keys, reference ``custom_modeling/__init__.py:4-7``
                     memory with exponential gates, ``mlstm``, each normed over the row and averaged); feed-forward dense
                     squared-relu or mixture of ungated GELU experts with softmax scores and identity experts; layers may
                     share another layer's weights; tied head.
+* ``nolavik``     - per-layer description: blocks normed before and after each sublayer, a stretch of layers repeated with
+                    the same weights (a learned vector added before every pass); mixers ``delta`` (gated delta rule),
+                    ``parallel`` (attention with unit queries and keys and a constant sink beside a selective scan, summed
+                    with two scales) and ``latent_attention`` (queries through a latent of their own, rotated key part
+                    shared by the heads); mixture of experts weighted by a softmax over the chosen logits, the shared
+                    expert behind a gate; untied head.
 """
 from __future__ import annotations
 
@@ -73,6 +79,7 @@ class MixerSpec:
     rot_dim: int = 0
     rot: Optional["RotarySpec"] = None
     gate: bool = False  # the concatenated heads are multiplied by sigmoid(W_g h) before the output projection
+    q_rank: int = 0  # > 0: the queries come from a latent of their own, W_uq rms_norm(W_dq h)
 
 
 @dataclass
@@ -94,7 +101,9 @@ class MoESpec:
     act: str = "glu_clamp"
     normalize: bool = True  # the chosen scores are divided by their sum
     weight_input: bool = False  # the score multiplies the expert's input (sum_e expert_e(w_e h)), not its output
-    score: str = "sigmoid"  # or "softmax" over all router outputs
+    score: str = "sigmoid"  # or "softmax" over all router outputs; "chosen": the largest logits, a softmax over them alone
+    bias: bool = False  # the router's logits have a bias
+    shared_gate: bool = False  # the shared expert's output is multiplied by sigmoid(w_sg . h), one number per token
     identity: int = 0  # router outputs after the experts': identity experts, whose output is the layer's input
 
 
@@ -102,11 +111,32 @@ class MoESpec:
 class RotarySpec:
     """Rotary positions on the first ``dims`` dimensions of a head, dimension i paired with i + dims / 2, frequency
     base^(-2 i / dims); ``scaling`` = (factor, original length, fast turns, slow turns) blends the frequencies
-    between the two turn counts towards f / factor and scales cos and sin by 0.1 ln(factor) + 1."""
+    between the two turn counts towards f / factor and scales cos and sin by 0.1 ln(factor) + 1; ``llama3`` = (factor,
+    low, high, original) blends the frequencies whose turns over the original length lie between low and high (below:
+    f / factor, above: f), cos and sin as they are."""
     dims: int
     base: float
     scaling: Optional[tuple] = None
     pairs: str = "half"  # "half": i with i + dims / 2; "neighbours": 2i with 2i + 1
+    llama3: Optional[tuple] = None
+
+    def steps(self) -> List[float]:
+        """Angular step per position of every pair (without ``scaling``, whose amplitude belongs to a table)."""
+        out = []
+        for i in range(self.dims // 2):
+            f = self.base ** (-2.0 * i / self.dims)
+            if self.llama3 is not None:
+                factor, low, high, original = self.llama3
+                turns = original * f / (2.0 * math.pi)
+                mix = min(1.0, max(0.0, (turns - low) / (high - low))) if high > low else float(turns >= low)
+                f = f * (mix + (1.0 - mix) / factor)
+            out.append(f)
+        return out
+
+    @property
+    def key(self) -> tuple:
+        """Layers with equal keys share a step's angles."""
+        return (self.dims, self.base) if self.llama3 is None else (self.dims, self.base) + self.llama3
 
 
 @dataclass
@@ -173,7 +203,8 @@ class WindowAttnSpec:
     the values are the keys as projected; ``sink``: exp of a learned number per head in the softmax denominator; ``bias``:
     the projections (output too) have biases; ``conv`` > 0: q, k and v pass a causal convolution of that many taps first;
     ``v_norm``: values divided per head by their root mean square; ``rot_values``: values turned by their position over
-    all vdim numbers (the keys' base) and every head's result turned back by its own."""
+    all vdim numbers (the keys' base) and every head's result turned back by its own; ``unit_qk``: queries and keys divided
+    per head by their root mean square, without a weight; ``unit_sink``: a constant one in the softmax denominator."""
     heads: int
     kv_heads: int
     dim: int
@@ -190,6 +221,8 @@ class WindowAttnSpec:
     conv: int = 0
     v_norm: bool = False
     rot_values: bool = False
+    unit_qk: bool = False
+    unit_sink: bool = False
     kind: str = "window_attention"
 
     @property
@@ -210,9 +243,11 @@ class MLSTMSpec:
 
 @dataclass
 class PairMixerSpec:
-    """Two mixers reading the same input; the result is half the sum of the two, each RMS-normed over the row first."""
+    """Two mixers reading the same input; the result is half the sum of the two, each RMS-normed over the row first, or,
+    with ``scales`` (left, right), the sum of the two times their scales."""
     left: Any
     right: Any
+    scales: Optional[tuple] = None
     kind: str = "pair"
 
     @property
@@ -241,6 +276,18 @@ class SSDSpec:
     @property
     def conv_channels(self) -> int:
         return self.inner + 2 * self.groups * self.state
+
+
+@dataclass
+class MambaSpec:
+    """Selective scan: ``inner`` channels with a state of ``state`` numbers each, a step size per channel and token through
+    ``dt_rank`` numbers, input and output vectors (B, C) shared by the channels; x through a causal convolution of ``conv``
+    taps with bias and SiLU, the result gated by silu(z)."""
+    inner: int
+    state: int
+    dt_rank: int
+    conv: int
+    kind: str = "mamba"
 
 
 @dataclass
@@ -350,6 +397,7 @@ class ModelConfig:
     sandwich: bool = False
     token_side_dim: int = 0  # > 0: after the feed-forward a layer adds a normed projection of its slice of a second token table
     loop: Optional[tuple] = None  # (start, stop, times): layers start .. stop - 1 run ``times`` times in a row
+    loop_step: bool = False  # a learned vector per pass is added before every pass, not the embedding before all but the first
     logit_scale: float = 1.0
     norm_groups: int = 1  # sandwich blocks: every norm is taken in that many equal consecutive parts of the row
     weights_of: Optional[List[int]] = None  # per layer: the layer whose weights it uses (itself: its own)
@@ -362,6 +410,14 @@ class ModelConfig:
             return list(range(n))
         a, b, times = self.loop
         return list(range(a)) + list(range(a, b)) * times + list(range(b, n))
+
+    def pass_before(self, run: int) -> Optional[int]:
+        """The pass of the looped stretch that layer run ``run`` opens (None: it opens none)."""
+        if not self.loop or (self.loop[2] <= 1 and not self.loop_step):
+            return None
+        a, b, times = self.loop
+        n = run - a
+        return n // (b - a) if 0 <= n < (b - a) * times and n % (b - a) == 0 else None
 
     # ---------------------------------------------------------------- derived
     @property
@@ -382,11 +438,11 @@ class ModelConfig:
 
     def num_params(self) -> int:
         h, f, v = self.hidden_size, self.intermediate_size, self.vocab_size
-        if self.layer_specs and self.model_type in ("babotar", "lamisun", "fizelix", "tefudra"):
-            from .weights import babotar_shapes, fizelix_shapes, lamisun_shapes, tefudra_shapes
+        if self.layer_specs and self.model_type in ("babotar", "lamisun", "fizelix", "tefudra", "nolavik"):
+            from .weights import babotar_shapes, fizelix_shapes, lamisun_shapes, nolavik_shapes, tefudra_shapes
 
             shapes = {"babotar": babotar_shapes, "lamisun": lamisun_shapes, "fizelix": fizelix_shapes,
-                      "tefudra": tefudra_shapes}[self.model_type](self)
+                      "tefudra": tefudra_shapes, "nolavik": nolavik_shapes}[self.model_type](self)
             return sum(math.prod(shp) for shp in shapes.values())
         if self.layer_specs:
             n = v * h + h
@@ -422,6 +478,8 @@ class ModelConfig:
             return _fizelix(cls, d)
         if mt is None and d.get("architecture") == "Tefudra":
             return _tefudra(cls, d)
+        if mt is None and d.get("architecture") == "Nolavik":
+            return _nolavik(cls, d)
         common = dict(
             bos_token_id=d.get("bos_token_id"),
             eos_token_id=_first(d.get("eos_token_id")),
@@ -793,6 +851,78 @@ def _tefudra(cls, d: Dict[str, Any]) -> "ModelConfig":
     )
 
 
+def _nolavik(cls, d: Dict[str, Any]) -> "ModelConfig":
+    """``{"architecture": "Nolavik", "vocab", "width", "norm": {"eps"}, "loop": {"start", "stop", "times"}, "layers":
+    [{"type": "delta" | "parallel" | "latent_attention", "mixer": {...}, "mlp": {"kind": "moe", "router": {"experts",
+    "top"}, "expert": {"ff"}, "shared": {"ff"}} | null}]}``. A delta mixer gives heads, kv_heads, dim, vdim, conv; a
+    parallel one ``left`` (heads, kv_heads, dim, vdim, scale, rot: {base, dims, scaling: {factor, low, high, original}}),
+    ``right`` (inner, state, dt_rank, conv), left_scale, right_scale; a latent one heads, dim, rot_dim, vdim, q_rank,
+    kv_rank, scale, rot: {base, dims}. Keys a config leaves out switch their mechanism off (no loop, no rotation, no
+    frequency scaling, no shared expert)."""
+    specs: List[LayerSpec] = []
+    for i, L in enumerate(d["layers"]):
+        m, typ = L["mixer"], L.get("type")
+        if typ == "delta":
+            mixer = DeltaSpec(int(m["heads"]), int(m.get("kv_heads") or m["heads"]), int(m["dim"]), int(m["vdim"]),
+                              int(m.get("conv") or 1))
+            if mixer.heads % mixer.kv_heads:
+                raise ValueError(f"Nolavik layer {i}: {mixer.heads} heads on {mixer.kv_heads} key heads")
+        elif typ == "parallel":
+            a, r = m["left"], m["right"]
+            rot = None
+            if a.get("rot") and int(a["rot"].get("dims") or 0):
+                sc = a["rot"].get("scaling")
+                rot = RotarySpec(int(a["rot"]["dims"]), float(a["rot"]["base"]),
+                                 llama3=None if not sc else tuple(float(sc[n]) for n in ("factor", "low", "high", "original")))
+                if rot.dims % 2 or rot.dims > int(a["dim"]):
+                    raise ValueError(f"Nolavik layer {i}: {rot.dims} rotary dimensions on heads of {a['dim']}")
+            left = WindowAttnSpec(int(a["heads"]), int(a.get("kv_heads") or a["heads"]), int(a["dim"]),
+                                  int(a.get("vdim") or a["dim"]), float(a["scale"]), rot=rot, unit_qk=True, unit_sink=True)
+            if left.heads % left.kv_heads:
+                raise ValueError(f"Nolavik layer {i}: {left.heads} heads on {left.kv_heads} key heads")
+            right = MambaSpec(int(r["inner"]), int(r["state"]), int(r["dt_rank"]), int(r.get("conv") or 1))
+            mixer = PairMixerSpec(left, right, (float(m.get("left_scale", 1.0)), float(m.get("right_scale", 1.0))))
+        elif typ == "latent_attention":
+            rd, rot = int(m.get("rot_dim") or 0), None
+            if rd:
+                rot = RotarySpec(int(m["rot"].get("dims") or rd), float(m["rot"]["base"]))
+                if rot.dims > rd or rot.dims % 2:
+                    raise ValueError(f"Nolavik layer {i}: {rot.dims} rotary dimensions on a rotated part of {rd}")
+            mixer = MixerSpec("latent_attention", int(m["heads"]), int(m["dim"]), int(m["vdim"]), int(m["kv_rank"]),
+                              float(m["scale"]), rot_dim=rd, rot=rot, q_rank=int(m["q_rank"]))
+        else:
+            raise ValueError(f"Nolavik layer {i}: unsupported mixer type {typ!r}")
+        f, mlp = L.get("mlp"), None
+        if f is not None:
+            if f.get("kind", "moe") != "moe":
+                raise ValueError(f"Nolavik layer {i}: unsupported feed-forward kind {f.get('kind')!r}")
+            sh = f.get("shared")
+            mlp = MoESpec(int(f["router"]["experts"]), int(f["router"]["top"]), ExpertSpec(int(f["expert"]["ff"])),
+                          None if not sh else ExpertSpec(int(sh["ff"])), act="silu", score="chosen", bias=True,
+                          shared_gate=bool(sh))
+            if not 1 <= mlp.top <= mlp.experts:
+                raise ValueError(f"Nolavik layer {i}: top {mlp.top} of {mlp.experts} experts")
+        specs.append(LayerSpec(mixer, mlp))
+    if not specs:
+        raise ValueError("Nolavik: no layers")
+    loop, lp = None, d.get("loop")
+    if lp:
+        loop = (int(lp["start"]), int(lp["stop"]), int(lp["times"]))
+        if not 0 <= loop[0] < loop[1] <= len(specs) or loop[2] < 1:
+            raise ValueError(f"Nolavik: loop over layers {loop[0]} .. {loop[1] - 1} of {len(specs)}, {loop[2]} times")
+    return cls(
+        model_type="nolavik", vocab_size=int(d["vocab"]), hidden_size=int(d["width"]), num_layers=len(specs),
+        num_heads=max(s.mixer.heads for s in specs), num_kv_heads=1, head_dim=1,
+        intermediate_size=max([s.mlp.expert.ff for s in specs if s.mlp] or [0]),
+        max_position_embeddings=1 << 20,  # the design has no positional limit of its own
+        norm="rmsnorm", norm_eps=float(d["norm"]["eps"]), activation="silu_glu", position="none", rotary_dim=0,
+        parallel_block=False, tie_word_embeddings=False, layer_specs=specs, residual_fp32=True, sandwich=True, loop=loop,
+        loop_step=loop is not None,
+        bos_token_id=d.get("bos_token_id"), eos_token_id=_first(d.get("eos_token_id")),
+        pad_token_id=d.get("pad_token_id"),
+    )
+
+
 def _first(x):
     if isinstance(x, (list, tuple)):
         return x[0] if x else None
@@ -934,6 +1064,25 @@ _PRESETS: Dict[str, Dict[str, Any]] = {
                                              mask=dict(size=7, keep_first=2), rot=dict(base=500.0, dims=8)),
                                   mlp=dict(kind="moe", router=dict(experts=5, top=2, identity=2), expert=dict(ff=20),
                                            shared=dict(ff=12))),
+                         ]),
+    # sandwich-normed per-layer design with a looped stretch: gated delta rule, unit-query attention with a constant sink
+    # beside a selective scan, latent attention with a query latent, experts with a gated shared expert
+    "tiny-nolavik": dict(architecture="Nolavik", vocab=211, width=48, norm=dict(eps=1e-5), loop=dict(start=1, stop=3, times=2),
+                         layers=[
+                             dict(type="latent_attention",
+                                  mixer=dict(heads=3, dim=16, rot_dim=8, vdim=12, q_rank=20, kv_rank=24, scale=0.2,
+                                             rot=dict(base=500.0, dims=8)),
+                                  mlp=None),
+                             dict(type="delta", mixer=dict(heads=4, kv_heads=2, dim=8, vdim=12, conv=4),
+                                  mlp=dict(kind="moe", router=dict(experts=5, top=2), expert=dict(ff=20),
+                                           shared=dict(ff=12))),
+                             dict(type="parallel",
+                                  mixer=dict(left=dict(heads=4, kv_heads=2, dim=8, vdim=12, scale=2.0,
+                                                       rot=dict(base=1000.0, dims=6,
+                                                                scaling=dict(factor=4.0, low=1.0, high=3.0, original=64))),
+                                             right=dict(inner=40, state=6, dt_rank=5, conv=4), left_scale=0.7,
+                                             right_scale=1.1),
+                                  mlp=dict(kind="moe", router=dict(experts=4, top=1), expert=dict(ff=16))),
                          ]),
     # TP up to 8 (16 q / kv heads: 2 per rank at TP=8, as Llama-2-7B's 32 give 4)
     "tiny-llama16h": dict(model_type="llama", hidden_size=256, num_hidden_layers=2, num_attention_heads=16,

@@ -1,7 +1,7 @@
 """Decoder whose layers are described one by one (``ModelConfig.layer_specs``) over an fp32 residual stream.
 
 The uniform families run through :class:`~llmss_amd.models.decoder.DecoderLM`; a per-layer design (Timisun, Babotar,
-Lamisun, Fizelix, Tefudra) runs through :class:`LayeredLM`, which offers the engine the same surface (``hidden_states`` / ``logits`` over a
+Lamisun, Fizelix, Tefudra, Nolavik) runs through :class:`LayeredLM`, which offers the engine the same surface (``hidden_states`` / ``logits`` over a
 :class:`StepInput`, ``allocate_kv_cache``, ``kv_bytes_per_block``, ``plan``) and so shares its scheduler, paged
 cache pool, decode graphs and sampler. A layer is either a parallel block (``cfg.parallel_block``)
 
@@ -26,7 +26,8 @@ the norms optionally taken in ``cfg.norm_groups`` equal parts of the row; layers
 
 optionally followed by a token input (x <- x + rms_norm(W_p (gelu(W_s x) * e)) * w, e the layer's slice of a second
 token table); a stretch of such layers may run several times in a row with the same weights (``cfg.loop``), each pass
-with cache and state of its own, the embedding added again before every pass but the first. The mixer and the feed-forward are looked up by kind
+with cache and state of its own, the embedding added again before every pass but the first, or a learned vector of the
+pass before each (``cfg.loop_step``). The mixer and the feed-forward are looked up by kind
 (``MIXERS`` / ``FFNS``), so another design can combine the same mechanisms with other constants or add its own
 beside them. Besides pages of the shared pool a mixer may own per-sequence state (a matrix state per head, the last
 inputs of a convolution): ``LayerCache.state`` tensors indexed by the scheduler's state slot of each sequence
@@ -44,7 +45,8 @@ over the causal (optionally windowed) keys, out = W_o concat_h(W_uv_h sum_j p_j 
 projects no latent of its own and reads the named layer's cache with its own W_uk / W_uv. With ``rot_dim`` > 0 every
 query head and the cached row carry a rotated part after the latent one (the key's is shared by all heads): the score
 is the dot product over the whole row [c | k_rot], the weighted sum reads c alone. ``gate``: the heads' outputs are
-multiplied by sigmoid(W_g h) before the output projection.
+multiplied by sigmoid(W_g h) before the output projection. ``q_rank``: the queries come from a latent of their own,
+W_uq rms_norm(W_dq h) (rms_cols), whose down-projection shares the input GEMM.
 
 Mixer ``attention`` (ops: linear_f, qk_norm_cache, sink_attn without a sink, diff_combine): differential attention -
 two softmax maps per head over the same values, o = a1 - lambda a2, RMS-normed per head - with RMS-normed queries
@@ -62,12 +64,15 @@ Mixer ``window_attention`` (ops: linear_f, rope_angles, head_prep_cache, window_
 window that keeps the sequence's first positions, with a learned sink per head, soft cap, short convolutions on q / k / v,
 query / key / value norms, rotated keys and values - each by the spec. Mixer ``mlstm`` (linear_f, mlstm_mix): matrix memory
 with exponential gates and a running maximum. Mixer ``pair``: two mixers on the same input, one input GEMM for both; their
-results go unjoined (``ops.PairPending``) into the block's closing op, which norms and averages them.
+results go unjoined (``ops.PairPending``) into the block's closing op, which norms and averages them or sums them with two
+scales. Mixer ``gated_delta`` (causal_conv, delta_recurrence, gated_group_norm): the gated delta rule on its own. Mixer
+``mamba`` (causal_conv with bias, linear_f, selective_scan), the right half of a pair: a state per channel with a step size,
+input and output vectors of its own per token.
 
 Feed-forward ``moe`` (ops: moe_router -> fp32 router logits and routing, moe_experts, glu_clamp): sigmoid scores, the
 choice made on score + correction, weights = chosen scores normalised; experts and the shared expert use the clamped
 gated activation g * sigmoid(1.702 g) * (u + 1); or, by the spec, unnormalised scores that multiply the expert's
-INPUT and plain silu(g) * u.
+INPUT and plain silu(g) * u, or weights from a softmax over the chosen logits and a gate on the shared expert.
 """
 from __future__ import annotations
 
@@ -97,12 +102,16 @@ class LatentAttention:
         dt = model.dtype
         H, dim, R, rot = spec.heads, spec.dim, spec.kv_rank, spec.rot_dim
         qc = ops.linear_f(h, W.qc, dt)  # [T, H * (dim + rot) (+ R + rot) (+ H * vdim)]: queries, raw latent, gate
+        src, off = qc, H * (dim + rot)
+        if spec.q_rank:  # [T, q_rank + R + rot]: the queries' latent, raw latent
+            off = spec.q_rank
+            qc = ops.linear_f(ops.rms_cols(src, 0, off, W.q_norm, model.cfg.norm_eps, dt), W.uq, dt)
         cache = caches[i if spec.kv_from is None else spec.kv_from][0]
         qa = ops.head_absorb(qc, W.uk_t, ops.latent_qa_dtype(cache), extra=rot)
         if W.own_kv:
             cs = model.angles(inp, W.rot_key, W.freqs) if rot else None
-            ops.latent_norm_cache(qc, H * (dim + rot), R, W.kv_norm, model.cfg.norm_eps, cache, inp.slots, rot, cs,
-                                  qa if rot else None, 0, dim)
+            ops.latent_norm_cache(src, off, R, W.kv_norm, model.cfg.norm_eps, cache, inp.slots, rot, cs,
+                                  qa if rot else None, 0, dim, q_src=qc)
         nd = inp.num_decode if inp.kind == "extend" else 0
         if nd and nd < qa.shape[0]:
             # mixed step: the single-token rows take the decode form of the kernel (their keys split over
@@ -160,7 +169,9 @@ class MoEFeedForward:
     @staticmethod
     def forward(model: "LayeredLM", W, spec, h):
         dt = model.dtype
-        idx, wts = ops.moe_router(h, W.router, W.correction, spec.top, spec.normalize, spec.score)
+        route = ops.moe_router(h, W.router, W.correction, spec.top, spec.normalize, spec.score, bias=W.bias,
+                               gate=spec.shared_gate)
+        idx, wts = route[:2]
         sh = None
         if spec.act == "gelu":  # experts without a gate
             if W.shared_gu is not None:
@@ -176,7 +187,49 @@ class MoEFeedForward:
                 sh = ops.linear_f(a, W.shared_down, dt)
         # combine=False: on the GPU the weighted sum over the chosen experts happens inside the next residual add
         return ops.moe_experts(h, idx, wts, W.gate, W.up, W.down, spec.expert.limit, GLU_ALPHA, shared=sh,
-                               combine=False, act=spec.act, weight_input=spec.weight_input)
+                               combine=False, act=spec.act, weight_input=spec.weight_input,
+                               shared_w=route[2] if spec.shared_gate else None)
+
+
+class DeltaMixer:
+    """Mixer ``gated_delta``: short convolution + SiLU on q | k | v, the gated delta rule over a matrix state per head, a
+    gated RMS norm per head."""
+
+    @staticmethod
+    def cache_row(spec) -> Optional[int]:
+        return None
+
+    @staticmethod
+    def allocate(model: "LayeredLM", spec, num_blocks: int, block_size: int, num_slots: int):
+        dev = model.device
+        return (None, None,
+                {"S": torch.zeros(num_slots, spec.heads, spec.dim, spec.vdim, dtype=torch.float32, device=dev),
+                 "tail": torch.zeros(num_slots, max(spec.conv - 1, 0), 2 * spec.kv_heads * spec.dim + spec.heads * spec.vdim,
+                                     dtype=torch.float32, device=dev)})
+
+    @staticmethod
+    def state_bytes(spec) -> int:
+        return 4 * (spec.heads * spec.dim * spec.vdim
+                    + max(spec.conv - 1, 0) * (2 * spec.kv_heads * spec.dim + spec.heads * spec.vdim))
+
+    @staticmethod
+    def mix(model: "LayeredLM", W, spec, proj, cols, inp: StepInput, cu, st, scale: float, out):
+        """The heads' results, gated and times ``scale``, into ``out`` [T, heads * vdim], from the projection rows (q | k | v
+        contiguous from cols["q"] on; g, a, b)."""
+        H, nqk, nv = spec.heads, spec.kv_heads * spec.dim, spec.heads * spec.vdim
+        qkv = ops.causal_conv(proj[:, cols["q"]:cols["q"] + 2 * nqk + nv], W.conv, st["tail"], cu, inp.ctx_lens,
+                              inp.state_slots, False, True, torch.float32)
+        o = ops.delta_recurrence(qkv[:, :nqk], qkv[:, nqk:2 * nqk], qkv[:, 2 * nqk:], proj[:, cols["a"]:cols["a"] + H],
+                                 proj[:, cols["b"]:cols["b"] + H], W.A_log, W.dt_bias, st["S"], cu, inp.ctx_lens,
+                                 inp.state_slots, H, spec.kv_heads, spec.dim, spec.vdim)
+        return ops.gated_group_norm(o, proj[:, cols["g"]:cols["g"] + nv], W.norm, model.cfg.norm_eps, "silu", scale, out=out)
+
+    @staticmethod
+    def forward(model: "LayeredLM", i: int, W, spec, h, inp: StepInput, cu, caches):
+        dt = model.dtype
+        y = torch.empty(h.shape[0], spec.heads * spec.vdim, dtype=dt, device=h.device)
+        DeltaMixer.mix(model, W, spec, ops.linear_f(h, W.proj, dt), W.cols, inp, cu, caches[i][2], 1.0, y)
+        return ops.linear_f(y, W.o, dt)
 
 
 class ParallelMixer:
@@ -191,20 +244,17 @@ class ParallelMixer:
     def allocate(model: "LayeredLM", spec, num_blocks: int, block_size: int, num_slots: int):
         a, r = spec.left, spec.right
         dt, dev = model.dtype, model.device
-        C = 2 * r.kv_heads * r.dim + r.heads * r.vdim
         return (torch.zeros(num_blocks, block_size, a.kv_heads * a.dim, dtype=dt, device=dev),
                 torch.zeros(num_blocks, block_size, a.kv_heads * a.vdim, dtype=dt, device=dev),
-                {"S": torch.zeros(num_slots, r.heads, r.dim, r.vdim, dtype=torch.float32, device=dev),
-                 "tail": torch.zeros(num_slots, max(r.conv - 1, 0), C, dtype=torch.float32, device=dev)})
+                DeltaMixer.allocate(model, r, num_blocks, block_size, num_slots)[2])
 
     @staticmethod
     def state_bytes(spec) -> int:
-        r = spec.right
-        return 4 * (r.heads * r.dim * r.vdim + max(r.conv - 1, 0) * (2 * r.kv_heads * r.dim + r.heads * r.vdim))
+        return DeltaMixer.state_bytes(spec.right)
 
     @staticmethod
     def forward(model: "LayeredLM", i: int, W, spec, h, inp: StepInput, cu, caches):
-        dt, eps = model.dtype, model.cfg.norm_eps
+        dt = model.dtype
         a, r, c = spec.left, spec.right, W.cols
         kc, vc, st = caches[i]
         T = h.shape[0]
@@ -214,21 +264,14 @@ class ParallelMixer:
                                 a.rot.dims if a.rot is not None else 0, kc, vc, inp.slots, a.heads, a.kv_heads, a.dim,
                                 a.vdim)
         single = inp.kind == "decode"
-        nl, nr = a.heads * a.vdim, r.heads * r.vdim
+        nl, nr = a.heads * a.vdim, r.heads * r.vdim  # (result columns of the two branches)
         both = torch.empty(T, nl + nr, dtype=dt, device=h.device)  # [left | right] rows for the one output GEMM
         ops.sink_attn_mix(q, kc, vc, inp.block_tables, cu, inp.ctx_lens, W.talk, spec.left_scale, a.heads, a.kv_heads,
                           a.dim, a.vdim, a.scale, a.softcap, both[:, :nl],
                           max_qlen=1 if single else max(1, inp.max_seqlen), num_decode=0 if single else inp.num_decode,
                           max_ctx=inp.max_ctx)
-        # right: short convolution + SiLU on q | k | v, then the gated delta rule over the sequence's matrix state
-        nqk = r.kv_heads * r.dim
-        qkv = ops.causal_conv(proj[:, c["rq"]:c["rq"] + 2 * nqk + nr], W.conv, st["tail"], cu, inp.ctx_lens,
-                              inp.state_slots, False, True, torch.float32)
-        o = ops.delta_recurrence(qkv[:, :nqk], qkv[:, nqk:2 * nqk], qkv[:, 2 * nqk:], proj[:, c["ra"]:c["ra"] + r.heads],
-                                 proj[:, c["rb"]:c["rb"] + r.heads], W.A_log, W.dt_bias, st["S"], cu, inp.ctx_lens,
-                                 inp.state_slots, r.heads, r.kv_heads, r.dim, r.vdim)
-        ops.gated_group_norm(o, proj[:, c["rg"]:c["rg"] + nr], W.norm, eps, "silu", spec.right_scale,
-                             out=both[:, nl:])
+        # right: the gated delta rule
+        DeltaMixer.mix(model, W, r, proj, {n: c["r" + n] for n in "qgab"}, inp, cu, st, spec.right_scale, both[:, nl:])
         return ops.linear_f(both, W.o, dt)
 
 
@@ -435,9 +478,40 @@ class MLSTMMixer:
         return ops.linear_f(MLSTMMixer.mix(model, W, spec, ops.linear_f(h, W.proj, dt), inp, cu, caches[i]), W.o, dt)
 
 
+class MambaMixer:
+    """Mixer ``mamba`` (in a pair): x through a short causal convolution with bias and SiLU; step sizes, input and output
+    vectors from it; the selective scan over a state per channel, gated by silu(z)."""
+
+    @staticmethod
+    def cache_row(spec) -> Optional[int]:
+        return None
+
+    @staticmethod
+    def allocate(model: "LayeredLM", spec, num_blocks: int, block_size: int, num_slots: int):
+        dev = model.device
+        return (None, None, {"S": torch.zeros(num_slots, spec.inner, spec.state, dtype=torch.float32, device=dev),
+                             "tail": torch.zeros(num_slots, max(spec.conv - 1, 0), spec.inner, dtype=torch.float32,
+                                                 device=dev)})
+
+    @staticmethod
+    def state_bytes(spec) -> int:
+        return 4 * spec.inner * (spec.state + max(spec.conv - 1, 0))
+
+    @staticmethod
+    def mix(model: "LayeredLM", W, spec, proj, inp: StepInput, cu, cache):
+        """The gated channels [T, inner], before the output projection, from the projection rows."""
+        dt, c, st, n, R, N = model.dtype, W.cols, cache[2], spec.inner, spec.dt_rank, spec.state
+        x = ops.causal_conv(proj[:, c["x"]:c["x"] + n], W.conv, st["tail"], cu, inp.ctx_lens, inp.state_slots, False, True,
+                            dt, bias=W.conv_b)
+        dbc = ops.linear_f(x, W.x, dt)
+        step = ops.linear_f(dbc[:, :R], W.dt, torch.float32)
+        return ops.selective_scan(x, step, W.dt_bias, dbc[:, R:R + N], dbc[:, R + N:R + 2 * N], W.A, W.D,
+                                  proj[:, c["z"]:c["z"] + n], st["S"], cu, inp.ctx_lens, inp.state_slots, dt)
+
+
 class PairMixer:
-    """Mixer ``pair``: two mixers side by side, each result RMS-normed over the row, averaged. One GEMM holds the input
-    projections of both; the join happens inside the block's closing op."""
+    """Mixer ``pair``: two mixers side by side, each result RMS-normed over the row, averaged; or summed with two scales. One
+    GEMM holds the input projections of both; the join happens inside the block's closing op."""
 
     @staticmethod
     def cache_row(spec) -> Optional[int]:
@@ -459,12 +533,12 @@ class PairMixer:
         yl = MIXERS[spec.left.kind].mix(model, W.left, spec.left, proj, inp, cu, caches[i])
         yr = MIXERS[spec.right.kind].mix(model, W.right, spec.right, proj, inp, cu, caches[i])
         return ops.PairPending(ops.linear_f(yl, W.left.o, dt, bias=W.left.o_bias), ops.linear_f(yr, W.right.o, dt), W.out_l,
-                               W.out_r)
+                               W.out_r, spec.scales)
 
 
 MIXERS = {"latent_attention": LatentAttention, "parallel": ParallelMixer, "lightning": DecayMixer,
           "attention": DiffAttention, "pool_attention": PoolAttention, "mamba2": SSDMixer,
-          "window_attention": WindowAttention, "mlstm": MLSTMMixer, "pair": PairMixer}
+          "window_attention": WindowAttention, "mlstm": MLSTMMixer, "pair": PairMixer, "gated_delta": DeltaMixer, "mamba": MambaMixer}
 FFNS = {"moe": MoEFeedForward, "dense": DenseFeedForward}
 
 
@@ -525,7 +599,7 @@ class LayeredLM:
                 out[f"{name}_{N}x{K}"] = GemmShape(N, K)
         for L in self.w.layers:
             for mx in (L.mix, getattr(L.mix, "left", None), getattr(L.mix, "right", None)):
-                for nm in ("qc", "proj", "o"):
+                for nm in ("qc", "uq", "proj", "x", "o"):
                     if getattr(mx, nm, None) is not None:
                         put(nm, getattr(mx, nm))
             for nm in ("shared_gu", "shared_down", "gu", "down"):
@@ -718,7 +792,7 @@ class LayeredLM:
     def _sandwich_blocks(self, inp: StepInput, kv_caches) -> torch.Tensor:
         """Blocks normed on both sides of their sublayers. Every sublayer's closing op (the gated, normed, scaled
         residual add, or the token input after it) also forms what the next reader takes - the next sublayer's normed
-        input, with the embedding added first where a new pass of a looped stretch begins - as the residual add and
+        input, with what a new pass of a looped stretch adds first where one begins - as the residual add and
         the next norm are one op for the other families. The gate logits come out of the sublayer's own first GEMM
         (``self.proj``). With a ``tap`` the closing ops run unfused, so that the tap sees the residual as the layer
         leaves it."""
@@ -730,15 +804,20 @@ class LayeredLM:
         self._angles = {}
         runs = cfg.layer_runs()
         x = ops.embed_scaled(inp.input_ids, w.wte, cfg.embedding_scale)
-        x0 = x.clone() if cfg.loop else None
+        x0 = x.clone() if cfg.loop and not cfg.loop_step else None
         W_, ng = cfg.hidden_size, cfg.norm_groups
-        h = ops.sandwich_add_norm(x, None, None, None, None, eps, None, w.layers[runs[0]].norm1, dt, ng)
+
+        def added(r):  # what comes on top of the residual before layer run r
+            t = cfg.pass_before(r)
+            if t is None or r == len(runs):
+                return None
+            return w.extra["loop_step"][t] if cfg.loop_step else (x0 if t else None)
+        h = ops.sandwich_add_norm(x, None, None, None, None, eps, added(0), w.layers[runs[0]].norm1, dt, ng)
         for r, i in enumerate(runs):
             L, spec = w.layers[i], cfg.layer_specs[i]
             last = r + 1 == len(runs)
             nxt = w.lnf_w if last else w.layers[runs[r + 1]].norm1
-            # the embedding comes back in before a pass of the looped stretch other than the first
-            add = x0 if not last and cfg.loop and runs[r + 1] == cfg.loop[0] and r + 1 > cfg.loop[0] else None
+            add = added(r + 1)
             if self.tap is not None:
                 tail = (None, None)  # close the layer first, tap, then add / norm on their own
             else:

@@ -22,7 +22,7 @@ from .config import ModelConfig
 from .decoder import StepInput
 from .layered import create_model
 from .weights import (load_babotar_weights, load_fizelix_weights, load_hf_weights, load_lamisun_weights,
-                      load_tefudra_weights, load_timisun_weights)
+                      load_nolavik_weights, load_tefudra_weights, load_timisun_weights)
 
 
 @dataclass
@@ -55,9 +55,10 @@ class CausalLM:
     def __init__(self, config, weights, max_blocks: int = 4096, block_size: int = 16, max_seqs: int = 16):
         cfg = config if isinstance(config, ModelConfig) else ModelConfig.from_hf_dict(config.to_dict())
         tp = getattr(weights, "tp", None) or TPGroup()
-        if cfg.layer_specs:  # per-layer designs (Timisun, Babotar, Lamisun, Fizelix, Tefudra)
+        if cfg.layer_specs:  # per-layer designs (Timisun, Babotar, Lamisun, Fizelix, Tefudra, Nolavik)
             load = {"babotar": load_babotar_weights, "lamisun": load_lamisun_weights,
-                    "fizelix": load_fizelix_weights, "tefudra": load_tefudra_weights}.get(cfg.model_type, load_timisun_weights)
+                    "fizelix": load_fizelix_weights, "tefudra": load_tefudra_weights,
+                    "nolavik": load_nolavik_weights}.get(cfg.model_type, load_timisun_weights)
             w = load(cfg, weights.reader, device=weights.device, dtype=weights.dtype)
         else:
             w = load_hf_weights(cfg, weights.reader, tp.size, tp.rank, device=weights.device, dtype=weights.dtype)
@@ -298,6 +299,14 @@ class TefudraForCausalLM(_FamilyLM):
     model_type = "tefudra"
 
 
+class NolavikForCausalLM(_FamilyLM):
+    """Per-layer design: blocks normed on both sides of their sublayers, gated delta rule, unit-query attention beside a
+    selective scan, latent attention with a query latent, experts with a gated shared expert, a looped stretch of layers
+    (models/layered.py)."""
+    model_type = "nolavik"
+
+
 MODEL_REGISTRY = {c.model_type: c for c in (GPT2LMHeadModel, GPTJForCausalLM, GPTBigCodeForCausalLM,
                                             LlamaForCausalLM, TimisunForCausalLM, BabotarForCausalLM,
-                                            LamisunForCausalLM, FizelixForCausalLM, TefudraForCausalLM)}
+                                            LamisunForCausalLM, FizelixForCausalLM, TefudraForCausalLM,
+                                            NolavikForCausalLM)}

@@ -555,16 +555,22 @@ class LatentAttnWeights:
     freqs: Optional[torch.Tensor] = None
     gate_col: Optional[int] = None
     rot_key: Optional[tuple] = None  # (dims, base): layers with the same rotation share a step's angles
+    # queries through a latent: ``qc`` holds the query down-projection's rows before the latent's, ``q_norm`` [q_rank] is
+    # that latent's norm weight and ``uq`` [heads * (dim + rot_dim), q_rank] the up-projection
+    q_norm: Optional[torch.Tensor] = None
+    uq: Optional[torch.Tensor] = None
 
     def tensors(self):
-        return [t for t in (self.qc, self.kv_norm, self.uk_t, self.uv, self.o, self.freqs) if t is not None]
+        return [t for t in (self.qc, self.kv_norm, self.uk_t, self.uv, self.o, self.freqs, self.q_norm, self.uq)
+                if t is not None]
 
 
 @dataclass
 class MoEWeights:
     """Experts stacked: ``gate`` / ``up`` [E, F, H] (``gate`` None: ungated experts), ``down`` [E, H, F]; ``router`` [E (+
     identity experts), H]; ``correction`` fp32 [router rows] (added to the scores for the choice only); the shared expert as
-    one gate | up matrix ``shared_gu`` [2 Fs, H] (ungated: [Fs, H]) and ``shared_down`` [H, Fs]."""
+    one gate | up matrix ``shared_gu`` [2 Fs, H] (ungated: [Fs, H]) and ``shared_down`` [H, Fs]; ``bias`` fp32 [experts],
+    added to the router's logits. A shared expert behind a gate has its gate's row after the router's last one."""
     router: torch.Tensor
     correction: Optional[torch.Tensor]
     gate: Optional[torch.Tensor]
@@ -572,10 +578,11 @@ class MoEWeights:
     down: torch.Tensor
     shared_gu: Optional[torch.Tensor] = None
     shared_down: Optional[torch.Tensor] = None
+    bias: Optional[torch.Tensor] = None
 
     def tensors(self):
         return [t for t in (self.router, self.correction, self.gate, self.up, self.down, self.shared_gu,
-                            self.shared_down) if t is not None]
+                            self.shared_down, self.bias) if t is not None]
 
 
 @dataclass
@@ -1443,13 +1450,14 @@ class MLSTMWeights:
 @dataclass
 class PairWeights:
     """Two mixers reading the same rows: ``proj`` [every input projection of both, rows padded to 8, W] with ``bias``, ``out_l``
-    / ``out_r`` fp32 [W] the weights of the norms their results pass before they are averaged."""
+    / ``out_r`` fp32 [W] the weights of the norms their results pass before they are averaged (None: they are summed with
+    the spec's scales)."""
     proj: torch.Tensor
     bias: Optional[torch.Tensor]
     left: WindowAttnWeights
-    right: MLSTMWeights
-    out_l: torch.Tensor
-    out_r: torch.Tensor
+    right: object
+    out_l: Optional[torch.Tensor] = None
+    out_r: Optional[torch.Tensor] = None
 
     def tensors(self):
         return [t for t in (self.proj, self.bias, self.out_l, self.out_r) if t is not None] + self.left.tensors() + \
@@ -1607,3 +1615,198 @@ def tefudra_state_dict(cfg: ModelConfig, seed: int = 0) -> Dict[str, torch.Tenso
     """The random weights of :func:`random_tefudra_weights` under their checkpoint names (bf16; tests, examples)."""
     get = _tefudra_random(cfg, seed)
     return {n: get(n).to(torch.bfloat16) for n in tefudra_shapes(cfg)}
+
+
+# --------------------------------------------------------- sandwich-normed per-layer designs with a selective scan (Nolavik)
+@dataclass
+class DeltaMixWeights:
+    """Gated delta rule: ``proj`` [q | k | v | g | b | a rows padded to 8, W], ``cols`` the first row of each part; ``conv``
+    [q | k | v channels, taps]; ``A_log``, ``dt_bias`` fp32 [heads]; ``norm`` [vdim]; ``o`` [W, heads * vdim]."""
+    proj: torch.Tensor
+    cols: Dict[str, int]
+    conv: torch.Tensor
+    A_log: torch.Tensor
+    dt_bias: torch.Tensor
+    norm: torch.Tensor
+    o: torch.Tensor
+
+    def tensors(self):
+        return [self.proj, self.conv, self.A_log, self.dt_bias, self.norm, self.o]
+
+
+@dataclass
+class MambaWeights:
+    """Selective scan: ``cols`` the first rows of x and z in the pair's matrix; ``conv`` [inner, taps] with ``conv_b``
+    [inner]; ``x`` [dt_rank + 2 state rows padded to 8, inner] gives step inputs | B | C; ``dt`` [inner, dt_rank];
+    ``dt_bias`` fp32 [inner], ``A`` fp32 [inner, state] = -exp(A_log), ``D`` fp32 [inner]; ``o`` [W, inner]."""
+    cols: Dict[str, int]
+    conv: torch.Tensor
+    conv_b: torch.Tensor
+    x: torch.Tensor
+    dt: torch.Tensor
+    dt_bias: torch.Tensor
+    A: torch.Tensor
+    D: torch.Tensor
+    o: torch.Tensor
+
+    def tensors(self):
+        return [self.conv, self.conv_b, self.x, self.dt, self.dt_bias, self.A, self.D, self.o]
+
+
+def nolavik_shapes(cfg: ModelConfig) -> Dict[str, tuple]:
+    """Checkpoint tensor names of a Nolavik config and their shapes."""
+    W = cfg.hidden_size
+    out = {"embed": (cfg.vocab_size, W), "final.norm": (W,), "head": (cfg.vocab_size, W)}
+    if cfg.loop:
+        out["loop.step"] = (cfg.loop[2], W)
+    for i, spec in enumerate(cfg.layer_specs):
+        p, m, f = f"l{i}.", spec.mixer, spec.mlp
+        q = p + "mix."
+        out[p + "norm1"] = out[p + "norm1b"] = (W,)
+        if m.kind == "gated_delta":
+            for n, c in (("q", m.kv_heads * m.dim), ("k", m.kv_heads * m.dim), ("v", m.heads * m.vdim)):
+                out.update({q + n: (c, W), q + n + ".conv": (c, m.conv)})
+            out.update({q + "g": (m.heads * m.vdim, W), q + "b": (m.heads, W), q + "a": (m.heads, W), q + "A_log": (m.heads,),
+                        q + "dt_bias": (m.heads,), q + "norm": (m.vdim,), q + "o": (W, m.heads * m.vdim)})
+        elif m.kind == "pair":
+            a, r, ql, qr = m.left, m.right, q + "left.", q + "right."
+            out.update({ql + "q": (a.heads * a.dim, W), ql + "k": (a.kv_heads * a.dim, W), ql + "v": (a.kv_heads * a.vdim, W),
+                        ql + "o": (W, a.heads * a.vdim), qr + "in": (2 * r.inner, W), qr + "conv": (r.inner, r.conv),
+                        qr + "conv.b": (r.inner,), qr + "x": (r.dt_rank + 2 * r.state, r.inner),
+                        qr + "dt": (r.inner, r.dt_rank), qr + "dt.b": (r.inner,), qr + "A_log": (r.inner, r.state),
+                        qr + "D": (r.inner,), qr + "o": (W, r.inner)})
+        else:
+            out.update({q + "dq": (m.q_rank, W), q + "dq.norm": (m.q_rank,), q + "uq": (m.heads * (m.dim + m.rot_dim), m.q_rank),
+                        q + "dkv": (m.kv_rank + m.rot_dim, W), q + "dkv.norm": (m.kv_rank,),
+                        q + "uk": (m.heads * m.dim, m.kv_rank), q + "uv": (m.heads * m.vdim, m.kv_rank),
+                        q + "o": (W, m.heads * m.vdim)})
+        if f is None:
+            continue
+        out[p + "norm2"] = out[p + "norm2b"] = (W,)
+        q = p + "mlp."
+        out.update({q + "router": (f.experts, W), q + "router.b": (f.experts,)})
+        for e, x in [(f"e{k}", f.expert) for k in range(f.experts)] + ([("shared", f.shared)] if f.shared is not None else []):
+            out.update({f"{q}{e}.gate": (x.ff, W), f"{q}{e}.up": (x.ff, W), f"{q}{e}.down": (W, x.ff)})
+        if f.shared is not None:
+            out[q + "shared.sg"] = (1, W)
+    return out
+
+
+def _pair_rows(t: torch.Tensor, heads: int, plain: int, rot: int, dims: int) -> torch.Tensor:
+    """Rows of a projection whose heads hold ``plain`` numbers and then a rotated part of ``rot``: inside that part the
+    partners i and i + dims / 2 become neighbours 2 i and 2 i + 1 (what the cache kernels turn), the numbers from ``dims``
+    on stay. A score is a sum over the part's numbers, so queries and keys permuted alike give the same one."""
+    half = dims // 2
+    order = [x for i in range(half) for x in (i, i + half)] + list(range(dims, rot))
+    t = t.view(heads, plain + rot, -1)
+    return torch.cat([t[:, :plain], t[:, plain:][:, order]], 1).reshape(heads * (plain + rot), -1)
+
+
+def _nolavik_finish(cfg: ModelConfig, get, device, dtype) -> ModelWeights:
+    """``get(name)`` returns the checkpoint tensor of that name. Shapes are checked against the config. All input projections
+    of a mixer (both branches of a pair) become one matrix; the shared expert's gate becomes the router's last row; norm
+    weights, router biases and the recurrences' constants are kept in fp32."""
+    shapes = nolavik_shapes(cfg)
+
+    def g(name):
+        t = get(name)
+        if tuple(t.shape) != shapes[name]:
+            raise ValueError(f"{name} has shape {tuple(t.shape)}, the config says {shapes[name]}")
+        return t
+
+    def dev(t, dt=dtype):
+        return None if t is None else t.to(device=device, dtype=dt).contiguous()
+
+    def f32(t):
+        return dev(t.float(), torch.float32)
+    layers = []
+    for i, spec in enumerate(cfg.layer_specs):
+        p, m, f = f"l{i}.", spec.mixer, spec.mlp
+        q = p + "mix."
+        if m.kind == "gated_delta":
+            proj, cols = _cat_rows([(n, g(q + n)) for n in ("q", "k", "v", "g", "b", "a")])
+            mix = DeltaMixWeights(dev(proj), cols, dev(torch.cat([g(q + n + ".conv") for n in "qkv"], 0)), f32(g(q + "A_log")),
+                                  f32(g(q + "dt_bias")), dev(g(q + "norm")), dev(g(q + "o")))
+        elif m.kind == "pair":
+            a, ql, qr = m.left, q + "left.", q + "right."
+            proj, cols = _cat_rows([(n, g(ql + n)) for n in "qkv"] + [("x", g(qr + "in"))])
+            ones = torch.ones(a.dim)  # (a rotation leaves the root mean square alone: the division may come before it)
+            left = WindowAttnWeights(None, None, cols, None, f32(ones), f32(ones), f32(torch.zeros(a.heads)),
+                                     f32(torch.tensor(a.rot.steps(), dtype=torch.float64)) if a.rot is not None else None,
+                                     a.rot.key if a.rot is not None else None, None, None, dev(g(ql + "o")), None)
+            dbc, _ = _cat_rows([("dbc", g(qr + "x"))])
+            right = MambaWeights({"x": cols["x"], "z": cols["x"] + m.right.inner}, dev(g(qr + "conv")), dev(g(qr + "conv.b")),
+                                 dev(dbc), dev(g(qr + "dt")), f32(g(qr + "dt.b")), f32(-torch.exp(g(qr + "A_log").float())),
+                                 f32(g(qr + "D")), dev(g(qr + "o")))
+            mix = PairWeights(dev(proj), None, left, right)
+        else:
+            uq, dkv = g(q + "uq"), g(q + "dkv")
+            if m.rot is not None:
+                uq = _pair_rows(uq, m.heads, m.dim, m.rot_dim, m.rot.dims)
+                dkv = _pair_rows(dkv, 1, m.kv_rank, m.rot_dim, m.rot.dims)
+            qc, _ = _cat_rows([("dq", g(q + "dq")), ("dkv", dkv)])
+            mix = LatentAttnWeights(
+                dev(qc), True, dev(g(q + "dkv.norm")), dev(_heads_t(g(q + "uk"), m.heads, m.dim, m.kv_rank, i)),
+                dev(g(q + "uv")), dev(g(q + "o")),
+                freqs=f32(torch.tensor(m.rot.steps(), dtype=torch.float64)) if m.rot is not None else None,
+                rot_key=m.rot.key if m.rot is not None else None, q_norm=dev(g(q + "dq.norm")), uq=dev(uq))
+        blk = SandwichBlockWeights(f32(g(p + "norm1")), f32(g(p + "norm1b")), None, mix)
+        if f is not None:
+            blk.norm2, blk.post2 = f32(g(p + "norm2")), f32(g(p + "norm2b"))
+            q, E, sh = p + "mlp.", f.experts, f.shared is not None
+            blk.mlp = MoEWeights(
+                router=dev(torch.cat([g(q + "router")] + ([g(q + "shared.sg")] if sh else []), 0)), correction=None,
+                gate=dev(torch.stack([g(f"{q}e{k}.gate") for k in range(E)])),
+                up=dev(torch.stack([g(f"{q}e{k}.up") for k in range(E)])),
+                down=dev(torch.stack([g(f"{q}e{k}.down") for k in range(E)])),
+                shared_gu=dev(torch.cat([g(q + "shared.gate"), g(q + "shared.up")], 0)) if sh else None,
+                shared_down=dev(g(q + "shared.down")) if sh else None, bias=f32(g(q + "router.b")))
+        layers.append(blk)
+    vp = math.ceil(cfg.vocab_size / 16) * 16
+    head = torch.zeros(vp, cfg.hidden_size, dtype=dtype, device=device)
+    head[:cfg.vocab_size].copy_(g("head").to(device=device, dtype=dtype))
+    extra = {"loop_step": f32(g("loop.step"))} if cfg.loop else {}
+    return ModelWeights(wte=dev(g("embed")), wpe=None, layers=layers, lnf_w=f32(g("final.norm")), lnf_b=None,
+                        head=Linear(head), extra=extra)
+
+
+def load_nolavik_weights(cfg: ModelConfig, reader, device="cpu", dtype=torch.bfloat16) -> ModelWeights:
+    return _nolavik_finish(cfg, lambda n: reader.get(n), device, dtype)
+
+
+def _nolavik_random(cfg: ModelConfig, seed: int, device="cpu"):
+    import zlib
+
+    shapes = nolavik_shapes(cfg)
+
+    def get(name: str) -> torch.Tensor:
+        gen = torch.Generator(device=device)
+        gen.manual_seed((seed * 1000003 + zlib.crc32(name.encode())) & 0x7FFFFFFF)
+        shp = shapes[name]
+        t = torch.randn(*shp, generator=gen, dtype=torch.float32, device=device)
+        last = name.split(".")[-1]
+        if last.startswith("norm"):
+            t = 1.0 + 0.1 * t
+        elif last == "A_log":
+            t = 0.5 * t + (0.0 if len(shp) == 2 else -1.0)
+        elif last == "dt_bias" or (last == "b" and len(shp) == 1):
+            t = 0.3 * t - (1.5 if name.endswith("dt.b") else 0.0)
+        elif last == "D":
+            t = 1.0 + 0.2 * t
+        elif last == "conv" or (len(shp) == 2 and name not in ("embed", "loop.step")):
+            t = t * shp[1] ** -0.5
+        return t.to(torch.bfloat16).float()
+    return get
+
+
+def random_nolavik_weights(cfg: ModelConfig, device="cpu", dtype=torch.bfloat16, seed: int = 0) -> ModelWeights:
+    """Random-init weights of a Nolavik config (values rounded to bf16, so a bf16 and an fp32 run hold the same model):
+    projections ~ N(0, 1 / fan_in), norm weights around one."""
+    gen = device if torch.device(device).type == "cuda" else "cpu"  # large models: draw on the GPU
+    return _nolavik_finish(cfg, _nolavik_random(cfg, seed, gen), device, dtype)
+
+
+def nolavik_state_dict(cfg: ModelConfig, seed: int = 0) -> Dict[str, torch.Tensor]:
+    """The random weights of :func:`random_nolavik_weights` under their checkpoint names (bf16; tests, examples)."""
+    get = _nolavik_random(cfg, seed)
+    return {n: get(n).to(torch.bfloat16) for n in nolavik_shapes(cfg)}

@@ -168,6 +168,7 @@ linear_f = _route("linear_f")
 head_absorb = _route("head_absorb")
 head_expand = _route("head_expand")
 latent_norm_cache = _route("latent_norm_cache")
+rms_cols = _route("rms_cols")
 latent_attn = _route("latent_attn")
 latent_qa_dtype = _route("latent_qa_dtype")
 glu_clamp = _route("glu_clamp")
@@ -205,6 +206,7 @@ rope_pairs_cache = _route("rope_pairs_cache")
 pool_update = _route("pool_update")
 pool_window_attn = _route("pool_window_attn")
 ssd_recurrence = _route("ssd_recurrence")
+selective_scan = _route("selective_scan")
 
 # ---------- heads on their way into the cache / softmax over a window with kept positions / exponential-gate recurrence
 PairPending = ref.PairPending

@@ -517,20 +517,27 @@ def _turn_neighbours(x: torch.Tensor, cs: torch.Tensor) -> torch.Tensor:
 
 def latent_norm_cache(src: torch.Tensor, off: int, R: int, w: torch.Tensor, eps: float, cache: torch.Tensor,
                       slots: torch.Tensor, rot: int = 0, cs: Optional[torch.Tensor] = None,
-                      qa: Optional[torch.Tensor] = None, off_q: int = 0, qdim: int = 0) -> None:
+                      qa: Optional[torch.Tensor] = None, off_q: int = 0, qdim: int = 0,
+                      q_src: Optional[torch.Tensor] = None) -> None:
     """cache[slot[t], :R] = rms_norm(src[t, off : off + R]) * w (slots < 0 are skipped); cache is [blocks, bs,
     R + rot]. ``rot`` > 0: the ``rot`` columns after the latent's are one key part shared by all heads; turned by
     ``cs`` [T, dims / 2, 2] (neighbouring pairs of the first ``dims`` <= rot numbers) they fill the cached row, and every query head's last ``rot`` numbers
-    (head h at src[t, off_q + h * (qdim + rot) + qdim]), turned the same way, fill qa[t, h, R:]."""
+    (head h at src[t, off_q + h * (qdim + rot) + qdim], or in ``q_src``), turned the same way, fill qa[t, h, R:]."""
     c = src[:, off:off + R].float()
     c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * w.float()
     if rot:
         c = torch.cat([c, _turn_neighbours(src[:, off + R:off + R + rot].float(), cs)], -1)
         T, H = qa.shape[0], qa.shape[1]
-        qr = src[:, off_q:off_q + H * (qdim + rot)].float().reshape(T, H, qdim + rot)[..., qdim:]
+        qr = (src if q_src is None else q_src)[:, off_q:off_q + H * (qdim + rot)].float().reshape(T, H, qdim + rot)[..., qdim:]
         qa[..., R:] = _turn_neighbours(qr, cs).to(qa.dtype)
     valid = slots >= 0
     cache.view(-1, R + rot)[slots[valid]] = c[valid].to(cache.dtype)
+
+
+def rms_cols(src: torch.Tensor, off: int, n: int, w: torch.Tensor, eps: float, out_dtype) -> torch.Tensor:
+    """rms_norm(src[t, off : off + n]) * w -> [T, n] in ``out_dtype``."""
+    x = src[:, off:off + n].float()
+    return (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
 
 
 def rope_angles(positions: torch.Tensor, freqs: torch.Tensor) -> torch.Tensor:
@@ -579,39 +586,46 @@ def glu_clamp(gu: torch.Tensor, F_: int, limit: float, alpha: float) -> torch.Te
 
 
 def moe_route(z: torch.Tensor, corr: Optional[torch.Tensor], top: int, normalize: bool = True,
-              score: str = "sigmoid"):
+              score: str = "sigmoid", bias: Optional[torch.Tensor] = None, gate: bool = False):
     """fp32 router logits [T, E] -> (idx int32 [T, top], weights fp32 [T, top]): scores sigmoid(z) (``score``
     "softmax": softmax(z) over all outputs), the ``top``
     largest of score + corr chosen (ties: lower index), weights = chosen scores / (their sum + 1e-20), or the chosen
-    scores themselves (``normalize`` false)."""
-    s = torch.softmax(z.float(), -1) if score == "softmax" else torch.sigmoid(z.float())
+    scores themselves (``normalize`` false). ``score`` "chosen": the ``top`` largest logits, weights = a softmax over those
+    alone. ``bias`` [E] is added to the logits first. ``gate``: z has one more column; its sigmoid [T] is returned third."""
+    if gate:
+        z, zg = z[:, :-1], z[:, -1]
+    z = z.float() if bias is None else z.float() + bias.float()
+    s = z if score == "chosen" else torch.softmax(z, -1) if score == "softmax" else torch.sigmoid(z)
     ch = s if corr is None else s + corr.float()
     # descending by value, ascending by index among equals
     order = torch.argsort(ch, dim=-1, descending=True, stable=True)
     idx = order[:, :top]
     w = torch.gather(s, 1, idx)
-    if normalize:
+    if score == "chosen":
+        w = torch.softmax(w, -1)
+    elif normalize:
         w = w / (w.sum(-1, keepdim=True) + 1e-20)
-    return idx.to(torch.int32), w
+    idx = idx.to(torch.int32)
+    return (idx, w, torch.sigmoid(zg.float())) if gate else (idx, w)
 
 
 def moe_router(h: torch.Tensor, router: torch.Tensor, corr: Optional[torch.Tensor], top: int,
-               normalize: bool = True, score: str = "sigmoid"):
+               normalize: bool = True, score: str = "sigmoid", bias: Optional[torch.Tensor] = None, gate: bool = False):
     """Router logits in fp32 from the layer input, then :func:`moe_route`."""
-    return moe_route(linear_f(h, router, torch.float32), corr, top, normalize, score)
+    return moe_route(linear_f(h, router, torch.float32), corr, top, normalize, score, bias, gate)
 
 
 def moe_experts(h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, gate: torch.Tensor, up: torch.Tensor,
                 down: torch.Tensor, limit: float, alpha: float, shared: Optional[torch.Tensor] = None,
                 combine: bool = True, act: str = "glu_clamp", weight_input: bool = False,
-                identity: bool = False) -> torch.Tensor:
+                identity: bool = False, shared_w: Optional[torch.Tensor] = None) -> torch.Tensor:
     """sum_j wts[t, j] * down_e(glu(gate_e h, up_e h)) (+ shared) with e = idx[t, j] -> fp32 [T, N]. Stacked expert
     weights gate / up [E, F, K], down [E, N, F]; the activation is rounded to the storage type between the
     products, as the grouped GEMMs do. ``act`` "silu": silu(g) * u without clamps. ``weight_input``: the weight
     multiplies the expert's input instead, sum_j down_e(act(w gate_e h, w up_e h)) (experts have no biases, so the
     weight is applied to the two products). ``act`` "gelu": experts without a gate (``gate`` None), down_e(gelu(up_e
     h)), the error-function form. ``identity``: an index from E on is an
-    identity expert, its output is h[t] itself."""
+    identity expert, its output is h[t] itself. ``shared_w`` fp32 [T] multiplies the shared rows."""
     T = h.shape[0]
     N = down.shape[1]
     out = torch.zeros(T, N, dtype=torch.float32, device=h.device)
@@ -633,7 +647,7 @@ def moe_experts(h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, gate: tor
             a = (g_ * torch.sigmoid(g_) * u_ if act == "silu" else glu_clamped(g_, u_, limit, alpha)).to(h.dtype).float()
             out[rows] += (a @ down[e].float().t()) * (1.0 if weight_input else wts[rows, j:j + 1])
     if shared is not None:
-        out += shared.float()
+        out += shared.float() if shared_w is None else shared.float() * shared_w[:, None]
     return out
 
 
@@ -987,12 +1001,13 @@ def diff_combine(O, lam: float, eps: float, mult: float, heads: int, kv_heads: i
 # ------------------- blocks normed on both sides / token input / windowed sigmoid attention with pooled blocks / SSD
 class PairPending:
     """The results of two mixers side by side before they are joined: y = 1/2 (rms_norm(yl) * wl + rms_norm(yr) * wr), the
-    norms over the whole row. sandwich_add_norm takes it as its ``y`` and joins while it reads."""
+    norms over the whole row, or, with ``scales`` (cl, cr), y = cl yl + cr yr. sandwich_add_norm takes it as its ``y`` and
+    joins while it reads."""
 
-    __slots__ = ("yl", "yr", "wl", "wr")
+    __slots__ = ("yl", "yr", "wl", "wr", "scales")
 
-    def __init__(self, yl, yr, wl, wr):
-        self.yl, self.yr, self.wl, self.wr = yl, yr, wl, wr
+    def __init__(self, yl, yr, wl, wr, scales=None):
+        self.yl, self.yr, self.wl, self.wr, self.scales = yl, yr, wl, wr, scales
 
 
 def _rms_parts(x, eps: float, groups: int):
@@ -1002,12 +1017,12 @@ def _rms_parts(x, eps: float, groups: int):
 
 def sandwich_add_norm(x, y, r, rb, wpost, eps: float, add, wnext, out_dtype, groups: int = 1):
     """x fp32 [T, W], in place: with ``y`` [T, W], x += rms_norm(y * sigmoid(r + rb)) * wpost (``r`` [T, W] gate
-    logits and ``rb`` [W] their bias, or None for no gate; ``wpost`` fp32 [W]); with ``add`` (fp32 [T, W]) x += add;
+    logits and ``rb`` [W] their bias, or None for no gate; ``wpost`` fp32 [W]); with ``add`` (fp32 [T, W] or [W]) x += add;
     with ``wnext`` (fp32 [W]) returns rms_norm(x) * wnext in ``out_dtype``, else None. ``groups``: both norms are taken in
     that many equal consecutive parts of the row. ``y`` may be a :class:`PairPending`."""
     if isinstance(y, PairPending):
         l, rr = y.yl.float(), y.yr.float()
-        y = 0.5 * (_rms_parts(l, eps, 1) * y.wl.float() + _rms_parts(rr, eps, 1) * y.wr.float())
+        y = y.scales[0] * l + y.scales[1] * rr if y.scales is not None else 0.5 * (_rms_parts(l, eps, 1) * y.wl.float() + _rms_parts(rr, eps, 1) * y.wr.float())
     if y is not None:
         yf = y.float()
         if r is not None:
@@ -1129,6 +1144,26 @@ def ssd_recurrence(x, Bm, Cm, dt, A_log, dt_bias, D, state, cu, ctx_lens, state_
             out[t0 + j] = (torch.einsum("hdv,hd->hv", S, CC[j]) + D.float()[:, None] * xx[j]).reshape(-1)
         state[slots[b]] = S
     return out
+
+
+def selective_scan(x, dt, dt_bias, Bm, Cm, A, D, z, state, cu, ctx_lens, state_slots, out_dtype):
+    """Per channel c and state n over each sequence's rows: d = softplus(dt_c + dt_bias_c); S <- exp(d A[c, n]) S + d x_c
+    B_n; y_c = sum_n S[c, n] C_n + D_c x_c; S fp32 [slots, inner, state] carried in the sequence's slot (zero when the
+    portion starts at position 0). x, z [T, inner], dt fp32 [T, inner], Bm / Cm [T, state], A fp32 [inner, state]. Returns
+    y * silu(z) [T, inner] in ``out_dtype``."""
+    T, inner = x.shape
+    out = torch.zeros(T, inner, dtype=torch.float32)
+    slots = state_slots.tolist()
+    for b, t0, n, p0 in _seq_rows(cu, ctx_lens):
+        S = state[slots[b]].clone() if p0 > 0 else torch.zeros_like(state[slots[b]])
+        xx = x[t0:t0 + n].float()
+        d = F.softplus(dt[t0:t0 + n] + dt_bias, threshold=20.0)
+        for j in range(n):
+            S = torch.exp(d[j][:, None] * A) * S + (d[j] * xx[j])[:, None] * Bm[t0 + j].float()[None, :]
+            out[t0 + j] = S @ Cm[t0 + j].float() + D * xx[j]
+        state[slots[b]] = S
+    zf = z.float()
+    return (out * zf * torch.sigmoid(zf)).to(out_dtype)
 
 
 # ------------- heads on their way into the cache / softmax over a window with kept positions / exponential-gate recurrence
