@@ -22,20 +22,21 @@
 // rot > 0: the cached row is [c | k_rot], k_rot = src[t, off + R : off + R + rot] with the neighbouring pairs
 // (2i, 2i + 1), i < rdims / 2, turned by cs[t, i] = (cos, sin) and the numbers from rdims on passed unchanged; and
 // every query head's rotated part - head h holds qdim plain numbers, then rot - is turned the same way into
-// qa[t, h, R : R + rot] (qa [T, H, R + rot] in its own type TQ).
+// qa[t, h, R : R + rot] (qa [T, H, R + rot] in its own type TQ). The queries are columns of src, or rows of their own (qsrc).
 template <typename T, typename TQ>
 __global__ __launch_bounds__(64) void latent_norm_cache_kernel(const T* __restrict__ src, int64_t lds_, int off,
                                                                const T* __restrict__ w, float eps,
                                                                T* __restrict__ cache, const int64_t* __restrict__ slots,
                                                                int R, int rot, int rdims,
                                                                const float* __restrict__ cs, TQ* __restrict__ qa,
-                                                               int off_q, int H, int qdim) {
+                                                               const T* __restrict__ qsrc, int64_t ldq, int H,
+                                                               int qdim) {
   const int t = blockIdx.x, lane = threadIdx.x;
   const int64_t slot = slots[t];
   const int half = rdims >> 1, rest = rot - rdims;
   const float* tab = cs + (int64_t)t * half * 2;
   if (rot) {
-    const T* q = src + (int64_t)t * lds_ + off_q;
+    const T* q = qsrc + (int64_t)t * ldq;
     TQ* dst = qa + (int64_t)t * H * (R + rot) + R;
     for (int e = lane; e < H * half; e += 64) {
       const int h = e / half, i = e - h * half;
@@ -68,16 +69,16 @@ __global__ __launch_bounds__(64) void latent_norm_cache_kernel(const T* __restri
   for (int i = rdims + lane; i < rot; i += 64) El<T>::st(dst + R + i, El<T>::ld(s + R + i));
 }
 
-// dq: storage type of qa (0 bf16, 1 fp32); only read when rot > 0
+// qsrc: the first head of the first row's queries. dq: storage type of qa (0 bf16, 1 fp32); only read when rot > 0
 void launch_latent_norm_cache(const void* src, int64_t ld, int off, const void* w, float eps, void* cache,
                               const void* slots, int T_, int R, int rot, int rdims, const void* cs, void* qa,
-                              int off_q, int H, int qdim, int dt, int dq, hipStream_t st) {
+                              const void* qsrc, int64_t ldq, int H, int qdim, int dt, int dq, hipStream_t st) {
   if (T_ == 0) return;
   if (rot < 0 || rdims < 0 || rdims > rot || (rdims & 1))
     throw std::runtime_error("latent_norm_cache: rotated dimensions must be even and fit the rotated part");
   DISPATCH_T(dt, T, DISPATCH_T(rot ? dq : 1, TQ, (latent_norm_cache_kernel<T, TQ><<<T_, 64, 0, st>>>(
       (const T*)src, ld, off, (const T*)w, eps, (T*)cache, (const int64_t*)slots, R, rot, rdims, (const float*)cs,
-      (TQ*)qa, off_q, H, qdim))));
+      (TQ*)qa, (const T*)qsrc, ldq, H, qdim))));
   HIP_CHECK_LAUNCH();
 }
 

@@ -94,15 +94,17 @@ void launch_moe_down_tile(const void* act, const void* wd, const void* meta, voi
                           int tile_rows, hipStream_t st);
 void launch_latent_norm_cache(const void* src, int64_t ld, int off, const void* w, float eps, void* cache,
                               const void* slots, int T_, int R, int rot, int rdims, const void* cs, void* qa,
-                              int off_q, int H, int qdim, int dt, int dq, hipStream_t st);
+                              const void* qsrc, int64_t ldq, int H, int qdim, int dt, int dq, hipStream_t st);
+void launch_rms_cols(const void* src, int64_t ld, const void* w, float eps, void* out, int T_, int n, int dt,
+                     hipStream_t st);
 void launch_rope_angles(const void* positions, const void* freqs, void* cs, int T_, int half, hipStream_t st);
 void launch_latent_attn(const void* qa, int64_t ldq, const void* cache, const void* bt, int maxb, const void* cu_q,
                         const void* ctx_lens, void* out, int64_t ldo, int T_, int B, int H, int R, int bs, int window,
                         float scale, int dt, hipStream_t st);
 void launch_moe_route(const void* z, const void* corr, void* idx, void* wts, int T_, int E, int top, int norm,
-                      int smax, hipStream_t st);
+                      int smax, const void* zb, void* sg, hipStream_t st);
 void launch_moe_router(const void* h, int64_t ldh, const void* wr, const void* corr, void* idx, void* wts, int T_,
-                       int E, int K, int top, int dt, int norm, int smax, hipStream_t st);
+                       int E, int K, int top, int dt, int norm, int smax, const void* zb, void* sg, hipStream_t st);
 void launch_moe_group(const void* idx, int P, int E, int maxt, void* meta, void* order, void* place, int tile_rows,
                       hipStream_t st);
 void launch_moe_gate_up(const void* h, int64_t ldh, const void* wg, const void* wu, const void* meta,
@@ -111,7 +113,8 @@ void launch_moe_gate_up(const void* h, int64_t ldh, const void* wg, const void* 
 void launch_moe_down(const void* act, const void* wd, const void* meta, void* y, int E, int maxt, int N, int F,
                      int dt, hipStream_t st);
 void launch_moe_combine(const void* y, const void* place, const void* wts, const void* shared_, int64_t lds_,
-                        void* out, int T_, int N, int top, int dt, const void* ident, int64_t ldi, hipStream_t st);
+                        void* out, int T_, int N, int top, int dt, const void* ident, int64_t ldi, const void* sw,
+                        hipStream_t st);
 void launch_glu_clamp(const void* gu, int64_t ldg, void* out, int64_t ldo, int T_, int F, float limit, float alpha,
                       int dt, hipStream_t st);
 
@@ -137,6 +140,10 @@ void launch_recurrence(int mode, const void* q, const void* k, const void* v, in
 void launch_mlstm_gates(const void* zi, const void* zf, int64_t ld, const void* bi, const void* bf, float cap,
                         void* mstate, const void* cu, const void* ctx, const void* sslots, void* gates, void* ab, int B,
                         int H, int dt, hipStream_t st);
+void launch_selective_scan(const void* x, int64_t ldx, const void* dt, int64_t ldt, const void* dt_bias, const void* Bm,
+                           const void* Cm, int64_t ldb, const void* A, const void* D, const void* z, int64_t ldz,
+                           void* state, const void* cu, const void* ctx, const void* sslots, void* out, int64_t ldo, int B,
+                           int inner, int N, int all_single, int dtype, hipStream_t st);
 bool mlstm_step_ok(int dim, int vdim);
 void launch_mlstm_step(const void* q, const void* k, const void* v, int64_t ldq, int64_t ldk, int64_t ldv, const void* zi,
                        const void* zf, int64_t ldz, const void* bi, const void* bf, float cap, void* S, void* n, void* m,
@@ -157,7 +164,8 @@ void launch_sandwich_add_norm(void* x, const void* y, int64_t ldy, const void* e
                               int top, const void* shared_, int64_t lds_, const void* r, int64_t ldr, const void* rb,
                               const void* wpost, const void* add, const void* wnext, void* h, int64_t ldh, float eps,
                               int groups, const void* ident, int64_t ldi, const void* y2, int64_t ldy2, const void* wl,
-                              const void* wr, int T_, int W, int dt, hipStream_t st);
+                              const void* wr, float cl, float cr, int64_t lda, const void* sw, int T_, int W, int dt,
+                              hipStream_t st);
 void launch_token_side_add(void* x, const void* ids, const void* table, int64_t ldt, int vocab, int col0, int d,
                            const void* wg, const void* wp, const void* wn, const void* add, const void* wnext, void* h,
                            int64_t ldh, float eps, int T_, int W, int dt, hipStream_t st);
@@ -384,10 +392,12 @@ PYBIND11_MODULE(_C, m) {
   });
   m.def("latent_norm_cache", [](uintptr_t src, int64_t ld, int off, uintptr_t w, float eps, uintptr_t cache,
                                 uintptr_t slots, int T, int R, int rot, int rdims, uintptr_t cs, uintptr_t qa,
-                                int off_q, int H, int qdim, int dt, int dq, uintptr_t st) {
-    launch_latent_norm_cache(CP(src), ld, off, CP(w), eps, P(cache), CP(slots), T, R, rot, rdims, CP(cs), P(qa), off_q,
-                             H, qdim, dt, dq, S(st));
+                                uintptr_t qsrc, int64_t ldq, int H, int qdim, int dt, int dq, uintptr_t st) {
+    launch_latent_norm_cache(CP(src), ld, off, CP(w), eps, P(cache), CP(slots), T, R, rot, rdims, CP(cs), P(qa), CP(qsrc),
+                             ldq, H, qdim, dt, dq, S(st));
   });
+  m.def("rms_cols", [](uintptr_t src, int64_t ld, uintptr_t w, float eps, uintptr_t out, int T, int n, int dt,
+                       uintptr_t st) { launch_rms_cols(CP(src), ld, CP(w), eps, P(out), T, n, dt, S(st)); });
   m.def("rope_angles", [](uintptr_t pos, uintptr_t freqs, uintptr_t cs, int T, int half, uintptr_t st) {
     launch_rope_angles(CP(pos), CP(freqs), P(cs), T, half, S(st));
   });
@@ -398,12 +408,12 @@ PYBIND11_MODULE(_C, m) {
                        scale, dt, S(st));
   });
   m.def("moe_route", [](uintptr_t z, uintptr_t corr, uintptr_t idx, uintptr_t wts, int T, int E, int top, int norm,
-                        int smax, uintptr_t st) {
-    launch_moe_route(CP(z), CP(corr), P(idx), P(wts), T, E, top, norm, smax, S(st));
+                        int smax, uintptr_t zb, uintptr_t sg, uintptr_t st) {
+    launch_moe_route(CP(z), CP(corr), P(idx), P(wts), T, E, top, norm, smax, CP(zb), P(sg), S(st));
   });
   m.def("moe_router", [](uintptr_t h, int64_t ldh, uintptr_t wr, uintptr_t corr, uintptr_t idx, uintptr_t wts, int T,
-                         int E, int K, int top, int dt, int norm, int smax, uintptr_t st) {
-    launch_moe_router(CP(h), ldh, CP(wr), CP(corr), P(idx), P(wts), T, E, K, top, dt, norm, smax, S(st));
+                         int E, int K, int top, int dt, int norm, int smax, uintptr_t zb, uintptr_t sg, uintptr_t st) {
+    launch_moe_router(CP(h), ldh, CP(wr), CP(corr), P(idx), P(wts), T, E, K, top, dt, norm, smax, CP(zb), P(sg), S(st));
   });
   m.def("moe_group", [](uintptr_t idx, int Pn, int E, int maxt, uintptr_t meta, uintptr_t order, uintptr_t place,
                         int tile_rows, uintptr_t st) {
@@ -418,8 +428,8 @@ PYBIND11_MODULE(_C, m) {
   m.def("moe_down", [](uintptr_t act, uintptr_t wd, uintptr_t meta, uintptr_t y, int E, int maxt, int N, int F, int dt,
                        uintptr_t st) { launch_moe_down(CP(act), CP(wd), CP(meta), P(y), E, maxt, N, F, dt, S(st)); });
   m.def("moe_combine", [](uintptr_t y, uintptr_t place, uintptr_t wts, uintptr_t sh, int64_t lds_, uintptr_t out, int T,
-                          int N, int top, int dt, uintptr_t ident, int64_t ldi, uintptr_t st) {
-    launch_moe_combine(CP(y), CP(place), CP(wts), CP(sh), lds_, P(out), T, N, top, dt, CP(ident), ldi, S(st));
+                          int N, int top, int dt, uintptr_t ident, int64_t ldi, uintptr_t sw, uintptr_t st) {
+    launch_moe_combine(CP(y), CP(place), CP(wts), CP(sh), lds_, P(out), T, N, top, dt, CP(ident), ldi, CP(sw), S(st));
   });
   m.def("glu_clamp", [](uintptr_t gu, int64_t ldg, uintptr_t out, int64_t ldo, int T, int F, float limit, float alpha,
                         int dt, uintptr_t st) { launch_glu_clamp(CP(gu), ldg, P(out), ldo, T, F, limit, alpha, dt, S(st)); });
@@ -461,6 +471,13 @@ PYBIND11_MODULE(_C, m) {
                           uintptr_t st) {
     launch_mlstm_gates(CP(zi), CP(zf), ld, CP(bi), CP(bf), cap, P(ms), CP(cu), CP(ctx), CP(ss), P(gates), P(ab), B, H,
                        dt, S(st));
+  });
+  m.def("selective_scan", [](uintptr_t x, int64_t ldx, uintptr_t dt, int64_t ldt, uintptr_t dtb, uintptr_t Bm, uintptr_t Cm,
+                             int64_t ldb, uintptr_t A, uintptr_t D, uintptr_t z, int64_t ldz, uintptr_t state, uintptr_t cu,
+                             uintptr_t ctx, uintptr_t ss, uintptr_t out, int64_t ldo, int B, int inner, int N,
+                             int all_single, int dtype, uintptr_t st) {
+    launch_selective_scan(CP(x), ldx, CP(dt), ldt, CP(dtb), CP(Bm), CP(Cm), ldb, CP(A), CP(D), CP(z), ldz, P(state), CP(cu),
+                          CP(ctx), CP(ss), P(out), ldo, B, inner, N, all_single, dtype, S(st));
   });
   m.def("mlstm_step_ok", &mlstm_step_ok);
   m.def("mlstm_chunk_ok", &mlstm_chunk_ok);
@@ -554,10 +571,11 @@ PYBIND11_MODULE(_C, m) {
                                 int top, uintptr_t sh, int64_t lds_, uintptr_t r, int64_t ldr, uintptr_t rb,
                                 uintptr_t wpost, uintptr_t add, uintptr_t wnext, uintptr_t h, int64_t ldh, float eps,
                                 int groups, uintptr_t ident, int64_t ldi, uintptr_t y2, int64_t ldy2, uintptr_t wl,
-                                uintptr_t wr, int T, int W, int dt, uintptr_t st) {
+                                uintptr_t wr, float cl, float cr, int64_t lda, uintptr_t sw, int T, int W, int dt,
+                                uintptr_t st) {
     launch_sandwich_add_norm(P(x), CP(y), ldy, CP(ey), CP(place), CP(wts), top, CP(sh), lds_, CP(r), ldr, CP(rb),
                              CP(wpost), CP(add), CP(wnext), P(h), ldh, eps, groups, CP(ident), ldi, CP(y2), ldy2,
-                             CP(wl), CP(wr), T, W, dt, S(st));
+                             CP(wl), CP(wr), cl, cr, lda, CP(sw), T, W, dt, S(st));
   });
   m.def("token_side_add", [](uintptr_t x, uintptr_t ids, uintptr_t table, int64_t ldt, int vocab, int col0, int d,
                              uintptr_t wg, uintptr_t wp, uintptr_t wn, uintptr_t add, uintptr_t wnext, uintptr_t h,

@@ -3,6 +3,8 @@
 //   z = W_router h (fp32, gemm_any)                                   [T, E]
 //   moe_route:   s = sigmoid(z), or softmax(z) over all experts; the `top` experts with the largest s + correction are chosen (ties: the lower
 //                index); weights = chosen s / (their sum + 1e-20)     -> idx [T, top] int32, wts [T, top] fp32
+//                or (score 2) s = z, the chosen ones weighted by a softmax over themselves. A bias may be added to z; one
+//                more column of z after the E routed ones may hold a gate, whose sigmoid goes to sg [T]
 //                A router may have more outputs than there are experts: the outputs from E on are identity experts,
 //                whose output is the layer's input row; their pairs are left out of the grouping (place -1).
 //   moe_group:   pairs p = t * top + j are bucketed by expert: off [E + 1], order [P] (pair at each sorted row),
@@ -10,7 +12,7 @@
 //                grouped GEMMs launch a grid whose size is known on the host (ceil(P / rows) + E tiles at most)
 //   moe_gate_up: act[r, f] = glu(h[token(r)] . gate_e[f], h[token(r)] . up_e[f])   for sorted row r of expert e
 //   moe_down:    y[r, n] = act[r, :] . down_e[n, :]                   (fp32)
-//   moe_combine: out[t, :] = sum_j wts[t, j] * y[place[t * top + j], :] (+ shared[t, :])   (fp32, j ascending;
+//   moe_combine: out[t, :] = sum_j wts[t, j] * y[place[t * top + j], :] (+ (sw[t] *) shared[t, :])   (fp32, j ascending;
 //                no wts: the plain sum, for layers whose weights went onto the experts' inputs in moe_gate_up)
 //
 // Expert activation (clamped, gated): g = min(g, limit), u = clamp(u, -limit, limit),
@@ -37,26 +39,29 @@ __device__ __forceinline__ float glu_value(float g, float u, float limit, float 
 // one wave per token; lanes over experts
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ z, const float* __restrict__ corr,
                                                        int* __restrict__ idx, float* __restrict__ wts, int E, int top,
-                                                       int norm, int smax) {
+                                                       int norm, int smax, const float* __restrict__ zb,
+                                                       float* __restrict__ sg) {
   extern __shared__ float sc[];  // [E] scores, [E] choice values
   float* ch = sc + E;
   const int t = blockIdx.x, lane = threadIdx.x;
+  const float* zr = z + (int64_t)t * (E + (sg ? 1 : 0));
+  if (sg && lane == 0) sg[t] = 1.f / (1.f + expf(-zr[E]));
   float mx = 0.f, den = 1.f;
-  if (smax) {
+  if (smax == 1) {
     mx = -INFINITY, den = 0.f;
-    for (int e = lane; e < E; e += 64) mx = fmaxf(mx, z[(int64_t)t * E + e]);
+    for (int e = lane; e < E; e += 64) mx = fmaxf(mx, zr[e] + (zb ? zb[e] : 0.f));
     mx = warp_max(mx);
-    for (int e = lane; e < E; e += 64) den += expf(z[(int64_t)t * E + e] - mx);
+    for (int e = lane; e < E; e += 64) den += expf(zr[e] + (zb ? zb[e] : 0.f) - mx);
     den = warp_sum(den);
   }
   for (int e = lane; e < E; e += 64) {
-    const float ze = z[(int64_t)t * E + e];
-    const float s = smax ? expf(ze - mx) / den : 1.f / (1.f + expf(-ze));
+    const float ze = zr[e] + (zb ? zb[e] : 0.f);
+    const float s = smax == 2 ? ze : smax ? expf(ze - mx) / den : 1.f / (1.f + expf(-ze));
     sc[e] = s;
     ch[e] = s + (corr ? corr[e] : 0.f);
   }
   __syncthreads();
-  float sum = 0.f;
+  float sum = 0.f, first = 0.f;
   for (int j = 0; j < top; ++j) {
     float best = -INFINITY;
     int bi = 0x7fffffff;
@@ -77,7 +82,11 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
       }
     }
     if (bi >= E) bi = 0;  // every value NaN: keep indices in range
-    const float s = sc[bi];
+    float s = sc[bi];
+    if (smax == 2) {  // the first one chosen is the largest
+      if (j == 0) first = s;
+      s = expf(s - first);
+    }
     sum += s;
     if (lane == 0) {
       idx[(int64_t)t * top + j] = bi;
@@ -86,17 +95,17 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
     }
     __syncthreads();
   }
-  if (!norm) return;  // the chosen scores themselves
-  const float inv = 1.f / (sum + 1e-20f);
+  if (!norm && smax != 2) return;  // the chosen scores themselves
+  const float inv = 1.f / (sum + (smax == 2 ? 0.f : 1e-20f));
   for (int j = lane; j < top; j += 64) wts[(int64_t)t * top + j] *= inv;
 }
 
 void launch_moe_route(const void* z, const void* corr, void* idx, void* wts, int T_, int E, int top, int norm,
-                      int smax, hipStream_t st) {
+                      int smax, const void* zb, void* sg, hipStream_t st) {
   if (T_ == 0) return;
   if (top > E || top <= 0) throw std::runtime_error("moe_route: top must be in [1, experts]");
   moe_route_kernel<<<T_, 64, 2 * E * sizeof(float), st>>>((const float*)z, (const float*)corr, (int*)idx, (float*)wts,
-                                                           E, top, norm, smax);
+                                                           E, top, norm, smax, (const float*)zb, (float*)sg);
   HIP_CHECK_LAUNCH();
 }
 
@@ -107,12 +116,13 @@ template <typename T>
 __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ h, int64_t ldh, const T* __restrict__ wr,
                                                          const float* __restrict__ corr, int* __restrict__ idx,
                                                          float* __restrict__ wts, int E, int K, int top, bool vec,
-                                                         int norm, int smax) {
+                                                         int norm, int smax, const float* __restrict__ zb,
+                                                         float* __restrict__ sg) {
   extern __shared__ float sc[];  // [E] scores, [E] choice values
   float* ch = sc + E;
   const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, nw = blockDim.x >> 6;
   const T* x = h + (int64_t)t * ldh;
-  for (int e = wv; e < E; e += nw) {
+  for (int e = wv; e < E + (sg ? 1 : 0); e += nw) {
     const T* w = wr + (int64_t)e * K;
     float acc = 0.f;
     if (vec) {  // K % 8 == 0, rows 16-byte aligned (bf16) - eight elements per lane and access
@@ -125,13 +135,18 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ 
     }
     acc = warp_sum(acc);
     if (lane == 0) {
+      if (e == E) {
+        sg[t] = 1.f / (1.f + expf(-acc));
+        continue;
+      }
+      if (zb) acc += zb[e];
       const float s = smax ? acc : 1.f / (1.f + expf(-acc));
       sc[e] = s;
       ch[e] = s + (corr ? corr[e] : 0.f);
     }
   }
   __syncthreads();
-  if (smax) {  // sc holds the logits: every wave forms their maximum and sum, then the scores replace them
+  if (smax == 1) {  // sc holds the logits: every wave forms their maximum and sum, then the scores replace them
     float mx = -INFINITY, den = 0.f;
     for (int e = lane; e < E; e += 64) mx = fmaxf(mx, sc[e]);
     mx = warp_max(mx);
@@ -145,7 +160,7 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ 
     }
     __syncthreads();
   }
-  float sum = 0.f;
+  float sum = 0.f, first = 0.f;
   for (int j = 0; j < top; ++j) {
     float best = -INFINITY;
     int bi = 0x7fffffff;
@@ -166,7 +181,11 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ 
       }
     }
     if (bi >= E) bi = 0;
-    const float s = sc[bi];
+    float s = sc[bi];
+    if (smax == 2) {
+      if (j == 0) first = s;
+      s = expf(s - first);
+    }
     sum += s;
     __syncthreads();  // every wave has read ch before the winner is struck out
     if (tid == 0) {
@@ -176,13 +195,13 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ 
     }
     __syncthreads();
   }
-  if (!norm) return;
-  const float inv = 1.f / (sum + 1e-20f);
+  if (!norm && smax != 2) return;
+  const float inv = 1.f / (sum + (smax == 2 ? 0.f : 1e-20f));
   for (int j = tid; j < top; j += blockDim.x) wts[(int64_t)t * top + j] *= inv;
 }
 
 void launch_moe_router(const void* h, int64_t ldh, const void* wr, const void* corr, void* idx, void* wts, int T_,
-                       int E, int K, int top, int dt, int norm, int smax, hipStream_t st) {
+                       int E, int K, int top, int dt, int norm, int smax, const void* zb, void* sg, hipStream_t st) {
   if (T_ == 0) return;
   if (top > E || top <= 0) throw std::runtime_error("moe_router: top must be in [1, experts]");
   const int es = dt == 0 ? 2 : 4;
@@ -190,7 +209,7 @@ void launch_moe_router(const void* h, int64_t ldh, const void* wr, const void* c
   const int threads = E >= 16 ? 1024 : (E >= 8 ? 512 : 256);  // a wave per expert up to 16 waves
   DISPATCH_T(dt, T, (moe_router_kernel<T><<<T_, threads, 2 * E * sizeof(float), st>>>(
                         (const T*)h, ldh, (const T*)wr, (const float*)corr, (int*)idx, (float*)wts, E, K, top, vec,
-                        norm, smax)));
+                        norm, smax, (const float*)zb, (float*)sg)));
   HIP_CHECK_LAUNCH();
 }
 
@@ -395,7 +414,8 @@ template <typename T>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ y, const int* __restrict__ place,
                                                           const float* __restrict__ wts, const T* __restrict__ shared_,
                                                           int64_t lds_, float* __restrict__ out, int N, int top,
-                                                          const T* __restrict__ ident, int64_t ldi) {
+                                                          const T* __restrict__ ident, int64_t ldi,
+                                                          const float* __restrict__ sw) {
   const int t = blockIdx.x;
   for (int c = threadIdx.x; c < N; c += blockDim.x) {
     float a = 0.f;
@@ -404,17 +424,18 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
       const float e = pl >= 0 ? y[(int64_t)pl * N + c] : (ident ? El<T>::ld(ident + (int64_t)t * ldi + c) : 0.f);
       a = fmaf(wts ? wts[(int64_t)t * top + j] : 1.0f, e, a);
     }
-    if (shared_) a += El<T>::ld(shared_ + (int64_t)t * lds_ + c);
+    if (shared_) a = fmaf(sw ? sw[t] : 1.0f, El<T>::ld(shared_ + (int64_t)t * lds_ + c), a);
     out[(int64_t)t * N + c] = a;
   }
 }
 
 void launch_moe_combine(const void* y, const void* place, const void* wts, const void* shared_, int64_t lds_,
-                        void* out, int T_, int N, int top, int dt, const void* ident, int64_t ldi, hipStream_t st) {
+                        void* out, int T_, int N, int top, int dt, const void* ident, int64_t ldi, const void* sw,
+                        hipStream_t st) {
   if (T_ == 0) return;
   DISPATCH_T(dt, T, (moe_combine_kernel<T><<<T_, 256, 0, st>>>((const float*)y, (const int*)place, (const float*)wts,
                                                                 (const T*)shared_, lds_, (float*)out, N, top,
-                                                                (const T*)ident, ldi)));
+                                                                (const T*)ident, ldi, (const float*)sw)));
   HIP_CHECK_LAUNCH();
 }
 

@@ -351,3 +351,26 @@ void launch_gate_mul(void* y, int64_t ldy, const void* src, int64_t lds_, int T_
   DISPATCH_T(dt, T, (gate_mul_kernel<T><<<g, 256, 0, st>>>((T*)y, ldy, (const T*)src, lds_, N)));
   HIP_CHECK_LAUNCH();
 }
+
+// out[t, :] = rms_norm(src[t, :n]) * w: the norm of a slice of projection rows (a latent), a wave per row
+template <typename T>
+__global__ __launch_bounds__(256) void rms_cols_kernel(const T* __restrict__ src, int64_t lds_, const T* __restrict__ w,
+                                                       float eps, T* __restrict__ out, int T_, int n) {
+  const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (t >= T_) return;
+  const T* s = src + (int64_t)t * lds_;
+  float ss = 0.f;
+  for (int c = lane; c < n; c += 64) {
+    const float v = El<T>::ld(s + c);
+    ss = fmaf(v, v, ss);
+  }
+  const float inv = 1.0f / sqrtf(warp_sum(ss) / (float)n + eps);
+  for (int c = lane; c < n; c += 64) El<T>::st(out + (int64_t)t * n + c, El<T>::ld(s + c) * inv * El<T>::ld(w + c));
+}
+
+void launch_rms_cols(const void* src, int64_t ld, const void* w, float eps, void* out, int T_, int n, int dt,
+                     hipStream_t st) {
+  if (T_ == 0) return;
+  DISPATCH_T(dt, T, (rms_cols_kernel<T><<<(T_ + 3) / 4, 256, 0, st>>>((const T*)src, ld, (const T*)w, eps, (T*)out, T_, n)));
+  HIP_CHECK_LAUNCH();
+}

@@ -1,7 +1,7 @@
 // Blocks normed on both sides of a sublayer, over the fp32 residual stream x [T, W]:
 //
 //   sandwich_add_norm:  x += rms_norm(y * sigmoid(r + rb)) * wpost      y the sublayer's result, r its gate logits
-//                       x += add                                        (optional fp32 rows)
+//                       x += add                                        (optional fp32 rows, or one row for all)
 //                       h  = rms_norm(x) * wnext                        (optional, in the storage type)
 //   token_side_add:     e = table[id, col0 : col0 + d]; g = gelu_tanh(Wg x) * e; y = Wp g;
 //                       x += rms_norm(y) * wn, then the same optional `add` and `h`
@@ -13,7 +13,8 @@
 // either a dense row in the storage type, or the still uncombined output of a mixture-of-experts layer (moe.hip):
 // y[t] = sum_j (wts ? wts[t, j] : 1) * ey[place[t * top + j]] (+ shared[t]), j ascending, then the shared expert.
 // A pair whose place is negative chose an identity expert: its output is ident[t], the sublayer's own input row. Or y
-// is the result of two mixers side by side, y = 1/2 (rms_norm(y) * wl + rms_norm(y2) * wr), both norms over the whole row.
+// is the result of two mixers side by side, y = 1/2 (rms_norm(y) * wl + rms_norm(y2) * wr), both norms over the whole row,
+// or (no wl, wr) y = cl * y + cr * y2. The shared expert's row may carry a factor per token, sw[t].
 // Norm weights, biases and layer scales are fp32. One workgroup per row; the gated row lives in LDS between the
 // pass that sums its squares and the pass that adds it, and the updated x between that pass and the norm.
 #include "anytype.h"
@@ -45,6 +46,9 @@ struct SandwichArgs {
   int64_t ldy2;
   const float* wl;
   const float* wr;
+  float cl, cr;
+  int64_t lda;      // row stride of add (0: one row for all)
+  const float* sw;  // [T] or null
 };
 
 template <typename T, int V>
@@ -120,7 +124,7 @@ __global__ __launch_bounds__(512) void sandwich_add_norm_kernel(SandwichArgs p) 
     const T* rr = p.r ? (const T*)p.r + (int64_t)t * p.ldr : nullptr;
     const T* y2r = p.y2 ? (const T*)p.y2 + (int64_t)t * p.ldy2 : nullptr;
     float il = 0.f, ir = 0.f;
-    if (y2r) {  // two mixers: the root mean square of each row first
+    if (y2r && p.wl) {  // two mixers: the root mean square of each row first
       float sl = 0.f, sr2 = 0.f;
       for (int c = threadIdx.x * V; c < W; c += blockDim.x * V) {
         float a[V], b[V];
@@ -136,17 +140,24 @@ __global__ __launch_bounds__(512) void sandwich_add_norm_kernel(SandwichArgs p) 
       il = 0.5f / sqrtf(s2[0] / (float)W + p.eps);
       ir = 0.5f / sqrtf(s2[1] / (float)W + p.eps);
     }
+    const float swt = p.sw ? p.sw[t] : 1.0f;
     float ss = 0.f;
     for (int c = threadIdx.x * V; c < W; c += blockDim.x * V) {
       float v[V];
       if (y2r) {
-        float a[V], b[V], wa[V], wb[V];
+        float a[V], b[V];
         ldv<T, V>(yr + c, a);
         ldv<T, V>(y2r + c, b);
-        ldv<float, V>(p.wl + c, wa);
-        ldv<float, V>(p.wr + c, wb);
+        if (p.wl) {
+          float wa[V], wb[V];
+          ldv<float, V>(p.wl + c, wa);
+          ldv<float, V>(p.wr + c, wb);
 #pragma unroll
-        for (int i = 0; i < V; ++i) v[i] = fmaf(a[i] * il, wa[i], b[i] * ir * wb[i]);
+          for (int i = 0; i < V; ++i) v[i] = fmaf(a[i] * il, wa[i], b[i] * ir * wb[i]);
+        } else {
+#pragma unroll
+          for (int i = 0; i < V; ++i) v[i] = fmaf(p.cl, a[i], p.cr * b[i]);
+        }
       } else if (yr) {
         ldv<T, V>(yr + c, v);
       } else {
@@ -165,7 +176,7 @@ __global__ __launch_bounds__(512) void sandwich_add_norm_kernel(SandwichArgs p) 
           float e[V];
           ldv<T, V>(sr + c, e);
 #pragma unroll
-          for (int i = 0; i < V; ++i) v[i] += e[i];
+          for (int i = 0; i < V; ++i) v[i] = fmaf(swt, e[i], v[i]);
         }
       }
       if (rr) {
@@ -188,7 +199,7 @@ __global__ __launch_bounds__(512) void sandwich_add_norm_kernel(SandwichArgs p) 
       inv = 1.0f / sqrtf(ss / (float)W + p.eps);
     }
   }
-  const float* ar = p.add ? p.add + (int64_t)t * W : nullptr;
+  const float* ar = p.add ? p.add + (int64_t)t * p.lda : nullptr;
   const int part = W / p.groups;
   float ss2 = 0.f;
   for (int c = threadIdx.x * V; c < W; c += blockDim.x * V) {
@@ -222,13 +233,14 @@ void launch_sandwich_add_norm(void* x, const void* y, int64_t ldy, const void* e
                               int top, const void* shared_, int64_t lds_, const void* r, int64_t ldr, const void* rb,
                               const void* wpost, const void* add, const void* wnext, void* h, int64_t ldh, float eps,
                               int groups, const void* ident, int64_t ldi, const void* y2, int64_t ldy2, const void* wl,
-                              const void* wr, int T_, int W, int dt, hipStream_t st) {
+                              const void* wr, float cl, float cr, int64_t lda, const void* sw, int T_, int W, int dt,
+                              hipStream_t st) {
   if (T_ == 0) return;
   if (groups < 1 || W % groups) throw std::runtime_error("sandwich_add_norm: the norm's parts must divide the row");
   if (((size_t)W + groups) * 4 > 64 * 1024) throw std::runtime_error("sandwich_add_norm: rows wider than 16384");
   SandwichArgs p{(float*)x, y, ldy, (const float*)ey, (const int*)place, (const float*)wts, top, shared_, lds_, r, ldr,
                  (const float*)rb, (const float*)wpost, (const float*)add, (const float*)wnext, h, ldh, eps, W, groups, ident, ldi, y2, ldy2,
-                 (const float*)wl, (const float*)wr};
+                 (const float*)wl, (const float*)wr, cl, cr, lda, (const float*)sw};
   const int es = dt == 0 ? 2 : 4;
   const auto alv = [&](const void* q, int64_t ld) { return !q || (((uintptr_t)q % (4 * es)) == 0 && ld % 4 == 0); };
   const bool vec = W % 4 == 0 && al16(x) && al16(ey) && al16(rb) && al16(wpost) && al16(add) && al16(wnext) &&

@@ -823,9 +823,10 @@ class MoEPending:
     pair, ``wts`` [T, top], ``shared`` [T, N] or None. resid_add_norm takes it as its fp32 addend and combines while
     it adds to the stream."""
 
-    __slots__ = ("y", "place", "wts", "shared", "top", "ident")
+    __slots__ = ("y", "place", "wts", "shared", "top", "ident", "shared_w")
 
-    def __init__(self, y, place, wts, shared, top=None, ident=None):
+    def __init__(self, y, place, wts, shared, top=None, ident=None, shared_w=None):
+        self.shared_w = shared_w  # fp32 [T]: factor of the shared rows (None: 1)
         self.ident = ident  # [T, N]: the output of the identity experts (pairs whose place is -1)
         self.y, self.place, self.wts, self.shared = y, place, wts, shared
         self.top = top if top is not None else wts.shape[1]  # wts None: the outputs are summed unweighted
@@ -840,7 +841,7 @@ def resid_add_norm(x, a, b, w, woff, eps, out_dtype, want_y=True):
         _check(a.shape[0] == T, "a rows")
     pend = b if isinstance(b, MoEPending) else None
     if pend is not None:
-        _check(pend.wts is not None and pend.ident is None, "resid_add_norm combines weighted expert outputs")
+        _check(pend.wts is not None and pend.ident is None and pend.shared_w is None, "resid_add_norm combines weighted expert outputs")
         top = pend.wts.shape[1]
         _check(pend.y.shape == (T * top, H) and pend.y.is_contiguous() and pend.place.numel() == T * top
                and pend.wts.shape[0] == T, "pending expert outputs do not fit the stream")
@@ -933,7 +934,8 @@ def head_expand(o, uv, out_dtype):
     return y
 
 
-def latent_norm_cache(src, off, R, w, eps, cache, slots, rot=0, cs=None, qa=None, off_q=0, qdim=0):
+def latent_norm_cache(src, off, R, w, eps, cache, slots, rot=0, cs=None, qa=None, off_q=0, qdim=0,
+                      q_src=None):
     T = src.shape[0]
     _rows(src, "src")
     rot = int(rot)
@@ -951,10 +953,24 @@ def latent_norm_cache(src, off, R, w, eps, cache, slots, rot=0, cs=None, qa=None
         _check(qa.is_contiguous() and qa.is_cuda and qa.dim() == 3 and qa.shape[0] == T and qa.shape[2] == R + rot,
                "qa [T, H, R + rot] contiguous")
         H, dq = qa.shape[1], _dt(qa, "qa")
-        _check(off_q >= 0 and off_q + H * (qdim + rot) <= src.shape[1], "query columns outside src")
+        qs = src if q_src is None else q_src
+        _rows(qs, "q_src", dtype=src.dtype)
+        _check(qs.shape[0] == T and off_q >= 0 and off_q + H * (qdim + rot) <= qs.shape[1], "query columns outside their rows")
     lib().latent_norm_cache(src.data_ptr(), src.stride(0), int(off), w.data_ptr(), float(eps), cache.data_ptr(),
-                            slots.data_ptr(), T, R, rot, rdims, _ptr(cs) if rot else 0, _ptr(qa) if rot else 0, int(off_q), H,
+                            slots.data_ptr(), T, R, rot, rdims, _ptr(cs) if rot else 0, _ptr(qa) if rot else 0,
+                            qs.data_ptr() + int(off_q) * qs.element_size() if rot else 0, qs.stride(0) if rot else 0, H,
                             int(qdim), _dt(src, "src"), dq, _stream())
+
+
+def rms_cols(src, off, n, w, eps, out_dtype):
+    T = src.shape[0]
+    _rows(src, "src", dtype=out_dtype)
+    _check(0 <= off and off + n <= src.shape[1], "columns outside src")
+    _check(w.dtype == src.dtype and w.is_contiguous() and w.numel() == n and w.is_cuda, "norm weight [n] in src's type")
+    out = torch.empty(T, n, dtype=out_dtype, device=src.device)
+    lib().rms_cols(src.data_ptr() + int(off) * src.element_size(), src.stride(0), w.data_ptr(), float(eps), out.data_ptr(), T,
+                   int(n), _dt(src, "src"), _stream())
+    return out
 
 
 def rope_angles(positions, freqs):
@@ -1024,50 +1040,57 @@ def glu_clamp(gu, F, limit, alpha):
     return out
 
 
-def moe_route(z, corr, top, normalize=True, score="sigmoid"):
-    T, E = z.shape
+_SCORE = {"sigmoid": 0, "softmax": 1, "chosen": 2}
+
+
+def _route_args(E, top, corr, bias, score):
+    _check(1 <= top <= E and E <= 4096, "1 <= top <= experts <= 4096")
+    _check(score in _SCORE and not (score == "chosen" and corr is not None), "score: sigmoid, softmax or chosen (no correction)")
+    for t, nm in ((corr, "correction"), (bias, "router bias")):
+        if t is not None:
+            _check(t.dtype == torch.float32 and t.is_contiguous() and t.numel() == E and t.is_cuda, f"{nm} fp32 [E]")
+
+
+def moe_route(z, corr, top, normalize=True, score="sigmoid", bias=None, gate=False):
+    T, E = z.shape[0], z.shape[1] - int(bool(gate))
     _rows(z, "z", dtype=torch.float32)
     _check(z.is_contiguous(), "router logits contiguous")
-    _check(1 <= top <= E and E <= 4096, "1 <= top <= experts <= 4096")
-    if corr is not None:
-        _check(corr.dtype == torch.float32 and corr.is_contiguous() and corr.numel() == E and corr.is_cuda,
-               "correction fp32 [E]")
+    _route_args(E, top, corr, bias, score)
     idx = torch.empty(T, top, dtype=torch.int32, device=z.device)
     wts = torch.empty(T, top, dtype=torch.float32, device=z.device)
+    sg = torch.empty(T, dtype=torch.float32, device=z.device) if gate else None
     lib().moe_route(z.data_ptr(), _ptr(corr), idx.data_ptr(), wts.data_ptr(), T, E, top, int(bool(normalize)),
-                    int(score == "softmax"), _stream())
-    return idx, wts
+                    _SCORE[score], _ptr(bias), _ptr(sg), _stream())
+    return (idx, wts, sg) if gate else (idx, wts)
 
 
 ROUTER_FUSED_MAX_ROWS = 1024  # steps of at most this many tokens compute logits and routing in one launch
 
 
-def moe_router(h, router, corr, top, normalize=True, score="sigmoid"):
-    """(idx [T, top] int32, wts [T, top] fp32) from the layer input: fp32 router logits, then moe_route. Few rows (a
-    decode step): one fused launch; a prompt: the matrix-core GEMM with fp32 output, then moe_route."""
+def moe_router(h, router, corr, top, normalize=True, score="sigmoid", bias=None, gate=False):
+    """(idx [T, top] int32, wts [T, top] fp32(, gate fp32 [T])) from the layer input: fp32 router logits, then moe_route. Few
+    rows (a decode step): one fused launch; a prompt: the matrix-core GEMM with fp32 output, then moe_route."""
     T, K = h.shape
-    E = router.shape[0]
+    E = router.shape[0] - int(bool(gate))
     if T > ROUTER_FUSED_MAX_ROWS:
-        return moe_route(linear_f(h, router, torch.float32), corr, top, normalize, score)
+        return moe_route(linear_f(h, router, torch.float32), corr, top, normalize, score, bias, gate)
     _rows(h, "h")
-    _check(router.dtype == h.dtype and router.is_contiguous() and router.shape == (E, K) and router.is_cuda,
-           "router [E, K] in h's storage type")
-    _check(1 <= top <= E and E <= 4096, "1 <= top <= experts <= 4096")
-    if corr is not None:
-        _check(corr.dtype == torch.float32 and corr.is_contiguous() and corr.numel() == E and corr.is_cuda,
-               "correction fp32 [E]")
+    _check(router.dtype == h.dtype and router.is_contiguous() and router.shape[1] == K and router.is_cuda,
+           "router [E (+ 1), K] in h's storage type")
+    _route_args(E, top, corr, bias, score)
     idx = torch.empty(T, top, dtype=torch.int32, device=h.device)
     wts = torch.empty(T, top, dtype=torch.float32, device=h.device)
+    sg = torch.empty(T, dtype=torch.float32, device=h.device) if gate else None
     lib().moe_router(h.data_ptr(), h.stride(0), router.data_ptr(), _ptr(corr), idx.data_ptr(), wts.data_ptr(), T, E, K,
-                     top, _dt(h, "h"), int(bool(normalize)), int(score == "softmax"), _stream())
-    return idx, wts
+                     top, _dt(h, "h"), int(bool(normalize)), _SCORE[score], _ptr(bias), _ptr(sg), _stream())
+    return (idx, wts, sg) if gate else (idx, wts)
 
 
 _MOE_PP = os.environ.get("LLMSS_MOE_PP", "1") != "0"  # 0: grouped products on the tile kernel at every size (A/B runs)
 
 
 def moe_experts(h, idx, wts, gate, up, down, limit, alpha, shared=None, combine=True, act="glu_clamp",
-                weight_input=False, identity=False):
+                weight_input=False, identity=False, shared_w=None):
     """``identity``: indices from E on are identity experts. ``combine=False``: leave the weighting and summing to the next residual add (returns a :class:`MoEPending`).
     ``weight_input``: the weights scale the two input products in the gate / up epilogue (the experts have no
     biases), and the outputs are summed plainly (``MoEPending.wts`` is None)."""
@@ -1085,6 +1108,9 @@ def moe_experts(h, idx, wts, gate, up, down, limit, alpha, shared=None, combine=
     if shared is not None:
         _rows(shared, "shared", N, h.dtype)
         _check(shared.shape[0] == T, "shared rows")
+    if shared_w is not None:
+        _check(shared_w.dtype == torch.float32 and shared_w.is_contiguous() and shared_w.numel() == T and shared_w.is_cuda
+               and shared is not None, "shared_w fp32 [T]")
     out = torch.empty(T, N, dtype=torch.float32, device=h.device) if combine or T == 0 else None
     if T == 0:
         return out
@@ -1125,10 +1151,10 @@ def moe_experts(h, idx, wts, gate, up, down, limit, alpha, shared=None, combine=
                       act_.data_ptr(), E, maxt, top, F, K, float(limit), float(alpha), dt, pw, silu, st)
         L.moe_down(act_.data_ptr(), down.data_ptr(), meta.data_ptr(), y.data_ptr(), E, maxt, N, F, dt, st)
     if not combine:
-        return MoEPending(y, place, None if weight_input else wts, shared, top, h if identity else None)
+        return MoEPending(y, place, None if weight_input else wts, shared, top, h if identity else None, shared_w)
     L.moe_combine(y.data_ptr(), place.data_ptr(), 0 if weight_input else wts.data_ptr(), _ptr(shared),
                   shared.stride(0) if shared is not None else 0, out.data_ptr(), T, N, top, dt,
-                  h.data_ptr() if identity else 0, h.stride(0), st)
+                  h.data_ptr() if identity else 0, h.stride(0), _ptr(shared_w), st)
     return out
 
 
@@ -1504,7 +1530,7 @@ def sandwich_add_norm(x, y, r, rb, wpost, eps, add, wnext, out_dtype, groups=1):
         for t_, nm in ((pair.yl, "left"), (pair.yr, "right")):
             _rows(t_, nm, W, out_dtype)
             _check(t_.shape[0] == T, "pair rows")
-        for t_ in (pair.wl, pair.wr):
+        for t_ in (pair.wl, pair.wr) if pair.scales is None else ():
             _f32c(t_, "pair weights")
             _check(t_.numel() == W, "pair weights [W]")
         y = pair.yl
@@ -1532,7 +1558,7 @@ def sandwich_add_norm(x, y, r, rb, wpost, eps, add, wnext, out_dtype, groups=1):
             _check(r.shape[0] == T and rb.numel() == W, "gate logits [T, W], bias [W]")
     if add is not None:
         _f32c(add, "add")
-        _check(tuple(add.shape) == (T, W), "add fp32 [T, W]")
+        _check(tuple(add.shape) in ((T, W), (W,)), "add fp32 [T, W] or [W]")
     h = None
     if wnext is not None:
         _f32c(wnext, "wnext")
@@ -1547,7 +1573,9 @@ def sandwich_add_norm(x, y, r, rb, wpost, eps, add, wnext, out_dtype, groups=1):
                             _ptr(wnext), _ptr(h), W, float(eps), int(groups),
                             _ptr(pend.ident) if pend else 0, pend.ident.stride(0) if pend and pend.ident is not None else 0,
                             _ptr(pair.yr) if pair else 0, pair.yr.stride(0) if pair else 0, _ptr(pair.wl) if pair else 0,
-                            _ptr(pair.wr) if pair else 0, T, W, _DT[out_dtype], _stream())
+                            _ptr(pair.wr) if pair else 0, *(pair.scales if pair and pair.scales else (0.0, 0.0)),
+                            W if add is not None and add.dim() == 2 else 0,
+                            _ptr(pend.shared_w) if pend else 0, T, W, _DT[out_dtype], _stream())
     return h
 
 
@@ -1704,6 +1732,34 @@ def ssd_recurrence(x, Bm, Cm, dt, A_log, dt_bias, D, state, cu, ctx_lens, state_
                          cu.data_ptr(), ctx_lens.data_ptr(), state_slots.data_ptr(), out.data_ptr(), heads * vdim, B,
                          heads, groups, N, vdim, 0, 0, _dt(x, "x"), _dt(dt, "dt"), D.data_ptr(), 0, 0,
                          _stream())
+    return out
+
+
+def selective_scan(x, dt, dt_bias, Bm, Cm, A, D, z, state, cu, ctx_lens, state_slots, out_dtype):
+    T, inner = x.shape
+    N = A.shape[1]
+    _rows(x, "x", dtype=out_dtype)
+    _rows(z, "z", inner, out_dtype)
+    _rows(dt, "dt", inner, torch.float32)
+    _rows(Bm, "B", N, out_dtype)
+    _rows(Cm, "C", N, out_dtype)
+    _check(z.shape[0] == T and dt.shape[0] == T and Bm.shape[0] == T and Cm.shape[0] == T and Bm.stride(0) == Cm.stride(0),
+           "rows of z / dt / B / C, one row stride for B and C")
+    for t, nm, shp in ((A, "A", (inner, N)), (D, "D", (inner,)), (dt_bias, "dt_bias", (inner,))):
+        _f32c(t, nm)
+        _check(tuple(t.shape) == shp, f"{nm} {shp}")
+    B = cu.numel() - 1
+    _i32(cu, "cu")
+    _i32(ctx_lens, "ctx_lens", B)
+    _i32(state_slots, "state_slots", B)
+    _f32c(state, "state")
+    _check(state.dim() == 3 and tuple(state.shape[1:]) == (inner, N), "state [slots, inner, N]")
+    out = torch.empty(T, inner, dtype=out_dtype, device=x.device)
+    if T:
+        lib().selective_scan(x.data_ptr(), x.stride(0), dt.data_ptr(), dt.stride(0), dt_bias.data_ptr(), Bm.data_ptr(),
+                             Cm.data_ptr(), Bm.stride(0), A.data_ptr(), D.data_ptr(), z.data_ptr(), z.stride(0),
+                             state.data_ptr(), cu.data_ptr(), ctx_lens.data_ptr(), state_slots.data_ptr(), out.data_ptr(),
+                             inner, B, inner, N, int(T == B), _dt(x, "x"), _stream())
     return out
 
 
