@@ -144,6 +144,16 @@ void launch_selective_scan(const void* x, int64_t ldx, const void* dt, int64_t l
                            const void* Cm, int64_t ldb, const void* A, const void* D, const void* z, int64_t ldz,
                            void* state, const void* cu, const void* ctx, const void* sslots, void* out, int64_t ldo, int B,
                            int inner, int N, int all_single, int dtype, hipStream_t st);
+bool delta_step_ok(int dim, int vdim);
+void launch_delta_step(const void* q, const void* k, const void* v, int64_t ldq, int64_t ldk, int64_t ldv, const void* a,
+                       const void* b, int64_t ldab, const void* A_log, const void* dt_bias, void* S, const void* cu,
+                       const void* ctx, const void* sslots, const void* gate, int64_t ldg, const void* w, float eps,
+                       float scale, void* y, int64_t ldy, int B, int H, int G, int dim, int vdim, int dt, hipStream_t st);
+bool delta_chunk_ok(int dim, int vdim);
+void launch_delta_chunk(const void* q, const void* k, const void* v, int64_t ldq, int64_t ldk, int64_t ldv, const void* a,
+                        const void* b, int64_t ldab, const void* A_log, const void* dt_bias, void* S, const void* cu,
+                        const void* ctx, const void* sslots, void* out, void* work, void* aux, int T_, int B, int max_qlen,
+                        int H, int G, int dim, int vdim, hipStream_t st);
 bool mlstm_step_ok(int dim, int vdim);
 void launch_mlstm_step(const void* q, const void* k, const void* v, int64_t ldq, int64_t ldk, int64_t ldv, const void* zi,
                        const void* zf, int64_t ldz, const void* bi, const void* bf, float cap, void* S, void* n, void* m,
@@ -478,6 +488,22 @@ PYBIND11_MODULE(_C, m) {
                              int all_single, int dtype, uintptr_t st) {
     launch_selective_scan(CP(x), ldx, CP(dt), ldt, CP(dtb), CP(Bm), CP(Cm), ldb, CP(A), CP(D), CP(z), ldz, P(state), CP(cu),
                           CP(ctx), CP(ss), P(out), ldo, B, inner, N, all_single, dtype, S(st));
+  });
+  m.def("delta_step_ok", &delta_step_ok);
+  m.def("delta_chunk_ok", &delta_chunk_ok);
+  m.def("delta_step", [](uintptr_t q, uintptr_t k, uintptr_t v, int64_t ldq, int64_t ldk, int64_t ldv, uintptr_t a,
+                         uintptr_t b, int64_t ldab, uintptr_t A_log, uintptr_t dtb, uintptr_t Sp, uintptr_t cu,
+                         uintptr_t ctx, uintptr_t ss, uintptr_t gate, int64_t ldg, uintptr_t w, float eps, float scale,
+                         uintptr_t y, int64_t ldy, int B, int H, int G, int dim, int vdim, int dt, uintptr_t st) {
+    launch_delta_step(CP(q), CP(k), CP(v), ldq, ldk, ldv, CP(a), CP(b), ldab, CP(A_log), CP(dtb), P(Sp), CP(cu), CP(ctx),
+                      CP(ss), CP(gate), ldg, CP(w), eps, scale, P(y), ldy, B, H, G, dim, vdim, dt, S(st));
+  });
+  m.def("delta_chunk", [](uintptr_t q, uintptr_t k, uintptr_t v, int64_t ldq, int64_t ldk, int64_t ldv, uintptr_t a,
+                          uintptr_t b, int64_t ldab, uintptr_t A_log, uintptr_t dtb, uintptr_t Sp, uintptr_t cu,
+                          uintptr_t ctx, uintptr_t ss, uintptr_t out, uintptr_t work, uintptr_t aux, int T, int B,
+                          int max_qlen, int H, int G, int dim, int vdim, uintptr_t st) {
+    launch_delta_chunk(CP(q), CP(k), CP(v), ldq, ldk, ldv, CP(a), CP(b), ldab, CP(A_log), CP(dtb), P(Sp), CP(cu), CP(ctx),
+                       CP(ss), P(out), P(work), P(aux), T, B, max_qlen, H, G, dim, vdim, S(st));
   });
   m.def("mlstm_step_ok", &mlstm_step_ok);
   m.def("mlstm_chunk_ok", &mlstm_chunk_ok);

@@ -33,8 +33,7 @@ beside them. Besides pages of the shared pool a mixer may own per-sequence state
 inputs of a convolution): ``LayerCache.state`` tensors indexed by the scheduler's state slot of each sequence
 (``StepInput.state_slots``); a portion that starts at position 0 starts from an empty state.
 
-Mixer ``parallel`` (ops: linear_f, rope_bias_cache, sink_attn_mix = sink_attn + talk_mix, causal_conv, delta_recurrence,
-gated_group_norm): softmax attention with a sink, soft cap, partial scaled rotation and head mixing beside a gated
+Mixer ``parallel`` (ops: linear_f, rope_bias_cache, sink_attn_mix = sink_attn + talk_mix, causal_conv, delta_mix): softmax attention with a sink, soft cap, partial scaled rotation and head mixing beside a gated
 delta rule, one input GEMM and one output GEMM for both. Mixer ``lightning`` (decay_recurrence, gated_group_norm):
 linear attention with a constant decay per head. Feed-forward ``dense`` (glu_act): gated, tanh-form GELU.
 
@@ -65,7 +64,7 @@ window that keeps the sequence's first positions, with a learned sink per head, 
 query / key / value norms, rotated keys and values - each by the spec. Mixer ``mlstm`` (linear_f, mlstm_mix): matrix memory
 with exponential gates and a running maximum. Mixer ``pair``: two mixers on the same input, one input GEMM for both; their
 results go unjoined (``ops.PairPending``) into the block's closing op, which norms and averages them or sums them with two
-scales. Mixer ``gated_delta`` (causal_conv, delta_recurrence, gated_group_norm): the gated delta rule on its own. Mixer
+scales. Mixer ``gated_delta`` (causal_conv, delta_mix): the gated delta rule on its own. Mixer
 ``mamba`` (causal_conv with bias, linear_f, selective_scan), the right half of a pair: a state per channel with a step size,
 input and output vectors of its own per token.
 
@@ -213,22 +212,26 @@ class DeltaMixer:
                     + max(spec.conv - 1, 0) * (2 * spec.kv_heads * spec.dim + spec.heads * spec.vdim))
 
     @staticmethod
-    def mix(model: "LayeredLM", W, spec, proj, cols, inp: StepInput, cu, st, scale: float, out):
+    def mix(model: "LayeredLM", W, spec, proj, cols, inp: StepInput, cu, st, scale: float, out,
+            conv_dtype):
         """The heads' results, gated and times ``scale``, into ``out`` [T, heads * vdim], from the projection rows (q | k | v
-        contiguous from cols["q"] on; g, a, b)."""
+        contiguous from cols["q"] on; g, a, b). ``conv_dtype``: type of the convolved q, k, v (in the model's own the
+        matrix cores and the fused single-row step take them)."""
         H, nqk, nv = spec.heads, spec.kv_heads * spec.dim, spec.heads * spec.vdim
         qkv = ops.causal_conv(proj[:, cols["q"]:cols["q"] + 2 * nqk + nv], W.conv, st["tail"], cu, inp.ctx_lens,
-                              inp.state_slots, False, True, torch.float32)
-        o = ops.delta_recurrence(qkv[:, :nqk], qkv[:, nqk:2 * nqk], qkv[:, 2 * nqk:], proj[:, cols["a"]:cols["a"] + H],
-                                 proj[:, cols["b"]:cols["b"] + H], W.A_log, W.dt_bias, st["S"], cu, inp.ctx_lens,
-                                 inp.state_slots, H, spec.kv_heads, spec.dim, spec.vdim)
-        return ops.gated_group_norm(o, proj[:, cols["g"]:cols["g"] + nv], W.norm, model.cfg.norm_eps, "silu", scale, out=out)
+                              inp.state_slots, False, True, conv_dtype)
+        single = inp.kind == "decode"
+        return ops.delta_mix(qkv[:, :nqk], qkv[:, nqk:2 * nqk], qkv[:, 2 * nqk:], proj[:, cols["a"]:cols["a"] + H],
+                             proj[:, cols["b"]:cols["b"] + H], W.A_log, W.dt_bias, st["S"], cu, inp.ctx_lens,
+                             inp.state_slots, H, spec.kv_heads, spec.dim, spec.vdim, proj[:, cols["g"]:cols["g"] + nv], W.norm,
+                             model.cfg.norm_eps, scale, out, max_qlen=1 if single else max(1, inp.max_seqlen),
+                             num_decode=0 if single else inp.num_decode)
 
     @staticmethod
     def forward(model: "LayeredLM", i: int, W, spec, h, inp: StepInput, cu, caches):
         dt = model.dtype
         y = torch.empty(h.shape[0], spec.heads * spec.vdim, dtype=dt, device=h.device)
-        DeltaMixer.mix(model, W, spec, ops.linear_f(h, W.proj, dt), W.cols, inp, cu, caches[i][2], 1.0, y)
+        DeltaMixer.mix(model, W, spec, ops.linear_f(h, W.proj, dt), W.cols, inp, cu, caches[i][2], 1.0, y, dt)
         return ops.linear_f(y, W.o, dt)
 
 
@@ -271,7 +274,8 @@ class ParallelMixer:
                           max_qlen=1 if single else max(1, inp.max_seqlen), num_decode=0 if single else inp.num_decode,
                           max_ctx=inp.max_ctx)
         # right: the gated delta rule
-        DeltaMixer.mix(model, W, r, proj, {n: c["r" + n] for n in "qgab"}, inp, cu, st, spec.right_scale, both[:, nl:])
+        DeltaMixer.mix(model, W, r, proj, {n: c["r" + n] for n in "qgab"}, inp, cu, st, spec.right_scale, both[:, nl:],
+                       torch.float32)
         return ops.linear_f(both, W.o, dt)
 
 

@@ -184,6 +184,7 @@ gated_group_norm = _route("gated_group_norm")
 glu_act = _route("glu_act")
 decay_recurrence = _route("decay_recurrence")
 delta_recurrence = _route("delta_recurrence")
+delta_mix = _route("delta_mix")
 rope_bias_cache = _route("rope_bias_cache")
 sink_attn = _route("sink_attn")
 sink_attn_mix = _route("sink_attn_mix")

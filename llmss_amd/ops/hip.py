@@ -1302,8 +1302,8 @@ def decay_recurrence(q, k, v, decay, state, cu, ctx_lens, state_slots, heads, di
     return out
 
 
-def delta_recurrence(q, k, v, a, b_, A_log, dt_bias, state, cu, ctx_lens, state_slots, heads, kv_heads, dim, vdim):
-    T, B, out = _rec_common(q, k, v, state, cu, ctx_lens, state_slots, heads, kv_heads, dim, vdim)
+def _delta_args(q, a, b_, A_log, dt_bias, heads):
+    T = q.shape[0]
     _f32c(A_log, "A_log")
     _f32c(dt_bias, "dt_bias")
     _check(A_log.numel() == heads and dt_bias.numel() == heads, "A_log, dt_bias [heads]")
@@ -1312,6 +1312,12 @@ def delta_recurrence(q, k, v, a, b_, A_log, dt_bias, state, cu, ctx_lens, state_
     # a and b are columns of one projection: addressed from a's base with b's offset in elements
     _check(a.dtype == b_.dtype and a.stride(0) == b_.stride(0) and a.shape[0] == T and b_.shape[0] == T
            and a.untyped_storage().data_ptr() == b_.untyped_storage().data_ptr(), "a and b: columns of one tensor")
+
+
+def delta_recurrence(q, k, v, a, b_, A_log, dt_bias, state, cu, ctx_lens, state_slots, heads, kv_heads, dim, vdim, first=0):
+    """``first``: the first sequence the walk takes (the rows of the sequences before it are left alone)."""
+    T, B, out = _rec_common(q, k, v, state, cu, ctx_lens, state_slots, heads, kv_heads, dim, vdim)
+    _delta_args(q, a, b_, A_log, dt_bias, heads)
     off_b = (b_.data_ptr() - a.data_ptr()) // a.element_size()
     ready = 0
     if T > B:  # portions: the per-token decay and write strength once per (token, head), not per workgroup
@@ -1322,9 +1328,57 @@ def delta_recurrence(q, k, v, a, b_, A_log, dt_bias, state, cu, ctx_lens, state_
     if T:
         lib().recurrence(1, q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0),
                          a.data_ptr(), a.stride(0), 0, int(off_b), A_log.data_ptr(), dt_bias.data_ptr(),
-                         state.data_ptr(), cu.data_ptr(), ctx_lens.data_ptr(), state_slots.data_ptr(), out.data_ptr(),
-                         heads * vdim, B, heads, kv_heads, dim, vdim, 0, ready, _dt(q, "q"), _dt(a, "a"), 0, 0, 0,
-                         _stream())
+                         state.data_ptr(), cu.data_ptr() + 4 * first, ctx_lens.data_ptr() + 4 * first,
+                         state_slots.data_ptr() + 4 * first, out.data_ptr(), heads * vdim, B - first, heads, kv_heads, dim,
+                         vdim, 0, ready, _dt(q, "q"), _dt(a, "a"), 0, 0, 0, _stream())
+    return out
+
+
+_DELTA_MFMA = os.environ.get("LLMSS_DELTA_MFMA", "1") != "0"  # 0: portions token by token (A/B runs)
+
+
+def delta_mix(q, k, v, a, b_, A_log, dt_bias, state, cu, ctx_lens, state_slots, heads, kv_heads, dim, vdim, gate, w, eps,
+              scale, out, max_qlen=0, num_decode=0):
+    """The ``num_decode`` leading single-row sequences (all of them when ``max_qlen`` is 1) take one fused launch; portions of
+    bf16 rows the chunked form on the matrix cores, everything else the token-by-token walk, then the per-head norm and
+    gate."""
+    N = heads * vdim
+    _rows(gate, "gate", N)
+    _rows(out, "out", N)
+    _check(w.is_contiguous() and w.numel() == vdim and gate.dtype == w.dtype == out.dtype and gate.shape[0] == q.shape[0]
+           and out.shape[0] == q.shape[0], "gate / norm weight / out in one storage type")
+    T, B = q.shape[0], cu.numel() - 1
+    if T == 0:
+        return out
+    L, st, dt, es = lib(), _stream(), _dt(out, "out"), out.element_size()
+    nd = B if max_qlen == 1 else int(num_decode)
+    _check(0 <= nd <= B and (nd < B or T == B), "num_decode outside the step")
+    same = q.dtype == k.dtype == v.dtype == a.dtype == out.dtype
+    if not (same and L.delta_step_ok(dim, vdim) and state.data_ptr() % 16 == 0):
+        nd = 0
+    qkv = (q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0))
+    ab = (a.data_ptr(), b_.data_ptr(), a.stride(0), A_log.data_ptr(), dt_bias.data_ptr(), state.data_ptr())
+    o = None
+    if nd < B and not (same and q.dtype == torch.bfloat16 and max_qlen > 0 and _DELTA_MFMA and L.delta_chunk_ok(dim, vdim)
+                       and not any(p % 16 for p in qkv[:2]) and not any(x % 8 for x in qkv[3:5])):
+        o = delta_recurrence(q, k, v, a, b_, A_log, dt_bias, state, cu, ctx_lens, state_slots, heads, kv_heads, dim, vdim, nd)
+    else:
+        _, _, o = _rec_common(q, k, v, state, cu, ctx_lens, state_slots, heads, kv_heads, dim, vdim)
+        _delta_args(q, a, b_, A_log, dt_bias, heads)
+        if nd < B:
+            work = torch.empty(4, T, heads, 64, dtype=torch.bfloat16, device=q.device)
+            aux = torch.empty(T, heads, 4, dtype=torch.float32, device=q.device)
+            L.delta_chunk(*qkv, *ab, cu.data_ptr() + 4 * nd, ctx_lens.data_ptr() + 4 * nd, state_slots.data_ptr() + 4 * nd,
+                          o.data_ptr(), work.data_ptr(), aux.data_ptr(), T, B - nd, int(max_qlen), heads, kv_heads, dim,
+                          vdim, st)
+    if nd:
+        L.delta_step(*qkv, *ab, cu.data_ptr(), ctx_lens.data_ptr(), state_slots.data_ptr(), gate.data_ptr(), gate.stride(0),
+                     w.data_ptr(), float(eps), float(scale), out.data_ptr(), out.stride(0), nd, heads, kv_heads, dim, vdim,
+                     dt, st)
+    if nd < B:  # the portions' rows: nd .. T - 1 (single-row sequences come first)
+        L.gated_group_norm(o.data_ptr() + 4 * nd * N, N, gate.data_ptr() + es * nd * gate.stride(0), gate.stride(0),
+                           w.data_ptr(), float(eps), 1, float(scale), out.data_ptr() + es * nd * out.stride(0),
+                           out.stride(0), T - nd, heads, vdim, dt, 0, 0, 0, 0, 1.0, st)
     return out
 
 

@@ -806,6 +806,15 @@ def delta_recurrence(q, k, v, a, b_, A_log, dt_bias, state, cu, ctx_lens, state_
     return out
 
 
+def delta_mix(q, k, v, a, b_, A_log, dt_bias, state, cu, ctx_lens, state_slots, heads: int, kv_heads: int, dim: int,
+              vdim: int, gate, w, eps: float, scale: float, out, max_qlen: int = 0, num_decode: int = 0):
+    """:func:`delta_recurrence`, then every head divided by its root mean square, times w [vdim], silu(gate) and ``scale``,
+    into ``out`` [T, heads * vdim]. ``max_qlen`` (the step's longest portion) and ``num_decode`` (leading single-row
+    sequences) only steer the GPU kernels."""
+    o = delta_recurrence(q, k, v, a, b_, A_log, dt_bias, state, cu, ctx_lens, state_slots, heads, kv_heads, dim, vdim)
+    return gated_group_norm(o, gate, w, eps, "silu", scale, out=out)
+
+
 def rope_angle_table(npos: int, dims: int, base: float, scaling=None) -> torch.Tensor:
     """fp32 [npos, dims / 2, 2] = (cos, sin) of position * f_i, f_i = base^(-2 i / dims). ``scaling`` = (factor,
     original, fast, slow): frequencies between the two turn counts are blended towards f_i / factor (YaRN) and both

@@ -70,13 +70,14 @@ def causal_attention(q, k, v, scale, sink=False):
     T, H, _ = q.shape
     G = k.shape[1]
     out = torch.zeros(T, H, v.shape[2], dtype=F64)
+    later = torch.arange(T)[None, :] > torch.arange(T)[:, None]
     for h in range(H):
         g = h // (H // G)
-        for i in range(T):
-            s = (k[:i + 1, g] @ q[i, h]) * scale
-            m = s.max().clamp(min=0.0) if sink else s.max()
-            e = torch.exp(s - m)
-            out[i, h] = (e @ v[:i + 1, g]) / (e.sum() + (torch.exp(-m) if sink else 0.0))
+        s = ((q[:, h] @ k[:, g].T) * scale).masked_fill(later, -math.inf)
+        m = s.max(-1, keepdim=True).values
+        m = m.clamp(min=0.0) if sink else m
+        e = torch.exp(s - m)
+        out[:, h] = (e @ v[:, g]) / (e.sum(-1, keepdim=True) + (torch.exp(-m) if sink else 0.0))
     return out
 
 
@@ -96,11 +97,10 @@ def delta_rule(q, k, v, beta, g):
     S = torch.zeros(H, dim, v.shape[2], dtype=F64)
     out = torch.zeros(T, H, v.shape[2], dtype=F64)
     for t in range(T):
-        for h in range(H):
-            S[h] = S[h] * g[t, h]
-            u = beta[t, h] * (v[t, h] - k[t, h] @ S[h])
-            S[h] = S[h] + torch.outer(k[t, h], u)
-            out[t, h] = q[t, h] @ S[h]
+        S = S * g[t, :, None, None]
+        u = beta[t, :, None] * (v[t] - (S * k[t, :, :, None]).sum(1))
+        S = S + k[t, :, :, None] * u[:, None, :]
+        out[t] = (S * q[t, :, :, None]).sum(1)
     return out
 
 
@@ -185,9 +185,9 @@ def latent_mixer(W, p, m, h, eps):
 def moe(W, p, f, h):
     idx, w = route(h @ W(p + "router").T + W(p + "router.b"), f["router"]["top"])
     out = torch.zeros_like(h)
-    for t in range(h.shape[0]):
-        for j, e in enumerate(idx[t].tolist()):
-            out[t] += w[t, j] * expert(W, f"{p}e{e}.", h[t:t + 1])[0]
+    for e in range(f["router"]["experts"]):
+        share = torch.where(idx == e, w, torch.zeros_like(w)).sum(-1, keepdim=True)
+        out = out + share * expert(W, f"{p}e{e}.", h)
     if f.get("shared"):
         out = out + sigmoid(h @ W(p + "shared.sg").T) * expert(W, p + "shared.", h)
     return out
@@ -226,3 +226,10 @@ def forward(cfg, sd, tokens, tap=None):
         if tap is not None:
             tap(r, x)
     return (rms(x, eps) * W("final.norm")) @ W("head").T
+
+
+def greedy(cfg, sd, prompt, n):
+    t = list(prompt)
+    for _ in range(n):
+        t.append(int(forward(cfg, sd, t)[-1].argmax()))
+    return t[len(prompt):]
