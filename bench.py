@@ -94,7 +94,22 @@ def main():
                     help="instead of the headline workload: prefill / decode throughput of the Tefudra design beside "
                          "the Llama family at equal size (bench/tefudra_compare.py), sizes by name, one GPU")
     ap.add_argument("--tefudra-kinds", default="tefudra,dense", help="which of the two models --tefudra runs")
+    ap.add_argument("--nolavik", nargs="?", const="w1024,w2048,w4096", default="",
+                    help="instead of the headline workload: prefill / decode throughput of the Nolavik design beside "
+                         "the Llama family at equal size (bench/nolavik_compare.py), sizes by name, one GPU")
+    ap.add_argument("--nolavik-kinds", default="nolavik,dense", help="which of the two models --nolavik runs")
     args = ap.parse_args()
+
+    if args.nolavik:
+        sys.path.insert(0, os.path.join(ROOT, "bench"))
+        import nolavik_compare
+
+        res = nolavik_compare.run(args.nolavik.split(","), args.batch_per_gpu, args.prompt_len, args.gen_len,
+                                  args.timisun_rounds,
+                                  lambda m: print(f"[bench] {m}", file=sys.stderr, flush=True),
+                                  kinds=tuple(args.nolavik_kinds.split(",")))
+        print(json.dumps(res), flush=True)
+        return
 
     if args.tefudra:
         sys.path.insert(0, os.path.join(ROOT, "bench"))

@@ -87,7 +87,7 @@ void launch_gemm_tile(const void* A, const void* B, void* C, int M, int N, int K
                       int64_t sBb, int64_t sBn, int64_t sCb, int64_t sCm, int dc, const void* bias, hipStream_t st);
 void launch_moe_gate_up_tile(const void* h, int64_t ldh, const void* wg, const void* wu, const void* meta,
                              const void* order, void* act, int E, int maxt, int top, int F, int K, float limit,
-                             float alpha, int tile_rows, const void* pw, int silu, hipStream_t st);
+                             float alpha, int tile_rows, const void* pw, int silu, int ilv, hipStream_t st);
 void launch_moe_pp(int mode, const void* A, int64_t lda, const void* W, const void* meta, const void* order, void* C, int E,
                    int maxt, int top, int N, int K, int act, hipStream_t st);
 void launch_moe_down_tile(const void* act, const void* wd, const void* meta, void* y, int E, int maxt, int N, int F,
@@ -126,7 +126,7 @@ void launch_stream_add_norm(void* x, const void* y, int64_t ldy, const void* mix
                             int W, int dt, int h_f32, hipStream_t st);
 void launch_causal_conv(const void* in, int64_t ldi, const void* w, void* state, const void* cu, const void* ctx,
                         const void* sslots, void* out, int64_t ldo, int T_, int B, int C, int taps, int res, int silu,
-                        int di, int dw, int dout, const void* bias, hipStream_t st);
+                        int di, int dw, int dout, const void* bias, int single, hipStream_t st);
 void launch_gated_group_norm(const void* o, int64_t ldo, const void* gate, int64_t ldg, const void* w, float eps,
                              int act, float c, void* out, int64_t ldout, int T_, int groups, int n, int dt, int wfull,
                              int first, const void* den, const void* gates, float qs, hipStream_t st);
@@ -388,9 +388,9 @@ PYBIND11_MODULE(_C, m) {
   });
   m.def("moe_gate_up_tile", [](uintptr_t h, int64_t ldh, uintptr_t wg, uintptr_t wu, uintptr_t meta, uintptr_t order,
                                uintptr_t act, int E, int maxt, int top, int F, int K, float limit, float alpha,
-                               int tile_rows, uintptr_t pw, int silu, uintptr_t st) {
+                               int tile_rows, uintptr_t pw, int silu, int ilv, uintptr_t st) {
     launch_moe_gate_up_tile(CP(h), ldh, CP(wg), CP(wu), CP(meta), CP(order), P(act), E, maxt, top, F, K, limit, alpha,
-                            tile_rows, CP(pw), silu, S(st));
+                            tile_rows, CP(pw), silu, ilv, S(st));
   });
   m.def("moe_pp", [](int mode, uintptr_t A, int64_t lda, uintptr_t W, uintptr_t meta, uintptr_t order, uintptr_t C, int E,
                      int maxt, int top, int N, int K, int act, uintptr_t st) {
@@ -455,9 +455,9 @@ PYBIND11_MODULE(_C, m) {
   });
   m.def("causal_conv", [](uintptr_t in, int64_t ldi, uintptr_t w, uintptr_t state, uintptr_t cu, uintptr_t ctx,
                           uintptr_t ss, uintptr_t out, int64_t ldo, int T, int B, int C, int taps, int res, int silu,
-                          int di, int dw, int dout, uintptr_t bias, uintptr_t st) {
+                          int di, int dw, int dout, uintptr_t bias, int single, uintptr_t st) {
     launch_causal_conv(CP(in), ldi, CP(w), P(state), CP(cu), CP(ctx), CP(ss), P(out), ldo, T, B, C, taps, res, silu,
-                       di, dw, dout, CP(bias), S(st));
+                       di, dw, dout, CP(bias), single, S(st));
   });
   m.def("gated_group_norm", [](uintptr_t o, int64_t ldo, uintptr_t gate, int64_t ldg, uintptr_t w, float eps, int act,
                                float c, uintptr_t out, int64_t ldout, int T, int groups, int n, int dt, int wfull,

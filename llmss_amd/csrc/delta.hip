@@ -196,18 +196,23 @@ __device__ __forceinline__ void split2(float x, bf16_t& hi, bf16_t& lo) {
   lo = f2bf(x - bf2f(hi));
 }
 
+constexpr int prep_kq_bytes(int kt) {  // K and Q rows, or P (value, remainder) and the fp32 inverse
+  return 2 * 64 * (16 * kt + 8) * 2 > 2 * 64 * 72 * 2 + 64 * 68 * 4 ? 2 * 64 * (16 * kt + 8) * 2 : 2 * 64 * 72 * 2 + 64 * 68 * 4;
+}
+
 // Workgroup (chunk of a portion, head, sequence), 4 waves
 template <int KT>
 __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaChunkArgs A) {
   constexpr int C = 64, DKP = 16 * KT, LDK = DKP + 8, LDP = 64 + 8, LDL = 64 + 4;
+  constexpr int KQ = prep_kq_bytes(KT);  // the rows' region; once their products are taken P and the inverse lie there
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   bf16_t* Ks = reinterpret_cast<bf16_t*>(smem);
   bf16_t* Qs = Ks + C * LDK;
-  bf16_t* Ph = Qs + C * LDK;
+  bf16_t* Ph = reinterpret_cast<bf16_t*>(smem);
   bf16_t* Pl = Ph + C * LDP;
-  float* Ls = reinterpret_cast<float*>(Pl + C * LDP);  // [64][LDL]
-  float* Xs = Ls + C * LDL;                            // [64][LDL]
-  float* bs = Xs + C * LDL;                            // [64] sum of the log decays
+  float* Xs = reinterpret_cast<float*>(Pl + C * LDP);     // [64][LDL]
+  float* Ls = reinterpret_cast<float*>(smem + KQ);        // [64][LDL]
+  float* bs = Ls + C * LDL;                               // [64] sum of the log decays
   float* be = bs + C;                                  // [64] write strength
   float* nk = be + C;                                  // [64] 1 / |k|
   float* nq = nk + C;                                  // [64] dim^-1/2 / |q|
@@ -238,11 +243,6 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaChunkArgs A) {
     }
     bs[lane] = F;
     be[lane] = in ? 1.0f / (1.0f + expf(-bf2f(A.b[tt]))) : 0.f;
-  }
-  // zero the blocks of the inverse above the diagonal
-  for (int e = tid; e < C * C; e += 256) {
-    const int r = e >> 6, c = e & 63;
-    if (c > r) Xs[r * LDL + c] = 0.f;
   }
   __syncthreads();
   {  // norms: four neighbouring lanes per row
@@ -283,6 +283,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaChunkArgs A) {
         pq[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qa, kb, pq[ct], 0, 0, 0);
       }
     }
+    __syncthreads();  // every wave has read its rows
 #pragma unroll
     for (int ct = 0; ct < 4; ++ct) {
       const int s = 16 * ct + li;
@@ -293,6 +294,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaChunkArgs A) {
         const float e = s <= t ? expf(bs[t] - bsv) * nks : 0.f;
         Ls[t * LDL + s] = s < t ? e * be[t] * nk[t] * pk[ct][i] : 0.f;
         split2(s <= t ? e * nq[t] * pq[ct][i] : 0.f, Ph[t * LDP + s], Pl[t * LDP + s]);
+        if (ct > w) Xs[t * LDL + s] = 0.f;  // the blocks of the inverse above the diagonal
       }
     }
   }
@@ -581,7 +583,7 @@ void launch_delta_chunk(const void* q, const void* k, const void* v, int64_t ldq
                    (const int*)sslots, (float*)out, (bf16_t*)work, (int64_t)T_ * H * 64, (f32x4*)aux, H, G, dim, vdim};
   dim3 g1((max_qlen + 63) / 64, H, B), g2(H, (vdim + 63) / 64, B);
   auto lds1 = [](int kt) {
-    return (size_t)2 * (2 * 64 * (16 * kt + 8) + 2 * 64 * 72) + (size_t)4 * (2 * 64 * 68 + 4 * 64);
+    return (size_t)prep_kq_bytes(kt) + (size_t)4 * (64 * 68 + 4 * 64);
   };
   auto lds2 = [](int kt) { return (size_t)2 * (2 * 64 * (16 * kt + 8) + 4 * 64 * 72) + (size_t)16 * 64; };
 #define LAUNCH_DC(KT_)                                                                                           \

@@ -2117,7 +2117,8 @@ void gemm_plan(int M, int N, int K, bool w_fp8, int* nt, int* splitk) {
 }
 
 // Grouped expert products on the ping-pong kernel, over a tile list of 256 rows per tile (moe_group): C = act(A[order / top]
-// W_e^T) in bf16 (mode 1) or C = A W_e^T in fp32 (mode 2). A [rows, K] with row stride lda, W [E, N, K].
+// W_e^T) in bf16 (mode 1), C = A W_e^T in fp32 (mode 2), or C [rows, N / 2] = silu(gate) * up in bf16 with W's rows gate and up
+// in alternating groups of 16 (mode 3). A [rows, K] with row stride lda, W [E, N, K].
 void launch_moe_pp(int mode, const void* A, int64_t lda, const void* W, const void* meta, const void* order, void* C, int E,
                    int maxt, int top, int N, int K, int act, hipStream_t st) {
   if (maxt <= 0) return;
@@ -2129,10 +2130,12 @@ void launch_moe_pp(int mode, const void* A, int64_t lda, const void* W, const vo
   gr.sB = (int64_t)N * K;
   gr.Yf = (float*)C;
   const char* z = K & 63 ? zero_page() : nullptr;
+  const int glu = mode == 3;
+  if (glu && N % 32) throw std::runtime_error("moe_pp: gate and up in groups of 16 rows");
 #define LAUNCH_PPG(KT_, G_)                                                                                         \
   gemm_pp_kernel<KT_, G_><<<(unsigned)nwg, 512, 0, st>>>((const bf16_t*)A, lda, (const bf16_t*)W, K, nullptr, (bf16_t*)C, \
-                                                         N, 0, N, K, act, 0, 1, z, gr)
-  if (mode == 1) {
+                                                         glu ? N / 2 : N, 0, N, K, glu ? 0 : act, glu, 1, z, gr)
+  if (mode == 1 || mode == 3) {
     if (K & 63) LAUNCH_PPG(true, 1);
     else LAUNCH_PPG(false, 1);
   } else if (mode == 2) {

@@ -34,6 +34,7 @@ struct GemmTileArgs {
   float limit, alpha;
   const float* pw;  // GATE_UP: weight of each (token, slot) pair on the expert's input (null: 1)
   int silu;         // GATE_UP: silu(g) * u instead of the clamped form
+  int ilv;          // GATE_UP: one weight matrix, gate and up rows in alternating groups of 16 (B the first gate row, B2 the first up row)
   const bf16_t* bias;  // PLAIN: [N] or null
 };
 
@@ -116,12 +117,14 @@ __global__ __launch_bounds__(256, BM * BN > 128 * 128 ? 2 : 1) void gemm_tile_ke
 #pragma unroll
   for (int i = 0; i < CB; ++i) {
     const int sr = (tid >> 3) + 32 * i;
-    brow[i] = (n0 + sr < p.N) ? B + (int64_t)(n0 + sr) * p.sBn : nullptr;
+    int nr = n0 + sr;  // row of the weights
+    if constexpr (DUAL) nr = p.ilv ? (nr >> 4) * 32 + (nr & 15) : nr;
+    brow[i] = (n0 + sr < p.N) ? B + (int64_t)nr * p.sBn : nullptr;
     bvec[i] = brow[i] && ((uintptr_t)brow[i] & 15) == 0;
     b2row[i] = nullptr;
     b2vec[i] = false;
     if constexpr (DUAL) {
-      b2row[i] = (n0 + sr < p.N) ? B2 + (int64_t)(n0 + sr) * p.sBn : nullptr;
+      b2row[i] = (n0 + sr < p.N) ? B2 + (int64_t)nr * p.sBn : nullptr;
       b2vec[i] = b2row[i] && ((uintptr_t)b2row[i] & 15) == 0;
     }
   }
@@ -230,7 +233,8 @@ void launch_gemm_tile(const void* A, const void* B, void* C, int M, int N, int K
 // per tile the list was built with (moe_group): 64 or 128
 void launch_moe_gate_up_tile(const void* h, int64_t ldh, const void* wg, const void* wu, const void* meta,
                              const void* order, void* act, int E, int maxt, int top, int F, int K, float limit,
-                             float alpha, int tile_rows, const void* pw, int silu, hipStream_t st) {
+                             float alpha, int tile_rows, const void* pw, int silu, int ilv, hipStream_t st) {
+  if (ilv && F % 16) throw std::runtime_error("moe_gate_up: gate and up in groups of 16 rows");
   if (tile_rows != 64 && tile_rows != 128) throw std::runtime_error("moe_gate_up: tile rows must be 64 or 128");
   if (maxt <= 0) return;
   if (maxt > 65535) throw std::runtime_error("moe_gate_up: too many row tiles");
@@ -239,6 +243,11 @@ void launch_moe_gate_up_tile(const void* h, int64_t ldh, const void* wg, const v
   a.N = F; a.K = K; a.sAm = ldh; a.sBb = (int64_t)F * K; a.sBn = K; a.sCm = F;
   a.meta = (const int*)meta; a.order = (const int*)order; a.E = E; a.maxt = maxt; a.top = top;
   a.limit = limit; a.alpha = alpha; a.pw = (const float*)pw; a.silu = silu;
+  if (ilv) {  // wg: [E, 2F, K]
+    a.ilv = 1;
+    a.B2 = a.B + (int64_t)16 * K;
+    a.sBb = (int64_t)2 * F * K;
+  }
   // 128-row tiles are 64 columns wide here: with two accumulator sets (gate and up) a 128x128 tile leaves one
   // workgroup per CU; at 128x64 two to three fit and hide each other's staging
   if (!wg) {

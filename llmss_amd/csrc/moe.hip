@@ -125,10 +125,16 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ 
   for (int e = wv; e < E + (sg ? 1 : 0); e += nw) {
     const T* w = wr + (int64_t)e * K;
     float acc = 0.f;
-    if (vec) {  // K % 8 == 0, rows 16-byte aligned (bf16) - eight elements per lane and access
+    if (vec) {  // K % 8 == 0, rows 16-byte aligned - eight elements per lane, two or four 16-byte accesses
+      typedef T vec8 __attribute__((ext_vector_type(8)));
+#pragma unroll 4
       for (int k = lane * 8; k < K; k += 512) {
+        const vec8 xv = *reinterpret_cast<const vec8*>(x + k), wv = *reinterpret_cast<const vec8*>(w + k);
 #pragma unroll
-        for (int i = 0; i < 8; ++i) acc = fmaf(El<T>::ld(x + k + i), El<T>::ld(w + k + i), acc);
+        for (int i = 0; i < 8; ++i) {
+          const T xi = xv[i], wi = wv[i];
+          acc = fmaf(El<T>::ld(&xi), El<T>::ld(&wi), acc);
+        }
       }
     } else {
       for (int k = lane; k < K; k += 64) acc = fmaf(El<T>::ld(x + k), El<T>::ld(w + k), acc);

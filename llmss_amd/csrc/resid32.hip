@@ -353,24 +353,65 @@ void launch_gate_mul(void* y, int64_t ldy, const void* src, int64_t lds_, int T_
 }
 
 // out[t, :] = rms_norm(src[t, :n]) * w: the norm of a slice of projection rows (a latent), a wave per row
-template <typename T>
+// (V: numbers per access, 8 bf16 or 4 fp32 = 16 bytes, or 1; rows of up to 64 * V * RC_N numbers stay in registers)
+#define RC_N 4
+template <typename T, int V>
 __global__ __launch_bounds__(256) void rms_cols_kernel(const T* __restrict__ src, int64_t lds_, const T* __restrict__ w,
                                                        float eps, T* __restrict__ out, int T_, int n) {
+  typedef T vec __attribute__((ext_vector_type(V == 1 ? 2 : V)));
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= T_) return;
   const T* s = src + (int64_t)t * lds_;
+  T* o = out + (int64_t)t * n;
   float ss = 0.f;
-  for (int c = lane; c < n; c += 64) {
-    const float v = El<T>::ld(s + c);
-    ss = fmaf(v, v, ss);
+  if constexpr (V == 1) {
+    for (int c = lane; c < n; c += 64) {
+      const float v = El<T>::ld(s + c);
+      ss = fmaf(v, v, ss);
+    }
+    const float inv = 1.0f / sqrtf(warp_sum(ss) / (float)n + eps);
+    for (int c = lane; c < n; c += 64) El<T>::st(o + c, El<T>::ld(s + c) * inv * El<T>::ld(w + c));
+  } else {
+    vec x[RC_N];
+#pragma unroll
+    for (int j = 0; j < RC_N; ++j) {
+      const int c = (lane + 64 * j) * V;
+      if (c >= n) continue;
+      x[j] = *reinterpret_cast<const vec*>(s + c);
+#pragma unroll
+      for (int i = 0; i < V; ++i) {
+        const T xi = x[j][i];
+        ss = fmaf(El<T>::ld(&xi), El<T>::ld(&xi), ss);
+      }
+    }
+    const float inv = 1.0f / sqrtf(warp_sum(ss) / (float)n + eps);
+#pragma unroll
+    for (int j = 0; j < RC_N; ++j) {
+      const int c = (lane + 64 * j) * V;
+      if (c >= n) continue;
+      const vec wv = *reinterpret_cast<const vec*>(w + c);
+      vec y;
+#pragma unroll
+      for (int i = 0; i < V; ++i) {
+        const T xi = x[j][i], wi = wv[i];
+        T yi;
+        El<T>::st(&yi, El<T>::ld(&xi) * inv * El<T>::ld(&wi));
+        y[i] = yi;
+      }
+      *reinterpret_cast<vec*>(o + c) = y;
+    }
   }
-  const float inv = 1.0f / sqrtf(warp_sum(ss) / (float)n + eps);
-  for (int c = lane; c < n; c += 64) El<T>::st(out + (int64_t)t * n + c, El<T>::ld(s + c) * inv * El<T>::ld(w + c));
 }
 
 void launch_rms_cols(const void* src, int64_t ld, const void* w, float eps, void* out, int T_, int n, int dt,
                      hipStream_t st) {
   if (T_ == 0) return;
-  DISPATCH_T(dt, T, (rms_cols_kernel<T><<<(T_ + 3) / 4, 256, 0, st>>>((const T*)src, ld, (const T*)w, eps, (T*)out, T_, n)));
+  const int v = dt == 0 ? 8 : 4;
+  const bool vec = n % v == 0 && ld % v == 0 && n <= 64 * v * RC_N && !(((uintptr_t)src | (uintptr_t)w | (uintptr_t)out) & 15);
+  DISPATCH_T(dt, T, {
+    constexpr int V = sizeof(T) == 2 ? 8 : 4;
+    if (vec) rms_cols_kernel<T, V><<<(T_ + 3) / 4, 256, 0, st>>>((const T*)src, ld, (const T*)w, eps, (T*)out, T_, n);
+    else rms_cols_kernel<T, 1><<<(T_ + 3) / 4, 256, 0, st>>>((const T*)src, ld, (const T*)w, eps, (T*)out, T_, n);
+  });
   HIP_CHECK_LAUNCH();
 }

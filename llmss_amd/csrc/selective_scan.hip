@@ -12,9 +12,11 @@
 // while staging; B and C once per workgroup), the next CT tokens' numbers in flight in registers behind the arithmetic. The
 // decay is exp2 of the fp32 product with A log2(e). The state is read from the sequence's slot unless the portion starts at
 // position 0 (then it is zero, whatever the slot held) and written back at the end. Rows of a padded sequence are zeroed.
+// Tokens past a portion's end are staged with step size 0, which leaves the state as it is.
 #include "anytype.h"
 
 #define SS_CH 64
+#define SS_LDY 80  // row stride of the sums: the four lanes of a channel write four rows, 16 banks apart
 
 struct ScanArgs {
   const void* x;  // [T, ldx]
@@ -43,11 +45,30 @@ __device__ __forceinline__ float ss_swap(float v) {
   return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xF, 0xF, false));
 }
 
+// softplus and silu: bf16 rows take the hardware's exponential, logarithm and reciprocal (a few units in the last place of
+// fp32; log(1 + e) corrected for the rounding of 1 + e), fp32 rows the library's functions
+template <typename T>
+__device__ __forceinline__ float ss_softplus(float q) {
+  if constexpr (sizeof(T) == 4) {
+    return q > 20.f ? q : log1pf(expf(q));
+  } else {
+    const float e = __builtin_amdgcn_exp2f(1.4426950408889634f * q), u = 1.0f + e, d = u - 1.0f;
+    const float l = 0.6931471805599453f * __builtin_amdgcn_logf(u) * e * __builtin_amdgcn_rcpf(d);
+    return q > 20.f ? q : (d == 0.f ? e : l);
+  }
+}
+template <typename T>
+__device__ __forceinline__ float ss_silu(float z) {
+  if constexpr (sizeof(T) == 4) return z / (1.0f + expf(-z));
+  else return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+}
+
 // CT: tokens staged at a time (16 in portions, 4 where every sequence has one row)
 template <typename T, int R, int CT>
 __global__ __launch_bounds__(256) void selective_scan_kernel(ScanArgs p) {
   constexpr int NP = 4 * R, NI = CT / 4, NB = (CT * 2 * NP + 255) / 256;
-  __shared__ __attribute__((aligned(16))) float sd[CT * SS_CH], sx[CT * SS_CH], sy[CT * SS_CH], sg[CT * SS_CH];
+  __shared__ __attribute__((aligned(16))) float sdx[CT * SS_CH * 2];  // (step size, step size * input)
+  __shared__ __attribute__((aligned(16))) float sy[CT * SS_LDY], sg[CT * SS_CH];
   __shared__ __attribute__((aligned(16))) float sbc[CT * 2 * NP];  // per token: B padded to NP, C padded to NP
   // sequences in reverse step order: the step's long portions come last and are dispatched first
   const int b = gridDim.y - 1 - blockIdx.y, tid = threadIdx.x;
@@ -117,12 +138,11 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(ScanArgs p) {
     const int nt = min(CT, qlen - j0);
 #pragma unroll
     for (int k = 0; k < NI; ++k) {
-      const int e = (it + 4 * k) * SS_CH + ic;
-      const float q = rd[k] + dtb, d = q > 20.f ? q : log1pf(expf(q));
-      sd[e] = d;
-      sx[e] = d * rx[k];
-      sy[e] = Dc * rx[k];
-      sg[e] = rz[k] / (1.0f + expf(-rz[k]));
+      const int j = it + 4 * k;
+      const float d = j < nt ? ss_softplus<T>(rd[k] + dtb) : 0.f;
+      *reinterpret_cast<f32x2*>(&sdx[(j * SS_CH + ic) * 2]) = f32x2{d, d * rx[k]};
+      sy[j * SS_LDY + ic] = Dc * rx[k];
+      sg[j * SS_CH + ic] = ss_silu<T>(rz[k]);
     }
 #pragma unroll
     for (int k = 0; k < NB; ++k) {
@@ -131,31 +151,40 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(ScanArgs p) {
     }
     __syncthreads();
     if (j0 + CT < qlen) fetch(j0 + CT);
-    for (int jj = 0; jj < nt; ++jj) {
-      const float d = sd[jj * SS_CH + ch], dx = sx[jj * SS_CH + ch];
-      const float* bp = sbc + jj * 2 * NP + d0;
-      float y = 0.f, y2 = 0.f;
+    constexpr int UNR = R <= 8 ? CT / 4 : 1;
+#pragma unroll UNR
+    for (int m = 0; m < CT / 4; ++m) {
+      float yv[4];
 #pragma unroll
-      for (int i = 0; i < R; i += 4) {
-        const f32x4 bv = *reinterpret_cast<const f32x4*>(bp + i), cv = *reinterpret_cast<const f32x4*>(bp + NP + i);
+      for (int q = 0; q < 4; ++q) {
+        const int jj = 4 * m + q;
+        const f32x2 dx = *reinterpret_cast<const f32x2*>(&sdx[(jj * SS_CH + ch) * 2]);
+        const float* bp = sbc + jj * 2 * NP + d0;
+        float y = 0.f, y2 = 0.f;
 #pragma unroll
-        for (int k = 0; k < 4; ++k) {
-          S[i + k] = fmaf(__builtin_amdgcn_exp2f(d * A2[i + k]), S[i + k], dx * bv[k]);
-          if (k & 1) y2 = fmaf(S[i + k], cv[k], y2);
-          else y = fmaf(S[i + k], cv[k], y);
+        for (int i = 0; i < R; i += 4) {
+          const f32x4 bv = *reinterpret_cast<const f32x4*>(bp + i), cv = *reinterpret_cast<const f32x4*>(bp + NP + i);
+#pragma unroll
+          for (int k = 0; k < 4; ++k) {
+            S[i + k] = fmaf(__builtin_amdgcn_exp2f(dx[0] * A2[i + k]), S[i + k], dx[1] * bv[k]);
+            if (k & 1) y2 = fmaf(S[i + k], cv[k], y2);
+            else y = fmaf(S[i + k], cv[k], y);
+          }
         }
+        y += y2;
+        y += ss_swap<0xB1>(y);  // lanes 0 <-> 1, 2 <-> 3
+        y += ss_swap<0x4E>(y);  // lanes 0 <-> 2, 1 <-> 3
+        yv[q] = y;
       }
-      y += y2;
-      y += ss_swap<0xB1>(y);  // lanes 0 <-> 1, 2 <-> 3
-      y += ss_swap<0x4E>(y);  // lanes 0 <-> 2, 1 <-> 3
-      if (part == 0) sy[jj * SS_CH + ch] += y;
+      // every lane of the channel holds the four tokens' sums; each adds one of them to its row
+      sy[(4 * m + part) * SS_LDY + ch] += part & 2 ? (part & 1 ? yv[3] : yv[2]) : (part & 1 ? yv[1] : yv[0]);
     }
     __syncthreads();  // the rows' sums are complete, and every reader of the staged numbers is done
     if (live_s) {
 #pragma unroll
       for (int k = 0; k < NI; ++k) {
         const int j = it + 4 * k;
-        if (j < nt) El<T>::st(outp + (int64_t)(j0 + j) * p.ldo, sy[j * SS_CH + ic] * sg[j * SS_CH + ic]);
+        if (j < nt) El<T>::st(outp + (int64_t)(j0 + j) * p.ldo, sy[j * SS_LDY + ic] * sg[j * SS_CH + ic]);
       }
     }
   }

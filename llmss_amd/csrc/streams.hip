@@ -129,13 +129,21 @@ void launch_stream_add_norm(void* x, const void* y, int64_t ldy, const void* mix
 
 // out[t, c] = act((res ? in[t, c] : 0) + sum_k w[c, k] * in_(pos - (taps - 1 - k))[c]); inputs before the portion come
 // from the sequence's tail (state[slot, i, c] holds position p0 - (taps - 1) + i), inputs before position 0 are zero.
+// single: every sequence of the step has one row; the thread that forms a channel's row then renews its tail as well.
+// sigmoid; results that leave in bf16 take the hardware's exponential and reciprocal (a unit in the last place of fp32)
+template <typename TO>
+__device__ __forceinline__ float sigm(float z) {
+  if constexpr (sizeof(TO) == 2) return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+  else return 1.0f / (1.0f + expf(-z));
+}
+
 template <typename TI, typename TW, typename TO>
 __global__ __launch_bounds__(256) void causal_conv_kernel(const TI* __restrict__ in, int64_t ldi,
-                                                          const TW* __restrict__ w, const float* __restrict__ state,
+                                                          const TW* __restrict__ w, float* __restrict__ state,
                                                           const int* __restrict__ cu, const int* __restrict__ ctx,
                                                           const int* __restrict__ sslots, TO* __restrict__ out,
                                                           int64_t ldo, int B, int C, int taps, int res, int silu,
-                                                          const TW* __restrict__ bias) {
+                                                          const TW* __restrict__ bias, int single) {
   const int t = blockIdx.x;
   const RowSeq r = row_seq(cu, ctx, B, t);  // once per workgroup: a thread walks CONV_CPT channels
   const int c_end = min(C, (int)(blockIdx.y + 1) * (int)blockDim.x * CONV_CPT);
@@ -157,8 +165,14 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const TI* __restrict__
       acc = fmaf(El<TW>::ld(w + (int64_t)c * taps + k), v, acc);
     }
     if (bias) acc += El<TW>::ld(bias + c);
-    if (silu) acc = acc / (1.0f + expf(-acc));
+    if (silu) acc = acc * sigm<TO>(acc);
     El<TO>::st(out + (int64_t)t * ldo + c, acc);
+    if (single) {
+      float* tail = state + (int64_t)slot * R * C + c;
+      for (int i = 0; i < R; ++i)  // (position pos - (R - 1) + i; inputs before position 0 are zero)
+        tail[(int64_t)i * C] = i == R - 1 ? El<TI>::ld(in + (int64_t)t * ldi + c)
+                                          : (r.pos - (R - 1) + i >= 0 ? tail[(int64_t)(i + 1) * C] : 0.f);
+    }
   }
 }
 
@@ -262,7 +276,7 @@ __global__ __launch_bounds__(256) void causal_conv_strip_kernel(const TI* __rest
       }
       if (silu) {
 #pragma unroll
-        for (int e = 0; e < CH; ++e) acc[e] = acc[e] / (1.0f + expf(-acc[e]));
+        for (int e = 0; e < CH; ++e) acc[e] = acc[e] * sigm<TO>(acc[e]);
       }
     }
     conv_st<TO, CH>(out + (int64_t)t * ldo + c, acc);
@@ -299,8 +313,8 @@ __global__ __launch_bounds__(256) void conv_tail_kernel(const TI* __restrict__ i
 template <typename TI, typename TW, typename TO>
 static void causal_conv_t(const void* in, int64_t ldi, const void* w, void* state, const void* cu, const void* ctx,
                           const void* sslots, void* out, int64_t ldo, int T_, int B, int C, int taps, int res,
-                          int silu, const void* bias, hipStream_t st) {
-  if (T_ >= 256 && T_ >= 8 * B && taps <= 9) {  // portions of eight rows and more on average
+                          int silu, const void* bias, int single, hipStream_t st) {
+  if (!single && T_ >= 256 && T_ >= 8 * B && taps <= 9) {  // portions of eight rows and more on average
     const auto al16 = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
     const bool four = C % 4 == 0 && ldi % 4 == 0 && ldo % 4 == 0 && al16(in) && al16(out) && al16(state);
 #define LAUNCH_STRIP(RMAX_, CH_)                                                                                    \
@@ -319,11 +333,11 @@ static void causal_conv_t(const void* in, int64_t ldi, const void* w, void* stat
 #undef LAUNCH_STRIP
   } else {
     dim3 g(T_, (C + 256 * CONV_CPT - 1) / (256 * CONV_CPT));
-    causal_conv_kernel<TI, TW, TO><<<g, 256, 0, st>>>((const TI*)in, ldi, (const TW*)w, (const float*)state,
+    causal_conv_kernel<TI, TW, TO><<<g, 256, 0, st>>>((const TI*)in, ldi, (const TW*)w, (float*)state,
                                                       (const int*)cu, (const int*)ctx, (const int*)sslots, (TO*)out,
-                                                      ldo, B, C, taps, res, silu, (const TW*)bias);
+                                                      ldo, B, C, taps, res, silu, (const TW*)bias, single);
   }
-  if (taps > 1) {
+  if (taps > 1 && !single) {
     dim3 g2(B, (C + 255) / 256);
     conv_tail_kernel<TI><<<g2, 256, 0, st>>>((const TI*)in, ldi, (float*)state, (const int*)cu, (const int*)ctx,
                                              (const int*)sslots, C, taps);
@@ -344,12 +358,13 @@ void launch_conv_tail(const void* in, int64_t ldi, void* state, const void* cu, 
 // di / dw / dout: storage types of the input, the weights and the output (0 bf16, 1 fp32)
 void launch_causal_conv(const void* in, int64_t ldi, const void* w, void* state, const void* cu, const void* ctx,
                         const void* sslots, void* out, int64_t ldo, int T_, int B, int C, int taps, int res, int silu,
-                        int di, int dw, int dout, const void* bias, hipStream_t st) {
+                        int di, int dw, int dout, const void* bias, int single, hipStream_t st) {
   if (T_ == 0 || B == 0) return;
+  if (single && T_ != B) throw std::runtime_error("causal_conv: single steps have one row per sequence");
   if (taps < 1 || taps - 1 > MAX_TAIL) throw std::runtime_error("causal_conv: 1 to 17 taps");
   if ((C + 255) / 256 > 65535) throw std::runtime_error("causal_conv: too many channels");
   DISPATCH_T(di, TI, DISPATCH_T(dw, TW, DISPATCH_T(dout, TO, (causal_conv_t<TI, TW, TO>(
-      in, ldi, w, state, cu, ctx, sslots, out, ldo, T_, B, C, taps, res, silu, bias, st)))));
+      in, ldi, w, state, cu, ctx, sslots, out, ldo, T_, B, C, taps, res, silu, bias, single, st)))));
   HIP_CHECK_LAUNCH();
 }
 
@@ -392,53 +407,48 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
     El<T>::st(dst + i, row[i] * inv * El<T>::ld(wr + i) * gate_of(i));
 }
 
-// The same, the gate after the norm, with a wave per group and 16-byte accesses, for groups of up to 1024 columns (whole fours): the
-// group's numbers stay in registers between the sum of squares and the result.
+// The same, the gate after the norm, for groups of 8 to 512 columns that are a power of two: L = n / 8 neighbouring lanes share
+// a group, eight columns each in 16-byte accesses; the numbers stay in registers between the sum of squares and the result.
 template <typename T>
 __global__ __launch_bounds__(256) void gated_group_norm_vec_kernel(const float* __restrict__ o, int64_t ldo,
                                                                    const T* __restrict__ gate, int64_t ldg,
                                                                    const T* __restrict__ w, float eps, int act, float c,
                                                                    T* __restrict__ out, int64_t ldout, int n, int wfull,
                                                                    const float* __restrict__ den,
-                                                                   const f32x4* __restrict__ gates, float qs, int groups) {
-  const int t = blockIdx.x, g = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (g >= groups) return;
-  const float* row = o + (int64_t)t * ldo + (int64_t)g * n;
-  const T* gr = gate + (int64_t)t * ldg + (int64_t)g * n;
-  const T* wr = wfull ? w + (int64_t)g * n : w;
+                                                                   const f32x4* __restrict__ gates, float qs, int groups,
+                                                                   int T_) {
+  const int L = n >> 3, i0 = 8 * (threadIdx.x & (L - 1));
+  const int64_t e = (int64_t)blockIdx.x * (256 / L) + threadIdx.x / L;  // row * groups + group
+  if (e >= (int64_t)T_ * groups) return;
+  const int64_t t = e / groups;
+  const int g = (int)(e - t * groups);
+  const float* row = o + t * ldo + (int64_t)g * n + i0;
+  const T* gr = gate + t * ldg + (int64_t)g * n + i0;
+  const T* wr = (wfull ? w + (int64_t)g * n : w) + i0;
   float pre = 1.0f;
-  if (den) {
-    const int64_t e = (int64_t)t * groups + g;
-    pre = qs / (fmaxf(fabsf(qs * den[e]), expf(-gates[e][2])) + 1e-6f);
-  }
-  float u[4][4], ga[4][4];
+  if (den) pre = qs / (fmaxf(fabsf(qs * den[e]), expf(-gates[e][2])) + 1e-6f);
+  float u[8], ga[8], wv[8];
   float ss = 0.f;
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int i0 = 4 * lane + 256 * j;
-    if (i0 >= n) continue;
-    conv_ld<float, 4>(row + i0, u[j]);
-    conv_ld<T, 4>(gr + i0, ga[j]);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const float sg = 1.0f / (1.0f + expf(-ga[j][i]));
-      ga[j][i] = act ? ga[j][i] * sg : sg;
-      u[j][i] *= pre;
-      ss = fmaf(u[j][i], u[j][i], ss);
-    }
+  for (int j = 0; j < 8; j += 4) {
+    conv_ld<float, 4>(row + j, u + j);
+    conv_ld<T, 4>(gr + j, ga + j);
+    conv_ld<T, 4>(wr + j, wv + j);
   }
-  const float inv = c / sqrtf(warp_sum(ss) / (float)n + eps);
-  T* dst = out + (int64_t)t * ldout + (int64_t)g * n;
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int i0 = 4 * lane + 256 * j;
-    if (i0 >= n) continue;
-    float wv[4];
-    conv_ld<T, 4>(wr + i0, wv);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) u[j][i] = u[j][i] * inv * wv[i] * ga[j][i];
-    conv_st<T, 4>(dst + i0, u[j]);
+  for (int i = 0; i < 8; ++i) {
+    const float sg = sigm<T>(ga[i]);
+    ga[i] = act ? ga[i] * sg : sg;
+    u[i] *= pre;
+    ss = fmaf(u[i], u[i], ss);
   }
+  for (int m = L >> 1; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
+  const float inv = c / sqrtf(ss / (float)n + eps);
+  T* dst = out + t * ldout + (int64_t)g * n + i0;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) u[i] = u[i] * inv * wv[i] * ga[i];
+  conv_st<T, 4>(dst, u);
+  conv_st<T, 4>(dst + 4, u + 4);
 }
 
 void launch_gated_group_norm(const void* o, int64_t ldo, const void* gate, int64_t ldg, const void* w, float eps,
@@ -448,12 +458,15 @@ void launch_gated_group_norm(const void* o, int64_t ldo, const void* gate, int64
   if (groups > 65535) throw std::runtime_error("gated_group_norm: too many groups");
   const int es = dt == 0 ? 2 : 4;
   const auto al = [](const void* p, int64_t b) { return ((uintptr_t)p % b) == 0; };
-  if (!first && n % 4 == 0 && n <= 1024 && n >= 64 && ldo % 4 == 0 && ldg % 4 == 0 && ldout % 4 == 0 && al(o, 16) && al(gate, 4 * es) &&
+  if (!first && n >= 8 && n <= 512 && (n & (n - 1)) == 0 && ldo % 4 == 0 && ldg % 4 == 0 && ldout % 4 == 0 && al(o, 16) && al(gate, 4 * es) &&
       al(w, 4 * es) && al(out, 4 * es)) {
-    dim3 gv(T_, (groups + 3) / 4);
+    const int per = 256 / (n / 8);
+    const int64_t blocks = ((int64_t)T_ * groups + per - 1) / per;
+    if (blocks > 0x7fffffff) throw std::runtime_error("gated_group_norm: too many rows");
+    const unsigned gv = (unsigned)blocks;
     DISPATCH_T(dt, T, (gated_group_norm_vec_kernel<T><<<gv, 256, 0, st>>>(
         (const float*)o, ldo, (const T*)gate, ldg, (const T*)w, eps, act, c, (T*)out, ldout, n, wfull,
-        (const float*)den, (const f32x4*)gates, qs, groups)));
+        (const float*)den, (const f32x4*)gates, qs, groups, T_)));
     HIP_CHECK_LAUNCH();
     return;
   }

@@ -177,7 +177,9 @@ class MoEFeedForward:
                 sh = ops.linear_f(ops.linear_f(h, W.shared_gu, dt, act="gelu"), W.shared_down, dt)
             return ops.moe_experts(h, idx, wts, None, W.up, W.down, 0.0, 0.0, shared=sh, combine=False, act="gelu",
                                    identity=spec.identity > 0)
-        if W.shared_gu is not None:
+        if W.shared_interleaved:
+            sh = ops.linear_f(ops.linear(h, W.shared_gu, None, "none", True), W.shared_down, dt)
+        elif W.shared_gu is not None:
             # (a sandwich block's gate logits ride in this GEMM as extra columns: model.proj)
             gu = model.proj = ops.linear_f(h, W.shared_gu, dt)
             if spec.shared is not None:
@@ -187,7 +189,7 @@ class MoEFeedForward:
         # combine=False: on the GPU the weighted sum over the chosen experts happens inside the next residual add
         return ops.moe_experts(h, idx, wts, W.gate, W.up, W.down, spec.expert.limit, GLU_ALPHA, shared=sh,
                                combine=False, act=spec.act, weight_input=spec.weight_input,
-                               shared_w=route[2] if spec.shared_gate else None)
+                               shared_w=route[2] if spec.shared_gate else None, interleaved=W.interleaved)
 
 
 class DeltaMixer:
@@ -219,7 +221,7 @@ class DeltaMixer:
         matrix cores and the fused single-row step take them)."""
         H, nqk, nv = spec.heads, spec.kv_heads * spec.dim, spec.heads * spec.vdim
         qkv = ops.causal_conv(proj[:, cols["q"]:cols["q"] + 2 * nqk + nv], W.conv, st["tail"], cu, inp.ctx_lens,
-                              inp.state_slots, False, True, conv_dtype)
+                              inp.state_slots, False, True, conv_dtype, single=inp.kind == "decode")
         single = inp.kind == "decode"
         return ops.delta_mix(qkv[:, :nqk], qkv[:, nqk:2 * nqk], qkv[:, 2 * nqk:], proj[:, cols["a"]:cols["a"] + H],
                              proj[:, cols["b"]:cols["b"] + H], W.A_log, W.dt_bias, st["S"], cu, inp.ctx_lens,
@@ -506,7 +508,7 @@ class MambaMixer:
         """The gated channels [T, inner], before the output projection, from the projection rows."""
         dt, c, st, n, R, N = model.dtype, W.cols, cache[2], spec.inner, spec.dt_rank, spec.state
         x = ops.causal_conv(proj[:, c["x"]:c["x"] + n], W.conv, st["tail"], cu, inp.ctx_lens, inp.state_slots, False, True,
-                            dt, bias=W.conv_b)
+                            dt, bias=W.conv_b, single=inp.kind == "decode")
         dbc = ops.linear_f(x, W.x, dt)
         step = ops.linear_f(dbc[:, :R], W.dt, torch.float32)
         return ops.selective_scan(x, step, W.dt_bias, dbc[:, R:R + N], dbc[:, R + N:R + 2 * N], W.A, W.D,
@@ -597,10 +599,10 @@ class LayeredLM:
             return {}
         out = {}
 
-        def put(name, w):
+        def put(name, w, glu=False):
             N, K = w.shape
-            if K % 16 == 0 and N % 8 == 0 and (N, K) not in {(s.N, s.K) for s in out.values()}:
-                out[f"{name}_{N}x{K}"] = GemmShape(N, K)
+            if K % 16 == 0 and N % 8 == 0 and (N, K, glu) not in {(s.N, s.K, s.glu) for s in out.values()}:
+                out[f"{name}_{N}x{K}"] = GemmShape(N, K, glu=glu)
         for L in self.w.layers:
             for mx in (L.mix, getattr(L.mix, "left", None), getattr(L.mix, "right", None)):
                 for nm in ("qc", "uq", "proj", "x", "o"):
@@ -609,7 +611,7 @@ class LayeredLM:
             for nm in ("shared_gu", "shared_down", "gu", "down"):
                 if getattr(L, "mlp", None) is not None and getattr(L.mlp, nm, None) is not None and \
                         getattr(L.mlp, nm).dim() == 2:
-                    put(nm, getattr(L.mlp, nm))
+                    put(nm, getattr(L.mlp, nm), nm == "shared_gu" and L.mlp.shared_interleaved)
         put("head", self.w.head.w)
         return out
 

@@ -570,7 +570,9 @@ class MoEWeights:
     """Experts stacked: ``gate`` / ``up`` [E, F, H] (``gate`` None: ungated experts), ``down`` [E, H, F]; ``router`` [E (+
     identity experts), H]; ``correction`` fp32 [router rows] (added to the scores for the choice only); the shared expert as
     one gate | up matrix ``shared_gu`` [2 Fs, H] (ungated: [Fs, H]) and ``shared_down`` [H, Fs]; ``bias`` fp32 [experts],
-    added to the router's logits. A shared expert behind a gate has its gate's row after the router's last one."""
+    added to the router's logits. A shared expert behind a gate has its gate's row after the router's last one.
+    ``interleaved``: ``up`` [E, 2F, H] holds gate and up rows in alternating groups of 16 (``gate`` None), for the products
+    whose epilogue applies the gated SiLU; ``shared_interleaved``: so does ``shared_gu``."""
     router: torch.Tensor
     correction: Optional[torch.Tensor]
     gate: Optional[torch.Tensor]
@@ -579,6 +581,8 @@ class MoEWeights:
     shared_gu: Optional[torch.Tensor] = None
     shared_down: Optional[torch.Tensor] = None
     bias: Optional[torch.Tensor] = None
+    interleaved: bool = False
+    shared_interleaved: bool = False
 
     def tensors(self):
         return [t for t in (self.router, self.correction, self.gate, self.up, self.down, self.shared_gu,
@@ -1706,7 +1710,9 @@ def _nolavik_finish(cfg: ModelConfig, get, device, dtype) -> ModelWeights:
     """``get(name)`` returns the checkpoint tensor of that name. Shapes are checked against the config. All input projections
     of a mixer (both branches of a pair) become one matrix; the shared expert's gate becomes the router's last row; norm
     weights, router biases and the recurrences' constants are kept in fp32."""
-    shapes = nolavik_shapes(cfg)
+    from ..ops.reference import glu_interleave
+
+    shapes, W = nolavik_shapes(cfg), cfg.hidden_size
 
     def g(name):
         t = get(name)
@@ -1754,13 +1760,20 @@ def _nolavik_finish(cfg: ModelConfig, get, device, dtype) -> ModelWeights:
         if f is not None:
             blk.norm2, blk.post2 = f32(g(p + "norm2")), f32(g(p + "norm2b"))
             q, E, sh = p + "mlp.", f.experts, f.shared is not None
+            # (the epilogue form needs bf16 rows of whole 16-byte pieces and whole groups of 16)
+            fused = [dtype == torch.bfloat16 and W % 16 == 0 and n % 16 == 0 for n in (f.expert.ff, f.shared.ff if sh else 1)]
+            gate = torch.stack([g(f"{q}e{k}.gate") for k in range(E)])
+            up = torch.stack([g(f"{q}e{k}.up") for k in range(E)])
+            sgu = None
+            if sh:
+                parts = (g(q + "shared.gate"), g(q + "shared.up"))
+                sgu = dev(glu_interleave(*parts) if fused[1] else torch.cat(parts, 0))
             blk.mlp = MoEWeights(
                 router=dev(torch.cat([g(q + "router")] + ([g(q + "shared.sg")] if sh else []), 0)), correction=None,
-                gate=dev(torch.stack([g(f"{q}e{k}.gate") for k in range(E)])),
-                up=dev(torch.stack([g(f"{q}e{k}.up") for k in range(E)])),
-                down=dev(torch.stack([g(f"{q}e{k}.down") for k in range(E)])),
-                shared_gu=dev(torch.cat([g(q + "shared.gate"), g(q + "shared.up")], 0)) if sh else None,
-                shared_down=dev(g(q + "shared.down")) if sh else None, bias=f32(g(q + "router.b")))
+                gate=None if fused[0] else dev(gate), up=dev(glu_interleave(gate, up, 1) if fused[0] else up),
+                down=dev(torch.stack([g(f"{q}e{k}.down") for k in range(E)])), shared_gu=sgu,
+                shared_down=dev(g(q + "shared.down")) if sh else None, bias=f32(g(q + "router.b")), interleaved=fused[0],
+                shared_interleaved=fused[1])
         layers.append(blk)
     vp = math.ceil(cfg.vocab_size / 16) * 16
     head = torch.zeros(vp, cfg.hidden_size, dtype=dtype, device=device)

@@ -886,6 +886,17 @@ def _mfma_ok(x, w, out_dtype) -> bool:
             and x.data_ptr() % 16 == 0 and (x.stride(0) * 2) % 16 == 0 and w.data_ptr() % 16 == 0)
 
 
+def prompt_plan(M: int, N: int, K: int):
+    """(nt_hint, split) of a prompt's product that is too narrow to fill the chip with 256 x 256 tiles: 128 x 256 tiles, K split
+    until there are about as many workgroups as compute units. (0, 0): the GEMM's own plan."""
+    if M < 2048 or -(-M // 256) * -(-N // 256) >= 192 or N < 128 or lib().gemm_tuned_get(M, N, K, False, 0) is not None:
+        return 0, 0
+    split = 1
+    while split < 4 and -(-M // 128) * -(-N // 256) * split * 2 <= 288 and K // (2 * split) >= 512:
+        split *= 2
+    return (12 | 16 | (512 if K % 64 == 0 else 0)) << 8, split
+
+
 def linear_f(x, w, out_dtype, bias=None, act="none"):
     """act(x [M, K] . w [N, K]^T + bias) -> [M, N] in ``out_dtype`` with fp32 accumulation: the MFMA GEMM where it applies
     (bias and activation in its epilogue), else the tile GEMM or the strided VALU GEMM (fp32 storage, fp32 output, odd
@@ -900,7 +911,8 @@ def linear_f(x, w, out_dtype, bias=None, act="none"):
     if M == 0:
         return torch.empty(0, N, dtype=out_dtype, device=x.device)
     if _mfma_ok(x, w, out_dtype):
-        return linear(x, w, bias, act)
+        nt, split = prompt_plan(M, N, K)
+        return linear(x, w, bias, act, nt_hint=nt, split_hint=split)
     y = torch.empty(M, N, dtype=out_dtype, device=x.device)
     gemm_any(x, w, y, M, N, K, 1, 0, x.stride(0), 0, K, 1, 0, N, bias)
     return y if act in ("none", None) else act_fn(y, act)
@@ -1090,18 +1102,23 @@ _MOE_PP = os.environ.get("LLMSS_MOE_PP", "1") != "0"  # 0: grouped products on t
 
 
 def moe_experts(h, idx, wts, gate, up, down, limit, alpha, shared=None, combine=True, act="glu_clamp",
-                weight_input=False, identity=False, shared_w=None):
+                weight_input=False, identity=False, shared_w=None, interleaved=False):
     """``identity``: indices from E on are identity experts. ``combine=False``: leave the weighting and summing to the next residual add (returns a :class:`MoEPending`).
     ``weight_input``: the weights scale the two input products in the gate / up epilogue (the experts have no
     biases), and the outputs are summed plainly (``MoEPending.wts`` is None)."""
     T, K = h.shape
     E, F, _ = up.shape
+    if interleaved:
+        _check(gate is None and act == "silu" and h.dtype == torch.bfloat16 and F % 32 == 0 and not weight_input,
+               "interleaved gate / up rows: bf16, silu, groups of 16 rows")
+        F //= 2
     N = down.shape[1]
     top = idx.shape[1]
     dt = _dt(h, "h")
     _rows(h, "h")
-    _check((gate is None) == (act == "gelu"), "experts without a gate: act gelu")
-    for t, nm, shp in ((up if gate is None else gate, "gate", (E, F, K)), (up, "up", (E, F, K)), (down, "down", (E, N, F))):
+    _check(interleaved or (gate is None) == (act == "gelu"), "experts without a gate: act gelu")
+    UF = 2 * F if interleaved else F
+    for t, nm, shp in ((up if gate is None else gate, "gate", (E, UF, K)), (up, "up", (E, UF, K)), (down, "down", (E, N, F))):
         _check(t.dtype == h.dtype and t.is_contiguous() and tuple(t.shape) == shp and t.is_cuda, f"{nm} {shp}")
     _check(idx.dtype == torch.int32 and idx.is_contiguous() and idx.shape == (T, top) and idx.is_cuda, "idx")
     _check(wts.dtype == torch.float32 and wts.is_contiguous() and wts.shape == (T, top) and wts.is_cuda, "wts")
@@ -1118,6 +1135,7 @@ def moe_experts(h, idx, wts, gate, up, down, limit, alpha, shared=None, combine=
     # rows per tile of the grouped GEMMs: 128 where the experts get enough rows to fill big tiles (bf16 only)
     rows = 128 if h.dtype == torch.bfloat16 and P >= 128 * E else 64
     # ungated experts with still more rows each: the dense GEMMs' 256x256 ping-pong kernel
+    # (gated ones with their gate and up rows interleaved, the activation in the epilogue)
     pp = (gate is None and h.dtype == torch.bfloat16 and P >= 384 * E and min(F, N) >= 256 and F % 8 == 0 and K % 8 == 0
           and h.stride(0) % 8 == 0 and not weight_input and h.data_ptr() % 16 == 0 and _MOE_PP)
     if pp:
@@ -1137,14 +1155,14 @@ def moe_experts(h, idx, wts, gate, up, down, limit, alpha, shared=None, combine=
     st = _stream()
     L.moe_group(idx.data_ptr(), P, E, maxt, meta.data_ptr(), order.data_ptr(), place.data_ptr(), rows, st)
     if pp:
-        L.moe_pp(1, h.data_ptr(), h.stride(0), up.data_ptr(), meta.data_ptr(), order.data_ptr(), act_.data_ptr(), E, maxt,
-                 top, F, K, _ACT["gelu"], st)
+        L.moe_pp(3 if interleaved else 1, h.data_ptr(), h.stride(0), up.data_ptr(), meta.data_ptr(), order.data_ptr(),
+                 act_.data_ptr(), E, maxt, top, UF, K, 0 if interleaved else _ACT["gelu"], st)
         L.moe_pp(2, act_.data_ptr(), F, down.data_ptr(), meta.data_ptr(), order.data_ptr(), y.data_ptr(), E, maxt, 1, N, F,
                  0, st)
     elif h.dtype == torch.bfloat16:  # matrix cores (csrc/gemm_tile.hip)
-        L.moe_gate_up_tile(h.data_ptr(), h.stride(0), _ptr(gate), up.data_ptr(), meta.data_ptr(),
-                           order.data_ptr(), act_.data_ptr(), E, maxt, top, F, K, float(limit), float(alpha), rows, pw,
-                           silu, st)
+        L.moe_gate_up_tile(h.data_ptr(), h.stride(0), up.data_ptr() if interleaved else _ptr(gate), up.data_ptr(),
+                           meta.data_ptr(), order.data_ptr(), act_.data_ptr(), E, maxt, top, F, K, float(limit), float(alpha),
+                           rows, pw, silu, int(interleaved), st)
         L.moe_down_tile(act_.data_ptr(), down.data_ptr(), meta.data_ptr(), y.data_ptr(), E, maxt, N, F, rows, st)
     else:
         L.moe_gate_up(h.data_ptr(), h.stride(0), _ptr(gate), up.data_ptr(), meta.data_ptr(), order.data_ptr(),
@@ -1215,7 +1233,8 @@ def stream_add_norm(x, y, mix, outw, c, inw, w, eps, rms, out_dtype):
     return h
 
 
-def causal_conv(x, w, state, cu, ctx_lens, state_slots, residual, silu, out_dtype, bias=None):
+def causal_conv(x, w, state, cu, ctx_lens, state_slots, residual, silu, out_dtype, bias=None, single=False):
+    """``single``: every sequence of the step has one row - the tails are renewed in the same launch."""
     T, C = x.shape
     _rows(x, "x")
     taps = w.shape[1]
@@ -1229,11 +1248,12 @@ def causal_conv(x, w, state, cu, ctx_lens, state_slots, residual, silu, out_dtyp
         _check(state.dim() == 3 and tuple(state.shape[1:]) == (taps - 1, C), "state [slots, taps - 1, C]")
     if bias is not None:
         _check(bias.dtype == w.dtype and bias.is_contiguous() and bias.numel() == C and bias.is_cuda, "conv bias [C]")
+    _check(not single or T == B, "single: one row per sequence")
     out = torch.empty(T, C, dtype=out_dtype, device=x.device)
     lib().causal_conv(x.data_ptr(), x.stride(0), w.data_ptr(), _ptr(state) if taps > 1 else 0, cu.data_ptr(),
                       ctx_lens.data_ptr(), state_slots.data_ptr(), out.data_ptr(), C, T, B, C, taps,
                       int(bool(residual)), int(bool(silu)), _dt(x, "x"), _dt(w, "w"), _DT[out_dtype], _ptr(bias),
-                      _stream())
+                      int(bool(single)), _stream())
     return out
 
 

@@ -618,14 +618,18 @@ def moe_router(h: torch.Tensor, router: torch.Tensor, corr: Optional[torch.Tenso
 def moe_experts(h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, gate: torch.Tensor, up: torch.Tensor,
                 down: torch.Tensor, limit: float, alpha: float, shared: Optional[torch.Tensor] = None,
                 combine: bool = True, act: str = "glu_clamp", weight_input: bool = False,
-                identity: bool = False, shared_w: Optional[torch.Tensor] = None) -> torch.Tensor:
+                identity: bool = False, shared_w: Optional[torch.Tensor] = None,
+                interleaved: bool = False) -> torch.Tensor:
     """sum_j wts[t, j] * down_e(glu(gate_e h, up_e h)) (+ shared) with e = idx[t, j] -> fp32 [T, N]. Stacked expert
     weights gate / up [E, F, K], down [E, N, F]; the activation is rounded to the storage type between the
     products, as the grouped GEMMs do. ``act`` "silu": silu(g) * u without clamps. ``weight_input``: the weight
     multiplies the expert's input instead, sum_j down_e(act(w gate_e h, w up_e h)) (experts have no biases, so the
     weight is applied to the two products). ``act`` "gelu": experts without a gate (``gate`` None), down_e(gelu(up_e
     h)), the error-function form. ``identity``: an index from E on is an
-    identity expert, its output is h[t] itself. ``shared_w`` fp32 [T] multiplies the shared rows."""
+    identity expert, its output is h[t] itself. ``shared_w`` fp32 [T] multiplies the shared rows.
+    ``interleaved`` (``gate`` None): up [E, 2F, K] holds gate and up rows in alternating groups of 16."""
+    if interleaved:
+        gate, up = glu_split(up, 1)
     T = h.shape[0]
     N = down.shape[1]
     out = torch.zeros(T, N, dtype=torch.float32, device=h.device)
@@ -681,11 +685,12 @@ def stream_add_norm(x, y, mix, outw, c: float, inw, w, eps: float, rms: bool, ou
     return (u * torch.rsqrt(u.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
 
 
-def causal_conv(x, w, state, cu, ctx_lens, state_slots, residual: bool, silu: bool, out_dtype, bias=None):
+def causal_conv(x, w, state, cu, ctx_lens, state_slots, residual: bool, silu: bool, out_dtype, bias=None,
+                single: bool = False):
     """Per-channel causal convolution over time of x [T, C] with w [C, taps] (last column: the current row), each
     sequence continuing from the taps - 1 inputs in its state slot (state fp32 [slots, taps - 1, C], renewed here;
     a portion starting at position 0 reads zeros). ``residual`` adds x itself; ``bias`` [C] is added to every row;
-    ``silu`` applies x * sigmoid(x)."""
+    ``silu`` applies x * sigmoid(x). ``single`` (every sequence has one row) only steers the GPU kernels."""
     T, C = x.shape
     taps = w.shape[1]
     R = taps - 1

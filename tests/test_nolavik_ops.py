@@ -106,6 +106,63 @@ def test_shared_expert_behind_a_gate(device, dtype, E, top, W, F, T):
     close(got, oracle.rms(xw, eps) * nxt, dtype, "next input")
 
 
+@pytest.mark.parametrize("device,dtype", [RUNS[0], RUNS[2]])
+@pytest.mark.parametrize("E,top,W,F,T", [(4, 2, 48, 32, 11), (3, 1, 64, 16, 700), (2, 2, 264, 272, 900), (3, 2, 256, 320, 1500)])
+def test_experts_with_interleaved_gate_and_up_rows(device, dtype, E, top, W, F, T):
+    """The layout whose epilogue applies the gated SiLU, from single rows to hundreds per expert (the larger cases run the
+    256-row products), one expert nobody chooses."""
+    h = rnd(T, W, seed=1, dtype=dtype)
+    gate, up = (rnd(E, F, W, seed=s, dtype=dtype, mul=W ** -0.5) for s in (2, 3))
+    down = rnd(E, W, F, seed=4, dtype=dtype, mul=F ** -0.5)
+    g = torch.Generator().manual_seed(5)
+    idx = torch.stack([torch.randperm(E, generator=g)[:top] for _ in range(T)])
+    if top == 1:
+        idx[idx == 1] = 0
+    w = torch.rand(T, top, generator=g).double()
+    want = torch.zeros(T, W, dtype=F64)
+    for e in range(E):
+        share = torch.where(idx == e, w, torch.zeros_like(w)).sum(-1, keepdim=True)
+        want += share * ((oracle.silu(h @ gate[e].T) * (h @ up[e].T)) @ down[e].T)
+    gu = ops.glu_interleave(gate, up, 1)
+    assert torch.equal(gu[:, :16], gate[:, :16]) and torch.equal(gu[:, 16:32], up[:, :16])
+    got = ops.moe_experts(to(h, device, dtype), i32(idx.tolist(), device), to(w, device), None, to(gu, device, dtype),
+                          to(down, device, dtype), 0.0, 0.0, act="silu", interleaved=True)
+    close(got, want, dtype, "experts")
+
+
+@pytest.mark.parametrize("device,dtype", [RUNS[0], RUNS[2]])
+@pytest.mark.parametrize("M,N,K", [(2048, 160, 1024), (2100, 1000, 192), (4096, 136, 2064), (2048, 512, 64), (3000, 96, 128)])
+def test_narrow_products_of_long_prompts(device, dtype, M, N, K):
+    x, w = rnd(M, K, seed=1, dtype=dtype), rnd(N, K, seed=2, dtype=dtype, mul=K ** -0.5)
+    for out in (dtype, torch.float32):
+        close(ops.linear_f(to(x, device, dtype), to(w, device, dtype), out), x @ w.T, dtype, f"product to {out}")
+
+
+# ------------------------------------------------------------------------------------------------- convolution
+@pytest.mark.parametrize("device,dtype", RUNS)
+@pytest.mark.parametrize("C,taps", [(40, 4), (7, 1), (264, 2), (1032, 6)])
+def test_convolution_of_single_rows_renews_its_tail(device, dtype, C, taps):
+    """Decode steps, where one launch forms the rows and renews the tails, against the portions' form; a slot that held
+    something else; a padded row."""
+    x, w, b = rnd(30, C, seed=1, dtype=dtype), rnd(C, taps, seed=2, dtype=dtype, mul=taps ** -0.5), rnd(C, seed=3, dtype=dtype)
+    want = oracle.silu(oracle.causal_conv(x, w, b))
+    for first in (0, 1, 17):
+        tail = torch.full((3, taps - 1, C), 9.0, device=device)
+        got = []
+        for p0, n in ([(0, first)] if first else []) + [(p, 1) for p in range(first, 30)]:
+            one = n == 1
+            rows = to(x[p0:p0 + n], device, dtype)
+            cu, ctx, ss = [0, n], [p0 + n], [1]
+            if one:  # a padded row rides along
+                rows = torch.cat([rows, rows])
+                cu, ctx, ss = [0, 1, 2], [p0 + 1, 0], [1, -1]
+            y = ops.causal_conv(rows, to(w, device, dtype), tail, i32(cu, device), i32(ctx, device), i32(ss, device), False, True,
+                                dtype, bias=to(b, device, dtype), single=one)
+            got.append(y[:n])
+        close(torch.cat(got), want, dtype, f"after {first} rows")
+        assert bool((tail[0] == 9.0).all()) and bool((tail[2] == 9.0).all())
+
+
 # ------------------------------------------------------------------------------------------------- rotation
 @pytest.mark.parametrize("dims,base,scaling", [(8, 1000.0, None), (32, 1e6, dict(factor=8.0, low=1.0, high=4.0, original=256)),
                                                (64, 500.0, dict(factor=3.0, low=2.0, high=2.5, original=90)),
