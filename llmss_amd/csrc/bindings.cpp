@@ -105,6 +105,9 @@ void launch_moe_route(const void* z, const void* corr, void* idx, void* wts, int
                       int smax, const void* zb, void* sg, hipStream_t st);
 void launch_moe_router(const void* h, int64_t ldh, const void* wr, const void* corr, void* idx, void* wts, int T_,
                        int E, int K, int top, int dt, int norm, int smax, const void* zb, void* sg, hipStream_t st);
+bool moe_router_mfma_ok(int E, int gate, int K);
+void launch_moe_router_mfma(const void* h, int64_t ldh, const void* wr, const void* corr, void* idx, void* wts, int T_,
+                            int E, int K, int top, int norm, int smax, const void* zb, void* sg, hipStream_t st);
 void launch_moe_group(const void* idx, int P, int E, int maxt, void* meta, void* order, void* place, int tile_rows,
                       hipStream_t st);
 void launch_moe_gate_up(const void* h, int64_t ldh, const void* wg, const void* wu, const void* meta,
@@ -424,6 +427,11 @@ PYBIND11_MODULE(_C, m) {
   m.def("moe_router", [](uintptr_t h, int64_t ldh, uintptr_t wr, uintptr_t corr, uintptr_t idx, uintptr_t wts, int T,
                          int E, int K, int top, int dt, int norm, int smax, uintptr_t zb, uintptr_t sg, uintptr_t st) {
     launch_moe_router(CP(h), ldh, CP(wr), CP(corr), P(idx), P(wts), T, E, K, top, dt, norm, smax, CP(zb), P(sg), S(st));
+  });
+  m.def("moe_router_mfma_ok", &moe_router_mfma_ok);
+  m.def("moe_router_mfma", [](uintptr_t h, int64_t ldh, uintptr_t wr, uintptr_t corr, uintptr_t idx, uintptr_t wts, int T,
+                              int E, int K, int top, int norm, int smax, uintptr_t zb, uintptr_t sg, uintptr_t st) {
+    launch_moe_router_mfma(CP(h), ldh, CP(wr), CP(corr), P(idx), P(wts), T, E, K, top, norm, smax, CP(zb), P(sg), S(st));
   });
   m.def("moe_group", [](uintptr_t idx, int Pn, int E, int maxt, uintptr_t meta, uintptr_t order, uintptr_t place,
                         int tile_rows, uintptr_t st) {

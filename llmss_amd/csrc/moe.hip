@@ -36,16 +36,75 @@ __device__ __forceinline__ float glu_value(float g, float u, float limit, float 
 }
 
 // ------------------------------------------------------------------------------------------------ routing
+// A wave routes one token of up to 128 outputs: lane e holds the logits of e and e + 64 (bias added; -inf past the last); an
+// output's rank among all choice values (ties: the lower index first) says whether and where it is chosen. row: LDS, 16-byte
+// aligned, room for the outputs in whole fours.
+__device__ __forceinline__ void route_ranked(float (&sc)[2], float* row, const float* __restrict__ corr, int* __restrict__ idx,
+                                             float* __restrict__ wts, int E, int top, int norm, int smax) {
+  const int lane = threadIdx.x & 63;
+  float ch[2];
+  float mx = -INFINITY, den = 0.f;
+  if (smax) mx = warp_max(fmaxf(sc[0], sc[1]));
+  if (smax == 1) {
+#pragma unroll
+    for (int j = 0; j < 2; ++j) den += lane + 64 * j < E ? expf(sc[j] - mx) : 0.f;
+    den = warp_sum(den);
+  }
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int e = lane + 64 * j;
+    if (smax != 2 && e < E) sc[j] = smax ? expf(sc[j] - mx) / den : 1.f / (1.f + expf(-sc[j]));
+    ch[j] = e < E ? sc[j] + (corr ? corr[e] : 0.f) : -INFINITY;
+    if (!(ch[j] == ch[j])) ch[j] = -INFINITY;  // (a NaN ranks last: the ranks stay a permutation)
+    if (e < ((E + 3) & ~3)) row[e] = ch[j];
+  }
+  __builtin_amdgcn_wave_barrier();
+  __threadfence_block();
+  int rank[2] = {0, 0};
+  for (int e0 = 0; e0 < E; e0 += 4) {
+    const f32x4 o = *reinterpret_cast<const f32x4*>(row + e0);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      if (e0 + i >= E) continue;
+#pragma unroll
+      for (int j = 0; j < 2; ++j) rank[j] += o[i] > ch[j] || (o[i] == ch[j] && e0 + i < lane + 64 * j) ? 1 : 0;
+    }
+  }
+  float sum = 0.f;
+  bool in[2];
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    in[j] = lane + 64 * j < E && rank[j] < top;
+    if (smax == 2) sc[j] = expf(sc[j] - mx);  // (the largest is always chosen)
+    sum += in[j] ? sc[j] : 0.f;
+  }
+  sum = warp_sum(sum);
+  const float inv = smax == 2 ? 1.f / sum : norm ? 1.f / (sum + 1e-20f) : 1.f;
+#pragma unroll
+  for (int j = 0; j < 2; ++j)
+    if (in[j]) {
+      idx[rank[j]] = lane + 64 * j;
+      wts[rank[j]] = sc[j] * inv;
+    }
+}
+
 // one wave per token; lanes over experts
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ z, const float* __restrict__ corr,
                                                        int* __restrict__ idx, float* __restrict__ wts, int E, int top,
                                                        int norm, int smax, const float* __restrict__ zb,
                                                        float* __restrict__ sg) {
-  extern __shared__ float sc[];  // [E] scores, [E] choice values
+  extern __shared__ __attribute__((aligned(16))) float sc[];  // [E] scores, [E] choice values
   float* ch = sc + E;
   const int t = blockIdx.x, lane = threadIdx.x;
   const float* zr = z + (int64_t)t * (E + (sg ? 1 : 0));
   if (sg && lane == 0) sg[t] = 1.f / (1.f + expf(-zr[E]));
+  if (E <= 128) {
+    float v[2];
+#pragma unroll
+    for (int j = 0; j < 2; ++j) v[j] = lane + 64 * j < E ? zr[lane + 64 * j] + (zb ? zb[lane + 64 * j] : 0.f) : -INFINITY;
+    route_ranked(v, sc, corr, idx + (int64_t)t * top, wts + (int64_t)t * top, E, top, norm, smax);
+    return;
+  }
   float mx = 0.f, den = 1.f;
   if (smax == 1) {
     mx = -INFINITY, den = 0.f;
@@ -104,7 +163,7 @@ void launch_moe_route(const void* z, const void* corr, void* idx, void* wts, int
                       int smax, const void* zb, void* sg, hipStream_t st) {
   if (T_ == 0) return;
   if (top > E || top <= 0) throw std::runtime_error("moe_route: top must be in [1, experts]");
-  moe_route_kernel<<<T_, 64, 2 * E * sizeof(float), st>>>((const float*)z, (const float*)corr, (int*)idx, (float*)wts,
+  moe_route_kernel<<<T_, 64, (2 * E + 4) * sizeof(float), st>>>((const float*)z, (const float*)corr, (int*)idx, (float*)wts,
                                                            E, top, norm, smax, (const float*)zb, (float*)sg);
   HIP_CHECK_LAUNCH();
 }
@@ -118,8 +177,9 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ 
                                                          float* __restrict__ wts, int E, int K, int top, bool vec,
                                                          int norm, int smax, const float* __restrict__ zb,
                                                          float* __restrict__ sg) {
-  extern __shared__ float sc[];  // [E] scores, [E] choice values
+  extern __shared__ __attribute__((aligned(16))) float sc[];  // [E] scores, [E] choice values
   float* ch = sc + E;
+  const bool ranked = E <= 128;
   const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, nw = blockDim.x >> 6;
   const T* x = h + (int64_t)t * ldh;
   for (int e = wv; e < E + (sg ? 1 : 0); e += nw) {
@@ -146,12 +206,25 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const T* __restrict__ 
         continue;
       }
       if (zb) acc += zb[e];
+      if (ranked) {
+        sc[e] = acc;
+        continue;
+      }
       const float s = smax ? acc : 1.f / (1.f + expf(-acc));
       sc[e] = s;
       ch[e] = s + (corr ? corr[e] : 0.f);
     }
   }
   __syncthreads();
+  if (ranked) {
+    if (wv) return;
+    float v[2];
+#pragma unroll
+    for (int j = 0; j < 2; ++j) v[j] = lane + 64 * j < E ? sc[lane + 64 * j] : -INFINITY;
+    __builtin_amdgcn_wave_barrier();
+    route_ranked(v, sc, corr, idx + (int64_t)t * top, wts + (int64_t)t * top, E, top, norm, smax);
+    return;
+  }
   if (smax == 1) {  // sc holds the logits: every wave forms their maximum and sum, then the scores replace them
     float mx = -INFINITY, den = 0.f;
     for (int e = lane; e < E; e += 64) mx = fmaxf(mx, sc[e]);
@@ -213,9 +286,103 @@ void launch_moe_router(const void* h, int64_t ldh, const void* wr, const void* c
   const int es = dt == 0 ? 2 : 4;
   const bool vec = K % 8 == 0 && ((uintptr_t)h % 16) == 0 && ((uintptr_t)wr % 16) == 0 && (ldh * es) % 16 == 0;
   const int threads = E >= 16 ? 1024 : (E >= 8 ? 512 : 256);  // a wave per expert up to 16 waves
-  DISPATCH_T(dt, T, (moe_router_kernel<T><<<T_, threads, 2 * E * sizeof(float), st>>>(
+  DISPATCH_T(dt, T, (moe_router_kernel<T><<<T_, threads, (2 * E + 4) * sizeof(float), st>>>(
                         (const T*)h, ldh, (const T*)wr, (const float*)corr, (int*)idx, (float*)wts, E, K, top, vec,
                         norm, smax, (const float*)zb, (float*)sg)));
+  HIP_CHECK_LAUNCH();
+}
+
+// The same for bf16 rows on the matrix cores, at any number of rows: a workgroup takes 16 tokens and all outputs (up to 16 *
+// MR_NT), its eight waves an eighth of K each (fragments straight from memory: lane (li, g) holds k = 8 g .. 8 g + 7 of row li);
+// the parts meet in LDS and every wave routes two of the tokens, a score per lane (lane e: outputs e, e + 64) whose rank among
+// all decides whether and where it is chosen.
+#define MR_NT 8
+template <int NT>
+__global__ __launch_bounds__(512) void moe_router_mfma_kernel(const bf16_t* __restrict__ h, int64_t ldh,
+                                                              const bf16_t* __restrict__ wr, const float* __restrict__ corr,
+                                                              int* __restrict__ idx, float* __restrict__ wts, int T_, int E,
+                                                              int K, int top, int norm, int smax,
+                                                              const float* __restrict__ zb, float* __restrict__ sg) {
+  constexpr int LD = 16 * NT + 4;
+  __shared__ __attribute__((aligned(16))) float part[4][16][LD];
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, li = lane & 15, g = lane >> 4;
+  const int t0 = blockIdx.x * 16, EG = E + (sg ? 1 : 0);
+  f32x4 acc[NT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const bf16_t* a = h + (int64_t)min(t0 + li, T_ - 1) * ldh + 8 * g;
+  const bf16_t* b[NT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) b[j] = wr + (int64_t)min(16 * j + li, EG - 1) * K + 8 * g;
+  const int ks = K / 32;  // (neighbouring waves take neighbouring steps: the halves of a 128-byte line meet in the cache)
+  constexpr int U = NT <= 4 ? 8 : 4;  // steps whose loads are in flight together
+  for (int k0 = w; k0 < ks; k0 += 8 * U) {  // (K a multiple of 32; steps past the end repeat the last one with a zero row)
+    s16x8 av[U], bv[U][NT];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int k = min(k0 + 8 * u, ks - 1);
+      av[u] = *reinterpret_cast<const s16x8*>(a + 32 * k);
+#pragma unroll
+      for (int j = 0; j < NT; ++j) bv[u][j] = *reinterpret_cast<const s16x8*>(b[j] + 32 * k);
+    }
+    __builtin_amdgcn_sched_barrier(0);  // all loads are issued before the first product waits for one
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      if (k0 + 8 * u >= ks) av[u] = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+      for (int j = 0; j < NT; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(av[u], bv[u][j], acc[j], 0, 0, 0);
+    }
+  }
+  if (w >= 4) {
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) part[w - 4][4 * g + i][16 * j + li] = acc[j][i];
+  }
+  __syncthreads();
+  if (w < 4) {
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) part[w][4 * g + i][16 * j + li] += acc[j][i];
+  }
+  __syncthreads();
+  auto z_of = [&](int r, int e) { return (part[0][r][e] + part[1][r][e]) + (part[2][r][e] + part[3][r][e]); };
+  for (int r = 2 * w; r < 2 * w + 2; ++r) {
+    const int64_t t = t0 + r;
+    if (t >= T_) return;
+    float sc[2];
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      const int e = lane + 64 * j;
+      sc[j] = e < E ? z_of(r, e) + (zb ? zb[e] : 0.f) : -INFINITY;
+    }
+    if (sg && lane == 0) sg[t] = 1.f / (1.f + expf(-z_of(r, E)));
+    __builtin_amdgcn_wave_barrier();
+    route_ranked(sc, &part[0][r][0], corr, idx + t * top, wts + t * top, E, top, norm, smax);  // (the row is this wave's alone)
+  }
+}
+
+// may a router of E outputs (+ gate) over bf16 rows of K numbers take the matrix-core form?
+bool moe_router_mfma_ok(int E, int gate, int K) { return E + (gate ? 1 : 0) <= 16 * MR_NT && E <= 128 && K % 32 == 0; }
+
+void launch_moe_router_mfma(const void* h, int64_t ldh, const void* wr, const void* corr, void* idx, void* wts, int T_,
+                            int E, int K, int top, int norm, int smax, const void* zb, void* sg, hipStream_t st) {
+  if (T_ == 0) return;
+  if (top > E || top <= 0) throw std::runtime_error("moe_router: top must be in [1, experts]");
+  if (!moe_router_mfma_ok(E, sg != nullptr, K) || (((uintptr_t)h | (uintptr_t)wr) & 15) || ldh % 8)
+    throw std::runtime_error("moe_router: shape of the matrix-core form");
+#define LAUNCH_MR(NT_)                                                                                                      \
+  moe_router_mfma_kernel<NT_><<<(T_ + 15) / 16, 512, 0, st>>>((const bf16_t*)h, ldh, (const bf16_t*)wr, (const float*)corr, \
+                                                              (int*)idx, (float*)wts, T_, E, K, top, norm, smax,            \
+                                                              (const float*)zb, (float*)sg)
+  const int nt = (E + (sg ? 1 : 0) + 15) / 16;
+  if (nt <= 1) LAUNCH_MR(1);
+  else if (nt <= 2) LAUNCH_MR(2);
+  else if (nt <= 3) LAUNCH_MR(3);
+  else if (nt <= 5) LAUNCH_MR(5);
+  else LAUNCH_MR(MR_NT);
+#undef LAUNCH_MR
   HIP_CHECK_LAUNCH();
 }
 

@@ -310,10 +310,73 @@ __global__ __launch_bounds__(256) void conv_tail_kernel(const TI* __restrict__ i
     if (i < R) state[((int64_t)slot * R + i) * C + c] = nv[i];
 }
 
+// A step of single rows (row t belongs to sequence t): the row and the renewed tail in one pass, four channels per thread, every
+// load in flight together
+template <typename TI, typename TW, typename TO, int RMAX>
+__global__ __launch_bounds__(256) void causal_conv_step_kernel(const TI* __restrict__ in, int64_t ldi,
+                                                               const TW* __restrict__ w, float* __restrict__ state,
+                                                               const int* __restrict__ ctx, const int* __restrict__ sslots,
+                                                               TO* __restrict__ out, int64_t ldo, int C, int taps, int res,
+                                                               int silu, const TW* __restrict__ bias) {
+  const int t = blockIdx.x, c = (blockIdx.y * blockDim.x + threadIdx.x) * 4;
+  if (c >= C) return;
+  const int R = taps - 1, pos = ctx[t] - 1, slot = sslots[t];
+  TO* o = out + (int64_t)t * ldo + c;
+  float acc[4] = {0.f, 0.f, 0.f, 0.f};
+  if (pos < 0 || slot < 0) {
+    conv_st<TO, 4>(o, acc);
+    return;
+  }
+  float x[4], old[RMAX][4], wv[RMAX + 1][4], bv[4];
+  float* tail = state + (int64_t)slot * R * C + c;  // [i] holds position pos - R + i
+  conv_ld<TI, 4>(in + (int64_t)t * ldi + c, x);
+#pragma unroll
+  for (int i = 0; i < RMAX; ++i) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) old[i][e] = 0.f;
+    if (i < R && pos - R + i >= 0) conv_ld<float, 4>(tail + (int64_t)i * C, old[i]);
+  }
+#pragma unroll
+  for (int k = 0; k <= RMAX; ++k)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) wv[k][e] = k <= R ? El<TW>::ld(w + (int64_t)(c + e) * taps + k) : 0.f;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) bv[e] = bias ? El<TW>::ld(bias + c + e) : 0.f;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    float a = res ? x[e] : 0.f;
+#pragma unroll
+    for (int k = 0; k < RMAX; ++k) a = fmaf(wv[k][e], k < R ? old[k][e] : 0.f, a);
+#pragma unroll
+    for (int k = 0; k <= RMAX; ++k)
+      if (k == R) a = fmaf(wv[k][e], x[e], a);
+    a += bv[e];
+    acc[e] = silu ? a * sigm<TO>(a) : a;
+  }
+  conv_st<TO, 4>(o, acc);
+#pragma unroll
+  for (int i = 0; i < RMAX; ++i) {
+    if (i + 1 < R) conv_st<float, 4>(tail + (int64_t)i * C, i + 1 < RMAX ? old[i + 1 < RMAX ? i + 1 : i] : x);
+    else if (i + 1 == R) conv_st<float, 4>(tail + (int64_t)i * C, x);
+  }
+}
+
 template <typename TI, typename TW, typename TO>
 static void causal_conv_t(const void* in, int64_t ldi, const void* w, void* state, const void* cu, const void* ctx,
                           const void* sslots, void* out, int64_t ldo, int T_, int B, int C, int taps, int res,
                           int silu, const void* bias, int single, hipStream_t st) {
+  const auto al16_ = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+  if (single && taps <= 9 && C % 4 == 0 && ldi % 4 == 0 && ldo % 4 == 0 && al16_(in) && al16_(out) && al16_(state)) {
+    dim3 gs(T_, (C / 4 + 255) / 256);
+#define LAUNCH_STEP(RMAX_)                                                                                       \
+  causal_conv_step_kernel<TI, TW, TO, RMAX_><<<gs, 256, 0, st>>>((const TI*)in, ldi, (const TW*)w, (float*)state, \
+                                                                 (const int*)ctx, (const int*)sslots, (TO*)out, ldo, C, taps, \
+                                                                 res, silu, (const TW*)bias)
+    if (taps <= 4) LAUNCH_STEP(3);
+    else LAUNCH_STEP(8);
+#undef LAUNCH_STEP
+    return;
+  }
   if (!single && T_ >= 256 && T_ >= 8 * B && taps <= 9) {  // portions of eight rows and more on average
     const auto al16 = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
     const bool four = C % 4 == 0 && ldi % 4 == 0 && ldo % 4 == 0 && al16(in) && al16(out) && al16(state);

@@ -115,11 +115,11 @@ class LatentAttention:
         if nd and nd < qa.shape[0]:
             # mixed step: the single-token rows take the decode form of the kernel (their keys split over
             # workgroups), the portions the prompt form - as DecoderLM sends its decode rows to the decode kernel
-            o = torch.cat([
-                ops.latent_attn(qa[:nd], cache, inp.block_tables[:nd], model.decode_cu(nd, qa.device),
-                                inp.ctx_lens[:nd], spec.window, spec.scale, max_qlen=1, max_ctx=inp.max_ctx),
-                ops.latent_attn(qa[nd:], cache, inp.block_tables[nd:], inp.cu_seqlens, inp.ctx_lens[nd:],
-                                spec.window, spec.scale, max_qlen=max(1, inp.max_seqlen))])
+            o = torch.empty_like(qa)
+            ops.latent_attn(qa[:nd], cache, inp.block_tables[:nd], model.decode_cu(nd, qa.device), inp.ctx_lens[:nd],
+                            spec.window, spec.scale, max_qlen=1, max_ctx=inp.max_ctx, out=o[:nd])
+            ops.latent_attn(qa[nd:], cache, inp.block_tables[nd:], inp.cu_seqlens, inp.ctx_lens[nd:], spec.window, spec.scale,
+                            max_qlen=max(1, inp.max_seqlen), out=o[nd:])
         else:
             single = inp.kind == "decode" or (nd and nd == qa.shape[0])
             o = ops.latent_attn(qa, cache, inp.block_tables, cu, inp.ctx_lens, spec.window, spec.scale,

@@ -1015,7 +1015,7 @@ def latent_key_split(B: int, window: int, max_ctx: int):
     return -(-tiles // per), per * 64
 
 
-def latent_attn(qa, cache, block_tables, cu_q, ctx_lens, window, scale, max_qlen=0, max_ctx=0):
+def latent_attn(qa, cache, block_tables, cu_q, ctx_lens, window, scale, max_qlen=0, max_ctx=0, out=None):
     """``qa`` [T, H, R]. bf16 queries over a bf16 cache of rank 64 / 128 / 256 run the MFMA extend kernel as
     multi-query attention whose one key/value head is the latent row (keys = values = cache, bf16 output); anything
     else runs the generic kernel (fp32 queries, fp32 output)."""
@@ -1030,12 +1030,14 @@ def latent_attn(qa, cache, block_tables, cu_q, ctx_lens, window, scale, max_qlen
         _check(latent_qa_dtype(cache) == torch.bfloat16 and max_qlen > 0, "bf16 queries: MFMA ranks and max_qlen only")
         kv = cache.view(cache.shape[0], 1, cache.shape[1], R)  # [blocks, one kv head, block_size, R]
         split = latent_key_split(T, window, max_ctx) if max_qlen == 1 and T == B and max_ctx > 0 else None
-        out = attn_extend(qa.view(T, H * R), kv, kv, block_tables, cu_q, ctx_lens[:B], max_qlen, H, 1, R, scale,
-                          window=window, key_split=split)
-        return out.view(T, H, R)
+        o = attn_extend(qa.view(T, H * R), kv, kv, block_tables, cu_q, ctx_lens[:B], max_qlen, H, 1, R, scale,
+                        window=window, key_split=split, out=None if out is None else out.view(T, H * R))
+        return o.view(T, H, R)
     _check(qa.dtype == torch.float32, "qa fp32")
     _check(R <= 1024, "latent rank above 1024")
-    out = torch.empty(T, H, R, dtype=torch.float32, device=qa.device)
+    if out is None:
+        out = torch.empty(T, H, R, dtype=torch.float32, device=qa.device)
+    _check(out.dtype == torch.float32 and out.is_contiguous() and tuple(out.shape) == (T, H, R), "out fp32 [T, H, R]")
     lib().latent_attn(qa.data_ptr(), H * R, cache.data_ptr(), block_tables.data_ptr(), block_tables.shape[1],
                       cu_q.data_ptr(), ctx_lens.data_ptr(), out.data_ptr(), H * R, T, B, H, R, cache.shape[1],
                       int(window), float(scale), _dt(cache, "cache"), _stream())
@@ -1076,23 +1078,31 @@ def moe_route(z, corr, top, normalize=True, score="sigmoid", bias=None, gate=Fal
     return (idx, wts, sg) if gate else (idx, wts)
 
 
+ROUTER_MFMA_MIN_ROWS = 256  # from here on a workgroup per token reads the router's weights too often
 ROUTER_FUSED_MAX_ROWS = 1024  # steps of at most this many tokens compute logits and routing in one launch
 
 
 def moe_router(h, router, corr, top, normalize=True, score="sigmoid", bias=None, gate=False):
     """(idx [T, top] int32, wts [T, top] fp32(, gate fp32 [T])) from the layer input: fp32 router logits, then moe_route. Few
-    rows (a decode step): one fused launch; a prompt: the matrix-core GEMM with fp32 output, then moe_route."""
+    rows (a decode step): one fused launch, a workgroup per token; a prompt of bf16 rows and up to 128 outputs: one launch on
+    the matrix cores, 16 tokens per workgroup; else the matrix-core GEMM with fp32 output, then moe_route."""
     T, K = h.shape
     E = router.shape[0] - int(bool(gate))
-    if T > ROUTER_FUSED_MAX_ROWS:
-        return moe_route(linear_f(h, router, torch.float32), corr, top, normalize, score, bias, gate)
     _rows(h, "h")
+    mfma = (h.dtype == torch.bfloat16 and T > ROUTER_MFMA_MIN_ROWS and lib().moe_router_mfma_ok(E, int(bool(gate)), K) and h.data_ptr() % 16 == 0
+            and h.stride(0) % 8 == 0 and router.data_ptr() % 16 == 0)
+    if T > ROUTER_FUSED_MAX_ROWS and not mfma:
+        return moe_route(linear_f(h, router, torch.float32), corr, top, normalize, score, bias, gate)
     _check(router.dtype == h.dtype and router.is_contiguous() and router.shape[1] == K and router.is_cuda,
            "router [E (+ 1), K] in h's storage type")
     _route_args(E, top, corr, bias, score)
     idx = torch.empty(T, top, dtype=torch.int32, device=h.device)
     wts = torch.empty(T, top, dtype=torch.float32, device=h.device)
     sg = torch.empty(T, dtype=torch.float32, device=h.device) if gate else None
+    if mfma:
+        lib().moe_router_mfma(h.data_ptr(), h.stride(0), router.data_ptr(), _ptr(corr), idx.data_ptr(), wts.data_ptr(), T, E, K,
+                              top, int(bool(normalize)), _SCORE[score], _ptr(bias), _ptr(sg), _stream())
+        return (idx, wts, sg) if gate else (idx, wts)
     lib().moe_router(h.data_ptr(), h.stride(0), router.data_ptr(), _ptr(corr), idx.data_ptr(), wts.data_ptr(), T, E, K,
                      top, _dt(h, "h"), int(bool(normalize)), _SCORE[score], _ptr(bias), _ptr(sg), _stream())
     return (idx, wts, sg) if gate else (idx, wts)

@@ -547,13 +547,13 @@ def rope_angles(positions: torch.Tensor, freqs: torch.Tensor) -> torch.Tensor:
 
 
 def latent_attn(qa: torch.Tensor, cache: torch.Tensor, block_tables, cu_q, ctx_lens, window: int,
-                scale: float, max_qlen: int = 0, max_ctx: int = 0) -> torch.Tensor:
+                scale: float, max_qlen: int = 0, max_ctx: int = 0, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Multi-query attention whose keys and values are the cached latent rows (csrc/attention_latent.hip):
     qa fp32 [T, H, R]; sequence b's rows cu_q[b]:cu_q[b+1] sit at positions ctx_lens[b] - qlen .. ctx_lens[b] - 1
     and see the positions j with 0 <= i - j (< window when window > 0). Returns fp32 [T, H, R]."""
     T, H, R = qa.shape
     bs = cache.shape[1]
-    out = torch.zeros(T, H, R, dtype=torch.float32, device=qa.device)
+    out = torch.zeros(T, H, R, dtype=torch.float32, device=qa.device) if out is None else out.zero_()
     cu = [int(c) for c in cu_q.tolist()]
     for b in range(len(cu) - 1):
         a, e = cu[b], cu[b + 1]

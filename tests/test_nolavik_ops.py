@@ -51,9 +51,10 @@ def test_closing_op_sums_two_mixers_with_scales(device, dtype, W):
 
 # ------------------------------------------------------------------------------------------------- experts
 @pytest.mark.parametrize("device,dtype", RUNS)
-@pytest.mark.parametrize("E,top,gate", [(4, 2, True), (3, 3, True), (6, 1, False), (70, 5, True), (1, 1, True), (20, 7, False)])
-def test_router_weighs_the_chosen_logits_alone(device, dtype, E, top, gate):
-    T, W = 13, 40
+@pytest.mark.parametrize("W,T", [(40, 13), (64, 300), (288, 259)])  # (many rows of whole 32s: the matrix cores take bf16)
+@pytest.mark.parametrize("E,top,gate", [(4, 2, True), (3, 3, True), (6, 1, False), (70, 5, True), (1, 1, True), (20, 7, False),
+                                        (128, 9, False), (127, 70, True)])
+def test_router_weighs_the_chosen_logits_alone(device, dtype, E, top, gate, W, T):
     h, rw = rnd(T, W, seed=1, dtype=dtype), rnd(E + gate, W, seed=2, dtype=dtype, mul=2 * W ** -0.5)
     bias = rnd(E, seed=3, mul=2.0)
     bias[0] += 100.0  # a logit far above the others: weights of the rest vanish, and its own logit alone must not overflow
