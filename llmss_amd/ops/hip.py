@@ -1007,10 +1007,11 @@ def latent_qa_dtype(cache) -> torch.dtype:
 
 def latent_key_split(B: int, window: int, max_ctx: int):
     """(nsplit, keys per split) for a decode step of B single-token rows whose visible range is at most
-    min(window, max_ctx) keys: about 1024 workgroups in flight, whole 64-key tiles per split."""
+    min(window, max_ctx) keys: about 512 workgroups, whole 64-key tiles per split (more splits write and read more partial
+    rows than their shorter key walks save)."""
     keys = min(window, max_ctx) if window > 0 else max_ctx
     tiles = -(-keys // 64) + (1 if window > 0 else 0)  # a window may straddle one more tile
-    nsplit = max(1, min(tiles, 1024 // max(1, B)))
+    nsplit = max(1, min(tiles, 512 // max(1, B)))
     per = -(-tiles // nsplit)
     return -(-tiles // per), per * 64
 
